@@ -1,8 +1,9 @@
 /*
  * wr_hip_mix.h — C ABI of the device steps of mixer-stack models: models whose
- * layers pair a mixer (decayed linear attention, or sliding-window attention
- * through a low-rank latent) with a feed-forward (dense or a mixture of
- * experts), each between norms, with bfloat16 weights.
+ * layers pair a mixer (decayed linear attention, sliding-window attention through
+ * a low-rank latent or over grouped keys and values, a matrix-state recurrence
+ * with input-made decays) with a feed-forward (dense or a mixture of experts),
+ * with norms before and, in some designs, after each, and bfloat16 weights.
  *
  * Conventions are those of wr_hip_attn.h: plain C, status returns, every call
  * enqueues on the calling thread's stream and returns without waiting unless it
@@ -37,6 +38,7 @@ extern "C" {
 #define WR_HIP_MIX_MAX_EXPERTS 1024u
 #define WR_HIP_MIX_MAX_TOP     64u
 #define WR_HIP_MIX_MAX_STATE_DIM 512u /* rows of a recurrent state matrix */
+#define WR_HIP_MIX_MAX_RECUR_DIM 256u /* head size of wr_hip_mix_recur */
 
 /* 1 when this build of the library runs mixer-stack models. */
 int wr_hip_mix_available(void);
@@ -51,8 +53,8 @@ void wr_hip_mix_mat_destroy(wr_hip_mat *w);
 
 /* ---- cache pool ----------------------------------------------------------
  * One pool per model, shared by its requests: `n_pages` pages of 64 positions
- * for each of `n_latent` attention layer runs (row of latent_dim[i] elements, a
- * multiple of 32) and `n_slots` state slots for each of `n_state` recurrent
+ * for each of `n_latent` attention layer runs (latent_dim[i] elements per position,
+ * a multiple of 32) and `n_slots` state slots for each of `n_state` recurrent
  * layer runs (state_elems[i] floats).  A slot has two buffers: a step reads one
  * and writes the other, so a step that fails has changed nothing. */
 typedef struct wr_hip_mix_pool wr_hip_mix_pool;
@@ -85,15 +87,17 @@ int  wr_hip_mix_step_set(wr_hip_mix_step *s, const wr_hip_mix_pool *pool, uint32
                          uint32_t n_want, const uint32_t *want_rows);
 
 /* ---- row steps ------------------------------------------------------------
- * x[r] = rmsnorm(table[token r]) * norm; x0, if not NULL, receives the same rows;
- * h (frag) = rmsnorm(x[r]) * next.  table: device bfloat16 [vocab][width]. */
+ * x[r] = rmsnorm(table[token r]) * norm, or table[token r] * scale without a norm;
+ * x0, if not NULL, receives the same rows; h (frag) = rmsnorm(x[r]) * next, when
+ * next is given.  table: device bfloat16 [vocab][width]. */
 int wr_hip_mix_embed(wr_hip_mix_step *s, int f32, const uint16_t *table_dev, uint32_t width,
-                     const float *norm_dev, float eps, float *x_dev, float *x0_dev,
+                     const float *norm_dev, float scale, float eps, float *x_dev, float *x0_dev,
                      const float *next_dev, void *h_dev);
 
 /* A sublayer's output joins the residual and the next sublayer's input is made:
- *   x += rmsnorm(y) * post           (when y is given; with `top` > 0, row r of y is
- *                                     sum_t gate[r][t] * y[slot[r][t]], the experts' rows)
+ *   x += rmsnorm(y) * post           (when y is given; x += y without `post`; with `top` > 0,
+ *                                     row r of y is sum_t gate[r][t] * y[slot[r][t]], the
+ *                                     experts' rows)
  *   x += add                         (when given)
  *   h = rmsnorm(x) * next            (when given; only the step's wanted rows, packed,
  *                                     with `wanted` set) */
@@ -109,20 +113,31 @@ typedef struct wr_hip_mix_resid {
     void *h;
 } wr_hip_mix_resid;
 int wr_hip_mix_residual(wr_hip_mix_step *s, int f32, const wr_hip_mix_resid *a);
+/* Token shift.  x += y first (y may be NULL).  With h[r] = rmsnorm(x[r]) * norm and p[r]
+ * the same request's h one position earlier (zeros at position 0, else state `run` of
+ * the pool, [width padded to 32] floats, which receives the request's last h):
+ * mix i = h + (p - h) * mu[i] goes to out (frag of n_mix * padded width inputs) at input
+ * i * padded width.  mu: n_mix vectors of the padded width.  With y the new residual
+ * goes to x_out (another buffer than x), which is where x lives from then on. */
+int wr_hip_mix_shift(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, int f32, uint32_t width,
+                     float eps, const float *x_dev, const float *y_dev, float *x_out_dev,
+                     const float *norm_dev, uint32_t n_mix, const float *mu_dev, void *out_dev);
 
 /* ---- matrix products -------------------------------------------------------
  * For every matrix z of the batch: outputs = x_z . W_z^T, x_z being the input
- * tiles [z * x_kt_z, ...) of frag rows with x_kt tiles in all (so x_kt_z = 0
+ * tiles [x_kt0 + z * x_kt_z, ...) of frag rows with x_kt tiles in all (so x_kt_z = 0
  * shares the input).  With group_expert (see route), group g of 16 rows takes
  * matrix group_expert[g], and groups with a negative entry are skipped.
  * out says where output n of row r goes:
- *   ROWS_F32   y_f32[r][n]                 32-bit rows, row stride ldy
+ *   ROWS_F32   y_f32[r][z * col_z + n]     32-bit rows, row stride ldy
  *   ROWS       y_act[r][n]                 activation type, row stride ldy
  *   FRAG       h (frag, h_kt tiles): row r, input z * col_z + n
  *   SPLIT      n < n_split: FRAG; else y_f32[r][n - n_split]
  *   GATED      tiles 2j / 2j+1 of W are gate / up: silu(gate) * up to FRAG
+ *              (with gelu: 0.5 g (1 + tanh(sqrt(2/pi) (g + 0.044715 g^3))) * up)
  * after an activation: SiLU for n < silu_end, else the logistic for n <
- * sigmoid_end; square of ReLU everywhere with relu2; times `scale` when not 0. */
+ * sigmoid_end, else the hyperbolic tangent for n < tanh_end; square of ReLU
+ * everywhere with relu2; times `scale` when not 0. */
 enum { WR_HIP_MIX_OUT_ROWS_F32 = 0, WR_HIP_MIX_OUT_ROWS = 1, WR_HIP_MIX_OUT_FRAG = 2,
        WR_HIP_MIX_OUT_SPLIT = 3, WR_HIP_MIX_OUT_GATED = 4 };
 typedef struct wr_hip_mix_gemm {
@@ -140,6 +155,8 @@ typedef struct wr_hip_mix_gemm {
     uint32_t h_kt, col_z;
     uint32_t n_split, silu_end, sigmoid_end, relu2;
     float scale;
+    uint32_t tanh_end, gelu;
+    uint32_t x_kt0;                /* first input tile of matrix 0 */
 } wr_hip_mix_gemm;
 int wr_hip_mix_gemm_run(int f32, const wr_hip_mix_gemm *a);
 
@@ -155,6 +172,61 @@ int wr_hip_mix_lightning(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run
 /* h (frag) = rmsnorm(o) * norm * g; g: activation-type rows. n features. */
 int wr_hip_mix_gate_norm(wr_hip_mix_step *s, int f32, const float *o_dev, uint32_t ldo, uint32_t n,
                          const void *g_dev, uint32_t ldg, const float *norm_dev, float eps, void *h_dev);
+
+/* ---- matrix-state recurrence with input-made decays -----------------------------
+ * Per head a state S [dim][dim], key channel by value column, 32-bit.  Every token
+ * brings r, k, v and a decay per key channel, w = exp(-exp(z + w0)), or
+ * exp(-gain * sigmoid(z + w0)) with `gain` > 0.  Two rules:
+ *   BONUS  o = (S + diag(u) k v^T)^T r;  then S <- diag(w) S + k v^T
+ *   DELTA  with n = k / sqrt(k . k + unit_eps) and a = sigmoid(za + a_bias):
+ *          S <- diag(w) S - (a n) (n^T S) + k v^T (old S on the right);  o = S^T r
+ * Then each head's o is divided by its root mean square (eps), times norm, times the
+ * gate (SiLU or logistic of the rows at col_g), times out_scale, and goes to h (frag,
+ * h_kt tiles) at input col_h + head * dim + column; inputs up to the next multiple of
+ * 32 are zeros.
+ * in: 32-bit rows, stride ld; r, k, v, za, g at their columns, head by head.
+ * z: 32-bit rows, stride ldz.  State `run` of the pool; position 0 starts from zero. */
+enum { WR_HIP_MIX_RULE_BONUS = 0, WR_HIP_MIX_RULE_DELTA = 1 };
+typedef struct wr_hip_mix_recurrence {
+    uint32_t heads, dim, rule;
+    float gain, unit_eps, eps, out_scale;
+    uint32_t gate_silu;                       /* 1: SiLU, 0: logistic */
+    const float *w0, *u, *a_bias, *norm;      /* device, heads * dim (u: BONUS, a_bias: DELTA) */
+    const float *in;
+    uint32_t ld, col_r, col_k, col_v, col_a, col_g;
+    const float *z;
+    uint32_t ldz;
+    void *h;
+    uint32_t h_kt, col_h;
+} wr_hip_mix_recurrence;
+int wr_hip_mix_recur(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, int f32,
+                     const wr_hip_mix_recurrence *a);
+
+/* ---- windowed attention over grouped keys and values ----------------------------
+ * `heads` query heads, `kv_heads` key/value heads (query head h reads h / (heads /
+ * kv_heads)), head sizes dim (queries, keys) and vdim (values), padded to dim_pad and
+ * vdim_pad (wr_hip_mix_window_pad).  The first 2 * rot_half dimensions are rotated, i
+ * with i + rot_half.  Cached per position: kv_heads * (dim_pad + vdim_pad) elements. */
+typedef struct wr_hip_mix_window {
+    uint32_t heads, kv_heads, dim, dim_pad, vdim, vdim_pad, rot_half;
+    uint32_t window;               /* keys a row sees, itself included */
+    float scale, out_scale;
+    uint32_t norm_values;          /* values divided by their root mean square (eps) ahead of the cache */
+    float eps;
+} wr_hip_mix_window;
+/* The padded head size to use: what the matrix kernels take, else a multiple of 32. */
+uint32_t wr_hip_mix_window_pad(uint32_t dim);
+/* From 32-bit rows (stride ld): queries at col_q rotated into q (frag, head h at input
+ * h * dim_pad); keys at col_k rotated and values at col_v, normed, into the cache. */
+int wr_hip_mix_window_append(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, int f32,
+                             const wr_hip_mix_window *g, const float *in_dev, uint32_t ld, uint32_t col_q,
+                             uint32_t col_k, uint32_t col_v, const float *table_dev, void *q_dev);
+/* Softmax attention over the cached rows inside the window; the denominator also holds
+ * exp(sink[head]) when sink is given.  Head h's output times out_scale goes to o (frag,
+ * o_kt tiles) at input h * vdim_pad. */
+int wr_hip_mix_window_attend(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, int f32,
+                             const wr_hip_mix_window *g, const void *q_dev, const float *sink_dev,
+                             void *o_dev, uint32_t o_kt);
 
 /* ---- attention through a latent -----------------------------------------------
  * Table of (cos, sin) of position * freq[i] for the step's rows, [rows][half][2];

@@ -143,16 +143,16 @@ static float inv_rms(const float *x, uint32_t n, float eps)
     return 1.0f / sqrtf((float)(ss / n) + eps);
 }
 
-int wr_hip_mix_embed(wr_hip_mix_step *s, int f32, const uint16_t *table, uint32_t width, const float *norm, float eps,
-                     float *x, float *x0, const float *next, void *h)
+int wr_hip_mix_embed(wr_hip_mix_step *s, int f32, const uint16_t *table, uint32_t width, const float *norm, float scale,
+                     float eps, float *x, float *x0, const float *next, void *h)
 {
     if (!f32) return WR_HIP_ERR_UNSUPPORTED;
     const uint32_t wp = p32(width);
     for (uint32_t r = 0; r < s->rows; r++) {
         float *xr = x + (size_t)r * wp;
         for (uint32_t k = 0; k < wp; k++) xr[k] = k < width ? widen(table[(size_t)s->tokens[r] * width + k]) : 0.0f;
-        const float inv = inv_rms(xr, width, eps);
-        for (uint32_t k = 0; k < wp; k++) xr[k] = xr[k] * inv * norm[k];
+        const float inv = norm ? inv_rms(xr, width, eps) : scale;
+        for (uint32_t k = 0; k < wp; k++) xr[k] = xr[k] * inv * (norm ? norm[k] : 1.0f);
         if (x0) memcpy(x0 + (size_t)r * wp, xr, wp * 4);
         if (next) {
             const float i2 = inv_rms(xr, width, eps);
@@ -176,8 +176,8 @@ int wr_hip_mix_residual(wr_hip_mix_step *s, int f32, const wr_hip_mix_resid *a)
                 for (uint32_t t = 0; t < a->top; t++)
                     y[k] += a->gate[(size_t)r * a->top + t] * a->y[(size_t)a->slot[(size_t)r * a->top + t] * wp + k];
             }
-            const float inv = inv_rms(y, a->width, a->eps);
-            for (uint32_t k = 0; k < wp; k++) x[k] += y[k] * inv * a->post[k];
+            const float inv = a->post ? inv_rms(y, a->width, a->eps) : 1.0f;
+            for (uint32_t k = 0; k < wp; k++) x[k] += a->post ? y[k] * inv * a->post[k] : y[k];
         }
         if (a->add)
             for (uint32_t k = 0; k < wp; k++) x[k] += a->add[(size_t)r * wp + k];
@@ -187,6 +187,34 @@ int wr_hip_mix_residual(wr_hip_mix_step *s, int f32, const wr_hip_mix_resid *a)
         }
     }
     free(y);
+    return WR_HIP_OK;
+}
+
+int wr_hip_mix_shift(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, int f32, uint32_t width, float eps,
+                     const float *x, const float *y, float *x_out, const float *norm, uint32_t n_mix, const float *mu,
+                     void *out)
+{
+    if (!f32) return WR_HIP_ERR_UNSUPPORTED;
+    const uint32_t wp = p32(width);
+    float *h = malloc(wp * 4), *p = malloc(wp * 4);
+    for (uint32_t i = 0; i < s->n_seq; i++) {
+        const wr_hip_mix_seq *q = &s->seqs[i];
+        const float *in = pool->state[run] + (size_t)(q->slot * 2 + q->buf_in) * wp;
+        for (uint32_t k = 0; k < wp; k++) p[k] = q->pos0 ? in[k] : 0.0f;
+        for (uint32_t r = s->row0[i]; r < s->row0[i] + q->rows; r++) {
+            for (uint32_t k = 0; k < wp; k++) h[k] = x[(size_t)r * wp + k] + (y ? y[(size_t)r * wp + k] : 0.0f);
+            if (y) memcpy(x_out + (size_t)r * wp, h, wp * 4);
+            const float inv = inv_rms(h, width, eps);
+            for (uint32_t k = 0; k < wp; k++) h[k] *= inv * norm[k];
+            for (uint32_t m = 0; m < n_mix; m++)
+                for (uint32_t k = 0; k < wp; k++)
+                    ((float *)out)[((size_t)r * n_mix + m) * wp + k] = h[k] + (p[k] - h[k]) * mu[m * wp + k];
+            memcpy(p, h, wp * 4);
+        }
+        memcpy(pool->state[run] + (size_t)(q->slot * 2 + q->buf_out) * wp, p, wp * 4);
+    }
+    free(h);
+    free(p);
     return WR_HIP_OK;
 }
 
@@ -204,7 +232,7 @@ int wr_hip_mix_gemm_run(int f32, const wr_hip_mix_gemm *a)
                 if (a->group_expert[r / 16] < 0) continue;
                 mat = (uint32_t)a->group_expert[r / 16];
             }
-            const float *x = (const float *)a->x + (size_t)r * ldx + (size_t)z * a->x_kt_z * 32;
+            const float *x = (const float *)a->x + (size_t)r * ldx + ((size_t)a->x_kt0 + (size_t)z * a->x_kt_z) * 32;
             const float *w = a->w->w + (size_t)mat * N * K;
             for (uint32_t n = 0; n < N; n++) {
                 float acc = 0;
@@ -215,7 +243,8 @@ int wr_hip_mix_gemm_run(int f32, const wr_hip_mix_gemm *a)
             if (a->out == WR_HIP_MIX_OUT_GATED) {
                 for (uint32_t n = 0; n < N / 2; n++) {
                     const float g = v[n / 16 * 32 + n % 16], u = v[n / 16 * 32 + 16 + n % 16];
-                    h[n] = g * sig(g) * u;
+                    h[n] = a->gelu ? 0.5f * g * (1.0f + tanhf(0.79788456080286536f * (g + 0.044715f * g * g * g))) * u
+                                   : g * sig(g) * u;
                 }
                 continue;
             }
@@ -223,9 +252,10 @@ int wr_hip_mix_gemm_run(int f32, const wr_hip_mix_gemm *a)
                 float o = v[n];
                 if (n < a->silu_end) o *= sig(o);
                 else if (n < sig_end) o = sig(o);
+                else if (n < a->tanh_end) o = tanhf(o);
                 else if (a->relu2) o = o > 0 ? o * o : 0;
                 if (a->scale != 0) o *= a->scale;
-                if (a->out == WR_HIP_MIX_OUT_ROWS_F32) a->y_f32[(size_t)r * a->ldy + n] = o;
+                if (a->out == WR_HIP_MIX_OUT_ROWS_F32) a->y_f32[(size_t)r * a->ldy + (size_t)z * a->col_z + n] = o;
                 else if (a->out == WR_HIP_MIX_OUT_ROWS) ((float *)a->y_act)[(size_t)r * a->ldy + n] = o;
                 else if (a->out == WR_HIP_MIX_OUT_SPLIT && n >= a->n_split) a->y_f32[(size_t)r * a->ldy + n - a->n_split] = o;
                 else h[n] = o;
@@ -285,6 +315,53 @@ int wr_hip_mix_rope_table(wr_hip_mix_step *s, const double *freq, uint32_t half,
             table[2 * ((size_t)r * half + i)] = (float)cos(s->pos[r] * freq[i]);
             table[2 * ((size_t)r * half + i) + 1] = (float)sin(s->pos[r] * freq[i]);
         }
+    return WR_HIP_OK;
+}
+
+int wr_hip_mix_recur(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, int f32, const wr_hip_mix_recurrence *a)
+{
+    if (!f32) return WR_HIP_ERR_UNSUPPORTED;
+    const uint32_t D = a->dim, hd = a->heads * D, delta = a->rule == WR_HIP_MIX_RULE_DELTA;
+    const size_t all = (size_t)hd * D;
+    if (pool->state_elems[run] != all) return WR_HIP_ERR_INVAL;
+    float w[WR_HIP_MIX_MAX_RECUR_DIM], b[WR_HIP_MIX_MAX_RECUR_DIM], n[WR_HIP_MIX_MAX_RECUR_DIM], o[WR_HIP_MIX_MAX_RECUR_DIM];
+    for (uint32_t i = 0; i < s->n_seq; i++) {
+        const wr_hip_mix_seq *q = &s->seqs[i];
+        float *S = calloc(all, 4);
+        if (q->pos0) memcpy(S, pool->state[run] + (size_t)(q->slot * 2 + q->buf_in) * all, all * 4);
+        for (uint32_t t = s->row0[i]; t < s->row0[i] + q->rows; t++)
+            for (uint32_t h = 0; h < a->heads; h++) {
+                const float *row = a->in + (size_t)t * a->ld + h * D, *r = row + a->col_r, *k = row + a->col_k,
+                            *v = row + a->col_v, *g = row + a->col_g, *z = a->z + (size_t)t * a->ldz + h * D;
+                float kk = 0, ss = 0;
+                for (uint32_t d = 0; d < D; d++) kk += k[d] * k[d];
+                for (uint32_t d = 0; d < D; d++) {
+                    const float y = z[d] + a->w0[h * D + d];
+                    w[d] = expf(a->gain > 0 ? -a->gain * sig(y) : -expf(y));
+                    n[d] = k[d] / sqrtf(kk + a->unit_eps);
+                    b[d] = delta ? sig(row[a->col_a + d] + a->a_bias[h * D + d]) * n[d] : 0.0f;
+                }
+                for (uint32_t c = 0; c < D; c++) {
+                    float *col = S + (size_t)h * D * D + c, seen = 0, out = 0;
+                    for (uint32_t d = 0; d < D; d++) seen += delta ? n[d] * col[d * D] : 0.0f;
+                    for (uint32_t d = 0; d < D; d++) {
+                        const float old = col[d * D];
+                        if (!delta) out += r[d] * (old + a->u[h * D + d] * k[d] * v[c]);
+                        col[d * D] = w[d] * old - b[d] * seen + k[d] * v[c];
+                        if (delta) out += r[d] * col[d * D];
+                    }
+                    o[c] = out;
+                    ss += out * out;
+                }
+                const float inv = a->out_scale / sqrtf(ss / D + a->eps);
+                float *to = (float *)a->h + (size_t)t * a->h_kt * 32 + a->col_h + h * D;
+                for (uint32_t c = 0; c < D; c++) to[c] = o[c] * inv * a->norm[h * D + c] * sig(g[c]) * (a->gate_silu ? g[c] : 1.0f);
+                if (h + 1 == a->heads)
+                    for (uint32_t c = hd; c < p32(hd); c++) to[c - h * D] = 0.0f;
+            }
+        memcpy(pool->state[run] + (size_t)(q->slot * 2 + q->buf_out) * all, S, all * 4);
+        free(S);
+    }
     return WR_HIP_OK;
 }
 
@@ -361,6 +438,72 @@ int wr_hip_mix_latent_attend(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t
                     a += w[j - lo] * pool->latent[run][((size_t)sq->pages[j / WR_HIP_MIX_PAGE] * WR_HIP_MIX_PAGE +
                                                         j % WR_HIP_MIX_PAGE) * dk + k];
                 o[k] = (float)(a / sum);
+            }
+        }
+        free(w);
+    }
+    return WR_HIP_OK;
+}
+
+uint32_t wr_hip_mix_window_pad(uint32_t dim) { return p32(dim); }
+
+static float *window_row(wr_hip_mix_pool *pool, uint32_t run, const wr_hip_mix_window *g, const wr_hip_mix_seq *q, uint32_t pos,
+                         uint32_t kvh)
+{
+    const uint32_t per = g->dim_pad + g->vdim_pad;
+    return pool->latent[run] + (((size_t)q->pages[pos / WR_HIP_MIX_PAGE] * g->kv_heads + kvh) * WR_HIP_MIX_PAGE +
+                                pos % WR_HIP_MIX_PAGE) * per;
+}
+
+int wr_hip_mix_window_append(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, int f32, const wr_hip_mix_window *g,
+                             const float *in, uint32_t ld, uint32_t col_q, uint32_t col_k, uint32_t col_v, const float *table,
+                             void *qv)
+{
+    if (!f32) return WR_HIP_ERR_UNSUPPORTED;
+    for (uint32_t r = 0; r < s->rows; r++) {
+        const float *row = in + (size_t)r * ld, *tab = table + (size_t)r * 2 * g->rot_half;
+        for (uint32_t h = 0; h < g->heads; h++) {
+            float *q = (float *)qv + ((size_t)r * g->heads + h) * g->dim_pad;
+            memset(q, 0, g->dim_pad * 4);
+            rotate(row + col_q + h * g->dim, tab, g->rot_half, g->dim, q);
+        }
+        for (uint32_t h = 0; h < g->kv_heads; h++) {
+            float *c = window_row(pool, run, g, &s->seqs[s->seq[r]], s->pos[r], h);
+            memset(c, 0, (g->dim_pad + g->vdim_pad) * 4);
+            rotate(row + col_k + h * g->dim, tab, g->rot_half, g->dim, c);
+            const float *v = row + col_v + h * g->vdim, inv = g->norm_values ? inv_rms(v, g->vdim, g->eps) : 1.0f;
+            for (uint32_t k = 0; k < g->vdim; k++) c[g->dim_pad + k] = v[k] * inv;
+        }
+    }
+    return WR_HIP_OK;
+}
+
+int wr_hip_mix_window_attend(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, int f32, const wr_hip_mix_window *g,
+                             const void *qv, const float *sink, void *ov, uint32_t o_kt)
+{
+    if (!f32) return WR_HIP_ERR_UNSUPPORTED;
+    for (uint32_t r = 0; r < s->rows; r++) {
+        const wr_hip_mix_seq *sq = &s->seqs[s->seq[r]];
+        const uint32_t pos = s->pos[r], lo = pos + 1 > g->window ? pos + 1 - g->window : 0;
+        double *w = malloc(sizeof(double) * (pos - lo + 1));
+        for (uint32_t h = 0; h < g->heads; h++) {
+            const uint32_t kvh = h / (g->heads / g->kv_heads);
+            const float *q = (const float *)qv + ((size_t)r * g->heads + h) * g->dim_pad;
+            float *o = (float *)ov + (size_t)r * o_kt * 32 + (size_t)h * g->vdim_pad;
+            double mx = sink ? sink[h] : -INFINITY;
+            for (uint32_t j = lo; j <= pos; j++) {
+                const float *c = window_row(pool, run, g, sq, j, kvh);
+                double a = 0;
+                for (uint32_t k = 0; k < g->dim_pad; k++) a += (double)q[k] * c[k];
+                w[j - lo] = a * g->scale;
+                if (w[j - lo] > mx) mx = w[j - lo];
+            }
+            double sum = sink ? exp(sink[h] - mx) : 0;
+            for (uint32_t j = lo; j <= pos; j++) sum += (w[j - lo] = exp(w[j - lo] - mx));
+            for (uint32_t k = 0; k < g->vdim_pad; k++) {
+                double a = 0;
+                for (uint32_t j = lo; j <= pos; j++) a += w[j - lo] * window_row(pool, run, g, sq, j, kvh)[g->dim_pad + k];
+                o[k] = (float)(a / sum * g->out_scale);
             }
         }
         free(w);

@@ -1,7 +1,7 @@
-"""Plain, slow restatement of the mixer-stack models (architecture "Bipotar"):
-one function per mechanism, numpy, one sequence at a time, every position from
-the definition (no cache, no chunks, no absorbed products).  Shares no code with
-the product path; the tests compare the engine with it.
+"""Plain, slow restatement of the mixer-stack models (architectures "Bipotar" and
+"Taredra"): one function per mechanism, numpy, one sequence at a time, every
+position from the definition (no cache, no chunks, no absorbed products).  Shares
+no code with the product path; the tests compare the engine with it.
 
 ``prec`` is the working dtype of every sum (float32 or float64).
 """
@@ -113,11 +113,102 @@ def moe_mlp(h, w, cfg):
     return out
 
 
-MIXERS = {"lightning": lambda *a: lightning(*a)[0], "latent_attention": latent_attention}
-
-
 def _sub(tensors, prefix):
     return {k[len(prefix):]: v for k, v in tensors.items() if k.startswith(prefix)}
+
+
+def gelu_tanh(z):
+    return 0.5 * z * (1.0 + np.tanh(np.sqrt(2.0 / np.pi) * (z + 0.044715 * z ** 3)))
+
+
+def unit_rms(x, eps):
+    return x / np.sqrt(np.mean(x * x, axis=-1, keepdims=True) + x.dtype.type(eps))
+
+
+def token_shift(h, mu, before=None):
+    """Every row moved towards the row before it (zeros, or `before`, ahead of the first)."""
+    prev = np.concatenate([np.zeros_like(h[:1]) if before is None else before[None], h[:-1]])
+    return h + (prev - h) * mu
+
+
+def wkv(h, w, cfg, eps):
+    """Matrix-state recurrence with a decay per head and key channel made from the input, and a bonus for the
+    current token; returns (out [T, width], final state [heads, dim, dim])."""
+    H, D = cfg["heads"], cfg["dim"]
+    T = h.shape[0]
+    mix = {s: token_shift(h, w["mu." + s]) for s in "rkvgw"}
+    r, k, v = ((mix[s] @ w[s].T).reshape(T, H, D) for s in "rkv")
+    decay = np.exp(-np.exp(np.tanh(mix["w"] @ w["w1"].T) @ w["w2"].T + w["w0"])).reshape(T, H, D)
+    S = np.zeros((H, D, D), dtype=h.dtype)
+    o = np.empty((T, H, D), dtype=h.dtype)
+    for t in range(T):
+        kv = k[t][:, :, None] * v[t][:, None, :]
+        o[t] = np.einsum("hdv,hd->hv", S + w["u"][:, :, None] * kv, r[t])
+        S = decay[t][:, :, None] * S + kv
+    o = unit_rms(o, eps).reshape(T, H * D) * w["norm"] * silu(mix["g"] @ w["g"].T)
+    return o @ w["o"].T, S
+
+
+def delta_rule(h, w, cfg, eps):
+    """Matrix-state recurrence that decays per key channel, removes along the unit key and adds k v^T; returns
+    (out [T, width], final state [heads, dim, dim])."""
+    H, D = cfg["heads"], cfg["dim"]
+    T = h.shape[0]
+    r, k, v = ((h @ w[s].T).reshape(T, H, D) for s in "rkv")
+    decay = np.exp(-np.exp(-0.5) * sigmoid(np.tanh(h @ w["w1"].T) @ w["w2"].T + w["w0"])).reshape(T, H, D)
+    rate = sigmoid(h @ w["a"].T + w["a.b"]).reshape(T, H, D)
+    u = k / np.sqrt((k * k).sum(-1, keepdims=True) + h.dtype.type(1e-6))
+    S = np.zeros((H, D, D), dtype=h.dtype)
+    o = np.empty((T, H, D), dtype=h.dtype)
+    for t in range(T):
+        seen = np.einsum("hd,hdv->hv", u[t], S)
+        S = (decay[t][:, :, None] * S - (rate[t] * u[t])[:, :, None] * seen[:, None, :]
+             + k[t][:, :, None] * v[t][:, None, :])
+        o[t] = np.einsum("hdv,hd->hv", S, r[t])
+    o = unit_rms(o, eps).reshape(T, H * D) * w["norm"] * sigmoid(h @ w["g"].T)
+    return o @ w["o"].T, S
+
+
+def window_attention(h, w, cfg, eps, positions=None):
+    """Grouped-query attention in a sliding window: rotated queries and keys, normed values, a sink in the softmax."""
+    H, G, D, V, rot = cfg["heads"], cfg["kv_heads"], cfg["dim"], cfg["vdim"], cfg["rot"]
+    T = h.shape[0]
+    pos = np.arange(T) if positions is None else np.asarray(positions)
+    q = rotate_half_pairs((h @ w["q"].T).reshape(T, H, D), pos, rot["base"], rot["dims"])
+    k = rotate_half_pairs((h @ w["k"].T).reshape(T, G, D), pos, rot["base"], rot["dims"])
+    v = unit_rms((h @ w["v"].T).reshape(T, G, V), eps)
+    gap = pos[:, None] - pos[None, :]
+    seen = (gap >= 0) & (gap < cfg["mask"]["size"])
+    out = np.empty((T, H, V), dtype=h.dtype)
+    for hh in range(H):
+        g = hh // (H // G)
+        s = np.where(seen, (q[:, hh] @ k[:, g].T) * h.dtype.type(cfg["scale"]), -np.inf)
+        top = np.maximum(s.max(axis=1, keepdims=True), w["sink"][hh])
+        e = np.exp(s - top)
+        out[:, hh] = (e / (e.sum(axis=1, keepdims=True) + np.exp(w["sink"][hh] - top))) @ v[:, g]
+    return out.reshape(T, H * V) @ w["o"].T
+
+
+def parallel(h, w, cfg, eps):
+    left = window_attention(h, _sub(w, "left."), cfg["left"], eps)
+    right, _ = delta_rule(h, _sub(w, "right."), cfg["right"], eps)
+    return h.dtype.type(cfg["left_scale"]) * left + h.dtype.type(cfg["right_scale"]) * right
+
+
+def gelu_mlp(h, w):
+    return (gelu_tanh(h @ w["gate"].T) * (h @ w["up"].T)) @ w["down"].T
+
+
+MIXERS = {"lightning": lambda *a: lightning(*a)[0], "latent_attention": latent_attention,
+          "wkv": lambda *a: wkv(*a)[0], "parallel": parallel}
+
+
+def prenorm_layer(x, w, cfg, eps):
+    """A layer with a norm ahead of each sublayer only, its weight stored around zero."""
+    x = x + MIXERS[cfg["type"]](rms_norm(x, 1 + w["norm1"], eps), _sub(w, "mix."), cfg["mixer"], eps)
+    if cfg.get("mlp"):
+        x = x + gelu_mlp(rms_norm(x, 1 + w["norm2"], eps), _sub(w, "mlp."))
+    return x
 
 
 def layer(x, w, cfg, eps, margins=None):
@@ -149,6 +240,13 @@ def forward(cfg, tensors, tokens, prec=np.float32, capture=None, margins=None):
     """Logits [T, vocab] of one sequence.  `capture`: a list that receives the rows after every layer run."""
     w = {k: (v if v.dtype == np.int32 else v.astype(prec)) for k, v in tensors.items()}
     eps = cfg["norm"]["eps"]
+    if cfg["architecture"] == "Taredra":
+        x = w["embed"][np.asarray(tokens)] * prec(cfg["embedding"]["scale"])
+        for i, c in enumerate(cfg["layers"]):
+            x = prenorm_layer(x, _sub(w, f"l{i}."), c, eps)
+            if capture is not None:
+                capture.append(x.copy())
+        return rms_norm(x, 1 + w["final.norm"], eps) @ w["embed"].T
     x = rms_norm(w["embed"][np.asarray(tokens)], w["embed.norm"], eps)
     x0 = x
     for i, again in layer_order(cfg):

@@ -24,7 +24,7 @@ struct MixGemmArgs {
     uint32_t x_kt, x_kt_z;
     uint32_t rows, groups;
     const int32_t* group_expert;
-    uint32_t out, ldy, h_kt, col_z, n_split, silu_end, sigmoid_end, relu2;
+    uint32_t out, ldy, h_kt, col_z, n_split, silu_end, sigmoid_end, tanh_end, relu2, gelu;
     float scale;
     float* y;
     void* ya;
@@ -62,7 +62,11 @@ __device__ __forceinline__ void mix_store_tile(const MixGemmArgs& a, f32x4 v, f3
     if (row >= a.rows || nt >= a.ntiles) return;
     if (a.out == kMixOutGated) {
 #pragma unroll
-        for (int i = 0; i < 4; i++) v[i] = v[i] * mix_sigmoid<F32>(v[i]) * up[i];
+        for (int i = 0; i < 4; i++) {
+            // the tanh form of GELU is x * logistic(2 y), y the argument of its tanh
+            const float y = a.gelu ? 1.5957691216057308f * (v[i] + 0.044715f * v[i] * v[i] * v[i]) : v[i];
+            v[i] = v[i] * mix_sigmoid<F32>(y) * up[i];
+        }
         mix_put4<F32>(a.h, frag_elem(row, nt / 2 * 16 + 4 * g, a.h_kt), v);
         return;
     }
@@ -72,6 +76,9 @@ __device__ __forceinline__ void mix_store_tile(const MixGemmArgs& a, f32x4 v, f3
             const float s = mix_sigmoid<F32>(v[i]);
             v[i] = n + i < a.silu_end ? v[i] * s : (n + i < a.sigmoid_end ? s : v[i]);
         }
+    } else if (n < a.tanh_end) {
+#pragma unroll
+        for (int i = 0; i < 4; i++) v[i] = n + i < a.tanh_end ? tanhf(v[i]) : v[i];
     } else if (a.relu2) {
 #pragma unroll
         for (int i = 0; i < 4; i++) {
@@ -84,7 +91,7 @@ __device__ __forceinline__ void mix_store_tile(const MixGemmArgs& a, f32x4 v, f3
         for (int i = 0; i < 4; i++) v[i] *= a.scale;
     }
     if (a.out == kMixOutRowsF32) {
-        *reinterpret_cast<f32x4*>(a.y + (size_t)row * a.ldy + n) = v;
+        *reinterpret_cast<f32x4*>(a.y + (size_t)row * a.ldy + (size_t)z * a.col_z + n) = v;
     } else if (a.out == kMixOutRows) {
         mix_put4<F32>(a.ya, (size_t)row * a.ldy + n, v);
     } else if (a.out == kMixOutSplit && n >= a.n_split) {

@@ -88,7 +88,8 @@ struct MixRowArgs {
     // embedding
     const uint16_t* table;
     const uint32_t* tokens;
-    const float* norm;
+    const float* norm;               // nullptr: times scale instead
+    float scale;
     float* x0;
 };
 
@@ -110,7 +111,8 @@ __device__ __forceinline__ void mix_sub_chunk(const MixRowArgs& a, uint32_t r, u
     }
 }
 
-// x <- x + rmsnorm(y) * post + add; h <- rmsnorm(x) * next (EMBED: x <- rmsnorm(table[token]) * norm first).
+// x <- x + rmsnorm(y) * post (or + y) + add; h <- rmsnorm(x) * next
+// (EMBED: x <- rmsnorm(table[token]) * norm, or table[token] * scale, first).
 template <bool F32, int RPW, bool EMBED, bool HELD>
 __global__ __launch_bounds__(MixRowShape<RPW>::kThreads) void mix_residual_kernel(const MixRowArgs a)
 {
@@ -150,9 +152,10 @@ __global__ __launch_bounds__(MixRowShape<RPW>::kThreads) void mix_residual_kerne
             mix_sub_chunk(a, r, q, v);
         }
     };
-    const bool normed = EMBED || a.y != nullptr;          // uniform
-    float inv = 0.f;
-    if (normed) {
+    const bool some = EMBED || a.y != nullptr;            // uniform: there is a value
+    const bool normed = EMBED ? a.norm != nullptr : a.post != nullptr;
+    float inv = EMBED ? a.scale : 1.0f;
+    if (some) {
         if constexpr (HELD) {
 #pragma unroll
             for (int i = 0; i < CH; i++) {
@@ -171,20 +174,28 @@ __global__ __launch_bounds__(MixRowShape<RPW>::kThreads) void mix_residual_kerne
                 for (int j = 0; j < 8; j++) ss = fmaf(v[j], v[j], ss);
             }
         }
-        inv = 1.0f / sqrtf(mix_row_sum<RPW>(ss, red) * invw + a.eps);
+        if (normed) inv = 1.0f / sqrtf(mix_row_sum<RPW>(ss, red) * invw + a.eps);
     }
 
     // x of one chunk, from the value above
     auto second = [&](uint32_t q, float (&v)[8]) {
         if constexpr (EMBED) {
-            float w[8];
-            mix_load8(a.norm + q * 8, w);
+            if (normed) {
+                float w[8];
+                mix_load8(a.norm + q * 8, w);
 #pragma unroll
-            for (int j = 0; j < 8; j++) v[j] = v[j] * inv * w[j];
+                for (int j = 0; j < 8; j++) v[j] = v[j] * inv * w[j];
+            } else {
+#pragma unroll
+                for (int j = 0; j < 8; j++) v[j] *= inv;
+            }
         } else {
             float x[8];
             mix_load8(xr + q * 8, x);
-            if (a.y) {
+            if (a.y && !normed) {
+#pragma unroll
+                for (int j = 0; j < 8; j++) x[j] += v[j];
+            } else if (a.y) {
                 float w[8];
                 mix_load8(a.post + q * 8, w);
 #pragma unroll
@@ -218,7 +229,7 @@ __global__ __launch_bounds__(MixRowShape<RPW>::kThreads) void mix_residual_kerne
     } else {
         for (uint32_t q = lr; q < nq; q += Sh::kPerRow) {
             float v[8];
-            if (normed) first(q, v);
+            if (some) first(q, v);
             second(q, v);
 #pragma unroll
             for (int j = 0; j < 8; j++) ss = fmaf(v[j], v[j], ss);
@@ -253,6 +264,81 @@ __global__ __launch_bounds__(MixRowShape<RPW>::kThreads) void mix_residual_kerne
                 mix_load8(xr + q * 8, v);
             }
             third(q, v);
+        }
+    }
+}
+
+// Token shift (wr_hip_mix_shift): one row of eight features a thread and turn; the row before is normed again
+// rather than waited for.
+struct MixShiftArgs {
+    const MixSeq* seqs;
+    const uint32_t* row_seq;
+    uint32_t rows, width, wpad, n_mix;
+    float eps;
+    const float *x, *y, *norm, *mu;
+    float* x_out;
+    float* state;                    // [buffer][wpad]
+    void* out;
+};
+template <bool F32, int RPW>
+__global__ __launch_bounds__(MixRowShape<RPW>::kThreads) void mix_shift_kernel(const MixShiftArgs a)
+{
+    using Sh = MixRowShape<RPW>;
+    __shared__ float red[64];
+    const uint32_t t = threadIdx.x, row = blockIdx.x * RPW + t % RPW, lr = t / RPW;
+    const bool live = row < a.rows;
+    const uint32_t r = live ? row : a.rows - 1, nq = a.wpad / 8;
+    const MixSeq s = a.seqs[a.row_seq[r]];
+    const bool first = r == s.row0, last = r + 1 == s.row0 + s.rows;
+    const uint32_t p = first ? r : r - 1;
+    auto load = [&](uint32_t rr, uint32_t q, float (&v)[8]) {
+        mix_load8(a.x + (size_t)rr * a.wpad + q * 8, v);
+        if (a.y) {
+            float w[8];
+            mix_load8(a.y + (size_t)rr * a.wpad + q * 8, w);
+#pragma unroll
+            for (int j = 0; j < 8; j++) v[j] += w[j];
+        }
+    };
+    float sr = 0.f, sp = 0.f;
+    for (uint32_t q = lr; q < nq; q += Sh::kPerRow) {
+        float v[8], w[8];
+        load(r, q, v);
+        load(p, q, w);
+#pragma unroll
+        for (int j = 0; j < 8; j++) {
+            sr = fmaf(v[j], v[j], sr);
+            sp = fmaf(w[j], w[j], sp);
+        }
+    }
+    const float invw = 1.0f / (float)a.width;
+    const float ir = 1.0f / sqrtf(mix_row_sum<RPW>(sr, red) * invw + a.eps);
+    const float ip = 1.0f / sqrtf(mix_row_sum<RPW>(sp, red) * invw + a.eps);
+    if (!live) return;
+    for (uint32_t q = lr; q < nq; q += Sh::kPerRow) {
+        float v[8], w[8], n[8];
+        load(r, q, v);
+        if (a.y) mix_store8(a.x_out + (size_t)r * a.wpad + q * 8, v);
+        mix_load8(a.norm + q * 8, n);
+        if (!first) {
+            load(p, q, w);
+#pragma unroll
+            for (int j = 0; j < 8; j++) w[j] *= ip * n[j];
+        } else if (s.pos0 > 0) {
+            mix_load8(a.state + (size_t)s.state_in * a.wpad + q * 8, w);
+        } else {
+#pragma unroll
+            for (int j = 0; j < 8; j++) w[j] = 0.f;
+        }
+#pragma unroll
+        for (int j = 0; j < 8; j++) v[j] *= ir * n[j];
+        if (last) mix_store8(a.state + (size_t)s.state_out * a.wpad + q * 8, v);
+        for (uint32_t m = 0; m < a.n_mix; m++) {
+            float u[8];
+            mix_load8(a.mu + (size_t)m * a.wpad + q * 8, u);
+#pragma unroll
+            for (int j = 0; j < 8; j++) u[j] = v[j] + (w[j] - v[j]) * u[j];
+            mix_store_unit<F32>(a.out, frag_unit(r, m * nq + q, a.n_mix * (a.wpad / 32)), u);
         }
     }
 }

@@ -19,6 +19,8 @@
 #include "kernels_lightning.hip.h"
 #include "kernels_latent.hip.h"
 #include "kernels_latent_mfma.hip.h"
+#include "kernels_recur.hip.h"
+#include "kernels_window.hip.h"
 
 using namespace wr;
 
@@ -60,7 +62,7 @@ struct wr_hip_mix_step {
     size_t o_tokens, o_seq, o_pos, o_want, o_seqs, o_chunks, o_all, o_short, o_long, o_short_rows, o_pages, bytes;
     uint32_t rows = 0, n_seq = 0, n_want = 0, n_chunks = 0, n_short = 0, n_long = 0, n_short_rows = 0;
     uint32_t long_rows[kMaxSeqs];           // rows of each request of the long list
-    Buffer chunk_state, state_frag, partial;
+    Buffer chunk_state, state_frag, partial, recur_ops, recur_out;
     template <typename T> T* d(size_t off) const { return reinterpret_cast<T*>(dev + off); }
     template <typename T> T* h(size_t off) const { return reinterpret_cast<T*>(host + off); }
 };
@@ -233,6 +235,8 @@ void wr_hip_mix_step_destroy(wr_hip_mix_step* s)
     wr_hip_attn_dev_free(s->chunk_state.p);
     wr_hip_attn_dev_free(s->state_frag.p);
     wr_hip_attn_dev_free(s->partial.p);
+    wr_hip_attn_dev_free(s->recur_ops.p);
+    wr_hip_attn_dev_free(s->recur_out.p);
     delete s;
 }
 
@@ -335,10 +339,10 @@ static int launch_residual(int f32, bool embed, const MixRowArgs& a)
 }
 
 int wr_hip_mix_embed(wr_hip_mix_step* s, int f32, const uint16_t* table_dev, uint32_t width, const float* norm_dev,
-                     float eps, float* x_dev, float* x0_dev, const float* next_dev, void* h_dev)
+                     float scale, float eps, float* x_dev, float* x0_dev, const float* next_dev, void* h_dev)
 {
     if (!g.inited) return WR_HIP_ERR_STATE;
-    if (!s || !s->rows || !table_dev || !width || !norm_dev || !x_dev || (next_dev && !h_dev)) return WR_HIP_ERR_INVAL;
+    if (!s || !s->rows || !table_dev || !width || !x_dev || (next_dev && !h_dev)) return WR_HIP_ERR_INVAL;
     ENTER();
     MixRowArgs a = {};
     a.rows = s->rows;
@@ -352,13 +356,14 @@ int wr_hip_mix_embed(wr_hip_mix_step* s, int f32, const uint16_t* table_dev, uin
     a.table = table_dev;
     a.tokens = s->d<uint32_t>(s->o_tokens);
     a.norm = norm_dev;
+    a.scale = scale;
     return launch_residual(f32, true, a);
 }
 
 int wr_hip_mix_residual(wr_hip_mix_step* s, int f32, const wr_hip_mix_resid* q)
 {
     if (!g.inited) return WR_HIP_ERR_STATE;
-    if (!s || !s->rows || !q || !q->width || !q->x || (q->y && !q->post) || (q->next && !q->h)) return WR_HIP_ERR_INVAL;
+    if (!s || !s->rows || !q || !q->width || !q->x || (q->post && !q->y) || (q->next && !q->h)) return WR_HIP_ERR_INVAL;
     if (q->top && (!q->y || !q->gate || !q->slot)) return WR_HIP_ERR_INVAL;
     if (q->wanted && (q->y || q->add || !s->n_want)) return WR_HIP_ERR_INVAL;
     ENTER();
@@ -378,6 +383,29 @@ int wr_hip_mix_residual(wr_hip_mix_step* s, int f32, const wr_hip_mix_resid* q)
     a.top = q->top;
     a.gather = q->wanted ? s->d<uint32_t>(s->o_want) : nullptr;
     return launch_residual(f32, false, a);
+}
+
+int wr_hip_mix_shift(wr_hip_mix_step* s, wr_hip_mix_pool* pool, uint32_t run, int f32, uint32_t width, float eps,
+                     const float* x_dev, const float* y_dev, float* x_out_dev, const float* norm_dev, uint32_t n_mix,
+                     const float* mu_dev, void* out_dev)
+{
+    if (!g.inited) return WR_HIP_ERR_STATE;
+    if (!s || !s->rows || !pool || run >= pool->state.size() || !width || pool->state_elems[run] != round32(width) || !x_dev ||
+        !norm_dev || !n_mix || !mu_dev || !out_dev || (y_dev && (!x_out_dev || x_out_dev == x_dev || x_out_dev == y_dev)))
+        return WR_HIP_ERR_INVAL;
+    ENTER();
+    MixShiftArgs a = {s->d<MixSeq>(s->o_seqs), s->d<uint32_t>(s->o_seq), s->rows, width, round32(width), n_mix, eps, x_dev, y_dev,
+                      norm_dev, mu_dev, x_out_dev, pool->state[run], out_dev};
+    if (s->rows >= 64) {
+        const dim3 grid((s->rows + 3) / 4), block(MixRowShape<4>::kThreads);
+        if (f32) MIX_LAUNCH((mix_shift_kernel<true, 4>), grid, block, 0, a);
+        else MIX_LAUNCH((mix_shift_kernel<false, 4>), grid, block, 0, a);
+    } else {
+        const dim3 grid(s->rows), block(MixRowShape<1>::kThreads);
+        if (f32) MIX_LAUNCH((mix_shift_kernel<true, 1>), grid, block, 0, a);
+        else MIX_LAUNCH((mix_shift_kernel<false, 1>), grid, block, 0, a);
+    }
+    return WR_HIP_OK;
 }
 
 // --------------------------------------------------------------- products --
@@ -408,7 +436,7 @@ int wr_hip_mix_gemm_run(int f32, const wr_hip_mix_gemm* q)
     if (!g.inited) return WR_HIP_ERR_STATE;
     if (!q || !q->w || !q->x || !q->rows) return WR_HIP_ERR_INVAL;
     const uint32_t ktiles = q->w->n_in / 32, batch = q->group_expert ? 1 : q->w->batch;
-    if ((uint64_t)q->x_kt_z * (batch - 1) + ktiles > q->x_kt) return WR_HIP_ERR_INVAL;
+    if ((uint64_t)q->x_kt0 + (uint64_t)q->x_kt_z * (batch - 1) + ktiles > q->x_kt) return WR_HIP_ERR_INVAL;
     const bool frag = q->out == WR_HIP_MIX_OUT_FRAG || q->out == WR_HIP_MIX_OUT_SPLIT || q->out == WR_HIP_MIX_OUT_GATED;
     if (q->out > WR_HIP_MIX_OUT_GATED || (frag && !q->h)) return WR_HIP_ERR_INVAL;
     const uint32_t n_frag = q->out == WR_HIP_MIX_OUT_SPLIT ? q->n_split : (q->out == WR_HIP_MIX_OUT_GATED ? q->w->n_out / 2 : q->w->n_out);
@@ -418,14 +446,16 @@ int wr_hip_mix_gemm_run(int f32, const wr_hip_mix_gemm* q)
     const bool rows32 = q->out == WR_HIP_MIX_OUT_ROWS_F32 || (q->out == WR_HIP_MIX_OUT_SPLIT && q->n_split < q->w->n_out);
     const uint32_t n_rows = q->out == WR_HIP_MIX_OUT_SPLIT ? q->w->n_out - q->n_split : q->w->n_out;
     if (rows32 && (!q->y_f32 || q->ldy % 4 || q->ldy < n_rows)) return WR_HIP_ERR_INVAL;
+    if (q->out == WR_HIP_MIX_OUT_ROWS_F32 && batch > 1 && (q->col_z % 4 || (uint64_t)q->col_z * (batch - 1) + n_rows > q->ldy))
+        return WR_HIP_ERR_INVAL;
     if (q->out == WR_HIP_MIX_OUT_ROWS && (!q->y_act || q->ldy % 8 || q->ldy < n_rows)) return WR_HIP_ERR_INVAL;
-    if ((q->out == WR_HIP_MIX_OUT_ROWS_F32 || q->out == WR_HIP_MIX_OUT_ROWS) && batch != 1) return WR_HIP_ERR_INVAL;
+    if (((q->out == WR_HIP_MIX_OUT_ROWS_F32 && !q->col_z) || q->out == WR_HIP_MIX_OUT_ROWS) && batch != 1) return WR_HIP_ERR_INVAL;
     if (q->group_expert && (q->rows % 16 || (q->tile_groups != 1 && q->tile_groups != 8))) return WR_HIP_ERR_INVAL;
     if (q->group_expert && q->rows / 16 % q->tile_groups) return WR_HIP_ERR_INVAL;
     ENTER();
     MixGemmArgs a = {};
     a.w = reinterpret_cast<const bf16x8*>(q->w->tiles);
-    a.x = q->x;
+    a.x = static_cast<const uint8_t*>(q->x) + (size_t)q->x_kt0 * 512 * (f32 ? 4 : 2);
     a.ntiles = q->w->n_out / 16;
     a.ktiles = ktiles;
     a.x_kt = q->x_kt;
@@ -440,7 +470,9 @@ int wr_hip_mix_gemm_run(int f32, const wr_hip_mix_gemm* q)
     a.n_split = q->n_split;
     a.silu_end = q->silu_end;
     a.sigmoid_end = std::max(q->sigmoid_end, q->silu_end);
+    a.tanh_end = q->tanh_end;
     a.relu2 = q->relu2;
+    a.gelu = q->gelu;
     a.scale = q->scale;
     a.y = q->y_f32;
     a.ya = q->y_act;
@@ -585,6 +617,104 @@ int wr_hip_mix_gate_norm(wr_hip_mix_step* s, int f32, const float* o_dev, uint32
         else MIX_LAUNCH((mix_gate_norm_kernel<false, 1>), grid, block, 0, a);
     }
     return WR_HIP_OK;
+}
+
+// ------------------------------------------------------------- recurrence --
+
+template <bool F32, bool DELTA>
+static int recur_steps(const RecurArgs& a, uint32_t n)
+{
+    if (n == 0) return WR_HIP_OK;
+    const dim3 grid(n, a.heads);
+    if (a.dim <= 16) MIX_LAUNCH((recur_step_kernel<F32, 16, DELTA>), grid, dim3(64), 0, a);
+    else if (a.dim <= 32) MIX_LAUNCH((recur_step_kernel<F32, 32, DELTA>), grid, dim3(128), 0, a);
+    else if (a.dim <= 64) MIX_LAUNCH((recur_step_kernel<F32, 64, DELTA>), grid, dim3(256), 0, a);
+    else if (a.dim <= 128) MIX_LAUNCH((recur_step_kernel<F32, 128, DELTA>), grid, dim3(512), 0, a);
+    else MIX_LAUNCH((recur_step_kernel<F32, 256, DELTA>), grid, dim3(1024), 0, a);
+    return WR_HIP_OK;
+}
+
+template <bool F32, int KT, bool DELTA, int VT>
+static int recur_chunks(wr_hip_mix_step* s, RecurArgs& a)
+{
+    a.vtiles = VT;
+    constexpr size_t unit = (size_t)recur_unit_kib(KT, DELTA, VT) * 1024;
+    int rc = ensure_device(s->recur_ops, (size_t)s->n_chunks * kRecurSubs * a.heads * unit);
+    if (rc == WR_HIP_OK) rc = ensure_device(s->recur_out, (size_t)s->n_chunks * kMixChunk * a.heads * VT * 16 * 4);
+    constexpr size_t l1 = (size_t)4 * recur_chunk_lds(KT, DELTA) * 4, l2 = recur_ring(KT) * unit;
+    if (rc == WR_HIP_OK) rc = allow_lds<recur_chunk_kernel<F32, KT, DELTA>>(l1);
+    if (rc == WR_HIP_OK) rc = allow_lds<recur_chain_kernel<F32, KT, DELTA, VT>>(l2);
+    if (rc) return rc;
+    a.ops = reinterpret_cast<unsigned char*>(s->recur_ops.p);
+    a.o = reinterpret_cast<float*>(s->recur_out.p);
+    const uint32_t whole = !((a.dim | a.ld | a.ldz | a.col_r | a.col_k | a.col_a) % 4);
+    MIX_LAUNCH((recur_chunk_kernel<F32, KT, DELTA>), dim3(s->n_chunks, a.heads), dim3(256), l1, a, whole);
+    MIX_LAUNCH((recur_chain_kernel<F32, KT, DELTA, VT>), dim3(s->n_long, a.heads), dim3(64 * VT), l2, a);
+    MIX_LAUNCH(recur_gate_kernel<F32>, dim3(s->n_chunks, a.heads), dim3(256), 0, a);
+    return WR_HIP_OK;
+}
+
+template <bool F32, bool DELTA>
+static int recur_run(wr_hip_mix_step* s, RecurArgs& a)
+{
+    const bool chunked = s->n_long && a.dim <= (uint32_t)kRecurMaxDim;
+    if (chunked) {
+        a.list = s->d<uint32_t>(s->o_long);
+        int rc;
+        if (a.dim <= 16) rc = recur_chunks<F32, 1, DELTA, 1>(s, a);
+        else if (a.dim <= 32) rc = recur_chunks<F32, 1, DELTA, 2>(s, a);
+        else if (a.dim <= 64) rc = recur_chunks<F32, 2, DELTA, 4>(s, a);
+        else rc = recur_chunks<F32, 4, DELTA, 8>(s, a);
+        if (rc) return rc;
+    }
+    a.list = s->d<uint32_t>(chunked ? s->o_short : s->o_all);
+    return recur_steps<F32, DELTA>(a, chunked ? s->n_short : s->n_seq);
+}
+
+int wr_hip_mix_recur(wr_hip_mix_step* s, wr_hip_mix_pool* pool, uint32_t run, int f32, const wr_hip_mix_recurrence* q)
+{
+    if (!g.inited) return WR_HIP_ERR_STATE;
+    if (!s || !s->rows || !pool || run >= pool->state.size() || !q || !q->heads || !q->dim || !q->w0 || !q->norm || !q->in ||
+        !q->z || !q->h || q->rule > WR_HIP_MIX_RULE_DELTA)
+        return WR_HIP_ERR_INVAL;
+    const bool delta = q->rule == WR_HIP_MIX_RULE_DELTA;
+    if (delta ? !q->a_bias : !q->u) return WR_HIP_ERR_INVAL;
+    if (q->dim > WR_HIP_MIX_MAX_RECUR_DIM) return WR_HIP_ERR_LIMIT;
+    const uint64_t hd = (uint64_t)q->heads * q->dim;
+    if (hd * q->dim != pool->state_elems[run]) return WR_HIP_ERR_INVAL;
+    if (q->ldz < hd || q->col_r + hd > q->ld || q->col_k + hd > q->ld || q->col_v + hd > q->ld || q->col_g + hd > q->ld ||
+        (delta && q->col_a + hd > q->ld) || q->col_h + (hd + 31) / 32 * 32 > (uint64_t)q->h_kt * 32)
+        return WR_HIP_ERR_INVAL;
+    ENTER();
+    RecurArgs a = {};
+    a.seqs = s->d<MixSeq>(s->o_seqs);
+    a.chunks = s->d<MixChunk>(s->o_chunks);
+    a.heads = q->heads;
+    a.dim = q->dim;
+    a.silu = q->gate_silu;
+    a.gain = q->gain;
+    a.unit_eps = q->unit_eps;
+    a.eps = q->eps;
+    a.out_scale = q->out_scale;
+    a.w0 = q->w0;
+    a.u = q->u;
+    a.ab = q->a_bias;
+    a.norm = q->norm;
+    a.in = q->in;
+    a.ld = q->ld;
+    a.col_r = q->col_r;
+    a.col_k = q->col_k;
+    a.col_v = q->col_v;
+    a.col_a = delta ? q->col_a : 0;
+    a.col_g = q->col_g;
+    a.z = q->z;
+    a.ldz = q->ldz;
+    a.state = pool->state[run];
+    a.h = q->h;
+    a.h_kt = q->h_kt;
+    a.col_h = q->col_h;
+    if (f32) return delta ? recur_run<true, true>(s, a) : recur_run<true, false>(s, a);
+    return delta ? recur_run<false, true>(s, a) : recur_run<false, false>(s, a);
 }
 
 // ----------------------------------------------------------------- latent --
@@ -785,6 +915,163 @@ int wr_hip_mix_latent_attend(wr_hip_mix_step* s, wr_hip_mix_pool* pool, uint32_t
     if (rc) return rc;
     if (f32) MIX_LAUNCH(latent_attend_any_kernel<true>, dim3(s->rows, q->heads), dim3(64), lds, a);
     else MIX_LAUNCH(latent_attend_any_kernel<false>, dim3(s->rows, q->heads), dim3(64), lds, a);
+    return WR_HIP_OK;
+}
+
+// --------------------------------------------------- windowed attention --
+
+uint32_t wr_hip_mix_window_pad(uint32_t dim)
+{
+    for (uint32_t p = 32; p <= 128; p *= 2)
+        if (dim <= p) return p;
+    return round32(dim);
+}
+
+static int check_window(const wr_hip_mix_step* s, const wr_hip_mix_pool* pool, uint32_t run, int f32, const wr_hip_mix_window* q)
+{
+    if (!s || !s->rows || !pool || run >= pool->latent.size() || pool->f32 != (f32 != 0) || !q || !q->heads || !q->kv_heads ||
+        q->heads % q->kv_heads || !q->dim || !q->vdim || q->dim_pad % 32 || q->vdim_pad % 32 || q->dim > q->dim_pad ||
+        q->vdim > q->vdim_pad || q->rot_half * 2 > q->dim || !q->window)
+        return WR_HIP_ERR_INVAL;
+    if ((uint64_t)q->kv_heads * (q->dim_pad + q->vdim_pad) != pool->latent_dim[run]) return WR_HIP_ERR_INVAL;
+    return WR_HIP_OK;
+}
+
+static WindowArgs window_args(const wr_hip_mix_step* s, const wr_hip_mix_pool* pool, uint32_t run, const wr_hip_mix_window* q)
+{
+    WindowArgs a = {};
+    a.seqs = s->d<MixSeq>(s->o_seqs);
+    a.row_seq = s->d<uint32_t>(s->o_seq);
+    a.row_pos = s->d<uint32_t>(s->o_pos);
+    a.pages = s->d<uint32_t>(s->o_pages);
+    a.rows = s->rows;
+    a.heads = q->heads;
+    a.kvh = q->kv_heads;
+    a.group = q->heads / q->kv_heads;
+    a.dim = q->dim;
+    a.dimp = q->dim_pad;
+    a.vdim = q->vdim;
+    a.vdimp = q->vdim_pad;
+    a.half = q->rot_half;
+    a.window = q->window;
+    a.norm_values = q->norm_values;
+    a.scale = q->scale;
+    a.out_scale = q->out_scale;
+    a.eps = q->eps;
+    a.cache = pool->latent[run];
+    return a;
+}
+
+int wr_hip_mix_window_append(wr_hip_mix_step* s, wr_hip_mix_pool* pool, uint32_t run, int f32, const wr_hip_mix_window* q,
+                             const float* in_dev, uint32_t ld, uint32_t col_q, uint32_t col_k, uint32_t col_v,
+                             const float* table_dev, void* q_dev)
+{
+    if (!g.inited) return WR_HIP_ERR_STATE;
+    int rc = check_window(s, pool, run, f32, q);
+    if (rc) return rc;
+    if (!in_dev || !q_dev || (q->rot_half && !table_dev) || (uint64_t)col_q + (uint64_t)q->heads * q->dim > ld ||
+        (uint64_t)col_k + (uint64_t)q->kv_heads * q->dim > ld || (uint64_t)col_v + (uint64_t)q->kv_heads * q->vdim > ld)
+        return WR_HIP_ERR_INVAL;
+    ENTER();
+    WindowArgs a = window_args(s, pool, run, q);
+    a.in = in_dev;
+    a.ld = ld;
+    a.col_q = col_q;
+    a.col_k = col_k;
+    a.col_v = col_v;
+    a.table = table_dev;
+    a.q = q_dev;
+    const dim3 grid((s->rows + 3) / 4, a.kvh + (4 * a.heads * (a.dimp / 8) + kWindowQUnits - 1) / kWindowQUnits);
+    if (f32) MIX_LAUNCH(window_append_kernel<true>, grid, dim3(256), 0, a);
+    else MIX_LAUNCH(window_append_kernel<false>, grid, dim3(256), 0, a);
+    return WR_HIP_OK;
+}
+
+template <int KQ, int VT>
+static int window_mfma(wr_hip_mix_step* s, WindowArgs& a)
+{
+    if (s->n_long) {
+        uint64_t tiles = 0;
+        for (uint32_t i = 0; i < s->n_long; i++) tiles += ((uint64_t)s->long_rows[i] * a.group + 127) / 128;
+        a.list = s->d<uint32_t>(s->o_long);
+        a.n_list = s->n_long;
+        constexpr size_t lds = window_prefill_lds(KQ, VT);
+        int rc = allow_lds<window_prefill_kernel<KQ, VT>>(lds);
+        if (rc) return rc;
+        launch_main(window_prefill_kernel<KQ, VT>, dim3((uint32_t)(tiles * a.kvh)), dim3(256), a, lds);
+        HIP_TRY(hipGetLastError(), "windowed prefill launch", 0);
+    }
+    const uint32_t n = s->n_short_rows;
+    if (n == 0) return WR_HIP_OK;
+    const LatentRow* rows = s->h<LatentRow>(s->o_short_rows);
+    uint32_t keys = 1;                                     // of the row that sees the most, from its first block on
+    for (uint32_t i = 0; i < n; i++) {
+        const uint32_t lo = rows[i].pos + 1 > a.window ? rows[i].pos + 1 - a.window : 0;
+        keys = std::max(keys, rows[i].pos + 1 - lo / 32 * 32);
+    }
+    const uint32_t groups = a.kvh * ((a.group + 15) / 16);
+    // Shares: two workgroups per compute unit at a time; a round costs about three iterations before its first and one
+    // for each it makes, and the shares' sums about two more to put together.
+    uint64_t best = ~(uint64_t)0;
+    for (uint32_t iters = 1; iters <= 256; iters++) {
+        const uint64_t share = (uint64_t)iters * 128, splits = (keys + share - 1) / share;
+        if (splits > kWindowSplits) continue;
+        const uint64_t rounds = ((uint64_t)n * groups * splits + 2 * g.n_cus - 1) / (2 * g.n_cus);
+        const uint64_t cost = rounds * (iters + 3) + (splits > 1 ? 2 : 0);
+        if (cost < best) {
+            best = cost;
+            a.split_keys = (uint32_t)share;
+            a.splits = (uint32_t)splits;
+        }
+        if (splits == 1) break;
+    }
+    a.drows = s->d<LatentRow>(s->o_short_rows);
+    if (a.splits > 1) {
+        const size_t part = (size_t)n * a.heads * a.splits;
+        int rc = ensure_device(s->partial, part * (VT * 32 + 2) * 4);
+        if (rc) return rc;
+        a.part_o = reinterpret_cast<float*>(s->partial.p);
+        a.part_ml = a.part_o + part * VT * 32;
+    }
+    launch_main(window_decode_kernel<KQ, VT>, dim3(n * groups, a.splits), dim3(256), a);
+    HIP_TRY(hipGetLastError(), "windowed decode launch", 0);
+    if (a.splits > 1) MIX_LAUNCH(window_combine_kernel<VT>, dim3(n, a.heads), dim3(64), 0, a);
+    return WR_HIP_OK;
+}
+
+template <int KQ>
+static int window_mfma_v(wr_hip_mix_step* s, WindowArgs& a)
+{
+    if (a.vdimp == 32) return window_mfma<KQ, 1>(s, a);
+    if (a.vdimp == 64) return window_mfma<KQ, 2>(s, a);
+    return window_mfma<KQ, 4>(s, a);
+}
+
+int wr_hip_mix_window_attend(wr_hip_mix_step* s, wr_hip_mix_pool* pool, uint32_t run, int f32, const wr_hip_mix_window* q,
+                             const void* q_dev, const float* sink_dev, void* o_dev, uint32_t o_kt)
+{
+    if (!g.inited) return WR_HIP_ERR_STATE;
+    int rc = check_window(s, pool, run, f32, q);
+    if (rc) return rc;
+    if (!q_dev || !o_dev || (uint64_t)q->heads * q->vdim_pad > (uint64_t)o_kt * 32) return WR_HIP_ERR_INVAL;
+    ENTER();
+    g.calls.fetch_add(s->n_seq, std::memory_order_relaxed);
+    WindowArgs a = window_args(s, pool, run, q);
+    a.q = const_cast<void*>(q_dev);
+    a.sink = sink_dev;
+    a.o = o_dev;
+    a.o_kt = o_kt;
+    auto fits = [](uint32_t p) { return p == 32 || p == 64 || p == 128; };
+    if (!f32 && !g.force_generic && fits(a.dimp) && fits(a.vdimp)) {
+        if (a.dimp == 32) return window_mfma_v<1>(s, a);
+        if (a.dimp == 64) return window_mfma_v<2>(s, a);
+        return window_mfma_v<4>(s, a);
+    }
+    const size_t lds = ((size_t)a.dimp + a.vdimp + 64) * 4;
+    rc = f32 ? allow_lds<window_attend_any_kernel<true>>(lds) : allow_lds<window_attend_any_kernel<false>>(lds);
+    if (rc) return rc;
+    if (f32) MIX_LAUNCH(window_attend_any_kernel<true>, dim3(s->rows, a.heads), dim3(64), lds, a);
+    else MIX_LAUNCH(window_attend_any_kernel<false>, dim3(s->rows, a.heads), dim3(64), lds, a);
     return WR_HIP_OK;
 }
 

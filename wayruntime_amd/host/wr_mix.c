@@ -130,6 +130,7 @@ static void *take(bump *b, size_t bytes)
 /* Rows shared by every layer. */
 typedef struct walk {
     float *x, *x0, *y;                     /* [R][width_p]: residual, embedding output, a sublayer's output */
+    float *x_next;                         /* the residual's other buffer: a token shift moves it there */
     void  *h;                              /* frag: a sublayer's input */
     float *rope[WRH_MAX_LAYERS];           /* rotary tables (one per distinct rotation) */
 } walk;
@@ -146,6 +147,16 @@ typedef struct latent_rows {
     float *qr;
     void  *q, *oc, *ov;
 } latent_rows;
+
+typedef struct wkv_rows {
+    void  *mix, *low, *oh;
+    float *in, *z;
+} wkv_rows;
+
+typedef struct parallel_rows {
+    void  *low, *q, *oh;
+    float *in, *z;
+} parallel_rows;
 
 typedef struct moe_rows {
     float    *z, *gate, *ys;
@@ -165,6 +176,7 @@ static walk take_walk(bump *b, const struct wrh_mix_model *mm, size_t R)
     const size_t e = mm->f32 ? 4 : 2;
     w.x = take(b, R * mm->width_p * 4);
     w.x0 = mm->looped ? take(b, R * mm->width_p * 4) : NULL;
+    w.x_next = mm->has_shift ? take(b, R * mm->width_p * 4) : NULL;
     w.y = take(b, R * mm->width_p * 4);
     w.h = take(b, r16(R) * mm->width_p * e);
     for (uint32_t i = 0; i < mm->n_ropes; i++) w.rope[i] = take(b, R * mm->ropes[i].dims * 4 + 4);
@@ -191,6 +203,32 @@ static latent_rows take_latent(bump *b, const wrh_mix_layer *L, size_t R, size_t
     r.q = take(b, r16(R) * H * (L->geo.rank_pad + L->geo.rot_pad) * e);
     r.oc = take(b, r16(R) * H * L->geo.rank_pad * e);
     r.ov = take(b, r16(R) * H * L->vdim_p * e);
+    return r;
+}
+
+static wkv_rows take_wkv(bump *b, const struct wrh_mix_model *mm, const wrh_mix_layer *L, size_t R)
+{
+    wkv_rows r;
+    const size_t e = mm->f32 ? 4 : 2;
+    r.mix = take(b, r16(R) * 5 * mm->width_p * e);
+    r.low = take(b, r16(R) * L->rec.rank_p * e);
+    r.in = take(b, R * 4 * L->rec.hd_p * 4);
+    r.z = take(b, R * L->rec.hd_p * 4);
+    r.oh = take(b, r16(R) * L->rec.hd_p * e);
+    return r;
+}
+
+/* Inputs of the layer's output product: the attention's heads, padded one by one, then the recurrence's. */
+static uint32_t parallel_out(const wrh_mix_layer *L) { return L->heads * L->win.vdim_pad + L->rec.hd_p; }
+
+static parallel_rows take_parallel(bump *b, const wrh_mix_layer *L, size_t R, size_t e)
+{
+    parallel_rows r;
+    r.low = take(b, r16(R) * L->rec.rank_p * e);
+    r.in = take(b, R * L->ld_in * 4);
+    r.z = take(b, R * L->rec.hd_p * 4);
+    r.q = take(b, r16(R) * L->heads * L->win.dim_pad * e);
+    r.oh = take(b, r16(R) * parallel_out(L) * e);
     return r;
 }
 
@@ -229,8 +267,12 @@ static size_t scratch_bytes(const struct wrh_mix_model *mm, size_t R)
     for (uint32_t i = 0; i < mm->n_layers; i++) {
         const wrh_mix_layer *L = &mm->layers[i];
         bump b = {NULL, 0};
-        if (L->kind == WRH_MIXER_LIGHTNING) (void)take_lightning(&b, L, R, e);
-        else (void)take_latent(&b, L, R, e);
+        switch (L->kind) {
+        case WRH_MIXER_LIGHTNING: (void)take_lightning(&b, L, R, e); break;
+        case WRH_MIXER_LATENT: (void)take_latent(&b, L, R, e); break;
+        case WRH_MIXER_WKV: (void)take_wkv(&b, mm, L, R); break;
+        case WRH_MIXER_PARALLEL: (void)take_parallel(&b, L, R, e); break;
+        }
         if (b.at > most) most = b.at;
         bump f = {NULL, 0};
         if (L->mlp == WRH_MLP_DENSE) (void)take(&f, r16(R) * L->ff_p * e);
@@ -340,6 +382,80 @@ static wr_status walk_latent(wr_model *m, const wrh_mix_layer *L, uint32_t r, co
     return WR_OK;
 }
 
+/* The decay's second product and the recurrence itself; `rec` has the rest filled in. */
+static wr_status walk_recur(wr_model *m, const wrh_mix_recur *q, uint32_t r, uint32_t store, const void *low, float *z,
+                            wr_hip_mix_recurrence *rec, uint32_t R)
+{
+    struct wrh_mix_model *mm = m->mix;
+    const wr_hip_mix_gemm decay = {.w = q->w_decay, .x = low, .x_kt = q->rank_p / 32, .rows = R,
+                                   .out = WR_HIP_MIX_OUT_ROWS_F32, .y_f32 = z, .ldy = q->hd_p};
+    TRY(wr_hip_mix_gemm_run(mm->f32, &decay), "decay product");
+    rec->heads = q->heads;
+    rec->dim = q->dim;
+    rec->eps = mm->eps;
+    rec->w0 = q->w0;
+    rec->norm = q->norm;
+    rec->z = z;
+    rec->ldz = q->hd_p;
+    TRY(wr_hip_mix_recur(mm->step, mm->pool, store, mm->f32, rec), "matrix-state recurrence");
+    return WR_OK;
+}
+
+/* Takes the residual from w->x and the sublayer output `y` waiting to join it (or NULL) to w->x_next. */
+static wr_status walk_wkv(wr_model *m, const wrh_mix_layer *L, uint32_t r, walk *w, bump b, uint32_t R, const float *y)
+{
+    struct wrh_mix_model *mm = m->mix;
+    const wkv_rows t = take_wkv(&b, mm, L, R);
+    const wrh_mix_recur *q = &L->rec;
+    const uint32_t wkt = mm->width_p / 32, hd = q->hd_p;
+    TRY(wr_hip_mix_shift(mm->step, mm->pool, mm->runs[r].store2, mm->f32, mm->width, mm->eps, w->x, y, w->x_next, L->norm1, 5,
+                         L->mu, t.mix), "token shift");
+    if (y) {
+        float *x = w->x;
+        w->x = w->x_next;
+        w->x_next = x;
+    }
+    const wr_hip_mix_gemm in = {.w = L->w_rkvg, .x = t.mix, .x_kt = 5 * wkt, .x_kt_z = wkt, .rows = R,
+                                .out = WR_HIP_MIX_OUT_ROWS_F32, .y_f32 = t.in, .ldy = 4 * hd, .col_z = hd};
+    TRY(wr_hip_mix_gemm_run(mm->f32, &in), "r/k/v/gate projection");
+    const wr_hip_mix_gemm low = {.w = L->w_low, .x = t.mix, .x_kt = 5 * wkt, .x_kt0 = 4 * wkt, .rows = R, .out = WR_HIP_MIX_OUT_FRAG,
+                                 .h = t.low, .h_kt = q->rank_p / 32, .tanh_end = q->rank_p};
+    TRY(wr_hip_mix_gemm_run(mm->f32, &low), "decay's low-rank product");
+    wr_hip_mix_recurrence rec = {.rule = WR_HIP_MIX_RULE_BONUS, .out_scale = 1.0f, .gate_silu = 1, .u = q->u, .in = t.in,
+                                 .ld = 4 * hd, .col_k = hd, .col_v = 2 * hd, .col_g = 3 * hd, .h = t.oh, .h_kt = hd / 32};
+    const wr_status st = walk_recur(m, q, r, mm->runs[r].store, t.low, t.z, &rec, R);
+    if (st != WR_OK) return st;
+    const wr_hip_mix_gemm out = {.w = L->w_o, .x = t.oh, .x_kt = hd / 32, .rows = R, .out = WR_HIP_MIX_OUT_ROWS_F32,
+                                 .y_f32 = w->y, .ldy = mm->width_p};
+    TRY(wr_hip_mix_gemm_run(mm->f32, &out), "output projection");
+    return WR_OK;
+}
+
+static wr_status walk_parallel(wr_model *m, const wrh_mix_layer *L, uint32_t r, const walk *w, bump b, uint32_t R)
+{
+    struct wrh_mix_model *mm = m->mix;
+    const parallel_rows t = take_parallel(&b, L, R, mm->f32 ? 4 : 2);
+    const wrh_mix_recur *q = &L->rec;
+    const uint32_t kt_o = parallel_out(L) / 32, store = mm->runs[r].store;
+    const wr_hip_mix_gemm in = {.w = L->w_in, .x = w->h, .x_kt = mm->width_p / 32, .rows = R, .out = WR_HIP_MIX_OUT_SPLIT,
+                                .h = t.low, .h_kt = q->rank_p / 32, .n_split = q->rank_p, .tanh_end = q->rank_p,
+                                .y_f32 = t.in, .ldy = L->ld_in};
+    TRY(wr_hip_mix_gemm_run(mm->f32, &in), "both halves' projections");
+    TRY(wr_hip_mix_window_append(mm->step, mm->pool, store, mm->f32, &L->win, t.in, L->ld_in, L->col_q, L->col_k, L->col_v,
+                                 w->rope[L->rope], t.q), "rotation + cache append");
+    TRY(wr_hip_mix_window_attend(mm->step, mm->pool, store, mm->f32, &L->win, t.q, L->sink, t.oh, kt_o), "windowed attention");
+    wr_hip_mix_recurrence rec = {.rule = WR_HIP_MIX_RULE_DELTA, .gain = WRH_DELTA_GAIN, .unit_eps = WRH_DELTA_UNIT_EPS,
+                                 .out_scale = L->right_scale, .a_bias = q->a_bias, .in = t.in, .ld = L->ld_in,
+                                 .col_r = L->col_rr, .col_k = L->col_rk, .col_v = L->col_rv, .col_a = L->col_ra,
+                                 .col_g = L->col_rg, .h = t.oh, .h_kt = kt_o, .col_h = L->heads * L->win.vdim_pad};
+    const wr_status st = walk_recur(m, q, r, mm->runs[r].store2, t.low, t.z, &rec, R);
+    if (st != WR_OK) return st;
+    const wr_hip_mix_gemm out = {.w = L->w_o, .x = t.oh, .x_kt = kt_o, .rows = R, .out = WR_HIP_MIX_OUT_ROWS_F32,
+                                 .y_f32 = w->y, .ldy = mm->width_p};
+    TRY(wr_hip_mix_gemm_run(mm->f32, &out), "output projection");
+    return WR_OK;
+}
+
 /* The feed-forward's output: plain rows in w->y, or expert rows that `res` is told to combine. */
 static wr_status walk_mlp(wr_model *m, const wrh_mix_layer *L, uint32_t r, const walk *w, bump b, uint32_t R,
                           wr_hip_mix_resid *res)
@@ -349,7 +465,7 @@ static wr_status walk_mlp(wr_model *m, const wrh_mix_layer *L, uint32_t r, const
     if (L->mlp == WRH_MLP_DENSE) {
         void *act = take(&b, r16(R) * L->ff_p * (mm->f32 ? 4 : 2));
         const wr_hip_mix_gemm gu = {.w = L->w_gu, .x = w->h, .x_kt = wkt, .rows = R, .out = WR_HIP_MIX_OUT_GATED, .h = act,
-                                    .h_kt = L->ff_p / 32};
+                                    .h_kt = L->ff_p / 32, .gelu = L->gelu};
         TRY(wr_hip_mix_gemm_run(mm->f32, &gu), "gate/up projection");
         const wr_hip_mix_gemm down = {.w = L->w_down, .x = act, .x_kt = L->ff_p / 32, .rows = R,
                                       .out = WR_HIP_MIX_OUT_ROWS_F32, .y_f32 = w->y, .ldy = mm->width_p};
@@ -392,20 +508,31 @@ static wr_status capture(struct wrh_mix_model *mm, const walk *w, uint32_t R)
 }
 
 /* All layers over the rows of mm->step; the residual ends up in w->x. */
-static wr_status walk_layers(wr_model *m, const walk *w, bump b, uint32_t R, int fail_run)
+static wr_status walk_layers(wr_model *m, walk *w, bump b, uint32_t R, int fail_run)
 {
     struct wrh_mix_model *mm = m->mix;
     uint32_t r = 0;
     for (uint32_t i = 0; i < mm->n_ropes; i++)
         if (mm->ropes[i].dims)
             TRY(wr_hip_mix_rope_table(mm->step, mm->ropes[i].freq_dev, mm->ropes[i].dims / 2, w->rope[i]), "angles");
-    TRY(wr_hip_mix_embed(mm->step, mm->f32, mm->embed_dev, mm->width, mm->embed_norm, mm->eps, w->x, w->x0,
-                         mm->layers[mm->runs[0].layer].norm1, w->h), "embedding");
+    const wrh_mix_layer *next = &mm->layers[mm->runs[0].layer];
+    /* a layer behind a token shift makes its input from the residual itself */
+    TRY(wr_hip_mix_embed(mm->step, mm->f32, mm->embed_dev, mm->width, mm->embed_norm, mm->embed_scale, mm->eps, w->x, w->x0,
+                         next->kind == WRH_MIXER_WKV ? NULL : next->norm1, w->h), "embedding");
+    const float *y = NULL;                                 /* a sublayer's output that waits for a token shift */
     for (r = 0; r < mm->n_runs; r++) {
-        const wrh_mix_layer *L = &mm->layers[mm->runs[r].layer];
+        const wrh_mix_layer *L = next;
+        next = r + 1 < mm->n_runs ? &mm->layers[mm->runs[r + 1].layer] : NULL;
         if (fail_run == (int)r) return op_fail(m, "mixer (injected)", r, WR_ERR_INTERNAL);
-        wr_status st = L->kind == WRH_MIXER_LIGHTNING ? walk_lightning(m, L, r, w, b, R) : walk_latent(m, L, r, w, b, R);
+        wr_status st = WR_ERR_INTERNAL;
+        switch (L->kind) {
+        case WRH_MIXER_LIGHTNING: st = walk_lightning(m, L, r, w, b, R); break;
+        case WRH_MIXER_LATENT: st = walk_latent(m, L, r, w, b, R); break;
+        case WRH_MIXER_WKV: st = walk_wkv(m, L, r, w, b, R, y); break;
+        case WRH_MIXER_PARALLEL: st = walk_parallel(m, L, r, w, b, R); break;
+        }
         if (st != WR_OK) return st;
+        y = NULL;
         wr_hip_mix_resid res = {.width = mm->width, .eps = mm->eps, .x = w->x, .y = w->y, .post = L->norm1b};
         if (L->mlp != WRH_MLP_NONE) {
             /* the mixer's output joins the residual and the feed-forward's input is made */
@@ -423,10 +550,15 @@ static wr_status walk_layers(wr_model *m, const walk *w, bump b, uint32_t R, int
             if (st != WR_OK) return st;
             res = (wr_hip_mix_resid){.width = mm->width, .eps = mm->eps, .x = w->x};
         }
-        if (r + 1 < mm->n_runs) {
-            res.next = mm->layers[mm->runs[r + 1].layer].norm1;
-            res.h = w->h;
+        if (next) {
             if (mm->runs[r + 1].add_embedding) res.add = w->x0;
+            if (next->kind != WRH_MIXER_WKV) {
+                res.next = next->norm1;
+                res.h = w->h;
+            } else if (res.y && !res.post && !res.top && !res.add) {
+                y = res.y;                                 /* the token shift adds it */
+                res.y = NULL;
+            }
         }
         if (res.y || res.add || res.next) TRY(wr_hip_mix_residual(mm->step, mm->f32, &res), "post-norm + residual");
     }
@@ -559,7 +691,7 @@ wr_status wrh_mix_step(wr_model *m, const wr_step_entry *entries, uint32_t n, fl
             break;
         }
         bump b = {mm->scratch, 0};
-        const walk w = take_walk(&b, mm, R);
+        walk w = take_walk(&b, mm, R);
         st = walk_layers(m, &w, b, R, fail_run);
         if (st == WR_OK && n_want) st = walk_logits(m, &w, n_want, dest, logits);
         /* the step's descriptors are in page-locked memory: they are free again after the wait */

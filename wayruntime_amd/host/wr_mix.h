@@ -1,8 +1,10 @@
 /*
  * wr_mix.h — mixer-stack models: a list of layers, each a mixer (decayed linear
- * attention or windowed attention through a latent) and an optional feed-forward
- * (dense or a mixture of experts), with norms before and after each, part of the
- * list possibly run several times.  Read from a folder with config.json and
+ * attention, windowed attention through a latent, a matrix-state recurrence behind
+ * a token shift, or windowed grouped-query attention and such a recurrence side by
+ * side) and an optional feed-forward (dense or a mixture of experts), with norms
+ * before and, in some designs, after each, part of the list possibly run several
+ * times.  A design (wrh_mix_design) says which of these its models use.  Read from a folder with config.json and
  * model.safetensors.  wr_mix_model.c reads and uploads, wr_mix.c keeps the cache
  * pool and walks the layers.
  */
@@ -13,8 +15,15 @@
 #include "wr_json.h"
 #include "../../include/wr_hip_mix.h"
 
-typedef enum { WRH_MIXER_LIGHTNING, WRH_MIXER_LATENT } wrh_mixer_kind;
+typedef enum { WRH_MIXER_LIGHTNING, WRH_MIXER_LATENT, WRH_MIXER_WKV, WRH_MIXER_PARALLEL } wrh_mixer_kind;
 typedef enum { WRH_MLP_NONE, WRH_MLP_DENSE, WRH_MLP_MOE } wrh_mlp_kind;
+
+/* A matrix-state recurrence: its own part of a layer's products and vectors. */
+typedef struct wrh_mix_recur {
+    uint32_t heads, dim, hd_p, rank_p;    /* hd = heads * dim; rank of the decay's low-rank product */
+    wr_hip_mat *w_decay;                  /* [hd_p][rank_p] */
+    const float *w0, *u, *a_bias, *norm;
+} wrh_mix_recur;
 
 /* Feature counts ending in _p are padded to a multiple of 32. */
 typedef struct wrh_mix_layer {
@@ -30,8 +39,19 @@ typedef struct wrh_mix_layer {
     wr_hip_mix_latent geo;
     wr_hip_mat *w_d, *w_uq, *w_uk, *w_uv;
     const float *dq_norm, *dkv_norm;
+    /* wkv: token shift, a batch of four products r, k, v, g, the decay's two; w_o */
+    wrh_mix_recur rec;
+    wr_hip_mat *w_rkvg, *w_low;
+    const float *mu;                      /* five vectors: r, k, v, g, w */
+    /* parallel: one stacked product [low | q | k | v | r | k | v | g | a], w_o over both halves' outputs */
+    wr_hip_mix_window win;
+    float right_scale;
+    wr_hip_mat *w_in;
+    uint32_t col_q, col_k, col_v, col_rr, col_rk, col_rv, col_rg, col_ra, ld_in;
+    const float *sink;
     /* feed-forward */
     wrh_mlp_kind mlp;
+    uint8_t gelu;
     uint32_t ff, ff_p, experts, experts_p, top;
     wr_hip_mat *w_gu, *w_down, *w_router, *w_eup, *w_edown;
     const float *norm1, *norm1b, *norm2, *norm2b;
@@ -40,7 +60,8 @@ typedef struct wrh_mix_layer {
 /* One run of a layer: a looped layer has several, each with its own cache or state. */
 typedef struct wrh_mix_run {
     uint32_t layer;
-    uint32_t store;                       /* index of its latent pages or state in the pool */
+    uint32_t store;                       /* index of its pages (attention) or state in the pool */
+    uint32_t store2;                      /* parallel: state of its recurrence; wkv: the previous token's input */
     uint8_t  add_embedding;               /* the embedding output joins the residual before it */
 } wrh_mix_run;
 
@@ -53,8 +74,8 @@ typedef struct wrh_mix_rope {
 struct wrh_mix_model {
     int      f32;                         /* 32-bit activations */
     uint32_t width, width_p, vocab, vocab_p, n_layers, n_runs, n_ropes, n_latent, n_state;
-    float    eps, logit_scale;
-    int      looped;
+    float    eps, logit_scale, embed_scale;
+    int      looped, has_shift;
     wrh_mix_layer *layers;
     wrh_mix_run   *runs;
     wrh_mix_rope  *ropes;
@@ -81,6 +102,10 @@ struct wrh_mix_model {
 };
 
 #define WRH_MIX_LOGIT_ROWS 64
+
+/* The delta rule's own constants: log w = -exp(-1/2) * logistic, unit keys over sqrt(k . k + 1e-6). */
+#define WRH_DELTA_GAIN     0.60653065971263342360f
+#define WRH_DELTA_UNIT_EPS 1e-6f
 
 typedef struct wrh_mix_session {
     uint32_t slot, buf;                   /* state slot; which of its buffers is current */

@@ -20,9 +20,27 @@
 static uint32_t p32(uint32_t n) { return (n + 31) / 32 * 32; }
 static uint32_t p16(uint32_t n) { return (n + 15) / 16 * 16; }
 
+/* What tells the designs of this family apart. */
+typedef enum { DESIGN_BIPOTAR = 1, DESIGN_TAREDRA = 2 } design_bit;
+typedef struct wrh_mix_design {
+    const char *arch;
+    design_bit  bit;
+    uint8_t post_norms;                   /* a sublayer's output is normed before it joins the residual */
+    uint8_t norms_around_zero;            /* stored w means 1 + w */
+    uint8_t embed_norm;                   /* the embedding is normed; else multiplied by embedding.scale */
+    uint8_t tied_head;                    /* the head is the embedding table */
+    uint8_t gelu;                         /* dense feed-forwards gate with the tanh form of GELU, else SiLU */
+} wrh_mix_design;
+
+static const wrh_mix_design designs[] = {
+    {.arch = "Bipotar", .bit = DESIGN_BIPOTAR, .post_norms = 1, .embed_norm = 1},
+    {.arch = "Taredra", .bit = DESIGN_TAREDRA, .norms_around_zero = 1, .tied_head = 1, .gelu = 1},
+};
+
 /* Everything the reading functions share; `st` keeps the first failure. */
 typedef struct loader {
     wr_engine            *e;
+    const wrh_mix_design *design;
     struct wrh_mix_model *mm;
     wrh_safetensors       f;
     float                *vec;            /* host copy of the vector block being gathered */
@@ -109,6 +127,24 @@ static const uint16_t *tensor(loader *l, const char *name, uint32_t rows, uint32
     return (const uint16_t *)t->data;
 }
 
+/* Rows of a matrix whose height only its shape tells; 0 after a failure. */
+static uint32_t tensor_rows(loader *l, uint32_t i, const char *name, uint32_t hi)
+{
+    char nb[128];
+    snprintf(nb, sizeof nb, "l%u.%s", i, name);
+    if (l->st != WR_OK) return 0;
+    const wrh_tensor *t = wrh_safetensors_find(&l->f, nb);
+    if (!t || t->n_dims != 2) {
+        fail(l, WR_ERR_FORMAT, "required matrix %s is missing", nb);
+        return 0;
+    }
+    if (t->shape[0] < 1 || t->shape[0] > hi) {
+        fail(l, WR_ERR_LIMIT, "tensor %s has too many rows", nb);
+        return 0;
+    }
+    return (uint32_t)t->shape[0];
+}
+
 /* layer tensor "l<i>.<name>" */
 static const uint16_t *ltensor(loader *l, uint32_t i, const char *name, uint32_t rows, uint32_t cols)
 {
@@ -154,6 +190,15 @@ static const float *vec_put(loader *l, const uint16_t *src, uint32_t n)
     if (!v) return NULL;
     for (uint32_t i = 0; i < n; i++) v[i] = widen(src[i]);
     return (const float *)(uintptr_t)(at + 1);
+}
+
+/* a norm's weights, as factors */
+static const float *norm_put(loader *l, const uint16_t *src, uint32_t n)
+{
+    const float *at = vec_put(l, src, n);
+    if (at && l->design->norms_around_zero)
+        for (uint32_t i = 0; i < n; i++) l->vec[(uintptr_t)at - 1 + i] += 1.0f;
+    return at;
 }
 
 static void vec_fix(const struct wrh_mix_model *mm, const float **p)
@@ -251,6 +296,33 @@ static void read_lightning(loader *l, uint32_t i, const wrh_json *c, wrh_mix_lay
     L->mix_norm = vec_put(l, ltensor(l, i, "mix.norm", hv, 0), hv);
 }
 
+/* The model's table of this rotation. */
+static uint32_t rope_index(loader *l, double base, uint32_t dims)
+{
+    struct wrh_mix_model *mm = l->mm;
+    uint32_t k = 0;
+    while (k < mm->n_ropes && !(mm->ropes[k].base == base && mm->ropes[k].dims == dims)) k++;
+    if (k == WRH_MAX_LAYERS) {
+        fail(l, WR_ERR_LIMIT, "config: more than %u different rotations", WRH_MAX_LAYERS);
+        return 0;
+    }
+    if (k == mm->n_ropes) {
+        mm->ropes[mm->n_ropes].base = base;
+        mm->ropes[mm->n_ropes++].dims = dims;
+    }
+    return k;
+}
+
+/* The output matrix over heads whose inputs are padded one by one: [Wp][H * vp], zeros between.  `at`: its first
+ * input inside a wider matrix. */
+static void put_heads_out(loader *l, operand *o, const uint16_t *wo, uint32_t at, uint32_t H, uint32_t v, uint32_t vp)
+{
+    if (l->st != WR_OK || !wo) return;
+    for (uint32_t r = 0; r < l->mm->width; r++)
+        for (uint32_t h = 0; h < H; h++)
+            memcpy(operand_row(o, 0, r) + at + (size_t)h * vp, wo + ((size_t)r * H + h) * v, (size_t)v * 2);
+}
+
 static void read_latent(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *L)
 {
     struct wrh_mix_model *mm = l->mm;
@@ -286,16 +358,8 @@ static void read_latent(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer 
     g->rot_half = dims / 2;
     g->window = window;
     g->scale = (float)scale;
-    for (L->rope = 0; L->rope < mm->n_ropes; L->rope++)
-        if (mm->ropes[L->rope].base == base && mm->ropes[L->rope].dims == dims) break;
-    if (L->rope == WRH_MAX_LAYERS) {
-        fail(l, WR_ERR_LIMIT, "config: more than %u different rotations", WRH_MAX_LAYERS);
-        return;
-    }
-    if (L->rope == mm->n_ropes) {
-        mm->ropes[mm->n_ropes].base = base;
-        mm->ropes[mm->n_ropes++].dims = dims;
-    }
+    L->rope = rope_index(l, base, dims);
+    if (l->st != WR_OK) return;
 
     const uint32_t kp = p32(L->kv_rank), rp = p32(L->rot_dim);
     operand o = operand_new(l, 1, L->q_rank_p + kp + rp, Wp);
@@ -332,12 +396,121 @@ static void read_latent(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer 
     for (uint32_t h = 0; h < H && uv; h++) operand_put(l, &o, h, 0, uv + (size_t)h * L->vdim * L->kv_rank, L->vdim, L->kv_rank);
     L->w_uv = operand_up(l, &o);
 
-    const uint16_t *wo = ltensor(l, i, "mix.o", W, H * L->vdim);
     o = operand_new(l, 1, Wp, H * L->vdim_p);
-    if (l->st == WR_OK)
-        for (uint32_t r = 0; r < W; r++)
-            for (uint32_t h = 0; h < H; h++)
-                memcpy(operand_row(&o, 0, r) + (size_t)h * L->vdim_p, wo + ((size_t)r * H + h) * L->vdim, (size_t)L->vdim * 2);
+    put_heads_out(l, &o, ltensor(l, i, "mix.o", W, H * L->vdim), 0, H, L->vdim, L->vdim_p);
+    L->w_o = operand_up(l, &o);
+}
+
+/* What the recurrences share: sizes, decay and norm; tensor names behind `prefix`. */
+static void read_recur(loader *l, uint32_t i, const char *prefix, const wrh_json *c, wrh_mix_recur *q)
+{
+    char nb[64];
+#define NAME(n) (snprintf(nb, sizeof nb, "%s%s", prefix, n), nb)
+    q->heads = need_u32(l, c, "heads", 1, HEADS_MAX);
+    q->dim = need_u32(l, c, "dim", 1, WR_HIP_MIX_MAX_RECUR_DIM);
+    const uint32_t rank = tensor_rows(l, i, NAME("w1"), DIM_MAX);
+    if (l->st != WR_OK) return;
+    const uint32_t hd = q->heads * q->dim;
+    q->hd_p = p32(hd);
+    q->rank_p = p32(rank);
+    q->w_decay = plain(l, ltensor(l, i, NAME("w2"), hd, rank), hd, rank, q->hd_p);
+    q->w0 = vec_put(l, ltensor(l, i, NAME("w0"), hd, 0), hd);
+    q->norm = vec_put(l, ltensor(l, i, NAME("norm"), hd, 0), hd);
+#undef NAME
+}
+
+static void read_wkv(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *L)
+{
+    struct wrh_mix_model *mm = l->mm;
+    const uint32_t W = mm->width, Wp = mm->width_p;
+    wrh_mix_recur *q = &L->rec;
+    L->kind = WRH_MIXER_WKV;
+    read_recur(l, i, "mix.", c, q);
+    if (l->st != WR_OK) return;
+    const uint32_t hd = q->heads * q->dim;
+    L->heads = q->heads;
+    L->dim = L->vdim = q->dim;
+    q->u = vec_put(l, ltensor(l, i, "mix.u", q->heads, q->dim), hd);
+    static const char *const mus[] = {"mix.mu.r", "mix.mu.k", "mix.mu.v", "mix.mu.g", "mix.mu.w"};
+    for (uint32_t k = 0; k < 5; k++) {                     /* one after the other: each takes the padded width */
+        const float *m = vec_put(l, ltensor(l, i, mus[k], W, 0), W);
+        if (k == 0) L->mu = m;
+    }
+    static const char *const ins[] = {"mix.r", "mix.k", "mix.v", "mix.g"};
+    operand o = operand_new(l, 4, q->hd_p, Wp);
+    for (uint32_t k = 0; k < 4; k++) operand_put(l, &o, k, 0, ltensor(l, i, ins[k], hd, W), hd, W);
+    L->w_rkvg = operand_up(l, &o);
+    const uint32_t rank = tensor_rows(l, i, "mix.w1", DIM_MAX);
+    L->w_low = plain(l, ltensor(l, i, "mix.w1", rank, W), rank, W, q->rank_p);
+    L->w_o = plain(l, ltensor(l, i, "mix.o", W, hd), W, hd, Wp);
+    mm->has_shift = 1;
+}
+
+static void read_parallel(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *L)
+{
+    struct wrh_mix_model *mm = l->mm;
+    const uint32_t W = mm->width, Wp = mm->width_p;
+    L->kind = WRH_MIXER_PARALLEL;
+    const wrh_json *left = need_obj(l, c, "left"), *right = need_obj(l, c, "right");
+    const double ls = need_num(l, c, "left_scale"), rs = need_num(l, c, "right_scale");
+    if (l->st != WR_OK) return;
+    wr_hip_mix_window *g = &L->win;
+    const uint32_t H = g->heads = L->heads = need_u32(l, left, "heads", 1, HEADS_MAX);
+    const uint32_t G = g->kv_heads = need_u32(l, left, "kv_heads", 1, HEADS_MAX);
+    const uint32_t D = g->dim = L->dim = need_u32(l, left, "dim", 1, 4096);
+    const uint32_t V = g->vdim = L->vdim = need_u32(l, left, "vdim", 1, 4096);
+    const wrh_json *rot = need_obj(l, left, "rot"), *mask = need_obj(l, left, "mask");
+    g->scale = (float)need_num(l, left, "scale");
+    if (l->st != WR_OK) return;
+    const double base = need_num(l, rot, "base");
+    const uint32_t dims = need_u32(l, rot, "dims", 0, D);
+    g->window = need_u32(l, mask, "size", 1, 0xFFFFFFFFu);
+    if (l->st == WR_OK && (dims % 2 || base <= 0)) fail(l, WR_ERR_FORMAT, "config: layer %u: rotation of %u dimensions, base %g", i, dims, base);
+    if (l->st == WR_OK && H % G) fail(l, WR_ERR_FORMAT, "config: layer %u: %u heads over %u key/value heads", i, H, G);
+    if (l->st != WR_OK) return;
+    g->dim_pad = wr_hip_mix_window_pad(D);
+    g->vdim_pad = wr_hip_mix_window_pad(V);
+    g->rot_half = dims / 2;
+    g->out_scale = (float)ls;
+    g->norm_values = 1;
+    g->eps = mm->eps;
+    L->right_scale = (float)rs;
+    if ((uint64_t)H * g->dim_pad > DIM_MAX || (uint64_t)H * g->vdim_pad > DIM_MAX) {
+        fail(l, WR_ERR_LIMIT, "config: layer %u is too wide", i);
+        return;
+    }
+    L->rope = rope_index(l, base, dims);
+    wrh_mix_recur *q = &L->rec;
+    read_recur(l, i, "mix.right.", right, q);
+    if (l->st != WR_OK) return;
+    const uint32_t hd = q->heads * q->dim;
+    q->a_bias = vec_put(l, ltensor(l, i, "mix.right.a.b", hd, 0), hd);
+    L->sink = vec_put(l, ltensor(l, i, "mix.left.sink", H, 0), H);
+
+    /* one product of the layer's input: the decay's low-rank part first, then 32-bit rows */
+    const uint32_t rank = tensor_rows(l, i, "mix.right.w1", DIM_MAX);
+    const struct {
+        const char *name;
+        uint32_t rows, *col;
+    } parts[] = {{"mix.left.q", H * D, &L->col_q},  {"mix.left.k", G * D, &L->col_k},  {"mix.left.v", G * V, &L->col_v},
+                 {"mix.right.r", hd, &L->col_rr},   {"mix.right.k", hd, &L->col_rk},   {"mix.right.v", hd, &L->col_rv},
+                 {"mix.right.g", hd, &L->col_rg},   {"mix.right.a", hd, &L->col_ra}};
+    const size_t n = sizeof parts / sizeof *parts;
+    L->ld_in = 0;
+    for (size_t k = 0; k < n; k++) {
+        *parts[k].col = L->ld_in;
+        L->ld_in += p32(parts[k].rows);
+    }
+    operand o = operand_new(l, 1, q->rank_p + L->ld_in, Wp);
+    operand_put(l, &o, 0, 0, ltensor(l, i, "mix.right.w1", rank, W), rank, W);
+    for (size_t k = 0; k < n; k++)
+        operand_put(l, &o, 0, q->rank_p + *parts[k].col, ltensor(l, i, parts[k].name, parts[k].rows, W), parts[k].rows, W);
+    L->w_in = operand_up(l, &o);
+
+    /* one product over both halves' outputs, which arrive scaled */
+    o = operand_new(l, 1, Wp, H * g->vdim_pad + q->hd_p);
+    put_heads_out(l, &o, ltensor(l, i, "mix.left.o", W, H * V), 0, H, V, g->vdim_pad);
+    put_heads_out(l, &o, ltensor(l, i, "mix.right.o", W, hd), H * g->vdim_pad, 1, hd, q->hd_p);
     L->w_o = operand_up(l, &o);
 }
 
@@ -345,6 +518,7 @@ static void read_dense(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *
 {
     const uint32_t W = l->mm->width, Wp = l->mm->width_p;
     L->mlp = WRH_MLP_DENSE;
+    L->gelu = l->design->gelu;
     L->ff = need_u32(l, c, "ff", 1, DIM_MAX);
     if (l->st != WR_OK) return;
     L->ff_p = p32(L->ff);
@@ -393,29 +567,35 @@ static void read_layer(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *
     static const struct {
         const char *name;
         void (*read)(loader *, uint32_t, const wrh_json *, wrh_mix_layer *);
-    } mixers[] = {{"lightning", read_lightning}, {"latent_attention", read_latent}},
-      mlps[] = {{"dense", read_dense}, {"moe", read_moe}};
+        unsigned designs;
+    } mixers[] = {{"lightning", read_lightning, DESIGN_BIPOTAR},
+                  {"latent_attention", read_latent, DESIGN_BIPOTAR},
+                  {"wkv", read_wkv, DESIGN_TAREDRA},
+                  {"parallel", read_parallel, DESIGN_TAREDRA}},
+      mlps[] = {{"dense", read_dense, DESIGN_BIPOTAR | DESIGN_TAREDRA}, {"moe", read_moe, DESIGN_BIPOTAR}};
+    const size_t n_mixers = sizeof mixers / sizeof *mixers, n_mlps = sizeof mlps / sizeof *mlps;
+    const wrh_mix_design *d = l->design;
     size_t k = 0;
-    while (k < 2 && strcmp(type, mixers[k].name)) k++;
-    if (k == 2) {
+    while (k < n_mixers && (strcmp(type, mixers[k].name) || !(mixers[k].designs & d->bit))) k++;
+    if (k == n_mixers) {
         fail(l, WR_ERR_UNSUPPORTED, "layer %u: mixer '%s' is not served by this engine", i, type);
         return;
     }
     mixers[k].read(l, i, mixer, L);
-    L->norm1 = vec_put(l, ltensor(l, i, "norm1", W, 0), W);
-    L->norm1b = vec_put(l, ltensor(l, i, "norm1b", W, 0), W);
+    L->norm1 = norm_put(l, ltensor(l, i, "norm1", W, 0), W);
+    if (d->post_norms) L->norm1b = norm_put(l, ltensor(l, i, "norm1b", W, 0), W);
     const wrh_json *mlp = wrh_json_get(c, "mlp");
     if (!mlp || mlp->type == WRH_JSON_NULL) return;
     const char *kind = need_str(l, mlp, "kind");
     if (l->st != WR_OK) return;
-    for (k = 0; k < 2 && strcmp(kind, mlps[k].name); k++) {}
-    if (k == 2) {
+    for (k = 0; k < n_mlps && (strcmp(kind, mlps[k].name) || !(mlps[k].designs & d->bit)); k++) {}
+    if (k == n_mlps) {
         fail(l, WR_ERR_UNSUPPORTED, "layer %u: feed-forward '%s' is not served by this engine", i, kind);
         return;
     }
     mlps[k].read(l, i, mlp, L);
-    L->norm2 = vec_put(l, ltensor(l, i, "norm2", W, 0), W);
-    L->norm2b = vec_put(l, ltensor(l, i, "norm2b", W, 0), W);
+    L->norm2 = norm_put(l, ltensor(l, i, "norm2", W, 0), W);
+    if (d->post_norms) L->norm2b = norm_put(l, ltensor(l, i, "norm2b", W, 0), W);
 }
 
 /* ------------------------------------------------------------------ model -- */
@@ -436,7 +616,7 @@ static void plan_runs(loader *l, const wrh_json *cfg)
     mm->n_runs = mm->n_layers + (times - 1) * (stop - start);
     mm->runs = calloc(mm->n_runs, sizeof *mm->runs);
     mm->latent_dim = calloc(mm->n_runs, sizeof *mm->latent_dim);
-    mm->state_elems = calloc(mm->n_runs, sizeof *mm->state_elems);
+    mm->state_elems = calloc((size_t)2 * mm->n_runs, sizeof *mm->state_elems);
     if (!mm->runs || !mm->latent_dim || !mm->state_elems) {
         fail(l, WR_ERR_NOMEM, "out of memory");
         return;
@@ -451,12 +631,28 @@ static void plan_runs(loader *l, const wrh_json *cfg)
     for (uint32_t i = stop; i < mm->n_layers; i++) mm->runs[n++].layer = i;
     for (uint32_t r = 0; r < n; r++) {
         const wrh_mix_layer *L = &mm->layers[mm->runs[r].layer];
-        if (L->kind == WRH_MIXER_LATENT) {
+        const uint64_t matrix = (uint64_t)L->rec.heads * L->rec.dim * L->rec.dim;
+        switch (L->kind) {
+        case WRH_MIXER_LATENT:
             mm->runs[r].store = mm->n_latent;
             mm->latent_dim[mm->n_latent++] = L->geo.rank_pad + L->geo.rot_pad;
-        } else {
+            break;
+        case WRH_MIXER_LIGHTNING:
             mm->runs[r].store = mm->n_state;
             mm->state_elems[mm->n_state++] = (uint64_t)L->heads * L->dim * L->vdim;
+            break;
+        case WRH_MIXER_WKV:
+            mm->runs[r].store = mm->n_state;
+            mm->state_elems[mm->n_state++] = matrix;
+            mm->runs[r].store2 = mm->n_state;
+            mm->state_elems[mm->n_state++] = mm->width_p;
+            break;
+        case WRH_MIXER_PARALLEL:
+            mm->runs[r].store = mm->n_latent;
+            mm->latent_dim[mm->n_latent++] = L->win.kv_heads * (L->win.dim_pad + L->win.vdim_pad);
+            mm->runs[r].store2 = mm->n_state;
+            mm->state_elems[mm->n_state++] = matrix;
+            break;
         }
     }
 }
@@ -474,7 +670,8 @@ static void upload_small(loader *l)
     vec_fix(mm, &mm->final_norm);
     for (uint32_t i = 0; i < mm->n_layers; i++) {
         wrh_mix_layer *L = &mm->layers[i];
-        const float **p[] = {&L->decay, &L->mix_norm, &L->dq_norm, &L->dkv_norm, &L->norm1, &L->norm1b, &L->norm2, &L->norm2b};
+        const float **p[] = {&L->decay, &L->mix_norm, &L->dq_norm, &L->dkv_norm, &L->norm1, &L->norm1b, &L->norm2, &L->norm2b,
+                             &L->mu, &L->sink, &L->rec.w0, &L->rec.u, &L->rec.a_bias, &L->rec.norm};
         for (size_t k = 0; k < sizeof p / sizeof *p; k++) vec_fix(mm, p[k]);
     }
     for (uint32_t r = 0; r < mm->n_ropes && l->st == WR_OK; r++) {
@@ -496,7 +693,8 @@ void wrh_mix_free(struct wrh_mix_model *mm)
     if (!mm) return;
     for (uint32_t i = 0; mm->layers && i < mm->n_layers; i++) {
         wrh_mix_layer *L = &mm->layers[i];
-        wr_hip_mat *w[] = {L->w_qkvg, L->w_o, L->w_d, L->w_uq, L->w_uk, L->w_uv, L->w_gu, L->w_down, L->w_router, L->w_eup, L->w_edown};
+        wr_hip_mat *w[] = {L->w_qkvg, L->w_o, L->w_d, L->w_uq, L->w_uk, L->w_uv, L->w_gu, L->w_down, L->w_router, L->w_eup,
+                           L->w_edown, L->w_rkvg, L->w_low, L->w_in, L->rec.w_decay};
         for (size_t k = 0; k < sizeof w / sizeof *w; k++) wr_hip_mix_mat_destroy(w[k]);
     }
     for (uint32_t r = 0; mm->ropes && r < mm->n_ropes; r++) wr_hip_attn_dev_free(mm->ropes[r].freq_dev);
@@ -530,7 +728,9 @@ wr_status wrh_mix_load(wr_engine *e, const char *dir, const char *arch, const wr
     struct wrh_mix_model *mm = calloc(1, sizeof *mm);
     if (!mm) return WR_ERR_NOMEM;
     pthread_mutex_init(&mm->lock, NULL);
-    loader l = {e, mm, {0}, NULL, 0, 0, WR_OK};
+    const wrh_mix_design *design = designs;
+    while (strcmp(design->arch, arch)) design++;           /* (the registry holds no other name) */
+    loader l = {e, design, mm, {0}, NULL, 0, 0, WR_OK};
     const wrh_json *layers = wrh_json_get(cfg, "layers");
     if (!layers || layers->type != WRH_JSON_ARRAY || layers->count == 0)
         fail(&l, WR_ERR_FORMAT, "config: 'layers' missing or empty");
@@ -544,6 +744,10 @@ wr_status wrh_mix_load(wr_engine *e, const char *dir, const char *arch, const wr
     double scale = 1.0;
     if (wrh_json_get(cfg, "logit_scale")) scale = need_num(&l, cfg, "logit_scale");
     mm->logit_scale = (float)scale;
+    if (!design->embed_norm) {
+        const wrh_json *emb = need_obj(&l, cfg, "embedding");
+        if (emb) mm->embed_scale = (float)need_num(&l, emb, "scale");
+    }
     if (l.st == WR_OK) {
         mm->n_layers = layers->count;
         mm->layers = calloc(mm->n_layers, sizeof *mm->layers);
@@ -563,9 +767,9 @@ wr_status wrh_mix_load(wr_engine *e, const char *dir, const char *arch, const wr
         const wrh_json *c = layers->first;
         for (uint32_t i = 0; i < mm->n_layers && l.st == WR_OK; i++, c = c->next) read_layer(&l, i, c, &mm->layers[i]);
         const uint16_t *emb = tensor(&l, "embed", mm->vocab, mm->width);
-        mm->embed_norm = vec_put(&l, tensor(&l, "embed.norm", mm->width, 0), mm->width);
-        mm->final_norm = vec_put(&l, tensor(&l, "final.norm", mm->width, 0), mm->width);
-        mm->head = plain(&l, tensor(&l, "head", mm->vocab, mm->width), mm->vocab, mm->width, mm->vocab_p);
+        if (design->embed_norm) mm->embed_norm = norm_put(&l, tensor(&l, "embed.norm", mm->width, 0), mm->width);
+        mm->final_norm = norm_put(&l, tensor(&l, "final.norm", mm->width, 0), mm->width);
+        mm->head = plain(&l, design->tied_head ? emb : tensor(&l, "head", mm->vocab, mm->width), mm->vocab, mm->width, mm->vocab_p);
         if (l.st == WR_OK) {
             const size_t bytes = (size_t)mm->vocab * mm->width * 2;
             mm->embed_dev = wr_hip_attn_dev_alloc(bytes);
@@ -588,6 +792,7 @@ wr_status wrh_mix_load(wr_engine *e, const char *dir, const char *arch, const wr
     m->hidden = mm->width;
     m->vocab = mm->vocab;
     m->rms_eps = mm->eps;
+    m->tied_head = design->tied_head;
     for (uint32_t i = 0; i < mm->n_layers; i++) {
         const wrh_mix_layer *L = &mm->layers[i];
         if (L->heads > m->n_q) m->n_q = L->heads;
@@ -597,6 +802,12 @@ wr_status wrh_mix_load(wr_engine *e, const char *dir, const char *arch, const wr
             m->has_swa = 1;
             m->n_kv = 1;                                   /* one latent row per position, shared by the heads */
             if (L->geo.window > m->sliding_window) m->sliding_window = L->geo.window;
+            m->rope_base = (float)mm->ropes[L->rope].base;
+        }
+        if (L->kind == WRH_MIXER_PARALLEL) {
+            m->has_swa = 1;
+            if (L->win.kv_heads > m->n_kv) m->n_kv = L->win.kv_heads;
+            if (L->win.window > m->sliding_window) m->sliding_window = L->win.window;
             m->rope_base = (float)mm->ropes[L->rope].base;
         }
     }

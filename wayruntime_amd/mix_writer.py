@@ -1,5 +1,5 @@
-"""Writes mixer-stack models (architecture "Bipotar") as a folder with config.json
-and model.safetensors: random-init models for the tests and the benchmark, and any
+"""Writes mixer-stack models (architectures "Bipotar" and "Taredra") as a folder with
+config.json and model.safetensors: random-init models for the tests and the benchmark, and any
 set of bfloat16 tensors a caller has."""
 from __future__ import annotations
 
@@ -24,6 +24,20 @@ def latent_attention(heads: int, dim: int, vdim: int, q_rank: int, kv_rank: int,
                       "scale": (dim + rot_dim) ** -0.5 if scale is None else scale}}
 
 
+def wkv(heads: int, dim: int) -> dict:
+    return {"type": "wkv", "mixer": {"heads": heads, "dim": dim}}
+
+
+def window_and_delta(heads: int, kv_heads: int, dim: int, vdim: int, window: int, right_heads: int, right_dim: int,
+                     rot_dims: int | None = None, base: float = 10000.0, scale: float | None = None,
+                     left_scale: float = 1.0, right_scale: float = 1.0) -> dict:
+    """Windowed grouped-query attention and a delta-rule recurrence side by side."""
+    left = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "mask": {"size": window},
+            "rot": {"base": base, "dims": dim if rot_dims is None else rot_dims}, "scale": dim ** -0.5 if scale is None else scale}
+    return {"type": "parallel", "mixer": {"left": left, "right": {"heads": right_heads, "dim": right_dim},
+                                          "left_scale": left_scale, "right_scale": right_scale}}
+
+
 def dense(ff: int) -> dict:
     return {"kind": "dense", "ff": ff}
 
@@ -39,7 +53,48 @@ def config(width: int, vocab: int, layers, loop=None, eps: float = 1e-6, logit_s
             "layers": [dict(m, mlp=f) for m, f in layers]}
 
 
-def tensor_shapes(cfg: dict) -> dict:
+def prenorm_config(width: int, vocab: int, layers, eps: float = 1e-6, embed_scale: float | None = None) -> dict:
+    """layers: [(mixer, feed-forward or None)] of wkv and window_and_delta mixers."""
+    return {"architecture": "Taredra", "width": width, "vocab": vocab, "norm": {"eps": eps},
+            "embedding": {"scale": width ** 0.5 if embed_scale is None else embed_scale},
+            "layers": [dict(m, mlp=f) for m, f in layers]}
+
+
+def _recur_shapes(p: str, hd: int, W: int, rank: int) -> dict:
+    out = {p + n: (hd, W) for n in "rkvg"}
+    out.update({p + "w1": (rank, W), p + "w2": (hd, rank), p + "w0": (hd,), p + "norm": (hd,), p + "o": (W, hd)})
+    return out
+
+
+def _prenorm_shapes(cfg: dict, rank: int) -> dict:
+    W, out = cfg["width"], {"embed": (cfg["vocab"], cfg["width"])}
+    for i, layer in enumerate(cfg["layers"]):
+        p, m, f = f"l{i}.", layer["mixer"], layer["mlp"]
+        for n in ("norm1",) + (("norm2",) if f else ()):
+            out[p + n] = (W,)
+        if layer["type"] == "wkv":
+            hd = m["heads"] * m["dim"]
+            out.update(_recur_shapes(p + "mix.", hd, W, rank))
+            out.update({p + "mix.mu." + n: (W,) for n in "rkvgw"})
+            out[p + "mix.u"] = (m["heads"], m["dim"])
+        else:
+            a, hd = m["left"], m["right"]["heads"] * m["right"]["dim"]
+            q = p + "mix.left."
+            out.update({q + "q": (a["heads"] * a["dim"], W), q + "k": (a["kv_heads"] * a["dim"], W),
+                        q + "v": (a["kv_heads"] * a["vdim"], W), q + "sink": (a["heads"],), q + "o": (W, a["heads"] * a["vdim"])})
+            q = p + "mix.right."
+            out.update(_recur_shapes(q, hd, W, rank))
+            out.update({q + "a": (hd, W), q + "a.b": (hd,)})
+        if f:
+            out.update({p + "mlp.gate": (f["ff"], W), p + "mlp.up": (f["ff"], W), p + "mlp.down": (W, f["ff"])})
+    out["final.norm"] = (W,)
+    return out
+
+
+def tensor_shapes(cfg: dict, rank: int = 24) -> dict:
+    """`rank`: of the decays' low-rank products, which no configuration names."""
+    if cfg["architecture"] == "Taredra":
+        return _prenorm_shapes(cfg, rank)
     W, out = cfg["width"], {"embed": (cfg["vocab"], cfg["width"]), "embed.norm": (cfg["width"],)}
     for i, layer in enumerate(cfg["layers"]):
         p, m, f = f"l{i}.", layer["mixer"], layer["mlp"]
@@ -72,28 +127,45 @@ def to_bf16(x: np.ndarray) -> np.ndarray:
     return ((u + np.uint32(0x7FFF) + ((u >> np.uint32(16)) & np.uint32(1))) >> np.uint32(16)).astype(np.uint16)
 
 
-def random_tensors(cfg: dict, seed: int = 0, gain: float = 1.0):
-    """Yields (name, bfloat16 bits): norms 1 + 0.1 N(0, 1), matrices gain * N(0, 1 / inputs), the embedding N(0, 1).
+# what the vectors of a pre-norm model are drawn around, and how widely
+_VECTORS = {"norm1": (0, 0.1), "norm2": (0, 0.1), "final.norm": (0, 0.1), "sink": (0, 1), "w0": (-3, 2), "a.b": (0, 1)}
+
+
+def random_tensors(cfg: dict, seed: int = 0, gain: float = 1.0, rank: int = 24):
+    """Yields (name, bfloat16 bits): norms 1 + 0.1 N(0, 1), matrices gain * N(0, 1 / inputs), the embedding N(0, 1);
+    of a pre-norm model the vectors as _VECTORS says, mixing factors in [0, 1], bonuses N(0, 1/4), the embedding N(0, 1 / width).
     Large matrices repeat a pool of samples at different offsets."""
+    prenorm = cfg["architecture"] == "Taredra"
     rng = np.random.default_rng(seed)
     pool = rng.standard_normal(1 << 22, dtype=np.float32)
-    for i, (name, shape) in enumerate(tensor_shapes(cfg).items()):
+    for i, (name, shape) in enumerate(tensor_shapes(cfg, rank).items()):
         n = int(np.prod(shape))
         at = int(rng.integers(0, pool.size))
         x = pool[(at + np.arange(n)) % pool.size] if n <= pool.size else np.resize(np.roll(pool, at), n)
-        if len(shape) == 1:
+        end = name.split(".", 2)[-1] if name.startswith("l") else name
+        end = end.removeprefix("left.").removeprefix("right.")
+        if prenorm and ".mu." in name:
+            x = 1.0 / (1.0 + np.exp(-x))
+        elif prenorm and end == "u":
+            x = 0.5 * x
+        elif prenorm and name == "embed":
+            x = x * np.float32(shape[1] ** -0.5)
+        elif prenorm and end in _VECTORS:
+            at, spread = _VECTORS[end]
+            x = at + spread * x
+        elif len(shape) == 1:
             x = 1.0 + 0.1 * x
         elif name != "embed":
             x = x * np.float32(gain / np.sqrt(shape[1]))
         yield name, to_bf16(x).reshape(shape)
 
 
-def write_model(folder: str, cfg: dict, tensors=None, seed: int = 0) -> str:
+def write_model(folder: str, cfg: dict, tensors=None, seed: int = 0, rank: int = 24) -> str:
     """tensors: {name: bfloat16 bits} or an iterable of such pairs; None draws random ones."""
     os.makedirs(folder, exist_ok=True)
     with open(os.path.join(folder, "config.json"), "w") as f:
         json.dump(cfg, f, indent=1)
-    shapes = tensor_shapes(cfg)
+    shapes = tensor_shapes(cfg, rank)
     header, at = {}, 0
     for name, shape in shapes.items():
         n = 2 * int(np.prod(shape))
@@ -102,7 +174,7 @@ def write_model(folder: str, cfg: dict, tensors=None, seed: int = 0) -> str:
     text = json.dumps(header).encode()
     text += b" " * (-len(text) % 8)
     if tensors is None:
-        tensors = random_tensors(cfg, seed)
+        tensors = random_tensors(cfg, seed, rank=rank)
     pairs = tensors.items() if isinstance(tensors, dict) else tensors
     with open(os.path.join(folder, "model.safetensors"), "wb") as f:
         f.write(struct.pack("<Q", len(text)) + text)
