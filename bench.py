@@ -198,19 +198,25 @@ def decode_config(hipattn, synth, oracle, pool16, name, nq, nkv, hd, ctxs, layer
 
 
 def mixer_workload(args) -> None:
-    """Mixer-stack models and the grouped-query model beside each, end to end through the host engine: one JSON line."""
+    """Mixer-stack models of one design and the models beside them, end to end through the host engine: one JSON line."""
     from wayruntime_amd import mix_timing
 
     steps = min(args.steps, 200)
-    figures = mix_timing.run(list(mix_timing.SIZES), reps=3, steps=steps, log=lambda *a: print(*a, file=sys.stderr, flush=True))
-    top = figures["w4096"]["mixer"]
+    kind = "taredra" if args.workload == "taredra" else "mixer"
+    beside = ("mixer", "gqa") if kind == "taredra" else ("gqa",)
+    model = {"mixer": "Bipotar, 4 layers (linear attention x 2, latent attention x 2; dense and expert feed-forwards), "
+                      "width 4096, random init",
+             "taredra": "Taredra, 4 layers (windowed attention beside a delta-rule recurrence x 2, wkv recurrence x 2; dense "
+                        "feed-forwards), width 4096, random init"}[kind]
+    figures = mix_timing.run(list(mix_timing.SIZES), reps=3, steps=steps, only=(kind,) + beside,
+                             log=lambda *a: print(*a, file=sys.stderr, flush=True))
+    top = figures["w4096"][kind]
     print(json.dumps({
         "metric": "mixer-stack decode tokens/s, 16 sessions x 2048 ctx; prefill tokens/s",
         "value": top["decode_b16_tok_s"], "unit": "tokens/s", "n_gpus": 1, "steps": steps, "warmup": 3,
         "ms_per_step": top["decode_b16_ms"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
         "dtype": "bf16", "data": "synthetic",
-        "config": {"model": "Bipotar, 4 layers (linear attention x 2, latent attention x 2; dense and expert feed-forwards), "
-                            "width 4096, random init", "global_batch": 16, "seq_len": 2048, "parallelism": "single GPU"},
+        "config": {"model": model, "global_batch": 16, "seq_len": 2048, "parallelism": "single GPU"},
         "prefill_tok_s": {n: top[f"prefill_{n}_tok_s"] for n in (512, 2048, 4096)},
         "sizes": figures}), flush=True)
 
@@ -232,7 +238,7 @@ def main() -> None:
     ap.add_argument("--no-decode-configs", action="store_true")
     ap.add_argument("--keys-per-wg", type=int, default=0)
     ap.add_argument("--workload", default="headline",
-                    choices=["headline", "ragged16", "long16", "long16-hd256", "batch1", "mixer"],
+                    choices=["headline", "ragged16", "long16", "long16-hd256", "batch1", "mixer", "taredra"],
                     help="headline: 16 sessions x --ctx, 32/8/128 (the metric's configuration), with "
                          "the other decode workloads as secondary keys; "
                          "ragged16: 16 sessions with contexts drawn from [256, 4096]; "
@@ -240,7 +246,8 @@ def main() -> None:
                          "batch1: one session, 16/8/128, --ctx keys.  Other than headline they "
                          "run that one workload as the timed steps and report the decode figures only; "
                          "mixer: prefill and decode throughput of mixer-stack models (Bipotar) with layers "
-                         "of real sizes, random weights, beside a grouped-query model of the same width")
+                         "of real sizes, random weights, beside a grouped-query model of the same width; "
+                         "taredra: the same of Taredra models, beside both")
     args = ap.parse_args()
 
     if args.gpus != 1:
@@ -248,7 +255,7 @@ def main() -> None:
               "(nothing here uses a second device)" % args.gpus, file=sys.stderr)
         sys.exit(2)
 
-    if args.workload == "mixer":
+    if args.workload in ("mixer", "taredra"):
         mixer_workload(args)
         return
 

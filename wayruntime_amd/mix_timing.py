@@ -2,12 +2,14 @@
 real sizes) beside a grouped-query model of the same width, through the host
 engine.
 
-    python -m wayruntime_amd.mix_timing [--size w2048 w4096] [--json]
+    python -m wayruntime_amd.mix_timing [--size w2048 w4096] [--only mixer taredra gqa] [--json]
 
-Each size has four layers: linear attention with a dense feed-forward and with
-experts, latent attention with experts and with a dense feed-forward.  The model
-beside it is the engine's Llama-style one with four layers of the same width,
-head dimension and feed-forward width (F16 weights)."""
+Each size has four layers.  mixer: linear attention with a dense feed-forward and
+with experts, latent attention with experts and with a dense feed-forward.
+taredra: windowed grouped-query attention beside a delta-rule recurrence, and a
+wkv recurrence, each twice, all with dense feed-forwards.  gqa: the engine's
+Llama-style model with four layers of the same width, head dimension and
+feed-forward width (F16 weights)."""
 from __future__ import annotations
 
 import argparse
@@ -32,10 +34,18 @@ def mixer_config(width: int, heads: int, q_rank: int, ff: int, experts: int, top
     return mw.config(width, VOCAB, [(light, d), (light, m), (latent, m), (latent, d)])
 
 
+def taredra_config(width: int, heads: int, ff: int) -> dict:
+    """Heads of 128 over eight key/value heads; recurrences with heads of 64 over the whole width."""
+    par = mw.window_and_delta(heads, 8, 128, 128, window=4096, right_heads=width // 64, right_dim=64)
+    return mw.prenorm_config(width, VOCAB, [(m, mw.dense(ff)) for m in (par, mw.wkv(width // 64, 64)) * 2])
+
+
+KINDS = ("mixer", "taredra", "gqa")
+RANK = 64                                   # of the decays' low-rank products
 SIZES = {
-    "w2048": (mixer_config(2048, 16, 768, 8192, 64, 6, 1024),
+    "w2048": (mixer_config(2048, 16, 768, 8192, 64, 6, 1024), taredra_config(2048, 16, 8192),
               gw.ModelShape(arch="llama", n_layers=4, hidden=2048, ffn=8192, n_q=16, n_kv=8, vocab=VOCAB, context=8192)),
-    "w4096": (mixer_config(4096, 32, 1536, 12288, 32, 4, 2048),
+    "w4096": (mixer_config(4096, 32, 1536, 12288, 32, 4, 2048), taredra_config(4096, 32, 12288),
               gw.ModelShape(arch="llama", n_layers=4, hidden=4096, ffn=12288, n_q=32, n_kv=8, vocab=VOCAB, context=8192)),
 }
 
@@ -91,26 +101,24 @@ def measure(eng, path: str, reps: int, steps: int) -> dict:
     return out
 
 
-def run(sizes, reps: int = 3, steps: int = 40, only: str = "both", log=print) -> dict:
+def run(sizes, reps: int = 3, steps: int = 40, only=KINDS, log=print) -> dict:
     figures = {}
     with tempfile.TemporaryDirectory() as tmp:
         eng = E.Engine(E.HOST_SO)
         for name in sizes:
-            cfg, shape = SIZES[name]
+            mixer, taredra, shape = SIZES[name]
             fig = figures[name] = {}
-            if only != "gqa":
+            for kind in only:
                 t = time.perf_counter()
-                path = mw.write_model(os.path.join(tmp, name), cfg)
-                log(f"{name}: model written in {time.perf_counter() - t:.1f} s")
-                fig["mixer"] = measure(eng, path, reps, steps)
-                log(f"{name}: mixer stack {fig['mixer']}")
-            if only != "mixer":
-                path = os.path.join(tmp, name + ".gguf")
-                t = time.perf_counter()
-                gw.write_model(path, shape)
-                log(f"{name}: model beside it written in {time.perf_counter() - t:.1f} s")
-                fig["gqa"] = measure(eng, path, reps, steps)
-                log(f"{name}: grouped-query {fig['gqa']}")
+                path = os.path.join(tmp, name + "_" + kind)
+                if kind == "gqa":
+                    path += ".gguf"
+                    gw.write_model(path, shape)
+                else:
+                    mw.write_model(path, mixer if kind == "mixer" else taredra, rank=RANK)
+                log(f"{name}: {kind} model written in {time.perf_counter() - t:.1f} s")
+                fig[kind] = measure(eng, path, reps, steps)
+                log(f"{name}: {kind} {fig[kind]}")
         eng.close()
     return figures
 
@@ -118,7 +126,7 @@ def run(sizes, reps: int = 3, steps: int = 40, only: str = "both", log=print) ->
 def main() -> int:
     ap = argparse.ArgumentParser(description=__doc__.split("\n\n")[0])
     ap.add_argument("--size", nargs="*", default=list(SIZES), choices=list(SIZES))
-    ap.add_argument("--only", default="both", choices=["both", "mixer", "gqa"])
+    ap.add_argument("--only", nargs="*", default=list(KINDS), choices=list(KINDS))
     ap.add_argument("--reps", type=int, default=3)
     ap.add_argument("--steps", type=int, default=40)
     ap.add_argument("--json", action="store_true", help="one JSON line with the figures at the end")
