@@ -176,7 +176,7 @@ int wr_hip_mix_gate_norm(wr_hip_mix_step *s, int f32, const float *o_dev, uint32
 /* ---- matrix-state recurrence with input-made decays -----------------------------
  * Per head a state S [dim][dim], key channel by value column, 32-bit.  Every token
  * brings r, k, v and a decay per key channel, w = exp(-exp(z + w0)), or
- * exp(-gain * sigmoid(z + w0)) with `gain` > 0.  Two rules:
+ * exp(-gain * sigmoid(z + w0)) with `gain` > 0, z = w_decay . low.  Two rules:
  *   BONUS  o = (S + diag(u) k v^T)^T r;  then S <- diag(w) S + k v^T
  *   DELTA  with n = k / sqrt(k . k + unit_eps) and a = sigmoid(za + a_bias):
  *          S <- diag(w) S - (a n) (n^T S) + k v^T (old S on the right);  o = S^T r
@@ -185,7 +185,8 @@ int wr_hip_mix_gate_norm(wr_hip_mix_step *s, int f32, const float *o_dev, uint32
  * h_kt tiles) at input col_h + head * dim + column; inputs up to the next multiple of
  * 32 are zeros.
  * in: 32-bit rows, stride ld; r, k, v, za, g at their columns, head by head.
- * z: 32-bit rows, stride ldz.  State `run` of the pool; position 0 starts from zero. */
+ * low: frag rows of w_decay's inputs; z: room for the products, 32-bit rows of w_decay's
+ * outputs (used where they are not made in passing).  State `run` of the pool; position 0 starts from zero. */
 enum { WR_HIP_MIX_RULE_BONUS = 0, WR_HIP_MIX_RULE_DELTA = 1 };
 typedef struct wr_hip_mix_recurrence {
     uint32_t heads, dim, rule;
@@ -194,8 +195,9 @@ typedef struct wr_hip_mix_recurrence {
     const float *w0, *u, *a_bias, *norm;      /* device, heads * dim (u: BONUS, a_bias: DELTA) */
     const float *in;
     uint32_t ld, col_r, col_k, col_v, col_a, col_g;
-    const float *z;
-    uint32_t ldz;
+    const wr_hip_mat *w_decay;                /* [heads * dim padded][rank padded] */
+    const void *low;
+    float *z;
     void *h;
     uint32_t h_kt, col_h;
 } wr_hip_mix_recurrence;

@@ -324,6 +324,11 @@ int wr_hip_mix_recur(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, in
     const uint32_t D = a->dim, hd = a->heads * D, delta = a->rule == WR_HIP_MIX_RULE_DELTA;
     const size_t all = (size_t)hd * D;
     if (pool->state_elems[run] != all) return WR_HIP_ERR_INVAL;
+    const uint32_t ldz = a->w_decay->n_out;
+    const wr_hip_mix_gemm decay = {.w = a->w_decay, .x = a->low, .x_kt = a->w_decay->n_in / 32, .rows = s->rows,
+                                   .out = WR_HIP_MIX_OUT_ROWS_F32, .y_f32 = a->z, .ldy = ldz};
+    const int rc = wr_hip_mix_gemm_run(f32, &decay);
+    if (rc != WR_HIP_OK) return rc;
     float w[WR_HIP_MIX_MAX_RECUR_DIM], b[WR_HIP_MIX_MAX_RECUR_DIM], n[WR_HIP_MIX_MAX_RECUR_DIM], o[WR_HIP_MIX_MAX_RECUR_DIM];
     for (uint32_t i = 0; i < s->n_seq; i++) {
         const wr_hip_mix_seq *q = &s->seqs[i];
@@ -332,7 +337,7 @@ int wr_hip_mix_recur(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, in
         for (uint32_t t = s->row0[i]; t < s->row0[i] + q->rows; t++)
             for (uint32_t h = 0; h < a->heads; h++) {
                 const float *row = a->in + (size_t)t * a->ld + h * D, *r = row + a->col_r, *k = row + a->col_k,
-                            *v = row + a->col_v, *g = row + a->col_g, *z = a->z + (size_t)t * a->ldz + h * D;
+                            *v = row + a->col_v, *g = row + a->col_g, *z = a->z + (size_t)t * ldz + h * D;
                 float kk = 0, ss = 0;
                 for (uint32_t d = 0; d < D; d++) kk += k[d] * k[d];
                 for (uint32_t d = 0; d < D; d++) {

@@ -280,17 +280,18 @@ struct MixShiftArgs {
     float* state;                    // [buffer][wpad]
     void* out;
 };
-template <bool F32, int RPW>
+constexpr uint32_t kShiftMixes = 5;  // factors fetched ahead of the norms where a row has a workgroup to itself
+
+template <bool F32, int RPW, bool HELD>
 __global__ __launch_bounds__(MixRowShape<RPW>::kThreads) void mix_shift_kernel(const MixShiftArgs a)
 {
     using Sh = MixRowShape<RPW>;
+    constexpr int CH = HELD ? Sh::kHeld : 1;
+    constexpr bool EARLY = HELD && RPW == 1;
     __shared__ float red[64];
     const uint32_t t = threadIdx.x, row = blockIdx.x * RPW + t % RPW, lr = t / RPW;
     const bool live = row < a.rows;
     const uint32_t r = live ? row : a.rows - 1, nq = a.wpad / 8;
-    const MixSeq s = a.seqs[a.row_seq[r]];
-    const bool first = r == s.row0, last = r + 1 == s.row0 + s.rows;
-    const uint32_t p = first ? r : r - 1;
     auto load = [&](uint32_t rr, uint32_t q, float (&v)[8]) {
         mix_load8(a.x + (size_t)rr * a.wpad + q * 8, v);
         if (a.y) {
@@ -300,45 +301,106 @@ __global__ __launch_bounds__(MixRowShape<RPW>::kThreads) void mix_shift_kernel(c
             for (int j = 0; j < 8; j++) v[j] += w[j];
         }
     };
+    float hr[CH][8], hp[CH][8], hn[EARLY ? CH : 1][8], hm[EARLY ? kShiftMixes : 1][EARLY ? CH : 1][8];
     float sr = 0.f, sp = 0.f;
-    for (uint32_t q = lr; q < nq; q += Sh::kPerRow) {
-        float v[8], w[8];
-        load(r, q, v);
-        load(p, q, w);
+    if constexpr (HELD) {                                  // (first what does not wait for the request's description)
+#pragma unroll
+        for (int i = 0; i < CH; i++) {
+            const uint32_t q = lr + i * Sh::kPerRow;
+            if (q >= nq) continue;
+            load(r, q, hr[i]);
+            if constexpr (EARLY) {
+                mix_load8(a.norm + q * 8, hn[i]);
+#pragma unroll
+                for (uint32_t m = 0; m < kShiftMixes; m++)
+                    if (m < a.n_mix) mix_load8(a.mu + (size_t)m * a.wpad + q * 8, hm[m][i]);
+            }
+        }
+    }
+    const MixSeq s = a.seqs[a.row_seq[r]];
+    const bool first = r == s.row0, last = r + 1 == s.row0 + s.rows;
+    const uint32_t p = first ? r : r - 1;
+    // h of the row before, not yet normed: its residual, or what the state holds (normed already)
+    auto before = [&](uint32_t q, float (&v)[8]) {
+        if (!first) {
+            load(p, q, v);
+        } else if (s.pos0 > 0) {
+            mix_load8(a.state + (size_t)s.state_in * a.wpad + q * 8, v);
+        } else {
+#pragma unroll
+            for (int j = 0; j < 8; j++) v[j] = 0.f;
+        }
+    };
+    auto square = [&](const float (&v)[8], const float (&w)[8]) {
 #pragma unroll
         for (int j = 0; j < 8; j++) {
             sr = fmaf(v[j], v[j], sr);
             sp = fmaf(w[j], w[j], sp);
         }
+    };
+    if constexpr (HELD) {
+#pragma unroll
+        for (int i = 0; i < CH; i++) {
+            const uint32_t q = lr + i * Sh::kPerRow;
+            if (q >= nq) continue;
+            before(q, hp[i]);
+            square(hr[i], hp[i]);
+        }
+    } else {
+        for (uint32_t q = lr; q < nq; q += Sh::kPerRow) {
+            load(r, q, hr[0]);
+            before(q, hp[0]);
+            square(hr[0], hp[0]);
+        }
     }
     const float invw = 1.0f / (float)a.width;
     const float ir = 1.0f / sqrtf(mix_row_sum<RPW>(sr, red) * invw + a.eps);
-    const float ip = 1.0f / sqrtf(mix_row_sum<RPW>(sp, red) * invw + a.eps);
+    float ip = 1.0f;
+    if (RPW > 1 || !first) ip = 1.0f / sqrtf(mix_row_sum<RPW>(sp, red) * invw + a.eps);      // (one row: uniform)
     if (!live) return;
-    for (uint32_t q = lr; q < nq; q += Sh::kPerRow) {
-        float v[8], w[8], n[8];
-        load(r, q, v);
+    auto mix = [&](uint32_t q, float (&v)[8], float (&w)[8], int i) {
+        float n[8];
         if (a.y) mix_store8(a.x_out + (size_t)r * a.wpad + q * 8, v);
-        mix_load8(a.norm + q * 8, n);
-        if (!first) {
-            load(p, q, w);
+        if constexpr (EARLY) {
 #pragma unroll
-            for (int j = 0; j < 8; j++) w[j] *= ip * n[j];
-        } else if (s.pos0 > 0) {
-            mix_load8(a.state + (size_t)s.state_in * a.wpad + q * 8, w);
+            for (int j = 0; j < 8; j++) n[j] = hn[i][j];
         } else {
-#pragma unroll
-            for (int j = 0; j < 8; j++) w[j] = 0.f;
+            mix_load8(a.norm + q * 8, n);
         }
 #pragma unroll
-        for (int j = 0; j < 8; j++) v[j] *= ir * n[j];
+        for (int j = 0; j < 8; j++) {
+            v[j] *= ir * n[j];
+            if (!first) w[j] *= ip * n[j];
+        }
         if (last) mix_store8(a.state + (size_t)s.state_out * a.wpad + q * 8, v);
-        for (uint32_t m = 0; m < a.n_mix; m++) {
+        auto put = [&](uint32_t m, const float (&u)[8]) {
+            float o[8];
+#pragma unroll
+            for (int j = 0; j < 8; j++) o[j] = v[j] + (w[j] - v[j]) * u[j];
+            mix_store_unit<F32>(a.out, frag_unit(r, m * nq + q, a.n_mix * (a.wpad / 32)), o);
+        };
+        if constexpr (EARLY) {
+#pragma unroll
+            for (uint32_t m = 0; m < kShiftMixes; m++)
+                if (m < a.n_mix) put(m, hm[m][i]);
+        }
+        for (uint32_t m = EARLY ? kShiftMixes : 0; m < a.n_mix; m++) {
             float u[8];
             mix_load8(a.mu + (size_t)m * a.wpad + q * 8, u);
+            put(m, u);
+        }
+    };
+    if constexpr (HELD) {
 #pragma unroll
-            for (int j = 0; j < 8; j++) u[j] = v[j] + (w[j] - v[j]) * u[j];
-            mix_store_unit<F32>(a.out, frag_unit(r, m * nq + q, a.n_mix * (a.wpad / 32)), u);
+        for (int i = 0; i < CH; i++) {
+            const uint32_t q = lr + i * Sh::kPerRow;
+            if (q < nq) mix(q, hr[i], hp[i], i);
+        }
+    } else {
+        for (uint32_t q = lr; q < nq; q += Sh::kPerRow) {
+            load(r, q, hr[0]);
+            before(q, hp[0]);
+            mix(q, hr[0], hp[0], 0);
         }
     }
 }

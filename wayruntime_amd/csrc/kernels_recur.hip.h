@@ -59,6 +59,9 @@ struct RecurArgs {
     uint32_t ld, col_r, col_k, col_v, col_a, col_g;
     const float* z;
     uint32_t ldz;
+    const bf16x8* wd;               // token by token: the decay's matrix, or nullptr where z is there already
+    const void* low;
+    uint32_t low_kt;
     float* state;                   // [buffer][heads][dim][dim]
     void* h;
     uint32_t h_kt, col_h;
@@ -87,6 +90,28 @@ __device__ __forceinline__ float recur_wave_sum(float v)
     return v;
 }
 
+// Row r's product with output n of the decay's matrix.
+template <bool F32>
+__device__ __forceinline__ float recur_z(const RecurArgs& a, uint32_t r, uint32_t n)
+{
+    using V8 = typename MixAct<F32>::V8;
+    float z = 0.f;
+    for (uint32_t kt = 0; kt < a.low_kt; kt++) {
+        bf16x8 w[4];
+        V8 x[4];
+#pragma unroll
+        for (int g = 0; g < 4; g++) {
+            w[g] = a.wd[((size_t)(n / 16) * a.low_kt + kt) * 64 + 16 * g + n % 16];
+            x[g] = reinterpret_cast<const V8*>(a.low)[frag_unit(r, kt * 4 + g, a.low_kt)];
+        }
+#pragma unroll
+        for (int g = 0; g < 4; g++)
+#pragma unroll
+            for (int j = 0; j < 8; j++) z = fmaf((float)w[g][j], (float)x[g][j], z);
+    }
+    return z;
+}
+
 // grid (requests, heads), 4 DP threads: thread t has value column t % DP, channels DPT (t / DP) .. +DPT
 template <bool F32, int DP, bool DELTA>
 __global__ __launch_bounds__(4 * DP) void recur_step_kernel(const RecurArgs a)
@@ -113,7 +138,7 @@ __global__ __launch_bounds__(4 * DP) void recur_step_kernel(const RecurArgs a)
         float g = 0.f;
         if (wave < WV) {
             const float rr = own ? row[a.col_r + c] : 0.f, kk = own ? row[a.col_k + c] : 0.f;
-            const float w = own ? recur_decay(a, a.z[(size_t)r * a.ldz + hd + c] + w0) : 0.f;
+            const float w = own ? recur_decay(a, (a.wd ? recur_z<F32>(a, r, hd + c) : a.z[(size_t)r * a.ldz + hd + c]) + w0) : 0.f;
             g = own ? row[a.col_g + c] : 0.f;
             if constexpr (DELTA) {
                 const float rate = own ? 1.0f / (1.0f + expf(-(row[a.col_a + c] + ub))) : 0.f;
@@ -225,10 +250,18 @@ template <> struct RecurOp4<false> {
     bf16x8 p;                                // four high terms, four low terms
 };
 
-__device__ __forceinline__ void recur_split(float x, __bf16& hi, __bf16& lo)
+// Two values as high and low terms (in pairs: one conversion instruction does two).
+typedef __bf16 bf16x2 __attribute__((ext_vector_type(2)));
+typedef float f32x2v __attribute__((ext_vector_type(2)));
+__device__ __forceinline__ void recur_split2(float x, float y, bf16x2& hi, bf16x2& lo)
 {
-    hi = (__bf16)x;
-    lo = (__bf16)(x - (float)hi);
+    hi = __builtin_convertvector((f32x2v{x, y}), bf16x2);
+    lo = __builtin_convertvector((f32x2v{x - (float)hi[0], y - (float)hi[1]}), bf16x2);
+}
+__device__ __forceinline__ bf16x8 recur_cat(bf16x2 a, bf16x2 b, bf16x2 c, bf16x2 d)
+{
+    return __builtin_shufflevector(__builtin_shufflevector(a, b, 0, 1, 2, 3), __builtin_shufflevector(c, d, 0, 1, 2, 3), 0, 1, 2, 3,
+                                   4, 5, 6, 7);
 }
 template <bool F32>
 __device__ __forceinline__ RecurOp8<F32> recur_op8(const float (&v)[8])
@@ -238,13 +271,11 @@ __device__ __forceinline__ RecurOp8<F32> recur_op8(const float (&v)[8])
         r.p[0] = f32x4{v[0], v[1], v[2], v[3]};
         r.p[1] = f32x4{v[4], v[5], v[6], v[7]};
     } else {
+        bf16x2 h[4], l[4];
 #pragma unroll
-        for (int j = 0; j < 8; j++) {
-            __bf16 h, l;
-            recur_split(v[j], h, l);
-            r.p[0][j] = h;
-            r.p[1][j] = l;
-        }
+        for (int j = 0; j < 4; j++) recur_split2(v[2 * j], v[2 * j + 1], h[j], l[j]);
+        r.p[0] = recur_cat(h[0], h[1], h[2], h[3]);
+        r.p[1] = recur_cat(l[0], l[1], l[2], l[3]);
     }
     return r;
 }
@@ -266,13 +297,10 @@ __device__ __forceinline__ RecurOp4<F32> recur_op4(f32x4 v)
     if constexpr (F32) {
         r.p = v;
     } else {
+        bf16x2 h[2], l[2];
 #pragma unroll
-        for (int j = 0; j < 4; j++) {
-            __bf16 h, l;
-            recur_split(v[j], h, l);
-            r.p[j] = h;
-            r.p[4 + j] = l;
-        }
+        for (int j = 0; j < 2; j++) recur_split2(v[2 * j], v[2 * j + 1], h[j], l[j]);
+        r.p = recur_cat(h[0], h[1], l[0], l[1]);
     }
     return r;
 }
@@ -283,15 +311,8 @@ __device__ __forceinline__ RecurOp8<true> recur_join(const RecurOp4<true>& a, co
 }
 __device__ __forceinline__ RecurOp8<false> recur_join(const RecurOp4<false>& a, const RecurOp4<false>& b)
 {
-    RecurOp8<false> r;
-#pragma unroll
-    for (int j = 0; j < 4; j++) {
-        r.p[0][j] = a.p[j];
-        r.p[0][4 + j] = b.p[j];
-        r.p[1][j] = a.p[4 + j];
-        r.p[1][4 + j] = b.p[4 + j];
-    }
-    return r;
+    return RecurOp8<false>{{__builtin_shufflevector(a.p, b.p, 0, 1, 2, 3, 8, 9, 10, 11),
+                            __builtin_shufflevector(a.p, b.p, 4, 5, 6, 7, 12, 13, 14, 15)}};
 }
 
 // acc + A B over 32 inputs
@@ -315,18 +336,14 @@ __device__ __forceinline__ f32x4 recur_mm(const RecurOp4<true>& a, const RecurOp
     return acc;
 }
 // The eight elements of a lane are its four high and four low terms: one product over 32 "inputs" of
-// (high, low) with (high, high), one of (high, high) with (low, 0).
+// (high, low) with (high, high), one of (high, low) with (low, 0).
 __device__ __forceinline__ f32x4 recur_mm(const RecurOp4<false>& a, const RecurOp4<false>& b, f32x4 acc)
 {
-    bf16x8 bh, ah, bl;
+    bf16x8 zero;
 #pragma unroll
-    for (int j = 0; j < 4; j++) {
-        bh[j] = bh[4 + j] = b.p[j];
-        ah[j] = ah[4 + j] = a.p[j];
-        bl[j] = b.p[4 + j];
-        bl[4 + j] = (__bf16)0.f;
-    }
-    return mix_mfma(a.p, bh, mix_mfma(ah, bl, acc));
+    for (int j = 0; j < 8; j++) zero[j] = (__bf16)0.f;
+    const bf16x8 bh = __builtin_shufflevector(b.p, b.p, 0, 1, 2, 3, 0, 1, 2, 3), bl = __builtin_shufflevector(b.p, zero, 4, 5, 6, 7, 8, 8, 8, 8);
+    return mix_mfma(a.p, bh, mix_mfma(a.p, bl, acc));
 }
 
 // KiB of a sub-chunk's operands for one head, and where each lies.
@@ -397,7 +414,7 @@ __host__ __device__ constexpr int recur_chunk_lds(int kt, bool delta)
 // grid (chunks of 64 rows, heads): wave w of four has rows 16w .. 16w + 15.  `whole`: dim and every column are
 // multiples of four.
 template <bool F32, int KT, bool DELTA>
-__global__ __launch_bounds__(256) void recur_chunk_kernel(const RecurArgs a, const uint32_t whole)
+__global__ __launch_bounds__(256, KT <= 2 ? 2 : 1) void recur_chunk_kernel(const RecurArgs a, const uint32_t whole)
 {
     using U = RecurUnit<KT, DELTA>;
     constexpr int LD = 32 * KT + 4;
@@ -627,17 +644,71 @@ __global__ __launch_bounds__(256) void recur_chunk_kernel(const RecurArgs a, con
 }
 
 // Sub-chunks whose operands lie in LDS at once.
-__host__ __device__ constexpr int recur_ring(int kt) { return kt >= 4 ? 3 : 4; }
+__host__ __device__ constexpr int recur_ring(int kt, bool delta) { return kt >= 4 || delta ? 3 : 4; }
 
-// grid (requests, heads), a wave per 16 value columns (1, 2, 4 or 8 of them, VT).
-template <bool F32, int KT, bool DELTA, int VT>
-__global__ __launch_bounds__(64 * VT) void recur_chain_kernel(const RecurArgs a)
+// One sub-chunk's operands in a wave's registers.
+template <bool F32, int KT, bool DELTA>
+struct RecurHeld {
+    RecurOp8<F32> R[KT], W[DELTA ? KT : 1], K8[DELTA ? 2 * KT : 1], A8;
+    RecurOp4<F32> K4[DELTA ? 1 : 2 * KT], A4, M, V;
+    f32x4 G[2 * KT];
+
+    __device__ __forceinline__ void fetch(const unsigned char* unit, uint32_t wave, int lane, int g)
+    {
+        using U = RecurUnit<KT, DELTA>;
+        V = recur_get4<F32>(unit, U::kV + wave, lane);
+        if constexpr (DELTA) {
+            M = recur_get4<F32>(unit, U::kM, lane);
+            A8 = recur_get8<F32>(unit, U::kA, lane);
+        } else {
+            A4 = recur_get4<F32>(unit, U::kA, lane);
+        }
+#pragma unroll
+        for (int t = 0; t < KT; t++) {
+            if constexpr (DELTA) W[t] = recur_get8<F32>(unit, U::kW + 2 * t, lane);
+            R[t] = recur_get8<F32>(unit, U::kR + 2 * t, lane);
+        }
+#pragma unroll
+        for (int t = 0; t < 2 * KT; t++) {
+            if constexpr (DELTA) K8[t] = recur_get8<F32>(unit, U::kK + 2 * t, lane);
+            else K4[t] = recur_get4<F32>(unit, U::kK + t, lane);
+            G[t] = *reinterpret_cast<const f32x4*>(unit + U::kG * 1024 + (16 * t + 4 * g) * 4);
+        }
+    }
+};
+
+// acc + sum over t of A[t] B[t], in chains of their own where there are several terms
+template <int N>
+__device__ __forceinline__ f32x4 recur_mm_many(const RecurOp8<true> (&a)[N], const RecurOp8<true> (&b)[N], f32x4 acc)
 {
-    using U = RecurUnit<KT, DELTA>;
-    constexpr int UNIT = recur_unit_kib(KT, DELTA, VT), RING = recur_ring(KT), AHEAD = RING - 1, CPW = (UNIT + VT - 1) / VT;
-    // what is on its way behind the stage waited for: AHEAD - 1 stages, and four stores of each step made since
-    constexpr int BEHIND = (AHEAD - 1) * CPW, FULL = BEHIND + 4 * AHEAD;
-    static_assert(FULL < 64, "vmcnt");
+#pragma unroll
+    for (int t = 0; t < N; t++) acc = recur_mm(a[t], b[t], acc);
+    return acc;
+}
+template <int N>
+__device__ __forceinline__ f32x4 recur_mm_many(const RecurOp8<false> (&a)[N], const RecurOp8<false> (&b)[N], f32x4 acc)
+{
+    f32x4 x = f32x4{0.f, 0.f, 0.f, 0.f}, y = x;
+#pragma unroll
+    for (int t = 0; t < N; t++) {
+        acc = mix_mfma(a[t].p[0], b[t].p[0], acc);
+        x = mix_mfma(a[t].p[0], b[t].p[1], x);
+        y = mix_mfma(a[t].p[1], b[t].p[0], y);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; i++) acc[i] += x[i] + y[i];
+    return acc;
+}
+
+// grid (requests, heads), a wave per 16 value columns (1, 2, 4 or 8 of them, VT).  A stage of the ring is read into
+// registers a step before it is used, and copied over from then on.
+template <bool F32, int KT, bool DELTA, int VT>
+__global__ __launch_bounds__(64 * VT, 2) void recur_chain_kernel(const RecurArgs a)
+{
+    constexpr int UNIT = recur_unit_kib(KT, DELTA, VT), RING = recur_ring(KT, DELTA), CPW = (UNIT + VT - 1) / VT;
+    // what is on its way behind the stage waited for: RING - 2 stages, and four stores of each step made since
+    constexpr int EARLY = (RING - 2) * CPW, FULL = (RING - 2) * (CPW + 4) + 4, FIRST = (RING - 1) * CPW;
+    static_assert(FULL < 64 && FIRST < 64, "vmcnt");
     extern __shared__ __attribute__((aligned(16))) unsigned char recur_lds[];
     const MixSeq s = a.seqs[a.list[blockIdx.x]];
     const uint32_t head = blockIdx.y, D = a.dim;
@@ -669,50 +740,53 @@ __global__ __launch_bounds__(64 * VT) void recur_chain_kernel(const RecurArgs a)
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     const uint32_t ldo = a.heads * VT * 16;
     float* o = a.o + ((size_t)sub0 * kRecurSub + 4 * g) * ldo + head * VT * 16 + col;
+    RecurHeld<F32, KT, DELTA> x, y;
 #pragma unroll
-    for (int i = 0; i < AHEAD; i++) issue(i);
-    for (uint32_t sub = 0; sub < n_sub; sub++) {                  // uniform
-        if (sub < (uint32_t)AHEAD)
-            asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)\n\ts_barrier" ::"n"(BEHIND) : "memory");
+    for (int i = 0; i < RING; i++) issue(i);
+    asm volatile("s_waitcnt vmcnt(%0)\n\ts_barrier" ::"n"(FIRST) : "memory");
+    x.fetch(recur_lds, wave, lane, g);
+    // a step: the next stage has landed and is fetched into `after`, the stage of `now` (in registers everywhere) is
+    // copied over, and `now` moves the state
+    auto step = [&](uint32_t sub, const RecurHeld<F32, KT, DELTA>& now, RecurHeld<F32, KT, DELTA>& after) {
+        if (sub < (uint32_t)RING - 1)
+            asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)\n\ts_barrier" ::"n"(EARLY) : "memory");
         else
             asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)\n\ts_barrier" ::"n"(FULL) : "memory");
-        issue(sub + AHEAD);                                       // (everybody is done with that stage)
-        const unsigned char* unit = recur_lds + sub % RING * UNIT * 1024;
+        issue(sub + RING);
+        after.fetch(recur_lds + (sub + 1) % RING * UNIT * 1024, wave, lane, g);
+        if constexpr (KT <= 2) __builtin_amdgcn_sched_barrier(0);         // (left alone, the reads sink to where they are used)
         RecurOp8<F32> So[KT];
 #pragma unroll
         for (int t = 0; t < KT; t++) So[t] = recur_op8<F32>(S[2 * t], S[2 * t + 1]);
-        const RecurOp4<F32> V = recur_get4<F32>(unit, U::kV + wave, lane);
         f32x4 O = f32x4{0.f, 0.f, 0.f, 0.f};
-        const float* G = reinterpret_cast<const float*>(unit + U::kG * 1024) + 4 * g;
-        f32x4 next[2 * KT];
-#pragma unroll
-        for (int t = 0; t < 2 * KT; t++) {
-            const f32x4 gg = *reinterpret_cast<const f32x4*>(G + 16 * t);
-#pragma unroll
-            for (int i = 0; i < 4; i++) next[t][i] = gg[i] * S[t][i];
-        }
         if constexpr (DELTA) {
-            f32x4 P = recur_mm(recur_get4<F32>(unit, U::kM, lane), V, O);
+            const f32x4 P = recur_mm_many<KT>(now.W, So, recur_mm(now.M, now.V, O));
+            O = recur_mm_many<KT>(now.R, So, O);
 #pragma unroll
-            for (int t = 0; t < KT; t++) P = recur_mm(recur_get8<F32>(unit, U::kW + 2 * t, lane), So[t], P);
+            for (int t = 0; t < 2 * KT; t++)
 #pragma unroll
-            for (int t = 0; t < KT; t++) O = recur_mm(recur_get8<F32>(unit, U::kR + 2 * t, lane), So[t], O);
-            const RecurOp8<F32> VP = recur_join(V, recur_op4<F32>(P));
+                for (int i = 0; i < 4; i++) S[t][i] *= now.G[t][i];
+            const RecurOp8<F32> VP = recur_join(now.V, recur_op4<F32>(P));
 #pragma unroll
-            for (int t = 0; t < 2 * KT; t++) S[t] = recur_mm(recur_get8<F32>(unit, U::kK + 2 * t, lane), VP, next[t]);
-            O = recur_mm(recur_get8<F32>(unit, U::kA, lane), VP, O);
+            for (int t = 0; t < 2 * KT; t++) S[t] = recur_mm(now.K8[t], VP, S[t]);
+            O = recur_mm(now.A8, VP, O);
         } else {
 #pragma unroll
-            for (int t = 0; t < 2 * KT; t++) S[t] = recur_mm(recur_get4<F32>(unit, U::kK + t, lane), V, next[t]);
-            O = recur_mm(recur_get4<F32>(unit, U::kA, lane), V, O);
+            for (int t = 0; t < 2 * KT; t++)
 #pragma unroll
-            for (int t = 0; t < KT; t++) O = recur_mm(recur_get8<F32>(unit, U::kR + 2 * t, lane), So[t], O);
+                for (int i = 0; i < 4; i++) S[t][i] *= now.G[t][i];
+#pragma unroll
+            for (int t = 0; t < 2 * KT; t++) S[t] = recur_mm(now.K4[t], now.V, S[t]);
+            O = recur_mm_many<KT>(now.R, So, recur_mm(now.A4, now.V, O));
         }
         // (rows past the request's end have room of their own)
 #pragma unroll
-        for (int i = 0; i < 4; i++)
-            o[(size_t)i * ldo] = O[i];
+        for (int i = 0; i < 4; i++) o[(size_t)i * ldo] = O[i];
         o += (size_t)kRecurSub * ldo;
+    };
+    for (uint32_t sub = 0; sub < n_sub; sub += 2) {               // uniform
+        step(sub, x, y);
+        if (sub + 1 < n_sub) step(sub + 1, y, x);
     }
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");              // the last copies still target the ring
 #pragma unroll

@@ -396,14 +396,17 @@ int wr_hip_mix_shift(wr_hip_mix_step* s, wr_hip_mix_pool* pool, uint32_t run, in
     ENTER();
     MixShiftArgs a = {s->d<MixSeq>(s->o_seqs), s->d<uint32_t>(s->o_seq), s->rows, width, round32(width), n_mix, eps, x_dev, y_dev,
                       norm_dev, mu_dev, x_out_dev, pool->state[run], out_dev};
-    if (s->rows >= 64) {
-        const dim3 grid((s->rows + 3) / 4), block(MixRowShape<4>::kThreads);
-        if (f32) MIX_LAUNCH((mix_shift_kernel<true, 4>), grid, block, 0, a);
-        else MIX_LAUNCH((mix_shift_kernel<false, 4>), grid, block, 0, a);
+    const bool many = s->rows >= 64, held = a.wpad <= 4096;
+    const dim3 g1(s->rows), b1(MixRowShape<1>::kThreads), g4((s->rows + 3) / 4), b4(MixRowShape<4>::kThreads);
+    if (f32) {                                             // (not the serving form: two shapes do)
+        if (many) MIX_LAUNCH((mix_shift_kernel<true, 4, false>), g4, b4, 0, a);
+        else MIX_LAUNCH((mix_shift_kernel<true, 1, false>), g1, b1, 0, a);
+    } else if (many) {
+        if (held) MIX_LAUNCH((mix_shift_kernel<false, 4, true>), g4, b4, 0, a);
+        else MIX_LAUNCH((mix_shift_kernel<false, 4, false>), g4, b4, 0, a);
     } else {
-        const dim3 grid(s->rows), block(MixRowShape<1>::kThreads);
-        if (f32) MIX_LAUNCH((mix_shift_kernel<true, 1>), grid, block, 0, a);
-        else MIX_LAUNCH((mix_shift_kernel<false, 1>), grid, block, 0, a);
+        if (held) MIX_LAUNCH((mix_shift_kernel<false, 1, true>), g1, b1, 0, a);
+        else MIX_LAUNCH((mix_shift_kernel<false, 1, false>), g1, b1, 0, a);
     }
     return WR_HIP_OK;
 }
@@ -641,7 +644,7 @@ static int recur_chunks(wr_hip_mix_step* s, RecurArgs& a)
     constexpr size_t unit = (size_t)recur_unit_kib(KT, DELTA, VT) * 1024;
     int rc = ensure_device(s->recur_ops, (size_t)s->n_chunks * kRecurSubs * a.heads * unit);
     if (rc == WR_HIP_OK) rc = ensure_device(s->recur_out, (size_t)s->n_chunks * kMixChunk * a.heads * VT * 16 * 4);
-    constexpr size_t l1 = (size_t)4 * recur_chunk_lds(KT, DELTA) * 4, l2 = recur_ring(KT) * unit;
+    constexpr size_t l1 = (size_t)4 * recur_chunk_lds(KT, DELTA) * 4, l2 = recur_ring(KT, DELTA) * unit;
     if (rc == WR_HIP_OK) rc = allow_lds<recur_chunk_kernel<F32, KT, DELTA>>(l1);
     if (rc == WR_HIP_OK) rc = allow_lds<recur_chain_kernel<F32, KT, DELTA, VT>>(l2);
     if (rc) return rc;
@@ -654,10 +657,28 @@ static int recur_chunks(wr_hip_mix_step* s, RecurArgs& a)
     return WR_HIP_OK;
 }
 
+// Ranks (in tiles of 32) up to which a decoded token's decays are made in passing.
+constexpr uint32_t kDecayTiles = 4;
+
 template <bool F32, bool DELTA>
-static int recur_run(wr_hip_mix_step* s, RecurArgs& a)
+static int recur_run(wr_hip_mix_step* s, RecurArgs& a, const wr_hip_mix_recurrence* q)
 {
     const bool chunked = s->n_long && a.dim <= (uint32_t)kRecurMaxDim;
+    if (!s->n_long && a.low_kt <= kDecayTiles) {
+        a.wd = reinterpret_cast<const bf16x8*>(q->w_decay->tiles);
+        a.low = q->low;
+    } else {
+        wr_hip_mix_gemm d = {};
+        d.w = q->w_decay;
+        d.x = q->low;
+        d.x_kt = a.low_kt;
+        d.rows = s->rows;
+        d.out = WR_HIP_MIX_OUT_ROWS_F32;
+        d.y_f32 = q->z;
+        d.ldy = a.ldz;
+        const int rc = wr_hip_mix_gemm_run(F32, &d);
+        if (rc) return rc;
+    }
     if (chunked) {
         a.list = s->d<uint32_t>(s->o_long);
         int rc;
@@ -675,14 +696,14 @@ int wr_hip_mix_recur(wr_hip_mix_step* s, wr_hip_mix_pool* pool, uint32_t run, in
 {
     if (!g.inited) return WR_HIP_ERR_STATE;
     if (!s || !s->rows || !pool || run >= pool->state.size() || !q || !q->heads || !q->dim || !q->w0 || !q->norm || !q->in ||
-        !q->z || !q->h || q->rule > WR_HIP_MIX_RULE_DELTA)
+        !q->w_decay || !q->low || !q->z || !q->h || q->rule > WR_HIP_MIX_RULE_DELTA)
         return WR_HIP_ERR_INVAL;
     const bool delta = q->rule == WR_HIP_MIX_RULE_DELTA;
     if (delta ? !q->a_bias : !q->u) return WR_HIP_ERR_INVAL;
     if (q->dim > WR_HIP_MIX_MAX_RECUR_DIM) return WR_HIP_ERR_LIMIT;
     const uint64_t hd = (uint64_t)q->heads * q->dim;
     if (hd * q->dim != pool->state_elems[run]) return WR_HIP_ERR_INVAL;
-    if (q->ldz < hd || q->col_r + hd > q->ld || q->col_k + hd > q->ld || q->col_v + hd > q->ld || q->col_g + hd > q->ld ||
+    if (q->w_decay->batch != 1 || q->w_decay->n_out < hd || q->col_r + hd > q->ld || q->col_k + hd > q->ld || q->col_v + hd > q->ld || q->col_g + hd > q->ld ||
         (delta && q->col_a + hd > q->ld) || q->col_h + (hd + 31) / 32 * 32 > (uint64_t)q->h_kt * 32)
         return WR_HIP_ERR_INVAL;
     ENTER();
@@ -708,13 +729,14 @@ int wr_hip_mix_recur(wr_hip_mix_step* s, wr_hip_mix_pool* pool, uint32_t run, in
     a.col_a = delta ? q->col_a : 0;
     a.col_g = q->col_g;
     a.z = q->z;
-    a.ldz = q->ldz;
+    a.ldz = q->w_decay->n_out;
+    a.low_kt = q->w_decay->n_in / 32;
     a.state = pool->state[run];
     a.h = q->h;
     a.h_kt = q->h_kt;
     a.col_h = q->col_h;
-    if (f32) return delta ? recur_run<true, true>(s, a) : recur_run<true, false>(s, a);
-    return delta ? recur_run<false, true>(s, a) : recur_run<false, false>(s, a);
+    if (f32) return delta ? recur_run<true, true>(s, a, q) : recur_run<true, false>(s, a, q);
+    return delta ? recur_run<false, true>(s, a, q) : recur_run<false, false>(s, a, q);
 }
 
 // ----------------------------------------------------------------- latent --

@@ -382,21 +382,19 @@ static wr_status walk_latent(wr_model *m, const wrh_mix_layer *L, uint32_t r, co
     return WR_OK;
 }
 
-/* The decay's second product and the recurrence itself; `rec` has the rest filled in. */
+/* The recurrence, the decay's second product included; `rec` has the rest filled in. */
 static wr_status walk_recur(wr_model *m, const wrh_mix_recur *q, uint32_t r, uint32_t store, const void *low, float *z,
-                            wr_hip_mix_recurrence *rec, uint32_t R)
+                            wr_hip_mix_recurrence *rec)
 {
     struct wrh_mix_model *mm = m->mix;
-    const wr_hip_mix_gemm decay = {.w = q->w_decay, .x = low, .x_kt = q->rank_p / 32, .rows = R,
-                                   .out = WR_HIP_MIX_OUT_ROWS_F32, .y_f32 = z, .ldy = q->hd_p};
-    TRY(wr_hip_mix_gemm_run(mm->f32, &decay), "decay product");
     rec->heads = q->heads;
     rec->dim = q->dim;
     rec->eps = mm->eps;
     rec->w0 = q->w0;
     rec->norm = q->norm;
+    rec->w_decay = q->w_decay;
+    rec->low = low;
     rec->z = z;
-    rec->ldz = q->hd_p;
     TRY(wr_hip_mix_recur(mm->step, mm->pool, store, mm->f32, rec), "matrix-state recurrence");
     return WR_OK;
 }
@@ -423,7 +421,7 @@ static wr_status walk_wkv(wr_model *m, const wrh_mix_layer *L, uint32_t r, walk 
     TRY(wr_hip_mix_gemm_run(mm->f32, &low), "decay's low-rank product");
     wr_hip_mix_recurrence rec = {.rule = WR_HIP_MIX_RULE_BONUS, .out_scale = 1.0f, .gate_silu = 1, .u = q->u, .in = t.in,
                                  .ld = 4 * hd, .col_k = hd, .col_v = 2 * hd, .col_g = 3 * hd, .h = t.oh, .h_kt = hd / 32};
-    const wr_status st = walk_recur(m, q, r, mm->runs[r].store, t.low, t.z, &rec, R);
+    const wr_status st = walk_recur(m, q, r, mm->runs[r].store, t.low, t.z, &rec);
     if (st != WR_OK) return st;
     const wr_hip_mix_gemm out = {.w = L->w_o, .x = t.oh, .x_kt = hd / 32, .rows = R, .out = WR_HIP_MIX_OUT_ROWS_F32,
                                  .y_f32 = w->y, .ldy = mm->width_p};
@@ -448,7 +446,7 @@ static wr_status walk_parallel(wr_model *m, const wrh_mix_layer *L, uint32_t r, 
                                  .out_scale = L->right_scale, .a_bias = q->a_bias, .in = t.in, .ld = L->ld_in,
                                  .col_r = L->col_rr, .col_k = L->col_rk, .col_v = L->col_rv, .col_a = L->col_ra,
                                  .col_g = L->col_rg, .h = t.oh, .h_kt = kt_o, .col_h = L->heads * L->win.vdim_pad};
-    const wr_status st = walk_recur(m, q, r, mm->runs[r].store2, t.low, t.z, &rec, R);
+    const wr_status st = walk_recur(m, q, r, mm->runs[r].store2, t.low, t.z, &rec);
     if (st != WR_OK) return st;
     const wr_hip_mix_gemm out = {.w = L->w_o, .x = t.oh, .x_kt = kt_o, .rows = R, .out = WR_HIP_MIX_OUT_ROWS_F32,
                                  .y_f32 = w->y, .ldy = mm->width_p};
