@@ -18,7 +18,8 @@ u32, vp = C.c_uint32, C.c_void_p
 class Gemm(C.Structure):
     _fields_ = [("w", vp), ("x", vp), ("x_kt", u32), ("x_kt_z", u32), ("rows", u32), ("group_expert", vp),
                 ("tile_groups", u32), ("out", u32), ("y_f32", vp), ("y_act", vp), ("ldy", u32), ("h", vp), ("h_kt", u32),
-                ("col_z", u32), ("n_split", u32), ("silu_end", u32), ("sigmoid_end", u32), ("relu2", u32), ("scale", C.c_float)]
+                ("col_z", u32), ("n_split", u32), ("silu_end", u32), ("sigmoid_end", u32), ("relu2", u32), ("scale", C.c_float),
+                ("tanh_end", u32), ("gelu", u32), ("x_kt0", u32)]
 
 
 @pytest.fixture(scope="module")
@@ -106,6 +107,11 @@ def test_rows_out(lib, f32, N, K, rows):
     act[:, :silu] = O.silu(want[:, :silu])
     act[:, silu:sig] = O.sigmoid(want[:, silu:sig])
     r.close(y.to_host((rows, N)), act)
+    r.go(xd, out=ROWS_F32, y_f32=y.p, ldy=N, silu_end=N // 4, tanh_end=N - 7)
+    act = want.copy()
+    act[:, :N // 4] = O.silu(want[:, :N // 4])
+    act[:, N // 4:N - 7] = np.tanh(want[:, N // 4:N - 7])
+    r.close(y.to_host((rows, N)), act)
     r.end()
     for b in (y, xd):
         b.free()
@@ -130,6 +136,8 @@ def test_frag_split_and_gated_out(lib, f32, N, K, rows):
     r.go(xd, out=GATED, h=h.p, h_kt=N // 64)
     t = want.reshape(rows, N // 32, 2, 16)
     r.close(r.frag_down(h, rows, N // 2), (O.silu(t[:, :, 0]) * t[:, :, 1]).reshape(rows, -1), eight_bits=True)
+    r.go(xd, out=GATED, h=h.p, h_kt=N // 64, gelu=1)
+    r.close(r.frag_down(h, rows, N // 2), (O.gelu_tanh(t[:, :, 0]) * t[:, :, 1]).reshape(rows, -1), eight_bits=True)
     r.end()
     for b in (y, xd, h):
         b.free()
@@ -146,8 +154,14 @@ def test_batch_of_matrices(lib, f32, batch, N, K, rows):
     r.go(xd, x_kt=batch * K // 32, x_kt_z=K // 32, out=FRAG, h=h.p, h_kt=batch * N // 32, col_z=N)
     want = np.einsum("rzk,znk->rzn", x.reshape(rows, batch, K).astype(np.float64), r.w.astype(np.float64)).reshape(rows, -1)
     r.close(r.frag_down(h, rows, batch * N), want, eight_bits=True)
+    # and to columns of shared 32-bit rows, from inputs that start further in
+    x = r.act(rows, (batch + 1) * K)
+    xd2, y = r.up(x), hipattn.DeviceBuffer(rows * batch * N * 4)
+    r.go(xd2, x_kt=(batch + 1) * K // 32, x_kt_z=K // 32, x_kt0=K // 32, out=ROWS_F32, y_f32=y.p, ldy=batch * N, col_z=N)
+    x = x.reshape(rows, batch + 1, K)[:, 1:]
+    r.close(y.to_host((rows, batch * N)), np.einsum("rzk,znk->rzn", x.astype(np.float64), r.w.astype(np.float64)).reshape(rows, -1))
     r.end()
-    for b in (xd, h):
+    for b in (xd, xd2, h, y):
         b.free()
 
 
@@ -177,7 +191,7 @@ def test_refusals(lib):
     y = hipattn.DeviceBuffer(16 * 32 * 4)
     ok = dict(w=r.h, x=y.p, x_kt=1, rows=16, out=ROWS_F32, y_f32=y.p, ldy=32)
     for change in (dict(x_kt=0), dict(ldy=28), dict(ldy=33), dict(y_f32=None), dict(out=9), dict(rows=0), dict(w=None),
-                   dict(out=FRAG, h=y.p, h_kt=0), dict(out=SPLIT, h=y.p, h_kt=1, n_split=8), dict(out=GATED)):
+                   dict(out=FRAG, h=y.p, h_kt=0), dict(out=SPLIT, h=y.p, h_kt=1, n_split=8), dict(out=GATED), dict(x_kt0=1)):
         assert lib.wr_hip_mix_gemm_run(0, C.byref(Gemm(**dict(ok, **change)))) == hipattn.ERR_INVAL, change
     h = vp()
     for shape in ((1, 8, 32), (1, 16, 16), (0, 16, 32)):
