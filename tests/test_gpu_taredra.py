@@ -292,6 +292,35 @@ def test_decays_from_none_to_all(eng, tmp_path, prec, w0):
     case.close()
 
 
+@pytest.mark.parametrize("dim", [12, 32, 60, 100, 128])
+@pytest.mark.parametrize("kind", ["wkv", "delta"])
+def test_long_prompts_walked_in_segments(eng, tmp_path, prec, kind, dim):
+    # prompts long enough for several segments, unequal ones side by side, and one that goes on from a state;
+    # decays slow enough for every segment to matter to the last
+    mixer = mw.wkv(2, dim) if kind == "wkv" else par((1, 1, 8, 8, 1), right=(2, dim), left_scale=0.1)
+    cfg = mw.prenorm_config(48, 90, [(mixer, None)])
+
+    def change(f):
+        p = "l0.mix." if kind == "wkv" else "l0.mix.right."
+        f[p + "w0"][:] = -7.0 + np.linspace(0, 3, 2 * dim)
+        if kind == "delta":
+            f[p + "a.b"][:] = np.linspace(-6, 1, 2 * dim)
+    case = Case(eng, tmp_path, cfg, prec, pool=2048, edit=f32_edit(change))
+    t, u = case.tokens(900), case.tokens(330, seed=8)
+    want, other = case.oracle(t), case.oracle(u)
+    a, b = case.m.session(), case.m.session()
+    rc, lg = E.mixed_step([(a, t[:617], range(617)), (b, u, range(330))])
+    assert rc == 947
+    case.check(lg[0], want[:617], f"{kind} {dim} beside a shorter one")
+    case.check(lg[1], other, f"{kind} {dim} the shorter one")
+    rc, lg = E.mixed_step([(a, t[617:], range(283))])
+    case.check(lg[0], want[617:], f"{kind} {dim} going on")
+    a.close()
+    b.close()
+    case.check(run_cut(case, t, [880, 1]), want, f"{kind} {dim} decoded behind it")
+    case.close()
+
+
 def test_repeated_keys_are_removed(eng, tmp_path, prec):
     # the same few tokens over and over: unit keys repeat, removal and unit norms carry the outcome;
     # one token's key is all but zero

@@ -28,7 +28,11 @@
 //                        T N~, R~, [K | -B], [A_rk | -A_rb], T A_nk and V
 //   recur_chain_kernel   a workgroup per (request, head), a wave per 16 value columns:
 //                        walks the chunks with S in registers, operands through LDS
-// and recur_gate_kernel norms and gates their rows.
+// and recur_gate_kernel norms and gates their rows.  Where requests times heads leave
+// most of the device idle, a request's chunks are walked in segments side by side: a
+// first walk takes every segment but the last from S = 0 (and, DELTA, from S = I
+// without values) without outputs, which gives the segment as S -> X S + C; the second
+// starts each segment from the earlier ones applied to the request's state.
 //
 // No decay is ever divided by: tokens s < t that differ first in bit L of their place
 // in the chunk meet in a product of two factors, rho from s to the end of its aligned
@@ -68,6 +72,8 @@ struct RecurArgs {
     // chunked
     unsigned char* ops;             // [sub-chunk][heads][recur_unit_kib KiB]
     float* o;                       // [sub-chunk][16][heads][16 vtiles]
+    uint32_t n_seg, seg_len;        // segments of a request, sub-chunks of one
+    float *seg_c, *seg_x;           // [request of the list][segment][heads]: C [32 KT][16 VT], X [32 KT][32 KT] or its diagonal
 };
 
 __device__ __forceinline__ float recur_decay(const RecurArgs& a, float z)
@@ -350,10 +356,10 @@ __device__ __forceinline__ f32x4 recur_mm(const RecurOp4<false>& a, const RecurO
 template <int KT, bool DELTA>
 struct RecurUnit {
     static constexpr int kR = 0;                                  // R~          [KT] op8
-    static constexpr int kG = kR + 2 * KT;                        // rho(chunk)  [32 KT] floats
+    static constexpr int kA = kR + 2 * KT;                        // A_rk, or [A_rk | -A_rb]: op4 / op8
+    static constexpr int kG = kA + (DELTA ? 2 : 1);               // rho(chunk)  [32 KT] floats; from here on: what moves S
     static constexpr int kK = kG + 1;                             // K^T, or [K | -B]^T: [2 KT tiles] op4 / op8
-    static constexpr int kA = kK + 2 * KT * (DELTA ? 2 : 1);      // A_rk, or [A_rk | -A_rb]: op4 / op8
-    static constexpr int kW = kA + (DELTA ? 2 : 1);               // T N~        [KT] op8
+    static constexpr int kW = kK + 2 * KT * (DELTA ? 2 : 1);      // T N~        [KT] op8
     static constexpr int kM = kW + (DELTA ? 2 * KT : 0);          // T A_nk      op4
     static constexpr int kV = kM + (DELTA ? 1 : 0);               // V           [value tiles] op4
 };
@@ -647,32 +653,36 @@ __global__ __launch_bounds__(256, KT <= 2 ? 2 : 1) void recur_chunk_kernel(const
 __host__ __device__ constexpr int recur_ring(int kt, bool delta) { return kt >= 4 || delta ? 3 : 4; }
 
 // One sub-chunk's operands in a wave's registers.
-template <bool F32, int KT, bool DELTA>
+template <bool F32, int KT, bool DELTA, bool CARRY>
 struct RecurHeld {
     RecurOp8<F32> R[KT], W[DELTA ? KT : 1], K8[DELTA ? 2 * KT : 1], A8;
     RecurOp4<F32> K4[DELTA ? 1 : 2 * KT], A4, M, V;
     f32x4 G[2 * KT];
 
-    __device__ __forceinline__ void fetch(const unsigned char* unit, uint32_t wave, int lane, int g)
+    __device__ __forceinline__ void fetch(const unsigned char* unit, uint32_t wave, int lane, int g, bool values)
     {
         using U = RecurUnit<KT, DELTA>;
-        V = recur_get4<F32>(unit, U::kV + wave, lane);
-        if constexpr (DELTA) {
-            M = recur_get4<F32>(unit, U::kM, lane);
-            A8 = recur_get8<F32>(unit, U::kA, lane);
-        } else {
-            A4 = recur_get4<F32>(unit, U::kA, lane);
+        constexpr int K0 = CARRY ? U::kG : 0;                     // first KiB that is there
+        V = recur_get4<F32>(unit, U::kV - K0 + wave, lane);
+        if (CARRY && DELTA && !values) {
+#pragma unroll
+            for (int j = 0; j < (int)(sizeof(V.p) / sizeof(V.p[0])); j++) V.p[j] = (std::remove_reference_t<decltype(V.p[0])>)0.f;
+        }
+        if constexpr (DELTA) M = recur_get4<F32>(unit, U::kM - K0, lane);
+        if constexpr (!CARRY) {
+            if constexpr (DELTA) A8 = recur_get8<F32>(unit, U::kA, lane);
+            else A4 = recur_get4<F32>(unit, U::kA, lane);
         }
 #pragma unroll
         for (int t = 0; t < KT; t++) {
-            if constexpr (DELTA) W[t] = recur_get8<F32>(unit, U::kW + 2 * t, lane);
-            R[t] = recur_get8<F32>(unit, U::kR + 2 * t, lane);
+            if constexpr (DELTA) W[t] = recur_get8<F32>(unit, U::kW - K0 + 2 * t, lane);
+            if constexpr (!CARRY) R[t] = recur_get8<F32>(unit, U::kR + 2 * t, lane);
         }
 #pragma unroll
         for (int t = 0; t < 2 * KT; t++) {
-            if constexpr (DELTA) K8[t] = recur_get8<F32>(unit, U::kK + 2 * t, lane);
-            else K4[t] = recur_get4<F32>(unit, U::kK + t, lane);
-            G[t] = *reinterpret_cast<const f32x4*>(unit + U::kG * 1024 + (16 * t + 4 * g) * 4);
+            if constexpr (DELTA) K8[t] = recur_get8<F32>(unit, U::kK - K0 + 2 * t, lane);
+            else K4[t] = recur_get4<F32>(unit, U::kK - K0 + t, lane);
+            G[t] = *reinterpret_cast<const f32x4*>(unit + (U::kG - K0) * 1024 + (16 * t + 4 * g) * 4);
         }
     }
 };
@@ -700,24 +710,32 @@ __device__ __forceinline__ f32x4 recur_mm_many(const RecurOp8<false> (&a)[N], co
     return acc;
 }
 
-// grid (requests, heads), a wave per 16 value columns (1, 2, 4 or 8 of them, VT).  A stage of the ring is read into
-// registers a step before it is used, and copied over from then on.
-template <bool F32, int KT, bool DELTA, int VT>
+// Grid (requests * segments, heads), a wave per 16 value columns (1, 2, 4 or 8 of them, VT).  A stage of the ring is
+// read into registers a step before it is used, and copied over from then on.  CARRY: the walk without outputs, of
+// every segment but the last; DELTA has z = 1 for the walk from S = I.
+template <bool F32, int KT, bool DELTA, int VT, bool CARRY>
 __global__ __launch_bounds__(64 * VT, 2) void recur_chain_kernel(const RecurArgs a)
 {
-    constexpr int UNIT = recur_unit_kib(KT, DELTA, VT), RING = recur_ring(KT, DELTA), CPW = (UNIT + VT - 1) / VT;
-    // what is on its way behind the stage waited for: RING - 2 stages, and four stores of each step made since
-    constexpr int EARLY = (RING - 2) * CPW, FULL = (RING - 2) * (CPW + 4) + 4, FIRST = (RING - 1) * CPW;
+    using U = RecurUnit<KT, DELTA>;
+    constexpr int ALL = recur_unit_kib(KT, DELTA, VT), K0 = CARRY ? U::kG : 0, UNIT = ALL - K0;
+    constexpr int RING = recur_ring(KT, DELTA), CPW = (UNIT + VT - 1) / VT, STORES = CARRY ? 0 : 4;
+    // what is on its way behind the stage waited for: RING - 2 stages, and the stores of each step made since
+    constexpr int EARLY = (RING - 2) * CPW, FULL = (RING - 2) * (CPW + STORES) + STORES, FIRST = (RING - 1) * CPW;
     static_assert(FULL < 64 && FIRST < 64, "vmcnt");
+    constexpr uint32_t KP = 32 * KT, CP = 16 * VT;
     extern __shared__ __attribute__((aligned(16))) unsigned char recur_lds[];
-    const MixSeq s = a.seqs[a.list[blockIdx.x]];
-    const uint32_t head = blockIdx.y, D = a.dim;
+    const uint32_t segs = CARRY ? a.n_seg - 1 : a.n_seg, item = blockIdx.x / segs, seg = blockIdx.x % segs;
+    const MixSeq s = a.seqs[a.list[item]];
+    const uint32_t n_sub = (s.rows + kRecurSub - 1) / kRecurSub, begin = seg * a.seg_len, end = min(n_sub, begin + a.seg_len);
+    if (begin >= n_sub || (CARRY && end == n_sub)) return;        // uniform over the workgroup
+    const bool values = !(CARRY && DELTA) || blockIdx.z == 0;     // (else: from S = I, without values)
+    const uint32_t head = blockIdx.y, D = a.dim, sub0 = s.chunk0 * kRecurSubs;
     const int lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4;
     const uint32_t wave = (uint32_t)__builtin_amdgcn_readfirstlane(threadIdx.x >> 6), col = wave * 16 + c;
-    const uint32_t n_sub = (s.rows + kRecurSub - 1) / kRecurSub, sub0 = s.chunk0 * kRecurSubs;
     const uint32_t lds0 = (uint32_t)__builtin_amdgcn_readfirstlane((uint32_t)(uintptr_t)recur_lds);
     auto issue = [&](uint32_t sub) {                              // (past the end: the last one again)
-        const unsigned char* base = uniform_ptr(a.ops + ((size_t)(sub0 + min(sub, n_sub - 1)) * a.heads + head) * UNIT * 1024);
+        const unsigned char* base =
+            uniform_ptr(a.ops + (((size_t)(sub0 + min(begin + sub, end - 1)) * a.heads + head) * ALL + K0) * 1024);
         const uint32_t to = lds0 + sub % RING * UNIT * 1024;
 #pragma unroll
         for (int i = 0; i < CPW; i++) {
@@ -728,40 +746,84 @@ __global__ __launch_bounds__(64 * VT, 2) void recur_chain_kernel(const RecurArgs
     const size_t head_elems = (size_t)D * D;
     const float* in = a.state + ((size_t)s.state_in * a.heads + head) * head_elems;
     float* out = a.state + ((size_t)s.state_out * a.heads + head) * head_elems;
-    f32x4 S[2 * KT];                                              // channels 16t + 4g + i, column col
+    auto seg_at = [&](uint32_t q) { return ((size_t)item * a.n_seg + q) * a.heads + head; };
+    f32x4 S[2 * KT], gp[2 * KT];                                  // channels 16t + 4g + i, column col
 #pragma unroll
     for (int t = 0; t < 2 * KT; t++)
 #pragma unroll
         for (int i = 0; i < 4; i++) {
             const uint32_t d = 16 * t + 4 * g + i;
-            S[t][i] = (s.pos0 > 0 && d < D && col < D) ? in[(size_t)d * D + col] : 0.f;
+            if constexpr (CARRY) S[t][i] = values || d != col ? 0.f : 1.0f;
+            else S[t][i] = (s.pos0 > 0 && d < D && col < D) ? in[(size_t)d * D + col] : 0.f;
+            gp[t][i] = 1.0f;
         }
+    if constexpr (!CARRY) {
+        for (uint32_t q = 0; q < seg; q++) {                      // S <- X S + C of the segments before
+            const float* C = a.seg_c + seg_at(q) * KP * CP + col;
+            f32x4 next[2 * KT];
+#pragma unroll
+            for (int t = 0; t < 2 * KT; t++)
+#pragma unroll
+                for (int i = 0; i < 4; i++) next[t][i] = C[(size_t)(16 * t + 4 * g + i) * CP];
+            if constexpr (DELTA) {
+                RecurOp8<F32> So[KT];
+#pragma unroll
+                for (int k = 0; k < KT; k++) So[k] = recur_op8<F32>(S[2 * k], S[2 * k + 1]);
+                const float* X = a.seg_x + seg_at(q) * KP * KP + (size_t)c * KP + 4 * g;
+#pragma unroll
+                for (int t = 0; t < 2 * KT; t++) {
+#pragma unroll
+                    for (int k = 0; k < KT; k++) {
+                        const f32x4 lo = *reinterpret_cast<const f32x4*>(X + (size_t)16 * t * KP + 32 * k);
+                        f32x4 hi = f32x4{0.f, 0.f, 0.f, 0.f};
+                        if (32 * k + 16 < (int)CP) hi = *reinterpret_cast<const f32x4*>(X + (size_t)16 * t * KP + 32 * k + 16);
+                        next[t] = recur_mm(recur_op8<F32>(lo, hi), So[k], next[t]);
+                    }
+                    if constexpr (KT >= 4) __builtin_amdgcn_sched_barrier(0);    // (not every row's operands at once)
+                }
+            } else {
+                const float* X = a.seg_x + seg_at(q) * KP + 4 * g;
+#pragma unroll
+                for (int t = 0; t < 2 * KT; t++) {
+                    const f32x4 x = *reinterpret_cast<const f32x4*>(X + 16 * t);
+#pragma unroll
+                    for (int i = 0; i < 4; i++) next[t][i] = fmaf(x[i], S[t][i], next[t][i]);
+                }
+            }
+#pragma unroll
+            for (int t = 0; t < 2 * KT; t++) S[t] = next[t];
+        }
+    }
     // nothing of the state is on its way any more: what follows counts loads and stores
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-    const uint32_t ldo = a.heads * VT * 16;
-    float* o = a.o + ((size_t)sub0 * kRecurSub + 4 * g) * ldo + head * VT * 16 + col;
-    RecurHeld<F32, KT, DELTA> x, y;
+    const uint32_t ldo = a.heads * CP, n = end - begin;
+    float* o = a.o + ((size_t)(sub0 + begin) * kRecurSub + 4 * g) * ldo + head * CP + col;
+    using Held = RecurHeld<F32, KT, DELTA, CARRY>;
+    Held x, y;
 #pragma unroll
     for (int i = 0; i < RING; i++) issue(i);
     asm volatile("s_waitcnt vmcnt(%0)\n\ts_barrier" ::"n"(FIRST) : "memory");
-    x.fetch(recur_lds, wave, lane, g);
+    x.fetch(recur_lds, wave, lane, g, values);
     // a step: the next stage has landed and is fetched into `after`, the stage of `now` (in registers everywhere) is
     // copied over, and `now` moves the state
-    auto step = [&](uint32_t sub, const RecurHeld<F32, KT, DELTA>& now, RecurHeld<F32, KT, DELTA>& after) {
+    auto step = [&](uint32_t sub, const Held& now, Held& after) {
         if (sub < (uint32_t)RING - 1)
             asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)\n\ts_barrier" ::"n"(EARLY) : "memory");
         else
             asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)\n\ts_barrier" ::"n"(FULL) : "memory");
         issue(sub + RING);
-        after.fetch(recur_lds + (sub + 1) % RING * UNIT * 1024, wave, lane, g);
-        if constexpr (KT <= 2) __builtin_amdgcn_sched_barrier(0);         // (left alone, the reads sink to where they are used)
+        after.fetch(recur_lds + (sub + 1) % RING * UNIT * 1024, wave, lane, g, values);
+        if constexpr (KT <= 2 && !DELTA) __builtin_amdgcn_sched_barrier(0);      // (left alone, the reads sink to their uses)
         RecurOp8<F32> So[KT];
+        if constexpr (DELTA || !CARRY) {
 #pragma unroll
-        for (int t = 0; t < KT; t++) So[t] = recur_op8<F32>(S[2 * t], S[2 * t + 1]);
-        f32x4 O = f32x4{0.f, 0.f, 0.f, 0.f};
+            for (int t = 0; t < KT; t++) So[t] = recur_op8<F32>(S[2 * t], S[2 * t + 1]);
+        }
+        const f32x4 zero = f32x4{0.f, 0.f, 0.f, 0.f};
+        f32x4 O = zero;
         if constexpr (DELTA) {
-            const f32x4 P = recur_mm_many<KT>(now.W, So, recur_mm(now.M, now.V, O));
-            O = recur_mm_many<KT>(now.R, So, O);
+            const f32x4 P = recur_mm_many<KT>(now.W, So, recur_mm(now.M, now.V, zero));
+            if constexpr (!CARRY) O = recur_mm_many<KT>(now.R, So, O);
 #pragma unroll
             for (int t = 0; t < 2 * KT; t++)
 #pragma unroll
@@ -769,26 +831,45 @@ __global__ __launch_bounds__(64 * VT, 2) void recur_chain_kernel(const RecurArgs
             const RecurOp8<F32> VP = recur_join(now.V, recur_op4<F32>(P));
 #pragma unroll
             for (int t = 0; t < 2 * KT; t++) S[t] = recur_mm(now.K8[t], VP, S[t]);
-            O = recur_mm(now.A8, VP, O);
+            if constexpr (!CARRY) O = recur_mm(now.A8, VP, O);
         } else {
 #pragma unroll
             for (int t = 0; t < 2 * KT; t++)
 #pragma unroll
-                for (int i = 0; i < 4; i++) S[t][i] *= now.G[t][i];
+                for (int i = 0; i < 4; i++) {
+                    S[t][i] *= now.G[t][i];
+                    if constexpr (CARRY) gp[t][i] *= now.G[t][i];
+                }
 #pragma unroll
             for (int t = 0; t < 2 * KT; t++) S[t] = recur_mm(now.K4[t], now.V, S[t]);
-            O = recur_mm_many<KT>(now.R, So, recur_mm(now.A4, now.V, O));
+            if constexpr (!CARRY) O = recur_mm_many<KT>(now.R, So, recur_mm(now.A4, now.V, O));
         }
-        // (rows past the request's end have room of their own)
+        if constexpr (!CARRY) {
+            // (rows past the request's end have room of their own)
 #pragma unroll
-        for (int i = 0; i < 4; i++) o[(size_t)i * ldo] = O[i];
-        o += (size_t)kRecurSub * ldo;
+            for (int i = 0; i < 4; i++) o[(size_t)i * ldo] = O[i];
+            o += (size_t)kRecurSub * ldo;
+        }
     };
-    for (uint32_t sub = 0; sub < n_sub; sub += 2) {               // uniform
+    for (uint32_t sub = 0; sub < n; sub += 2) {                   // uniform
         step(sub, x, y);
-        if (sub + 1 < n_sub) step(sub + 1, y, x);
+        if (sub + 1 < n) step(sub + 1, y, x);
     }
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");              // the last copies still target the ring
+    if constexpr (CARRY) {
+        float* to = values ? a.seg_c + seg_at(seg) * KP * CP + col : a.seg_x + seg_at(seg) * KP * KP + col;
+        const uint32_t ld = values ? CP : KP;
+#pragma unroll
+        for (int t = 0; t < 2 * KT; t++)
+#pragma unroll
+            for (int i = 0; i < 4; i++) to[(size_t)(16 * t + 4 * g + i) * ld] = S[t][i];
+        if (!DELTA && wave == 0 && c == 0) {
+#pragma unroll
+            for (int t = 0; t < 2 * KT; t++) *reinterpret_cast<f32x4*>(a.seg_x + seg_at(seg) * KP + 16 * t + 4 * g) = gp[t];
+        }
+        return;
+    }
+    if (end < n_sub) return;
 #pragma unroll
     for (int t = 0; t < 2 * KT; t++)
 #pragma unroll

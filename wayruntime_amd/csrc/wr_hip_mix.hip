@@ -62,7 +62,7 @@ struct wr_hip_mix_step {
     size_t o_tokens, o_seq, o_pos, o_want, o_seqs, o_chunks, o_all, o_short, o_long, o_short_rows, o_pages, bytes;
     uint32_t rows = 0, n_seq = 0, n_want = 0, n_chunks = 0, n_short = 0, n_long = 0, n_short_rows = 0;
     uint32_t long_rows[kMaxSeqs];           // rows of each request of the long list
-    Buffer chunk_state, state_frag, partial, recur_ops, recur_out;
+    Buffer chunk_state, state_frag, partial, recur_ops, recur_out, recur_segs;
     template <typename T> T* d(size_t off) const { return reinterpret_cast<T*>(dev + off); }
     template <typename T> T* h(size_t off) const { return reinterpret_cast<T*>(host + off); }
 };
@@ -237,6 +237,7 @@ void wr_hip_mix_step_destroy(wr_hip_mix_step* s)
     wr_hip_attn_dev_free(s->partial.p);
     wr_hip_attn_dev_free(s->recur_ops.p);
     wr_hip_attn_dev_free(s->recur_out.p);
+    wr_hip_attn_dev_free(s->recur_segs.p);
     delete s;
 }
 
@@ -637,6 +638,8 @@ static int recur_steps(const RecurArgs& a, uint32_t n)
     return WR_HIP_OK;
 }
 
+constexpr uint32_t kSegMax = 8, kSegSubs = 6;
+
 template <bool F32, int KT, bool DELTA, int VT>
 static int recur_chunks(wr_hip_mix_step* s, RecurArgs& a)
 {
@@ -645,14 +648,34 @@ static int recur_chunks(wr_hip_mix_step* s, RecurArgs& a)
     int rc = ensure_device(s->recur_ops, (size_t)s->n_chunks * kRecurSubs * a.heads * unit);
     if (rc == WR_HIP_OK) rc = ensure_device(s->recur_out, (size_t)s->n_chunks * kMixChunk * a.heads * VT * 16 * 4);
     constexpr size_t l1 = (size_t)4 * recur_chunk_lds(KT, DELTA) * 4, l2 = recur_ring(KT, DELTA) * unit;
+    constexpr size_t l3 = l2 - (size_t)recur_ring(KT, DELTA) * RecurUnit<KT, DELTA>::kG * 1024;      // without the outputs' part
     if (rc == WR_HIP_OK) rc = allow_lds<recur_chunk_kernel<F32, KT, DELTA>>(l1);
-    if (rc == WR_HIP_OK) rc = allow_lds<recur_chain_kernel<F32, KT, DELTA, VT>>(l2);
+    if (rc == WR_HIP_OK) rc = allow_lds<recur_chain_kernel<F32, KT, DELTA, VT, false>>(l2);
+    if (rc == WR_HIP_OK) rc = allow_lds<recur_chain_kernel<F32, KT, DELTA, VT, true>>(l2);
     if (rc) return rc;
+    uint32_t longest = 0;
+    for (uint32_t i = 0; i < s->n_long; i++) longest = std::max(longest, (s->long_rows[i] + kRecurSub - 1) / kRecurSub);
+    // Segments: as many as give every compute unit a walk (below three the two walks cost more than one), none shorter
+    // than kSegSubs.
+    a.n_seg = std::min({(uint32_t)g.n_cus / (s->n_long * a.heads), longest / kSegSubs, kSegMax});
+    if (a.n_seg < 3) a.n_seg = 1;
+    a.seg_len = (longest + a.n_seg - 1) / a.n_seg;
+    if (a.n_seg > 1) {
+        constexpr size_t c = (size_t)32 * KT * 16 * VT, x = DELTA ? (size_t)32 * KT * 32 * KT : 32 * KT;
+        const size_t items = (size_t)s->n_long * a.n_seg * a.heads;
+        rc = ensure_device(s->recur_segs, items * (c + x) * 4);
+        if (rc) return rc;
+        a.seg_c = reinterpret_cast<float*>(s->recur_segs.p);
+        a.seg_x = a.seg_c + items * c;
+    }
     a.ops = reinterpret_cast<unsigned char*>(s->recur_ops.p);
     a.o = reinterpret_cast<float*>(s->recur_out.p);
     const uint32_t whole = !((a.dim | a.ld | a.ldz | a.col_r | a.col_k | a.col_a) % 4);
     MIX_LAUNCH((recur_chunk_kernel<F32, KT, DELTA>), dim3(s->n_chunks, a.heads), dim3(256), l1, a, whole);
-    MIX_LAUNCH((recur_chain_kernel<F32, KT, DELTA, VT>), dim3(s->n_long, a.heads), dim3(64 * VT), l2, a);
+    if (a.n_seg > 1)
+        MIX_LAUNCH((recur_chain_kernel<F32, KT, DELTA, VT, true>), dim3(s->n_long * (a.n_seg - 1), a.heads, DELTA ? 2 : 1),
+                   dim3(64 * VT), l3, a);
+    MIX_LAUNCH((recur_chain_kernel<F32, KT, DELTA, VT, false>), dim3(s->n_long * a.n_seg, a.heads), dim3(64 * VT), l2, a);
     MIX_LAUNCH(recur_gate_kernel<F32>, dim3(s->n_chunks, a.heads), dim3(256), 0, a);
     return WR_HIP_OK;
 }
