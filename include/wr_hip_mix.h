@@ -223,8 +223,8 @@ uint32_t wr_hip_mix_window_pad(uint32_t dim);
 int wr_hip_mix_window_append(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, int f32,
                              const wr_hip_mix_window *g, const float *in_dev, uint32_t ld, uint32_t col_q,
                              uint32_t col_k, uint32_t col_v, const float *table_dev, void *q_dev);
-/* Softmax attention over the cached rows inside the window; the denominator also holds
- * exp(sink[head]) when sink is given.  Head h's output times out_scale goes to o (frag,
+/* Softmax attention over the cached rows inside the window; with `sink`, a head's weights
+ * are exp(score) / (exp(sink[head]) + sum of exp(score)).  Head h's output times out_scale goes to o (frag,
  * o_kt tiles) at input h * vdim_pad. */
 int wr_hip_mix_window_attend(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, int f32,
                              const wr_hip_mix_window *g, const void *q_dev, const float *sink_dev,

@@ -204,7 +204,7 @@ MIXERS = {"lightning": lambda *a: lightning(*a)[0], "latent_attention": latent_a
 
 
 def prenorm_layer(x, w, cfg, eps):
-    """A layer with a norm ahead of each sublayer only, its weight stored around zero."""
+    """A layer with a norm ahead of each sublayer only; stored w means the factor 1 + w."""
     x = x + MIXERS[cfg["type"]](rms_norm(x, 1 + w["norm1"], eps), _sub(w, "mix."), cfg["mixer"], eps)
     if cfg.get("mlp"):
         x = x + gelu_mlp(rms_norm(x, 1 + w["norm2"], eps), _sub(w, "mlp."))

@@ -1,5 +1,6 @@
-// Sliding-window attention over grouped keys and values, with an optional sink in the
-// softmax's denominator (a learned number per head: no key, no value, not scaled).
+// Sliding-window attention over grouped keys and values.  Optionally each head has a sink
+// s: its weights are exp(score) / (exp(s) + sum of exp(score)), so a row may attend to
+// nothing at all.
 //
 // A page (64 positions) holds each key/value head's block one after the other:
 //

@@ -95,8 +95,8 @@ typedef struct wr_model_params {
 
 /* A GGUF v2/v3 file (architectures "llama", "qwen3" and "gemma4", F16 / F32
  * tensors), or a folder with config.json and model.safetensors (bfloat16) whose
- * config names an architecture of the mixer-stack family ("Bipotar").  For the
- * latter, keep_quantized == WR_QUANT_F32 asks for 32-bit activations and caches. */
+ * config names an architecture of the mixer-stack family ("Bipotar", "Taredra").
+ * For the latter, keep_quantized == WR_QUANT_F32 asks for 32-bit activations and caches. */
 wr_status wr_model_load(wr_engine *e, const char *gguf_path,
                         const wr_model_params *params, wr_model **out);
 void      wr_model_free(wr_model *m);
