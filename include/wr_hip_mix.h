@@ -97,10 +97,13 @@ int wr_hip_mix_embed(wr_hip_mix_step *s, int f32, const uint16_t *table_dev, uin
 /* A sublayer's output joins the residual and the next sublayer's input is made:
  *   x += rmsnorm(y) * post           (when y is given; x += y without `post`; with `top` > 0,
  *                                     row r of y is sum_t gate[r][t] * y[slot[r][t]], the
- *                                     experts' rows)
+ *                                     experts' rows, slots of ~0 left out; with `side` as well
+ *                                     + side[r][0] * ident[r] + side[r][1] * shared[r])
  *   x += add                         (when given)
  *   h = rmsnorm(x) * next            (when given; only the step's wanted rows, packed,
- *                                     with `wanted` set) */
+ *                                     with `wanted` set)
+ * ident: frag rows of the width, may be h itself; shared: 32-bit rows like y; either may
+ * be NULL. */
 typedef struct wr_hip_mix_resid {
     uint32_t width;
     float eps;
@@ -111,6 +114,9 @@ typedef struct wr_hip_mix_resid {
     uint32_t top;
     uint32_t wanted;
     void *h;
+    const float *side;
+    const void *ident;
+    const float *shared;
 } wr_hip_mix_resid;
 int wr_hip_mix_residual(wr_hip_mix_step *s, int f32, const wr_hip_mix_resid *a);
 /* Token shift.  x += y first (y may be NULL).  With h[r] = rmsnorm(x[r]) * norm and p[r]
@@ -134,12 +140,15 @@ int wr_hip_mix_shift(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, in
  *   FRAG       h (frag, h_kt tiles): row r, input z * col_z + n
  *   SPLIT      n < n_split: FRAG; else y_f32[r][n - n_split]
  *   GATED      tiles 2j / 2j+1 of W are gate / up: silu(gate) * up to FRAG
- *              (with gelu: 0.5 g (1 + tanh(sqrt(2/pi) (g + 0.044715 g^3))) * up)
- * after an activation: SiLU for n < silu_end, else the logistic for n <
+ *              (with gelu: 0.5 g (1 + tanh(sqrt(2/pi) (g + 0.044715 g^3))) * up;
+ *              with limit > 0: g = min(gate, limit), u = up within [-limit, limit],
+ *              g * logistic(slope * g) * (u + up_bias))
+ *   SPLIT_GATED n < n_split (a multiple of 32): y_f32[r][n]; the tiles behind as GATED
+ * after `bias` (n_out floats, batch 1) and an activation: SiLU for n < silu_end, else the logistic for n <
  * sigmoid_end, else the hyperbolic tangent for n < tanh_end; square of ReLU
- * everywhere with relu2; times `scale` when not 0. */
+ * everywhere with relu2; times `scale` when not 0.  (GATED outputs take neither.) */
 enum { WR_HIP_MIX_OUT_ROWS_F32 = 0, WR_HIP_MIX_OUT_ROWS = 1, WR_HIP_MIX_OUT_FRAG = 2,
-       WR_HIP_MIX_OUT_SPLIT = 3, WR_HIP_MIX_OUT_GATED = 4 };
+       WR_HIP_MIX_OUT_SPLIT = 3, WR_HIP_MIX_OUT_GATED = 4, WR_HIP_MIX_OUT_SPLIT_GATED = 5 };
 typedef struct wr_hip_mix_gemm {
     const wr_hip_mat *w;
     const void *x;
@@ -157,6 +166,9 @@ typedef struct wr_hip_mix_gemm {
     float scale;
     uint32_t tanh_end, gelu;
     uint32_t x_kt0;                /* first input tile of matrix 0 */
+    const float *bias;
+    float limit, slope, up_bias;
+    const uint32_t *x_perm;        /* with group_expert and tile_groups 1: row i is row x_perm[i] of x (any row for ~0) */
 } wr_hip_mix_gemm;
 int wr_hip_mix_gemm_run(int f32, const wr_hip_mix_gemm *a);
 
@@ -207,28 +219,42 @@ int wr_hip_mix_recur(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, in
 /* ---- windowed attention over grouped keys and values ----------------------------
  * `heads` query heads, `kv_heads` key/value heads (query head h reads h / (heads /
  * kv_heads)), head sizes dim (queries, keys) and vdim (values), padded to dim_pad and
- * vdim_pad (wr_hip_mix_window_pad).  The first 2 * rot_half dimensions are rotated, i
- * with i + rot_half.  Cached per position: kv_heads * (dim_pad + vdim_pad) elements. */
+ * vdim_pad (wr_hip_mix_window_pad).  With maps = 2 every head has two queries and every
+ * key/value head two keys, one behind the other, and both maps weigh the same values.
+ * Queries and keys may be normed (each map's vector over its root mean square, times a
+ * weight of dim), then the first 2 * rot_half dimensions are rotated, i with
+ * i + rot_half, or with `neighbours` 2i with 2i + 1.
+ * Cached per position: kv_heads * (maps * dim_pad + vdim_pad) elements. */
 typedef struct wr_hip_mix_window {
     uint32_t heads, kv_heads, dim, dim_pad, vdim, vdim_pad, rot_half;
     uint32_t window;               /* keys a row sees, itself included */
     float scale, out_scale;
     uint32_t norm_values;          /* values divided by their root mean square (eps) ahead of the cache */
     float eps;
+    uint32_t maps;                 /* 1 or 2 */
+    uint32_t neighbours;
+    float softcap;                 /* > 0: scores are softcap * tanh(score / softcap) */
+    float diff;                    /* maps = 2: how much of the second map's output is taken off */
+    const float *q_norm, *k_norm;  /* device, dim floats each, or NULL */
 } wr_hip_mix_window;
 /* The padded head size to use: what the matrix kernels take, else a multiple of 32. */
 uint32_t wr_hip_mix_window_pad(uint32_t dim);
-/* From 32-bit rows (stride ld): queries at col_q rotated into q (frag, head h at input
- * h * dim_pad); keys at col_k rotated and values at col_v, normed, into the cache. */
+/* From 32-bit rows (stride ld): queries at col_q, normed and rotated, into q (frag, head h
+ * at input h * maps * dim_pad); keys at col_k, normed and rotated, and values at col_v,
+ * normed with norm_values, into the cache.  col_v may be col_k.  With col_k =
+ * WR_HIP_MIX_NO_KEYS the queries alone: another layer's keys and values serve. */
+#define WR_HIP_MIX_NO_KEYS 0xFFFFFFFFu
 int wr_hip_mix_window_append(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, int f32,
                              const wr_hip_mix_window *g, const float *in_dev, uint32_t ld, uint32_t col_q,
                              uint32_t col_k, uint32_t col_v, const float *table_dev, void *q_dev);
 /* Softmax attention over the cached rows inside the window; with `sink`, a head's weights
- * are exp(score) / (exp(sink[head]) + sum of exp(score)).  Head h's output times out_scale goes to o (frag,
- * o_kt tiles) at input h * vdim_pad. */
+ * are exp(score) / (exp(sink[head]) + sum of exp(score)).  With two maps a head's output is
+ * first - diff * second, over its root mean square (eps).  Head h's output times out_scale,
+ * and times logistic(gate[row * ldg + h]) where `gate` is given, goes to o (frag, o_kt
+ * tiles) at input h * vdim_pad. */
 int wr_hip_mix_window_attend(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, int f32,
                              const wr_hip_mix_window *g, const void *q_dev, const float *sink_dev,
-                             void *o_dev, uint32_t o_kt);
+                             const float *gate_dev, uint32_t ldg, void *o_dev, uint32_t o_kt);
 
 /* ---- attention through a latent -----------------------------------------------
  * Table of (cos, sin) of position * freq[i] for the step's rows, [rows][half][2];
@@ -261,15 +287,31 @@ int wr_hip_mix_latent_attend(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t
                              const wr_hip_mix_latent *g, const void *q_dev, void *o_dev);
 
 /* ---- mixture of experts ---------------------------------------------------------
- * From router logits (32-bit rows, row stride ldz): the `top` largest of each row
- * (lowest index first among equals), gate = softmax over them, and an order of the
- * (row, choice) pairs by expert: each expert's pairs take runs of tile_groups
- * groups of 16 slots.  slot[r][t]: the pair's slot; perm: row of each slot, or
- * ~0; group_expert: expert of each group of 16 slots, or -1.
+ * From router logits (32-bit rows, row stride ldz) over `experts` experts and `identity`
+ * outputs that pass the layer's input on: the `top` outputs with the largest choice value
+ * (lowest index first among equals), their weights, and an order of the (row, choice)
+ * pairs by expert: each expert's pairs take runs of tile_groups groups of 16 slots.
+ * The choice value is the logit and the weights are the softmax over the chosen; with
+ * softmax_all it is the softmax over all outputs plus `correction`, and the weights are
+ * the chosen outputs' softmax over (their sum + 1e-20), times scale.  With groups > 0 the
+ * outputs form that many equal groups of neighbours, and only those of the `keep` groups
+ * with the largest choice value in them can be chosen.
+ * slot[r][t]: the pair's slot, ~0 for an identity output; perm: row of each slot, or ~0;
+ * group_expert: expert of each group of 16 slots, or -1; side[r] (may be NULL): the sum of
+ * the identity outputs' weights, and, with shared_gate, the logistic of the logit behind
+ * the outputs' (else 0).
  * wr_hip_mix_route_groups: how many groups that can take at most. */
+typedef struct wr_hip_mix_router {
+    uint32_t experts, identity, top;
+    uint32_t groups, keep;
+    uint32_t softmax_all, shared_gate;
+    float scale;
+    const float *correction;       /* device, or NULL */
+} wr_hip_mix_router;
+#define WR_HIP_MIX_MAX_GROUPS 64u
 uint32_t wr_hip_mix_route_groups(uint32_t rows, uint32_t experts, uint32_t top, uint32_t tile_groups);
-int wr_hip_mix_route(wr_hip_mix_step *s, const float *z_dev, uint32_t ldz, uint32_t experts, uint32_t top,
-                     uint32_t tile_groups, float *gate_dev, uint32_t *slot_dev, uint32_t *perm_dev,
+int wr_hip_mix_route(wr_hip_mix_step *s, const float *z_dev, uint32_t ldz, const wr_hip_mix_router *g,
+                     uint32_t tile_groups, float *gate_dev, float *side_dev, uint32_t *slot_dev, uint32_t *perm_dev,
                      int32_t *group_expert_dev);
 /* The rows of h in slot order: xs (frag). */
 int wr_hip_mix_route_gather(wr_hip_mix_step *s, int f32, const void *h_dev, uint32_t kt, uint32_t n_groups,

@@ -173,8 +173,12 @@ int wr_hip_mix_residual(wr_hip_mix_step *s, int f32, const wr_hip_mix_resid *a)
         if (a->y) {
             for (uint32_t k = 0; k < wp; k++) {
                 y[k] = a->top ? 0.0f : a->y[(size_t)r * wp + k];
-                for (uint32_t t = 0; t < a->top; t++)
-                    y[k] += a->gate[(size_t)r * a->top + t] * a->y[(size_t)a->slot[(size_t)r * a->top + t] * wp + k];
+                for (uint32_t t = 0; t < a->top; t++) {
+                    const uint32_t slot = a->slot[(size_t)r * a->top + t];
+                    if (slot != ~0u) y[k] += a->gate[(size_t)r * a->top + t] * a->y[(size_t)slot * wp + k];
+                }
+                if (a->side && a->ident) y[k] += a->side[2 * r] * ((const float *)a->ident)[(size_t)r * wp + k];
+                if (a->side && a->shared) y[k] += a->side[2 * r + 1] * a->shared[(size_t)r * wp + k];
             }
             const float inv = a->post ? inv_rms(y, a->width, a->eps) : 1.0f;
             for (uint32_t k = 0; k < wp; k++) x[k] += a->post ? y[k] * inv * a->post[k] : y[k];
@@ -218,6 +222,16 @@ int wr_hip_mix_shift(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, in
     return WR_HIP_OK;
 }
 
+static float gated_unit(const wr_hip_mix_gemm *a, float g, float u)
+{
+    if (a->limit > 0) {
+        g = fminf(g, a->limit);
+        u = fminf(fmaxf(u, -a->limit), a->limit);
+        return g * sig(a->slope * g) * (u + a->up_bias);
+    }
+    return a->gelu ? 0.5f * g * (1.0f + tanhf(0.79788456080286536f * (g + 0.044715f * g * g * g))) * u : g * sig(g) * u;
+}
+
 int wr_hip_mix_gemm_run(int f32, const wr_hip_mix_gemm *a)
 {
     if (!f32) return WR_HIP_ERR_UNSUPPORTED;
@@ -232,7 +246,8 @@ int wr_hip_mix_gemm_run(int f32, const wr_hip_mix_gemm *a)
                 if (a->group_expert[r / 16] < 0) continue;
                 mat = (uint32_t)a->group_expert[r / 16];
             }
-            const float *x = (const float *)a->x + (size_t)r * ldx + ((size_t)a->x_kt0 + (size_t)z * a->x_kt_z) * 32;
+            const uint32_t from = !a->x_perm ? r : a->x_perm[r] == ~0u ? 0 : a->x_perm[r];
+            const float *x = (const float *)a->x + (size_t)from * ldx + ((size_t)a->x_kt0 + (size_t)z * a->x_kt_z) * 32;
             const float *w = a->w->w + (size_t)mat * N * K;
             for (uint32_t n = 0; n < N; n++) {
                 float acc = 0;
@@ -240,16 +255,15 @@ int wr_hip_mix_gemm_run(int f32, const wr_hip_mix_gemm *a)
                 v[n] = acc;
             }
             float *h = a->h ? (float *)a->h + (size_t)r * a->h_kt * 32 + (size_t)z * a->col_z : NULL;
-            if (a->out == WR_HIP_MIX_OUT_GATED) {
-                for (uint32_t n = 0; n < N / 2; n++) {
-                    const float g = v[n / 16 * 32 + n % 16], u = v[n / 16 * 32 + 16 + n % 16];
-                    h[n] = a->gelu ? 0.5f * g * (1.0f + tanhf(0.79788456080286536f * (g + 0.044715f * g * g * g))) * u
-                                   : g * sig(g) * u;
-                }
+            if (a->out >= WR_HIP_MIX_OUT_GATED) {
+                const uint32_t rows = a->out == WR_HIP_MIX_OUT_SPLIT_GATED ? a->n_split : 0;
+                for (uint32_t n = 0; n < rows; n++) a->y_f32[(size_t)r * a->ldy + n] = v[n];
+                for (uint32_t n = 0; n < (N - rows) / 2; n++)
+                    h[n] = gated_unit(a, v[rows + n / 16 * 32 + n % 16], v[rows + n / 16 * 32 + 16 + n % 16]);
                 continue;
             }
             for (uint32_t n = 0; n < N; n++) {
-                float o = v[n];
+                float o = v[n] + (a->bias ? a->bias[n] : 0.0f);
                 if (n < a->silu_end) o *= sig(o);
                 else if (n < sig_end) o = sig(o);
                 else if (n < a->tanh_end) o = tanhf(o);
@@ -455,9 +469,28 @@ uint32_t wr_hip_mix_window_pad(uint32_t dim) { return p32(dim); }
 static float *window_row(wr_hip_mix_pool *pool, uint32_t run, const wr_hip_mix_window *g, const wr_hip_mix_seq *q, uint32_t pos,
                          uint32_t kvh)
 {
-    const uint32_t per = g->dim_pad + g->vdim_pad;
+    const uint32_t per = g->maps * g->dim_pad + g->vdim_pad;
     return pool->latent[run] + (((size_t)q->pages[pos / WR_HIP_MIX_PAGE] * g->kv_heads + kvh) * WR_HIP_MIX_PAGE +
                                 pos % WR_HIP_MIX_PAGE) * per;
+}
+
+/* One query or key of one map: normed, rotated, padded. */
+static void window_turn(const wr_hip_mix_window *g, const float *x, const float *norm, const float *tab, float *out)
+{
+    float *y = malloc(g->dim * 4);
+    const float inv = norm ? inv_rms(x, g->dim, g->eps) : 1.0f;
+    for (uint32_t i = 0; i < g->dim; i++) y[i] = norm ? x[i] * inv * norm[i] : x[i];
+    memset(out, 0, g->dim_pad * 4);
+    if (!g->neighbours) {
+        rotate(y, tab, g->rot_half, g->dim, out);
+    } else {
+        memcpy(out, y, g->dim * 4);
+        for (uint32_t i = 0; i < g->rot_half; i++) {
+            out[2 * i] = y[2 * i] * tab[2 * i] - y[2 * i + 1] * tab[2 * i + 1];
+            out[2 * i + 1] = y[2 * i + 1] * tab[2 * i] + y[2 * i] * tab[2 * i + 1];
+        }
+    }
+    free(y);
 }
 
 int wr_hip_mix_window_append(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, int f32, const wr_hip_mix_window *g,
@@ -467,51 +500,62 @@ int wr_hip_mix_window_append(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t
     if (!f32) return WR_HIP_ERR_UNSUPPORTED;
     for (uint32_t r = 0; r < s->rows; r++) {
         const float *row = in + (size_t)r * ld, *tab = table + (size_t)r * 2 * g->rot_half;
-        for (uint32_t h = 0; h < g->heads; h++) {
-            float *q = (float *)qv + ((size_t)r * g->heads + h) * g->dim_pad;
-            memset(q, 0, g->dim_pad * 4);
-            rotate(row + col_q + h * g->dim, tab, g->rot_half, g->dim, q);
-        }
-        for (uint32_t h = 0; h < g->kv_heads; h++) {
-            float *c = window_row(pool, run, g, &s->seqs[s->seq[r]], s->pos[r], h);
-            memset(c, 0, (g->dim_pad + g->vdim_pad) * 4);
-            rotate(row + col_k + h * g->dim, tab, g->rot_half, g->dim, c);
+        for (uint32_t h = 0; h < g->heads * g->maps; h++)
+            window_turn(g, row + col_q + h * g->dim, g->q_norm, tab, (float *)qv + ((size_t)r * g->heads * g->maps + h) * g->dim_pad);
+        for (uint32_t h = 0; h < g->kv_heads && col_k != WR_HIP_MIX_NO_KEYS; h++) {
+            float *c = window_row(pool, run, g, &s->seqs[s->seq[r]], s->pos[r], h), *cv = c + g->maps * g->dim_pad;
+            for (uint32_t m = 0; m < g->maps; m++)
+                window_turn(g, row + col_k + (h * g->maps + m) * g->dim, g->k_norm, tab, c + m * g->dim_pad);
+            memset(cv, 0, g->vdim_pad * 4);
             const float *v = row + col_v + h * g->vdim, inv = g->norm_values ? inv_rms(v, g->vdim, g->eps) : 1.0f;
-            for (uint32_t k = 0; k < g->vdim; k++) c[g->dim_pad + k] = v[k] * inv;
+            for (uint32_t k = 0; k < g->vdim; k++) cv[k] = v[k] * inv;
         }
     }
     return WR_HIP_OK;
 }
 
 int wr_hip_mix_window_attend(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, int f32, const wr_hip_mix_window *g,
-                             const void *qv, const float *sink, void *ov, uint32_t o_kt)
+                             const void *qv, const float *sink, const float *gate, uint32_t ldg, void *ov, uint32_t o_kt)
 {
     if (!f32) return WR_HIP_ERR_UNSUPPORTED;
+    const uint32_t V = g->vdim_pad;
     for (uint32_t r = 0; r < s->rows; r++) {
         const wr_hip_mix_seq *sq = &s->seqs[s->seq[r]];
         const uint32_t pos = s->pos[r], lo = pos + 1 > g->window ? pos + 1 - g->window : 0;
-        double *w = malloc(sizeof(double) * (pos - lo + 1));
+        double *w = malloc(sizeof(double) * (pos - lo + 1)), *a2 = malloc(sizeof(double) * 2 * V);
         for (uint32_t h = 0; h < g->heads; h++) {
             const uint32_t kvh = h / (g->heads / g->kv_heads);
-            const float *q = (const float *)qv + ((size_t)r * g->heads + h) * g->dim_pad;
-            float *o = (float *)ov + (size_t)r * o_kt * 32 + (size_t)h * g->vdim_pad;
-            double mx = sink ? sink[h] : -INFINITY;
-            for (uint32_t j = lo; j <= pos; j++) {
-                const float *c = window_row(pool, run, g, sq, j, kvh);
-                double a = 0;
-                for (uint32_t k = 0; k < g->dim_pad; k++) a += (double)q[k] * c[k];
-                w[j - lo] = a * g->scale;
-                if (w[j - lo] > mx) mx = w[j - lo];
+            float *o = (float *)ov + (size_t)r * o_kt * 32 + (size_t)h * V;
+            for (uint32_t m = 0; m < g->maps; m++) {
+                const float *q = (const float *)qv + (((size_t)r * g->heads + h) * g->maps + m) * g->dim_pad;
+                double mx = sink ? sink[h] : -INFINITY;
+                for (uint32_t j = lo; j <= pos; j++) {
+                    const float *c = window_row(pool, run, g, sq, j, kvh) + m * g->dim_pad;
+                    double a = 0;
+                    for (uint32_t k = 0; k < g->dim_pad; k++) a += (double)q[k] * c[k];
+                    a *= g->scale;
+                    w[j - lo] = g->softcap > 0 ? g->softcap * tanh(a / g->softcap) : a;
+                    if (w[j - lo] > mx) mx = w[j - lo];
+                }
+                double sum = sink ? exp(sink[h] - mx) : 0;
+                for (uint32_t j = lo; j <= pos; j++) sum += (w[j - lo] = exp(w[j - lo] - mx));
+                for (uint32_t k = 0; k < V; k++) {
+                    double a = 0;
+                    for (uint32_t j = lo; j <= pos; j++)
+                        a += w[j - lo] * window_row(pool, run, g, sq, j, kvh)[g->maps * g->dim_pad + k];
+                    a2[m * V + k] = a / sum;
+                }
             }
-            double sum = sink ? exp(sink[h] - mx) : 0;
-            for (uint32_t j = lo; j <= pos; j++) sum += (w[j - lo] = exp(w[j - lo] - mx));
-            for (uint32_t k = 0; k < g->vdim_pad; k++) {
-                double a = 0;
-                for (uint32_t j = lo; j <= pos; j++) a += w[j - lo] * window_row(pool, run, g, sq, j, kvh)[g->dim_pad + k];
-                o[k] = (float)(a / sum * g->out_scale);
+            double f = gate ? g->out_scale * sig(gate[(size_t)r * ldg + h]) : g->out_scale, ss = 0;
+            for (uint32_t k = 0; g->maps == 2 && k < V; k++) {
+                a2[k] -= g->diff * a2[V + k];
+                ss += a2[k] * a2[k];
             }
+            if (g->maps == 2) f /= sqrt(ss / g->vdim + g->eps);
+            for (uint32_t k = 0; k < V; k++) o[k] = (float)(a2[k] * f);
         }
         free(w);
+        free(a2);
     }
     return WR_HIP_OK;
 }
@@ -522,30 +566,55 @@ uint32_t wr_hip_mix_route_groups(uint32_t rows, uint32_t experts, uint32_t top, 
     return (pairs / (tile_groups * 16) + (pairs < experts ? pairs : experts)) * tile_groups;
 }
 
-int wr_hip_mix_route(wr_hip_mix_step *s, const float *z, uint32_t ldz, uint32_t experts, uint32_t top, uint32_t tile_groups,
-                     float *gate, uint32_t *slot, uint32_t *perm, int32_t *group_expert)
+int wr_hip_mix_route(wr_hip_mix_step *s, const float *z, uint32_t ldz, const wr_hip_mix_router *g, uint32_t tile_groups,
+                     float *gate, float *side, uint32_t *slot, uint32_t *perm, int32_t *group_expert)
 {
+    const uint32_t experts = g->experts, top = g->top, N = experts + g->identity;
     const uint32_t groups = wr_hip_mix_route_groups(s->rows, experts, top, tile_groups), run = tile_groups * 16;
-    uint8_t *taken = malloc(experts);
+    if (ldz < N + (g->shared_gate != 0) || (g->groups && N % g->groups)) return WR_HIP_ERR_INVAL;
+    float *c = malloc(N * 4), *p = malloc(N * 4), *lead = malloc((g->groups + 1) * 4);
     for (uint32_t r = 0; r < s->rows; r++) {
-        memset(taken, 0, experts);
-        float sum = 0, first = 0;
-        for (uint32_t t = 0; t < top; t++) {
-            uint32_t best = experts;
-            for (uint32_t e = 0; e < experts; e++)
-                if (!taken[e] && (best == experts || z[(size_t)r * ldz + e] > z[(size_t)r * ldz + best])) best = e;
-            taken[best] = 1;
-            if (t == 0) first = z[(size_t)r * ldz + best];
-            slot[r * top + t] = best;
-            sum += gate[r * top + t] = expf(z[(size_t)r * ldz + best] - first);
+        const float *zr = z + (size_t)r * ldz;
+        float most = zr[0], all = 0;
+        for (uint32_t e = 1; e < N; e++) most = fmaxf(most, zr[e]);
+        for (uint32_t e = 0; e < N; e++) all += (p[e] = expf(zr[e] - most));
+        for (uint32_t e = 0; e < N; e++) c[e] = g->softmax_all ? p[e] / all + (g->correction ? g->correction[e] : 0) : zr[e];
+        for (uint32_t k = 0; k < g->groups; k++) {
+            lead[k] = -INFINITY;
+            for (uint32_t e = k * (N / g->groups); e < (k + 1) * (N / g->groups); e++) lead[k] = fmaxf(lead[k], c[e]);
         }
-        for (uint32_t t = 0; t < top; t++) gate[r * top + t] /= sum;
+        for (uint32_t k = 0; k < g->groups; k++) {
+            uint32_t ahead = 0;
+            for (uint32_t j = 0; j < g->groups; j++) ahead += lead[j] > lead[k] || (lead[j] == lead[k] && j < k);
+            for (uint32_t e = 0; ahead >= g->keep && e < N / g->groups; e++) c[k * (N / g->groups) + e] = -INFINITY;
+        }
+        float sum = 0, own = 0;
+        for (uint32_t t = 0; t < top; t++) {
+            uint32_t best = 0;
+            for (uint32_t e = 1; e < N; e++)
+                if (c[e] > c[best]) best = e;
+            c[best] = -INFINITY;
+            slot[r * top + t] = best;
+            sum += gate[r * top + t] = g->softmax_all ? p[best] / all : p[best];
+        }
+        for (uint32_t t = 0; t < top; t++) {
+            float *w = &gate[r * top + t];
+            *w = g->softmax_all ? *w / (sum + 1e-20f) * g->scale : *w / sum;
+            if (slot[r * top + t] >= experts) own += *w;
+        }
+        if (side) {
+            side[2 * r] = own;
+            side[2 * r + 1] = g->shared_gate ? sig(zr[N]) : 0;
+        }
     }
-    free(taken);
+    free(c);
+    free(p);
+    free(lead);
     for (uint32_t i = 0; i < groups * 16; i++) perm[i] = ~0u;
     for (uint32_t i = 0; i < groups; i++) group_expert[i] = -1;
     uint32_t at = 0;
     uint32_t *out = malloc((size_t)s->rows * top * 4);
+    memset(out, 0xFF, (size_t)s->rows * top * 4);          /* (the input itself takes no slot) */
     for (uint32_t e = 0; e < experts; e++) {
         const uint32_t begin = at;
         for (uint32_t i = 0; i < s->rows * top; i++)
@@ -554,7 +623,7 @@ int wr_hip_mix_route(wr_hip_mix_step *s, const float *z, uint32_t ldz, uint32_t 
                 out[i] = at++;
             }
         at = (at + run - 1) / run * run;
-        for (uint32_t g = begin / 16; g < at / 16; g++) group_expert[g] = (int32_t)e;
+        for (uint32_t i = begin / 16; i < at / 16; i++) group_expert[i] = (int32_t)e;
     }
     memcpy(slot, out, (size_t)s->rows * top * 4);
     free(out);

@@ -1,5 +1,5 @@
-"""Plain, slow restatement of the mixer-stack models (architectures "Bipotar" and
-"Taredra"): one function per mechanism, numpy, one sequence at a time, every
+"""Plain, slow restatement of the mixer-stack models (architectures "Bipotar",
+"Taredra" and "Fedirax"): one function per mechanism, numpy, one sequence at a time, every
 position from the definition (no cache, no chunks, no absorbed products).  Shares
 no code with the product path; the tests compare the engine with it.
 
@@ -199,6 +199,161 @@ def gelu_mlp(h, w):
     return (gelu_tanh(h @ w["gate"].T) * (h @ w["up"].T)) @ w["down"].T
 
 
+def rotate_neighbours(x, positions, base, dims):
+    """x [T, ..., >= dims]: dimension 2i turns with dimension 2i + 1."""
+    freq = float(base) ** (-2.0 * np.arange(dims // 2) / dims)
+    ang = np.asarray(positions, dtype=np.float64)[:, None] * freq[None]
+    out = x.copy()
+    for i in range(dims // 2):
+        shape = (len(positions),) + (1,) * (x.ndim - 2)
+        c, s = np.cos(ang[:, i]).reshape(shape).astype(x.dtype), np.sin(ang[:, i]).reshape(shape).astype(x.dtype)
+        out[..., 2 * i] = x[..., 2 * i] * c - x[..., 2 * i + 1] * s
+        out[..., 2 * i + 1] = x[..., 2 * i + 1] * c + x[..., 2 * i] * s
+    return out
+
+
+def in_window(pos, size):
+    """[T, T]: row i sees its own position and the size - 1 before it."""
+    gap = pos[:, None] - pos[None, :]
+    return (gap >= 0) & (gap < size)
+
+
+def soft_cap(score, cap):
+    return score if not cap else cap * np.tanh(score / cap)
+
+
+def keys_as_values_attention(h, w, cfg, eps, positions=None):
+    """Grouped-query attention whose values are the projected keys ahead of their rotation: biases, capped scores, a sink
+    per head, and each head's output times a logistic gate of its own."""
+    H, G, D = cfg["heads"], cfg["kv_heads"], cfg["dim"]
+    assert cfg["vdim"] == D
+    T = h.shape[0]
+    pos = np.arange(T) if positions is None else np.asarray(positions)
+    rot = cfg["rot"]
+    q = rotate_neighbours((h @ w["q"].T + w["q.b"]).reshape(T, H, D), pos, rot["base"], rot["dims"])
+    v = (h @ w["k"].T + w["k.b"]).reshape(T, G, D)
+    k = rotate_neighbours(v, pos, rot["base"], rot["dims"])
+    seen = in_window(pos, cfg["mask"]["size"])
+    out = np.empty((T, H, D), dtype=h.dtype)
+    for hh in range(H):
+        g = hh // (H // G)
+        s = np.where(seen, soft_cap((q[:, hh] @ k[:, g].T) * h.dtype.type(cfg["scale"]), cfg.get("softcap")), -np.inf)
+        top = np.maximum(s.max(axis=1, keepdims=True), w["sink"][hh])
+        e = np.exp(s - top)
+        out[:, hh] = (e / (e.sum(axis=1, keepdims=True) + np.exp(w["sink"][hh] - top))) @ v[:, g]
+    out = out * sigmoid(h @ w["g"].T)[:, :, None]
+    return out.reshape(T, H * D) @ w["o"].T
+
+
+def differential_weight(w, diff):
+    """How much of the second map's output is taken off the first's."""
+    return np.exp((w["lq1"] * w["lk1"]).sum()) - np.exp((w["lq2"] * w["lk2"]).sum()) + w["lq1"].dtype.type(diff)
+
+
+def differential_keys(h, w, cfg, eps, pos):
+    """Keys [T, G, 2, dim] as a cache holds them, and values [T, G, vdim]."""
+    G, D, V, T = cfg["kv_heads"], cfg["dim"], cfg["vdim"], h.shape[0]
+    k = rms_norm((h @ w["k"].T).reshape(T, G, 2, D), w["k.norm"], eps)
+    return rotate_neighbours(k, pos, cfg["rot"]["base"], cfg["rot"]["dims"]), (h @ w["v"].T).reshape(T, G, V)
+
+
+def differential_attention(h, w, cfg, eps, kv=None, positions=None):
+    """Two softmax maps per head over the same values, the second taken off the first, the difference over its root
+    mean square.  `kv`: another layer's keys and values; returns (out [T, width], the keys and values used)."""
+    H, G, D, V = cfg["heads"], cfg["kv_heads"], cfg["dim"], cfg["vdim"]
+    T = h.shape[0]
+    pos = np.arange(T) if positions is None else np.asarray(positions)
+    q = rms_norm((h @ w["q"].T).reshape(T, H, 2, D), w["q.norm"], eps)
+    q = rotate_neighbours(q, pos, cfg["rot"]["base"], cfg["rot"]["dims"])
+    k, v = differential_keys(h, w, cfg, eps, pos) if kv is None else kv
+    seen = in_window(pos, cfg["mask"]["size"])
+    lam, keep = differential_weight(w, cfg["diff"]), h.dtype.type(1.0 - cfg["diff"])
+    out = np.empty((T, H, V), dtype=h.dtype)
+    for hh in range(H):
+        g = hh // (H // G)
+        maps = []
+        for m in range(2):
+            s = np.where(seen, (q[:, hh, m] @ k[:, g, m].T) * h.dtype.type(cfg["scale"]), -np.inf)
+            e = np.exp(s - s.max(axis=1, keepdims=True))
+            maps.append((e / e.sum(axis=1, keepdims=True)) @ v[:, g])
+        out[:, hh] = unit_rms(maps[0] - lam * maps[1], eps) * keep
+    return out.reshape(T, H * V) @ w["o"].T, (k, v)
+
+
+def clamped_expert(h, w, limit):
+    """One feed-forward part of clamped gated units; h is one row or several."""
+    g = np.minimum(h @ w["gate"].T, h.dtype.type(limit))
+    u = np.clip(h @ w["up"].T, -h.dtype.type(limit), h.dtype.type(limit))
+    return (g * sigmoid(h.dtype.type(1.702) * g) * (u + 1)) @ w["down"].T
+
+
+def grouped_choice(z, correction, top, groups):
+    """One token's logits: the chosen outputs (by corrected score, best groups only) and the uncorrected scores of all."""
+    e = np.exp(z - z.max())
+    s = e / e.sum()
+    c = s + correction
+    if groups:
+        by_group = c.reshape(groups["count"], -1)
+        best = np.argsort(-by_group.max(axis=1), kind="stable")[:groups["keep"]]
+        allowed = np.isin(np.arange(len(z)) // by_group.shape[1], best)
+        c = np.where(allowed, c, -np.inf)
+    return np.argsort(-c, kind="stable")[:top], s
+
+
+def grouped_moe(h, w, cfg):
+    """Experts and outputs that pass the input on, chosen inside the best groups; a gated shared expert beside them."""
+    r, n = cfg["router"], cfg["router"]["experts"]
+    out = np.zeros_like(h)
+    for t in range(h.shape[0]):
+        chosen, s = grouped_choice(w["router"] @ h[t], w["correction"], r["top"], r.get("groups"))
+        weight = s[chosen] / (s[chosen].sum() + 1e-20) * h.dtype.type(r["scale"])
+        for g, e in zip(weight, chosen):
+            out[t] += g * (clamped_expert(h[t], _sub(w, f"e{e}."), cfg["expert"]["limit"]) if e < n else h[t])
+    if cfg.get("shared"):
+        out = out + sigmoid(h @ w["shared.sg"].T) * clamped_expert(h, _sub(w, "shared."), cfg["shared"]["limit"])
+    return out
+
+
+def grouped_margin(h, w, cfg):
+    """How little would change a token's choice: the gap between the last group kept and the first left out, and
+    between the last output chosen and the first not, over the scores' spread."""
+    r, out = cfg["router"], np.full(h.shape[0], np.inf)
+    for t in range(h.shape[0]):
+        z = w["router"] @ h[t]
+        chosen, s = grouped_choice(z, w["correction"], r["top"], r.get("groups"))
+        c, g = s + w["correction"], r.get("groups")
+        if g:
+            best = c.reshape(g["count"], -1).max(axis=1)
+            if g["keep"] < g["count"]:
+                order = np.sort(best)[::-1]
+                out[t] = min(out[t], (order[g["keep"] - 1] - order[g["keep"]]) / s.std())
+            kept = np.argsort(-best, kind="stable")[:g["keep"]]
+            c = c[np.isin(np.arange(len(z)) // (len(z) // g["count"]), kept)]
+        c = np.sort(c)[::-1]
+        if r["top"] < len(c):
+            out[t] = min(out[t], (c[r["top"] - 1] - c[r["top"]]) / s.std())
+    return out
+
+
+def shared_kv_layer(x, w, cfg, eps, kvs, margins=None):
+    """A pre-norm layer of differential or keys-as-values attention with an expert feed-forward.  `kvs`: the keys and
+    values of the layers so far, which receives this layer's."""
+    m, h = cfg["mixer"], rms_norm(x, 1 + w["norm1"], eps)
+    if cfg["type"] == "attention_2":
+        j = m.get("kv_from")
+        y, kv = differential_attention(h, _sub(w, "mix."), m, eps, None if j is None else kvs[j])
+    else:
+        y, kv = keys_as_values_attention(h, _sub(w, "mix."), m, eps), None
+    kvs.append(kv)
+    x = x + y
+    if cfg.get("mlp"):
+        h = rms_norm(x, 1 + w["norm2"], eps)
+        if margins is not None:
+            margins.append(grouped_margin(h, _sub(w, "mlp."), cfg["mlp"]))
+        x = x + grouped_moe(h, _sub(w, "mlp."), cfg["mlp"])
+    return x
+
+
 MIXERS = {"lightning": lambda *a: lightning(*a)[0], "latent_attention": latent_attention,
           "wkv": lambda *a: wkv(*a)[0], "parallel": parallel}
 
@@ -247,6 +402,13 @@ def forward(cfg, tensors, tokens, prec=np.float32, capture=None, margins=None):
             if capture is not None:
                 capture.append(x.copy())
         return rms_norm(x, 1 + w["final.norm"], eps) @ w["embed"].T
+    if cfg["architecture"] == "Fedirax":
+        x, kvs = w["embed"][np.asarray(tokens)] * prec(cfg["embedding"]["scale"]), []
+        for i, c in enumerate(cfg["layers"]):
+            x = shared_kv_layer(x, _sub(w, f"l{i}."), c, eps, kvs, margins)
+            if capture is not None:
+                capture.append(x.copy())
+        return rms_norm(x, 1 + w["final.norm"], eps) @ w["head"].T
     x = rms_norm(w["embed"][np.asarray(tokens)], w["embed.norm"], eps)
     x0 = x
     for i, again in layer_order(cfg):

@@ -15,7 +15,8 @@
 
 namespace wr {
 
-constexpr uint32_t kMixOutRowsF32 = 0, kMixOutRows = 1, kMixOutFrag = 2, kMixOutSplit = 3, kMixOutGated = 4;
+constexpr uint32_t kMixOutRowsF32 = 0, kMixOutRows = 1, kMixOutFrag = 2, kMixOutSplit = 3, kMixOutGated = 4,
+                   kMixOutSplitGated = 5;
 
 struct MixGemmArgs {
     const bf16x8* w;
@@ -25,7 +26,9 @@ struct MixGemmArgs {
     uint32_t rows, groups;
     const int32_t* group_expert;
     uint32_t out, ldy, h_kt, col_z, n_split, silu_end, sigmoid_end, tanh_end, relu2, gelu;
-    float scale;
+    float scale, limit, slope, up_bias;
+    const float* bias;
+    const uint32_t* x_perm;
     float* y;
     void* ya;
     void* h;
@@ -52,23 +55,44 @@ __device__ __forceinline__ void mix_put4(void* p, size_t elem, f32x4 v)
     *reinterpret_cast<typename MixAct<F32>::V4*>(reinterpret_cast<typename MixAct<F32>::E*>(p) + elem) = o;
 }
 
+// The gated unit of one gate and one up output.
+template <bool F32>
+__device__ __forceinline__ float mix_gated(const MixGemmArgs& a, float gate, float up)
+{
+    if (a.limit > 0.f) {                                   // (uniform, like gelu)
+        gate = fminf(gate, a.limit);
+        up = fminf(fmaxf(up, -a.limit), a.limit) + a.up_bias;
+        return gate * mix_sigmoid<F32>(a.slope * gate) * up;
+    }
+    // the tanh form of GELU is x * logistic(2 y), y the argument of its tanh
+    const float y = a.gelu ? 1.5957691216057308f * (gate + 0.044715f * gate * gate * gate) : gate;
+    return gate * mix_sigmoid<F32>(y) * up;
+}
+
 // Accumulator tile nt of row group `group`: lane 16g + c holds outputs
-// 16 nt + 4g .. +3 of row 16 group + c.  `up`: the tile's partner (GATED).
+// 16 nt + 4g .. +3 of row 16 group + c.  `up`: the tile's partner (GATED, SPLIT_GATED).
 template <bool F32>
 __device__ __forceinline__ void mix_store_tile(const MixGemmArgs& a, f32x4 v, f32x4 up, uint32_t nt, uint32_t group,
                                                uint32_t z, int lane)
 {
     const uint32_t c = lane & 15, g = lane >> 4, row = group * 16 + c, n = nt * 16 + 4 * g;
     if (row >= a.rows || nt >= a.ntiles) return;
-    if (a.out == kMixOutGated) {
-#pragma unroll
-        for (int i = 0; i < 4; i++) {
-            // the tanh form of GELU is x * logistic(2 y), y the argument of its tanh
-            const float y = a.gelu ? 1.5957691216057308f * (v[i] + 0.044715f * v[i] * v[i] * v[i]) : v[i];
-            v[i] = v[i] * mix_sigmoid<F32>(y) * up[i];
+    if (a.out >= kMixOutGated) {
+        if (a.out == kMixOutSplitGated && nt * 16 < a.n_split) {
+            *reinterpret_cast<f32x4*>(a.y + (size_t)row * a.ldy + n) = v;
+            *reinterpret_cast<f32x4*>(a.y + (size_t)row * a.ldy + n + 16) = up;
+            return;
         }
-        mix_put4<F32>(a.h, frag_elem(row, nt / 2 * 16 + 4 * g, a.h_kt), v);
+#pragma unroll
+        for (int i = 0; i < 4; i++) v[i] = mix_gated<F32>(a, v[i], up[i]);
+        const uint32_t to = nt - (a.out == kMixOutSplitGated ? a.n_split / 16 : 0u);
+        mix_put4<F32>(a.h, frag_elem(row, to / 2 * 16 + 4 * g, a.h_kt), v);
         return;
+    }
+    if (a.bias) {
+        const f32x4 b = *reinterpret_cast<const f32x4*>(a.bias + n);
+#pragma unroll
+        for (int i = 0; i < 4; i++) v[i] += b[i];
     }
     if (n < a.sigmoid_end) {
 #pragma unroll
@@ -127,6 +151,12 @@ __global__ __launch_bounds__(256) void mix_gemm_stream_kernel(const MixGemmArgs 
 #pragma unroll
     for (int i = 0; i < GR; i++)
         xp[i] = reinterpret_cast<const V8*>(a.x) + ((size_t)min(group0 + i, a.groups - 1) * a.x_kt + (size_t)z * a.x_kt_z) * 64 + lane;
+    if constexpr (GR == 1) {
+        if (a.x_perm) {                                    // rows picked one by one: the operand's lanes fetch their own
+            const uint32_t pick = a.x_perm[group0 * 16 + (lane & 15)], row = pick == 0xFFFFFFFFu ? 0 : pick;
+            xp[0] = reinterpret_cast<const V8*>(a.x) + (size_t)(row >> 4) * a.x_kt * 64 + (lane & 48) + (row & 15);
+        }
+    }
 
     f32x4 acc[NT][GR];
 #pragma unroll
@@ -187,7 +217,7 @@ __global__ __launch_bounds__(256) void mix_gemm_stream_kernel(const MixGemmArgs 
                 for (int j = 0; j < 4; j++) acc[t][i][j] += o[j];
             }
     }
-    if (a.out == kMixOutGated) {
+    if (a.out >= kMixOutGated) {
         if constexpr (NT % 2 == 0) {
 #pragma unroll
             for (int t = 0; t < NT; t += 2)
@@ -291,7 +321,7 @@ __global__ __launch_bounds__(256, 2) void mix_gemm_lds_kernel(const MixGemmArgs 
 
     const uint32_t nt0 = nt_wg + wn * NT, group0 = g_wg + wr * GROUPS;
     if (nt0 >= a.ntiles || group0 >= a.groups) return;
-    if (a.out == kMixOutGated) {
+    if (a.out >= kMixOutGated) {
 #pragma unroll
         for (int t = 0; t < NT; t += 2)
 #pragma unroll

@@ -83,6 +83,8 @@ struct MixRowArgs {
     const float* gate;
     const uint32_t* slot;
     uint32_t top;
+    const float *side, *shared;      // weights of the input's own row and of the shared expert's, [rows][2]
+    const void* ident;               // frag rows of the sublayer's input; may be h
     const uint32_t* gather;          // rows to read (the step's wanted rows), or nullptr
     void* h;
     // embedding
@@ -94,6 +96,7 @@ struct MixRowArgs {
 };
 
 // the sublayer output's chunk q of row r: plain, or the experts' rows weighted
+template <bool F32>
 __device__ __forceinline__ void mix_sub_chunk(const MixRowArgs& a, uint32_t r, uint32_t q, float (&v)[8])
 {
     if (!a.top) {
@@ -104,8 +107,24 @@ __device__ __forceinline__ void mix_sub_chunk(const MixRowArgs& a, uint32_t r, u
     for (int j = 0; j < 8; j++) v[j] = 0.f;
     for (uint32_t t = 0; t < a.top; t++) {
         const float gt = a.gate[(size_t)r * a.top + t];
+        const uint32_t slot = a.slot[(size_t)r * a.top + t];
+        if (slot == 0xFFFFFFFFu) continue;
         float e[8];
-        mix_load8(a.y + (size_t)a.slot[(size_t)r * a.top + t] * a.wpad + q * 8, e);
+        mix_load8(a.y + (size_t)slot * a.wpad + q * 8, e);
+#pragma unroll
+        for (int j = 0; j < 8; j++) v[j] = fmaf(gt, e[j], v[j]);
+    }
+    if (!a.side) return;
+    float e[8];
+    if (a.ident) {                                         // (read by the thread that writes this unit of h later)
+        const float own = a.side[(size_t)r * 2];
+        mix_load8(reinterpret_cast<const typename MixAct<F32>::E*>(a.ident) + frag_unit(r, q, a.wpad / 32) * 8, e);
+#pragma unroll
+        for (int j = 0; j < 8; j++) v[j] = fmaf(own, e[j], v[j]);
+    }
+    if (a.shared) {
+        const float gt = a.side[(size_t)r * 2 + 1];
+        mix_load8(a.shared + (size_t)r * a.wpad + q * 8, e);
 #pragma unroll
         for (int j = 0; j < 8; j++) v[j] = fmaf(gt, e[j], v[j]);
     }
@@ -149,7 +168,7 @@ __global__ __launch_bounds__(MixRowShape<RPW>::kThreads) void mix_residual_kerne
                 v[j] = k < a.width ? __uint_as_float((uint32_t)e[k] << 16) : 0.f;
             }
         } else {
-            mix_sub_chunk(a, r, q, v);
+            mix_sub_chunk<F32>(a, r, q, v);
         }
     };
     const bool some = EMBED || a.y != nullptr;            // uniform: there is a value
@@ -450,15 +469,25 @@ __global__ __launch_bounds__(MixRowShape<RPW>::kThreads) void mix_gate_norm_kern
 
 struct MixRouteArgs {
     const float* z;
-    uint32_t ldz, rows, experts, top, tile_groups, n_groups;
-    float* gate;
-    uint32_t* slot;                  // first the chosen expert, then the slot
+    uint32_t ldz, rows, outputs, experts, top, tile_groups, n_groups;     // outputs: experts, then those that pass the input on
+    uint32_t kinds, keep, softmax_all, shared_gate;                       // kinds: groups of neighbouring outputs, or 0
+    float scale;
+    const float* correction;
+    float *gate, *side;
+    uint32_t* slot;                  // first the chosen output, then the slot
     uint32_t* perm;
     int32_t* group_expert;
 };
 
-// One wave: the `top` largest logits of a row (lowest index among equals) and
-// the softmax over them.  Lane l holds logits l, l + 64, ...
+__device__ __forceinline__ float mix_wave_max(float v)
+{
+#pragma unroll
+    for (int off = 32; off >= 1; off >>= 1) v = fmaxf(v, wave_xor_f32(v, off));
+    return v;
+}
+
+// One wave: the `top` outputs of a row with the largest choice value (lowest index among equals) and their weights.
+// Lane l holds outputs l, l + 64, ...
 __device__ __forceinline__ void mix_top(const MixRouteArgs& a, uint32_t row, int lane)
 {
     constexpr int PER = (int)(1024 / 64);
@@ -467,17 +496,63 @@ __device__ __forceinline__ void mix_top(const MixRouteArgs& a, uint32_t row, int
 #pragma unroll
     for (int i = 0; i < PER; i++) {
         const uint32_t e = lane + 64 * i;
-        v[i] = e < a.experts ? z[e] : -INFINITY;
+        v[i] = e < a.outputs ? z[e] : -INFINITY;
     }
-    uint32_t taken = 0;                                    // bit i: this lane's logit i is chosen
-    float best0 = 0.f, sum = 0.f, mine = 0.f;
+    float zmax = 0.f, zinv = 1.f;
+    if (a.softmax_all) {                                   // choice: the softmax over all outputs, corrected
+        zmax = v[0];
+#pragma unroll
+        for (int i = 1; i < PER; i++) zmax = fmaxf(zmax, v[i]);
+        zmax = mix_wave_max(zmax);
+        float zs = 0.f;
+#pragma unroll
+        for (int i = 0; i < PER; i++) {
+            v[i] = expf(v[i] - zmax);                      // (zero past the outputs)
+            zs += v[i];
+        }
+#pragma unroll
+        for (int off = 32; off >= 1; off >>= 1) zs += wave_xor_f32(zs, off);
+        zinv = 1.0f / zs;
+#pragma unroll
+        for (int i = 0; i < PER; i++) {
+            const uint32_t e = lane + 64 * i;
+            if (e < a.outputs) v[i] = v[i] * zinv + (a.correction ? a.correction[e] : 0.f);
+        }
+    }
+    if (a.kinds) {                                         // lane g holds the largest choice value of group g
+        const uint32_t size = a.outputs / a.kinds;
+        float mine = -INFINITY;
+        for (uint32_t k = 0; k < a.kinds; k++) {
+            float best = -INFINITY;
+#pragma unroll
+            for (int i = 0; i < PER; i++) {
+                const uint32_t e = lane + 64 * i;
+                if (e >= k * size && e < (k + 1) * size) best = fmaxf(best, v[i]);
+            }
+            best = mix_wave_max(best);
+            if ((uint32_t)lane == k) mine = best;
+        }
+        uint32_t ahead = 0;                                // groups that are better than this lane's
+        for (uint32_t k = 0; k < a.kinds; k++) {
+            const float other = __shfl(mine, (int)k, 64);
+            ahead += other > mine || (other == mine && k < (uint32_t)lane);
+        }
+        const uint64_t kept = __ballot((uint32_t)lane < a.kinds && ahead < a.keep);
+#pragma unroll
+        for (int i = 0; i < PER; i++) {
+            const uint32_t e = lane + 64 * i;
+            if (e < a.outputs && !((kept >> (e / size)) & 1u)) v[i] = -INFINITY;
+        }
+    }
+    uint32_t taken = 0;                                    // bit i: this lane's output i is chosen
+    float best0 = 0.f, sum = 0.f, mine = 0.f, own = 0.f;
     for (uint32_t t = 0; t < a.top; t++) {
         float bv = -INFINITY;
         uint32_t be = 0xFFFFFFFFu;
 #pragma unroll
         for (int i = 0; i < PER; i++) {
             const uint32_t e = lane + 64 * i;
-            if (e < a.experts && !((taken >> i) & 1u) && (be == 0xFFFFFFFFu || v[i] > bv)) {
+            if (e < a.outputs && !((taken >> i) & 1u) && (be == 0xFFFFFFFFu || v[i] > bv)) {
                 bv = v[i];
                 be = e;
             }
@@ -491,17 +566,23 @@ __device__ __forceinline__ void mix_top(const MixRouteArgs& a, uint32_t row, int
                 be = oe;
             }
         }
-        be = min(be, a.experts - 1);                       // NaN logits: still an expert
+        be = min(be, a.outputs - 1);                       // NaN logits: still an output
         if ((be & 63u) == (uint32_t)lane) taken |= 1u << (be >> 6);
         if (t == 0) best0 = bv;
-        const float g = expf(bv - best0);
+        const float g = a.softmax_all ? expf(z[be] - zmax) * zinv : expf(bv - best0);
         sum += g;
+        if (be >= a.experts) own += g;
         if ((uint32_t)lane == t) {
             mine = g;
             a.slot[(size_t)row * a.top + t] = be;
         }
     }
-    if ((uint32_t)lane < a.top) a.gate[(size_t)row * a.top + lane] = mine / sum;
+    const float over = a.softmax_all ? a.scale / (sum + 1e-20f) : 1.0f;
+    if ((uint32_t)lane < a.top) a.gate[(size_t)row * a.top + lane] = a.softmax_all ? mine * over : mine / sum;
+    if (a.side && lane == 0) {
+        a.side[(size_t)row * 2] = a.softmax_all ? own * over : own / sum;
+        a.side[(size_t)row * 2 + 1] = a.shared_gate ? 1.0f / (1.0f + expf(-z[a.outputs])) : 0.f;
+    }
 }
 
 __global__ __launch_bounds__(256) void mix_top_kernel(const MixRouteArgs a)
@@ -526,7 +607,8 @@ __global__ __launch_bounds__(1024) void mix_order_kernel(const MixRouteArgs a)
     for (uint32_t i = t; i < n_slots; i += 1024) a.perm[i] = 0xFFFFFFFFu;
     for (uint32_t i = t; i < a.n_groups; i += 1024) a.group_expert[i] = -1;
     __syncthreads();
-    for (uint32_t i = t; i < pairs; i += 1024) atomicAdd(&count[a.slot[i]], 1u);
+    for (uint32_t i = t; i < pairs; i += 1024)
+        if (a.slot[i] < a.experts) atomicAdd(&count[a.slot[i]], 1u);
     __syncthreads();
     const uint32_t mine = (count[t] + run - 1) / run * run;
     scan[t] = mine;
@@ -542,7 +624,12 @@ __global__ __launch_bounds__(1024) void mix_order_kernel(const MixRouteArgs a)
     count[t] = 0;
     __syncthreads();
     for (uint32_t i = t; i < pairs; i += 1024) {
-        const uint32_t e = a.slot[i], s = base[e] + atomicAdd(&count[e], 1u);
+        const uint32_t e = a.slot[i];
+        if (e >= a.experts) {                              // the input itself: nothing to compute
+            a.slot[i] = 0xFFFFFFFFu;
+            continue;
+        }
+        const uint32_t s = base[e] + atomicAdd(&count[e], 1u);
         a.slot[i] = s;
         a.perm[s] = i / a.top;
     }

@@ -1,10 +1,17 @@
 // Sliding-window attention over grouped keys and values.  Optionally each head has a sink
 // s: its weights are exp(score) / (exp(s) + sum of exp(score)), so a row may attend to
-// nothing at all.
+// nothing at all.  Scores may be capped (cap * tanh(score / cap)) and a head's output gated.
+//
+// With two maps every head weighs the same values twice, by two queries over two keys, and
+// its output is the first sum less `diff` times the second, over its root mean square.
+// Prefill gives a wave the two maps of sixteen rows where it has 32 rows otherwise, so each
+// value operand feeds both and the difference is taken in registers.  Decode takes both maps
+// as columns of one product over keys twice as long, a column's query being zero where the
+// other map's keys lie: one running softmax and one product with the values serve both.
 //
 // A page (64 positions) holds each key/value head's block one after the other:
 //
-//   K  [64/16][dim_pad/32][64][8]     lane 16g + c of a tile: position 16s + c, elements 32k + 8g .. +8
+//   K  [64/16][maps * dim_pad/32][64][8]  lane 16g + c of a tile: position 16s + c, elements 32k + 8g .. +8
 //   V  [64/32][vdim_pad/16][64][8]    lane 16g + c of a tile: column 16t + c, element e of its eight:
 //                                     position 32b + 16 (e / 4) + 4g + e % 4
 //
@@ -12,8 +19,8 @@
 // positions 4g .. 4g+3 of two 16-position halves for row c, which is the B operand of
 // O^T = V^T P^T in the order V is stored.
 //
-//   window_append_kernel    queries rotated into an operand, keys rotated and values normed into the cache
-//   window_prefill_kernel   128 (token, head) rows of one key/value head a workgroup, a page at a time
+//   window_append_kernel    queries normed and rotated into an operand, keys the same way and values into the cache
+//   window_prefill_kernel   128 (token, head, map) rows of one key/value head a workgroup, a page at a time
 //                           through LDS
 //   window_decode_kernel    a workgroup per (token, key/value head, share of the keys)
 //   window_attend_any_kernel  any geometry, both activation types
@@ -28,7 +35,10 @@ struct WindowArgs {
     const uint32_t *row_seq, *row_pos, *pages;
     uint32_t rows, heads, kvh, group;            // group = heads / kvh
     uint32_t dim, dimp, vdim, vdimp, half, window, norm_values;
-    float scale, out_scale, eps;
+    uint32_t maps, dimk, neighbours, key_heads;  // dimk = maps * dimp; key_heads: key/value heads to append (0 or kvh)
+    float scale, out_scale, eps, softcap, diff;
+    const float *q_norm, *k_norm, *gate;
+    uint32_t ldg;
     void* cache;
     const float* in;
     uint32_t ld, col_q, col_k, col_v;
@@ -51,44 +61,102 @@ __device__ __forceinline__ uint32_t window_v_elem(uint32_t at, uint32_t d, uint3
 
 constexpr uint32_t kWindowQUnits = 512;          // query units of eight a workgroup rotates
 
-// grid (rows / 4, kvh + slices of 4 rows' query units)
+// Eight elements i0 .. i0 + 7 of the vector x, times inv and the norm's weights where there are any, rotated.
+__device__ __forceinline__ void window_turn8(const WindowArgs& a, const float* x, const float* norm, float inv, const float* tab,
+                                             uint32_t i0, float (&v)[8])
+{
+    if (!norm && !a.neighbours) {
+        latent_rotate8(x, tab, i0, a.dim, a.half, v);
+        return;
+    }
+    auto at = [&](uint32_t i) { return i < a.dim ? (norm ? x[i] * inv * norm[i] : x[i]) : 0.f; };
+#pragma unroll
+    for (uint32_t j = 0; j < 8; j += 2) {
+        const uint32_t i = i0 + j;
+        const float e = at(i), o = at(i + 1);
+        if (a.neighbours) {
+            const bool turn = i < 2 * a.half;
+            const float c = turn ? tab[i] : 1.0f, sn = turn ? tab[i + 1] : 0.f;
+            v[j] = e * c - o * sn;
+            v[j + 1] = o * c + e * sn;
+        } else {
+#pragma unroll
+            for (uint32_t k = 0; k < 2; k++) {
+                const uint32_t d = i + k;
+                const float own = k ? o : e;
+                if (d < a.half) v[j + k] = own * tab[2 * d] - at(d + a.half) * tab[2 * d + 1];
+                else if (d < 2 * a.half) v[j + k] = own * tab[2 * (d - a.half)] + at(d - a.half) * tab[2 * (d - a.half) + 1];
+                else v[j + k] = own;
+            }
+        }
+    }
+}
+
+// One over the root mean square of the vector x, whose units of eight (this thread's: i0 ..) are held by every fourth
+// lane of a run of lanes.
+__device__ __forceinline__ float window_inv_rms(const WindowArgs& a, const float* x, uint32_t i0)
+{
+    float ss = 0.f;
+    if (a.dimp == 32 || a.dimp == 64 || a.dimp == 128) {
+#pragma unroll
+        for (uint32_t j = 0; j < 8; j++) {
+            const float e = i0 + j < a.dim ? x[i0 + j] : 0.f;
+            ss = fmaf(e, e, ss);
+        }
+        ss += wave_xor_f32(ss, 4);
+        ss += wave_xor_f32(ss, 8);
+        if (a.dimp >= 64) ss += wave_xor_f32(ss, 16);
+        if (a.dimp >= 128) ss += wave_xor_f32(ss, 32);
+    } else {
+        for (uint32_t i = 0; i < a.dim; i++) ss = fmaf(x[i], x[i], ss);
+    }
+    return 1.0f / sqrtf(ss / (float)a.dim + a.eps);
+}
+
+// grid (rows / 4, key_heads + slices of 4 rows' query units)
 template <bool F32>
 __global__ __launch_bounds__(256) void window_append_kernel(const WindowArgs a)
 {
     using E = typename MixAct<F32>::E;
     using V4 = typename MixAct<F32>::V4;
     __shared__ float s_inv[4];
-    const uint32_t t = threadIdx.x, r0 = blockIdx.x * 4, n = min(4u, a.rows - r0);
-    if (blockIdx.y >= a.kvh) {
-        const uint32_t per = a.heads * (a.dimp / 8), u0 = (blockIdx.y - a.kvh) * kWindowQUnits;
+    const uint32_t t = threadIdx.x, r0 = blockIdx.x * 4, n = min(4u, a.rows - r0), per_map = a.dimp / 8;
+    if (blockIdx.y >= a.key_heads) {
+        const uint32_t per = a.heads * a.maps * per_map, u0 = (blockIdx.y - a.key_heads) * kWindowQUnits;
         for (uint32_t u = u0 + t; u < min(u0 + kWindowQUnits, 4 * per); u += 256) {
-            const uint32_t i = u % 4, q = u / 4, h = q / (a.dimp / 8), r = r0 + i;
+            const uint32_t i = u % 4, q = u / 4, r = r0 + min(i, n - 1);
+            const float* x = a.in + (size_t)r * a.ld + a.col_q + q / per_map * a.dim;
+            const float inv = a.q_norm ? window_inv_rms(a, x, q % per_map * 8) : 1.0f;
             if (i >= n) continue;
             float v[8];
-            latent_rotate8(a.in + (size_t)r * a.ld + a.col_q + h * a.dim, a.table + (size_t)r * 2 * a.half, q % (a.dimp / 8) * 8,
-                           a.dim, a.half, v);
-            mix_store_unit<F32>(a.q, frag_unit(r, q, a.heads * (a.dimp / 32)), v);
+            window_turn8(a, x, a.q_norm, inv, a.table + (size_t)r * 2 * a.half, q % per_map * 8, v);
+            mix_store_unit<F32>(a.q, frag_unit(r, q, a.heads * (a.dimk / 32)), v);
         }
         return;
     }
-    const uint32_t kvh = blockIdx.y, block = kMixPage * (a.dimp + a.vdimp);
+    const uint32_t kvh = blockIdx.y, block = kMixPage * (a.dimk + a.vdimp);
     auto head_block = [&](uint32_t r) {
         const MixSeq s = a.seqs[a.row_seq[r]];
         return reinterpret_cast<E*>(a.cache) + ((size_t)a.pages[s.page0 + a.row_pos[r] / kMixPage] * a.kvh + kvh) * block;
     };
-    for (uint32_t u = t; u < n * (a.dimp / 8); u += 256) {
-        const uint32_t i = u % n, q = u / n, r = r0 + i;
+    for (uint32_t u = t; u < 4 * a.maps * per_map; u += 256) {
+        const uint32_t i = u % 4, q = u / 4, r = r0 + min(i, n - 1);
+        const float* x = a.in + (size_t)r * a.ld + a.col_k + (kvh * a.maps + q / per_map) * a.dim;
+        const float inv = a.k_norm ? window_inv_rms(a, x, q % per_map * 8) : 1.0f;
+        if (i >= n) continue;
         float v[8];
-        latent_rotate8(a.in + (size_t)r * a.ld + a.col_k + kvh * a.dim, a.table + (size_t)r * 2 * a.half, q * 8, a.dim, a.half, v);
-        mix_store_unit<F32>(head_block(r), frag_unit(a.row_pos[r] % kMixPage, q, a.dimp / 32), v);
+        window_turn8(a, x, a.k_norm, inv, a.table + (size_t)r * 2 * a.half, q % per_map * 8, v);
+        mix_store_unit<F32>(head_block(r), frag_unit(a.row_pos[r] % kMixPage, q, a.dimk / 32), v);
     }
     const uint32_t wave = t >> 6, lane = t & 63;
     if (wave < n) {
-        const float* v = a.in + (size_t)(r0 + wave) * a.ld + a.col_v + kvh * a.vdim;
         float ss = 0.f;
-        for (uint32_t d = lane; d < a.vdim; d += 64) ss = fmaf(v[d], v[d], ss);
+        if (a.norm_values) {
+            const float* v = a.in + (size_t)(r0 + wave) * a.ld + a.col_v + kvh * a.vdim;
+            for (uint32_t d = lane; d < a.vdim; d += 64) ss = fmaf(v[d], v[d], ss);
 #pragma unroll
-        for (int off = 32; off >= 1; off >>= 1) ss += wave_xor_f32(ss, off);
+            for (int off = 32; off >= 1; off >>= 1) ss += wave_xor_f32(ss, off);
+        }
         if (lane == 0) s_inv[wave] = a.norm_values ? 1.0f / sqrtf(ss / (float)a.vdim + a.eps) : 1.0f;
     }
     __syncthreads();
@@ -100,92 +168,134 @@ __global__ __launch_bounds__(256) void window_append_kernel(const WindowArgs a)
         for (uint32_t i = 0; i < 4; i++)
             x[i] = (E)(i < n && d < a.vdim ? a.in[(size_t)(r0 + min(i, n - 1)) * a.ld + a.col_v + kvh * a.vdim + d] * s_inv[i] : 0.f);
         if (run) {                                         // four positions of one column side by side
-            *reinterpret_cast<V4*>(head_block(r0) + kMixPage * a.dimp + window_v_elem(p0 % kMixPage, d, a.vdimp)) = x;
+            *reinterpret_cast<V4*>(head_block(r0) + kMixPage * a.dimk + window_v_elem(p0 % kMixPage, d, a.vdimp)) = x;
         } else {
             for (uint32_t i = 0; i < n; i++)
-                head_block(r0 + i)[kMixPage * a.dimp + window_v_elem(a.row_pos[r0 + i] % kMixPage, d, a.vdimp)] = x[i];
+                head_block(r0 + i)[kMixPage * a.dimk + window_v_elem(a.row_pos[r0 + i] % kMixPage, d, a.vdimp)] = x[i];
         }
     }
 }
 
-// One wave per (row, head), a lane per key of a page.  LDS: the query row and the output row as floats, 64 weights.
+// What head h's output of row r is multiplied by, besides what its own sum calls for.
+template <bool F32>
+__device__ __forceinline__ float window_factor(const WindowArgs& a, uint32_t r, uint32_t h)
+{
+    return a.gate ? a.out_scale * mix_sigmoid<F32>(a.gate[(size_t)r * a.ldg + h]) : a.out_scale;
+}
+
+// One wave per (row, head), a lane per key of a page.  LDS: a query row and every map's output row as floats, 64 weights.
 template <bool F32>
 __global__ __launch_bounds__(64) void window_attend_any_kernel(const WindowArgs a)
 {
     using E = typename MixAct<F32>::E;
     using V8 = typename MixAct<F32>::V8;
     extern __shared__ __attribute__((aligned(16))) float window_smem[];
-    const uint32_t lane = threadIdx.x, r = blockIdx.x, h = blockIdx.y, kd = a.dimp / 32;
-    float *q = window_smem, *o = q + a.dimp, *w = o + a.vdimp;
+    const uint32_t lane = threadIdx.x, r = blockIdx.x, h = blockIdx.y, kd = a.dimk / 32, per_map = a.dimp / 8;
+    float *q = window_smem, *w = q + a.dimp, *outs = w + 64;
     const V8* qf = reinterpret_cast<const V8*>(a.q);
-    for (uint32_t u = lane; u < a.dimp / 8; u += 64) {
-        const V8 x = qf[frag_unit(r, h * kd * 4 + u, a.heads * kd)];
-#pragma unroll
-        for (int j = 0; j < 8; j++) q[u * 8 + j] = (float)x[j];
-    }
-    for (uint32_t k = lane; k < a.vdimp; k += 64) o[k] = 0.f;
-    __syncthreads();
     const MixSeq s = a.seqs[a.row_seq[r]];
     const uint32_t pos = a.row_pos[r], lo = pos + 1 > a.window ? pos + 1 - a.window : 0;
-    float mx = a.sink ? a.sink[h] : -INFINITY, sum = a.sink ? 1.0f : 0.f;
-    for (uint32_t j0 = lo / kMixPage * kMixPage; j0 <= pos; j0 += kMixPage) {
-        const uint32_t j = j0 + lane;
-        const V8* page = reinterpret_cast<const V8*>(
-            reinterpret_cast<const E*>(a.cache) +
-            ((size_t)a.pages[s.page0 + j0 / kMixPage] * a.kvh + h / a.group) * kMixPage * (a.dimp + a.vdimp));
-        float sc = 0.f;
-        for (uint32_t u = 0; u < a.dimp / 8; u++) {
-            const V8 x = page[frag_unit(lane, u, kd)];
+    for (uint32_t m = 0; m < a.maps; m++) {
+        float* o = outs + m * a.vdimp;
+        for (uint32_t u = lane; u < per_map; u += 64) {
+            const V8 x = qf[frag_unit(r, h * kd * 4 + m * per_map + u, a.heads * kd)];
 #pragma unroll
-            for (int e = 0; e < 8; e++) sc = fmaf((float)x[e], q[u * 8 + e], sc);
+            for (int j = 0; j < 8; j++) q[u * 8 + j] = (float)x[j];
         }
-        sc = (j >= lo && j <= pos) ? sc * a.scale : -INFINITY;
-        float bm = sc;
-#pragma unroll
-        for (int off = 32; off >= 1; off >>= 1) bm = fmaxf(bm, wave_xor_f32(bm, off));
-        const float nm = fmaxf(mx, bm), p = expf(sc - nm), corr = expf(mx - nm);
-        float bs = p;
-#pragma unroll
-        for (int off = 32; off >= 1; off >>= 1) bs += wave_xor_f32(bs, off);
-        sum = sum * corr + bs;
-        mx = nm;
-        w[lane] = p;
+        for (uint32_t k = lane; k < a.vdimp; k += 64) o[k] = 0.f;
         __syncthreads();
-        const V8* vb = page + kMixPage * a.dimp / 8;
-        for (uint32_t k = lane; k < a.vdimp; k += 64) {
-            float acc = o[k] * corr;
-            for (uint32_t u = 0; u < 8; u++) {             // 32-position block u / 4, lane group u % 4
-                const V8 x = vb[(u / 4 * (a.vdimp / 16) + k / 16) * 64 + 16 * (u % 4) + k % 16];
+        float mx = a.sink ? a.sink[h] : -INFINITY, sum = a.sink ? 1.0f : 0.f;
+        for (uint32_t j0 = lo / kMixPage * kMixPage; j0 <= pos; j0 += kMixPage) {
+            const uint32_t j = j0 + lane;
+            const V8* page = reinterpret_cast<const V8*>(
+                reinterpret_cast<const E*>(a.cache) +
+                ((size_t)a.pages[s.page0 + j0 / kMixPage] * a.kvh + h / a.group) * kMixPage * (a.dimk + a.vdimp));
+            float sc = 0.f;
+            for (uint32_t u = 0; u < per_map; u++) {
+                const V8 x = page[frag_unit(lane, m * per_map + u, kd)];
 #pragma unroll
-                for (int e = 0; e < 8; e++) {
-                    // (positions past the row's own may hold anything: their weight is zero, their value is not used)
-                    const float p8 = w[32 * (u / 4) + 16 * (e / 4) + 4 * (u % 4) + e % 4];
-                    acc = fmaf(p8, p8 != 0.f ? (float)x[e] : 0.f, acc);
-                }
+                for (int e = 0; e < 8; e++) sc = fmaf((float)x[e], q[u * 8 + e], sc);
             }
-            o[k] = acc;
+            sc *= a.scale;
+            if (a.softcap > 0.f) sc = a.softcap * tanhf(sc / a.softcap);
+            sc = (j >= lo && j <= pos) ? sc : -INFINITY;
+            float bm = sc;
+#pragma unroll
+            for (int off = 32; off >= 1; off >>= 1) bm = fmaxf(bm, wave_xor_f32(bm, off));
+            const float nm = fmaxf(mx, bm), p = expf(sc - nm), corr = expf(mx - nm);
+            float bs = p;
+#pragma unroll
+            for (int off = 32; off >= 1; off >>= 1) bs += wave_xor_f32(bs, off);
+            sum = sum * corr + bs;
+            mx = nm;
+            w[lane] = p;
+            __syncthreads();
+            const V8* vb = page + kMixPage * a.dimk / 8;
+            for (uint32_t k = lane; k < a.vdimp; k += 64) {
+                float acc = o[k] * corr;
+                for (uint32_t u = 0; u < 8; u++) {         // 32-position block u / 4, lane group u % 4
+                    const V8 x = vb[(u / 4 * (a.vdimp / 16) + k / 16) * 64 + 16 * (u % 4) + k % 16];
+#pragma unroll
+                    for (int e = 0; e < 8; e++) {
+                        // (positions past the row's own may hold anything: their weight is zero, their value is not used)
+                        const float p8 = w[32 * (u / 4) + 16 * (e / 4) + 4 * (u % 4) + e % 4];
+                        acc = fmaf(p8, p8 != 0.f ? (float)x[e] : 0.f, acc);
+                    }
+                }
+                o[k] = acc;
+            }
+            __syncthreads();
         }
-        __syncthreads();
+        for (uint32_t k = lane; k < a.vdimp; k += 64) o[k] /= sum;     // (this lane's own columns, here and below)
     }
-    const float inv = a.out_scale / sum;
+    float factor = window_factor<F32>(a, r, h);
+    if (a.maps == 2) {
+        float ss = 0.f;
+        for (uint32_t k = lane; k < a.vdimp; k += 64) {
+            outs[k] -= a.diff * outs[a.vdimp + k];
+            ss = fmaf(outs[k], outs[k], ss);
+        }
+#pragma unroll
+        for (int off = 32; off >= 1; off >>= 1) ss += wave_xor_f32(ss, off);
+        factor /= sqrtf(ss / (float)a.vdim + a.eps);
+    }
     E* out = reinterpret_cast<E*>(a.o);
-    for (uint32_t k = lane; k < a.vdimp; k += 64) out[frag_elem(r, h * a.vdimp + k, a.o_kt)] = (E)(o[k] * inv);
+    for (uint32_t k = lane; k < a.vdimp; k += 64) out[frag_elem(r, h * a.vdimp + k, a.o_kt)] = (E)(outs[k] * factor);
 }
 
 // ---- matrix forms (bfloat16; head sizes padded to 32, 64 or 128) -------------
 
-// The running softmax of one row tile over N x 16 keys from j0 on; s[n][i]: score of key j0 + 16n + 4g + i.
+// Products to scores in units of log2 e: times mul, and with cap > 0 (its own log2 e in it) capped; a capped score's mul
+// is 2 log2 e times scale over cap.
+struct WindowScore {
+    float mul, cap;
+    __device__ __forceinline__ explicit WindowScore(const WindowArgs& a)
+        : mul(a.softcap > 0.f ? a.scale / a.softcap * 2.0f * kLog2e : a.scale * kLog2e), cap(a.softcap * kLog2e) {}
+};
+
+// The running softmax of one row tile over N x 16 keys from j0 on; s[n][i]: product with key j0 + 16n + 4g + i.
 // Leaves the probabilities in s and returns by how much the old sums shrink.
 template <int N, bool MASK>
-__device__ __forceinline__ float window_softmax(f32x4 (&s)[N], uint32_t j0, int g, uint32_t lo, uint32_t pos, float scale,
+__device__ __forceinline__ float window_softmax(f32x4 (&s)[N], uint32_t j0, int g, uint32_t lo, uint32_t pos, WindowScore score,
                                                 float& mx, float& sum)
 {
     float bm = kLatentNone;
+    if (score.cap > 0.f) {                                 // uniform; tanh(x) = 1 - 2 / (exp(2x) + 1)
+#pragma unroll
+        for (int n = 0; n < N; n++)
+#pragma unroll
+            for (int i = 0; i < 4; i++)
+                s[n][i] = score.cap - 2.0f * score.cap * __builtin_amdgcn_rcpf(fast_exp2(s[n][i] * score.mul) + 1.0f);
+    } else {
+#pragma unroll
+        for (int n = 0; n < N; n++)
+#pragma unroll
+            for (int i = 0; i < 4; i++) s[n][i] *= score.mul;
+    }
 #pragma unroll
     for (int n = 0; n < N; n++)
 #pragma unroll
         for (int i = 0; i < 4; i++) {
-            s[n][i] *= scale;
             if constexpr (MASK) {
                 const uint32_t j = j0 + 16 * n + 4 * g + i;
                 if (j < lo || j > pos) s[n][i] = kLatentNone;
@@ -226,47 +336,68 @@ __device__ __forceinline__ bf16x8 window_pack(f32x4 a, f32x4 b)
 
 constexpr size_t window_prefill_lds(int kq, int vt) { return (size_t)2 * 4 * (kq + vt) * 1024; }
 
-// KQ, VT: head sizes in tiles of 32.  Grid: tiles of 128 (token, head of the group) rows times key/value heads, the
-// key/value head innermost: with eight of them each XCD keeps to one.
-template <int KQ, int VT>
+// The difference of two maps' outputs of one row, each over its own sum: over its root mean square times factor.
+// a, b: this lane's columns; the row's others are held by the lanes 16 and 32 away.
+template <int N>
+__device__ __forceinline__ float window_difference(const WindowArgs& a, f32x4 (&x)[N], const f32x4 (&y)[N], float ix, float iy)
+{
+    float ss = 0.f;
+    iy *= a.diff;
+#pragma unroll
+    for (int k = 0; k < N; k++)
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            x[k][i] = x[k][i] * ix - y[k][i] * iy;
+            ss = fmaf(x[k][i], x[k][i], ss);
+        }
+    ss += wave_xor_f32(ss, 16);
+    ss += wave_xor_f32(ss, 32);
+    return 1.0f / sqrtf(ss / (float)a.vdim + a.eps);
+}
+
+// KQ, VT: head sizes in tiles of 32.  Grid: tiles of 128 (token, head of the group, map) rows times key/value heads, the
+// key/value head innermost: with eight of them each XCD keeps to one.  A wave's two row tiles are 32 rows, or the two
+// maps of 16.
+template <int KQ, int VT, int MAPS>
 __global__ __launch_bounds__(256, 2) void window_prefill_kernel(const WindowArgs a)
 {
-    constexpr int NR = 2, STAGE = 4 * (KQ + VT) * 1024, CPW = KQ + VT;
+    constexpr int NR = 2, CPW = MAPS * KQ + VT, STAGE = 4 * CPW * 1024, WROWS = 32 / MAPS, ROWS = 4 * WROWS;
     extern __shared__ __attribute__((aligned(16))) unsigned char window_lds[];
     const int lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4;
     const uint32_t wave = (uint32_t)__builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const uint32_t kvh = blockIdx.x % a.kvh, H = a.group;
     uint32_t tile = blockIdx.x / a.kvh, pick_seq = 0, n_tiles = 0;
     for (uint32_t i = 0; i < a.n_list; i++) {
-        n_tiles = (a.seqs[a.list[i]].rows * H + 127) / 128;
+        n_tiles = (a.seqs[a.list[i]].rows * H + ROWS - 1) / ROWS;
         pick_seq = a.list[i];
         if (tile < n_tiles) break;
         tile -= n_tiles;
     }
     tile = n_tiles - 1 - tile;                             // the last tiles see the most keys and go first
     const MixSeq s = a.seqs[pick_seq];
-    const uint32_t m_end = s.rows * H, m0 = tile * 128;
-    const uint32_t pos_first = s.pos0 + m0 / H, pos_last = s.pos0 + (min(m0 + 128, m_end) - 1) / H;
+    const uint32_t m_end = s.rows * H, m0 = tile * ROWS;
+    const uint32_t pos_first = s.pos0 + m0 / H, pos_last = s.pos0 + (min(m0 + ROWS, m_end) - 1) / H;
     const uint32_t j_begin = (pos_first + 1 > a.window ? pos_first + 1 - a.window : 0) / kMixPage * kMixPage, j_end = pos_last + 1;
-    const float scale = a.scale * kLog2e;
+    const WindowScore score(a);
 
     uint32_t m[NR], pos[NR], lo[NR];
     bf16x8 qv[NR][KQ];
     float mx[NR], sum[NR];
 #pragma unroll
     for (int t = 0; t < NR; t++) {
-        m[t] = m0 + (wave * NR + t) * 16 + c;
+        m[t] = m0 + wave * WROWS + (MAPS == 1 ? t * 16 : 0) + c;
         const uint32_t mm = min(m[t], m_end - 1), head = kvh * H + mm % H;
         pos[t] = s.pos0 + mm / H;
         lo[t] = pos[t] + 1 > a.window ? pos[t] + 1 - a.window : 0;
 #pragma unroll
         for (int k = 0; k < KQ; k++)
-            qv[t][k] = reinterpret_cast<const bf16x8*>(a.q)[frag_unit(s.row0 + mm / H, (head * KQ + k) * 4 + g, a.heads * KQ)];
+            qv[t][k] = reinterpret_cast<const bf16x8*>(a.q)[frag_unit(
+                s.row0 + mm / H, ((MAPS == 1 ? head : head * MAPS + t) * KQ + k) * 4 + g, a.heads * MAPS * KQ)];
         mx[t] = a.sink ? a.sink[head] * kLog2e : kLatentNone;
         sum[t] = a.sink ? 1.0f : 0.f;
     }
     // positions this wave's rows span: a page between them needs no mask
-    const uint32_t w0 = min(m0 + wave * NR * 16, m_end - 1), w1 = min(m0 + wave * NR * 16 + NR * 16 - 1, m_end - 1);
+    const uint32_t w0 = min(m0 + wave * WROWS, m_end - 1), w1 = min(m0 + wave * WROWS + WROWS - 1, m_end - 1);
     const uint32_t w_pos0 = s.pos0 + w0 / H, w_pos1 = s.pos0 + w1 / H, w_lo1 = w_pos1 + 1 > a.window ? w_pos1 + 1 - a.window : 0;
     const uint32_t w_lo0 = w_pos0 + 1 > a.window ? w_pos0 + 1 - a.window : 0;
     f32x4 acc[NR][2 * VT];
@@ -293,7 +424,7 @@ __global__ __launch_bounds__(256, 2) void window_prefill_kernel(const WindowArgs
         if (j0 + kMixPage < j_end) issue(j0 + kMixPage, stage ^ 1);
         if (j0 > w_pos1 || j0 + kMixPage <= w_lo0) continue;              // uniform over the wave: none of its keys
         const bf16x8* kt = reinterpret_cast<const bf16x8*>(window_lds + stage * STAGE) + lane;
-        const bf16x8* vt = kt + 4 * KQ * 64;
+        const bf16x8* vt = kt + 4 * MAPS * KQ * 64;
         f32x4 sc[NR][4];
 #pragma unroll
         for (int t = 0; t < NR; t++)
@@ -303,16 +434,21 @@ __global__ __launch_bounds__(256, 2) void window_prefill_kernel(const WindowArgs
         for (int k = 0; k < KQ; k++)
 #pragma unroll
             for (int n = 0; n < 4; n++) {
-                const bf16x8 kv = kt[(n * KQ + k) * 64];
+                if constexpr (MAPS == 1) {
+                    const bf16x8 kv = kt[(n * KQ + k) * 64];
 #pragma unroll
-                for (int t = 0; t < NR; t++) sc[t][n] = mix_mfma(kv, qv[t][k], sc[t][n]);
+                    for (int t = 0; t < NR; t++) sc[t][n] = mix_mfma(kv, qv[t][k], sc[t][n]);
+                } else {
+#pragma unroll
+                    for (int t = 0; t < NR; t++) sc[t][n] = mix_mfma(kt[((n * MAPS + t) * KQ + k) * 64], qv[t][k], sc[t][n]);
+                }
             }
         const bool inside = j0 + kMixPage - 1 <= w_pos0 && j0 >= w_lo1;
         bf16x8 p[NR][2];
 #pragma unroll
         for (int t = 0; t < NR; t++) {
-            const float corr = inside ? window_softmax<4, false>(sc[t], j0, g, lo[t], pos[t], scale, mx[t], sum[t])
-                                      : window_softmax<4, true>(sc[t], j0, g, lo[t], pos[t], scale, mx[t], sum[t]);
+            const float corr = inside ? window_softmax<4, false>(sc[t], j0, g, lo[t], pos[t], score, mx[t], sum[t])
+                                      : window_softmax<4, true>(sc[t], j0, g, lo[t], pos[t], score, mx[t], sum[t]);
             if (__any(corr != 1.0f)) {
 #pragma unroll
                 for (int k = 0; k < 2 * VT; k++)
@@ -332,11 +468,13 @@ __global__ __launch_bounds__(256, 2) void window_prefill_kernel(const WindowArgs
             }
     }
     __bf16* out = reinterpret_cast<__bf16*>(a.o);
+    float norm = 1.0f;
+    if constexpr (MAPS == 2) norm = window_difference(a, acc[0], acc[1], 1.0f / sum[0], 1.0f / sum[1]);
 #pragma unroll
-    for (int t = 0; t < NR; t++) {
+    for (int t = 0; t < NR / MAPS; t++) {
         if (m[t] >= m_end) continue;
         const uint32_t r = s.row0 + m[t] / H, h = kvh * H + m[t] % H;
-        const float inv = a.out_scale / sum[t];
+        const float inv = window_factor<false>(a, r, h) * (MAPS == 2 ? norm : 1.0f / sum[t]);
 #pragma unroll
         for (int k = 0; k < 2 * VT; k++) {
             bf16x4 o;
@@ -347,21 +485,21 @@ __global__ __launch_bounds__(256, 2) void window_prefill_kernel(const WindowArgs
     }
 }
 
-// grid (rows of the launch * kvh * tiles of 16 heads of a group, splits).  The four waves take every fourth block of 32
-// keys of the share, straight into registers, one block ahead.
-template <int KQ, int VT>
-__global__ __launch_bounds__(256, 2) void window_decode_kernel(const WindowArgs a)
+// grid (rows of the launch * kvh * tiles of 16 (head, map) columns of a group, splits).  The four waves take every fourth
+// block of 32 keys of the share, straight into registers, one block ahead.  KQ: tiles of all maps' keys.
+template <int KQ, int VT, int MAPS>
+__global__ __launch_bounds__(256, KQ + VT > 8 ? 1 : 2) void window_decode_kernel(const WindowArgs a)
 {
     __shared__ f32x4 box[3 * (2 * VT + 1) * 64];
     const int lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4;
     const uint32_t wave = (uint32_t)__builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-    const uint32_t tiles = (a.group + 15) / 16, split = blockIdx.y;
+    const uint32_t columns = a.group * MAPS, tiles = (columns + 15) / 16, split = blockIdx.y;
     const uint32_t kvh = blockIdx.x % a.kvh, tile = blockIdx.x / a.kvh % tiles, ri = blockIdx.x / a.kvh / tiles;
     const LatentRow lr = a.drows[ri];
     const uint32_t r = lr.row, pos = lr.pos, lo = pos + 1 > a.window ? pos + 1 - a.window : 0;
     const uint32_t first = lo / 32 * 32 + split * a.split_keys, end = min(pos + 1, first + a.split_keys);
-    const float scale = a.scale * kLog2e;
-    const uint32_t member = tile * 16 + c, head = kvh * a.group + min(member, a.group - 1);
+    const WindowScore score(a);
+    const uint32_t member = tile * 16 + c, column = min(member, columns - 1), head = kvh * a.group + column / MAPS, map = column % MAPS;
 
     bf16x8 kA[2 * KQ], vA[2 * VT], kB[2 * KQ], vB[2 * VT];
     const uint32_t j_last = pos / 32 * 32;                 // (a block past the end reads the last one again)
@@ -376,7 +514,13 @@ __global__ __launch_bounds__(256, 2) void window_decode_kernel(const WindowArgs 
     };
     bf16x8 qv[KQ];
 #pragma unroll
-    for (int k = 0; k < KQ; k++) qv[k] = reinterpret_cast<const bf16x8*>(a.q)[frag_unit(r, (head * KQ + k) * 4 + g, a.heads * KQ)];
+    for (int k = 0; k < KQ; k++) {
+        qv[k] = reinterpret_cast<const bf16x8*>(a.q)[frag_unit(r, (head * KQ + k) * 4 + g, a.heads * KQ)];
+        if (MAPS > 1 && (uint32_t)k / (KQ / MAPS) != map) {
+#pragma unroll
+            for (int i = 0; i < 8; i++) qv[k][i] = (__bf16)0.f;
+        }
+    }
     f32x4 acc[2 * VT];
 #pragma unroll
     for (int k = 0; k < 2 * VT; k++) acc[k] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -391,7 +535,7 @@ __global__ __launch_bounds__(256, 2) void window_decode_kernel(const WindowArgs 
             sc[0] = mix_mfma(k[i], qv[i], sc[0]);
             sc[1] = mix_mfma(k[KQ + i], qv[i], sc[1]);
         }
-        const float corr = window_softmax<2, true>(sc, j0, g, lo, end - 1, scale, mx, sum);
+        const float corr = window_softmax<2, true>(sc, j0, g, lo, end - 1, score, mx, sum);
         if (__any(corr != 1.0f)) {
 #pragma unroll
             for (int i = 0; i < 2 * VT; i++)
@@ -434,9 +578,20 @@ __global__ __launch_bounds__(256, 2) void window_decode_kernel(const WindowArgs 
             for (int i = 0; i < 4; i++) acc[k][i] = acc[k][i] * s0 + v[i] * s1;
         }
     }
-    if (member >= a.group) return;
+    if (member >= columns) return;                         // (the two maps of a head go together)
     if (a.splits == 1) {
-        const float inv = a.out_scale / sum;
+        float inv = window_factor<false>(a, r, head);
+        if constexpr (MAPS == 2) {                         // the other map is the next lane's
+            f32x4 other[2 * VT];
+#pragma unroll
+            for (int k = 0; k < 2 * VT; k++)
+#pragma unroll
+                for (int i = 0; i < 4; i++) other[k][i] = wave_xor_f32(acc[k][i], 1);
+            inv *= window_difference(a, acc, other, 1.0f / sum, 1.0f / wave_xor_f32(sum, 1));
+            if (map) return;
+        } else {
+            inv /= sum;
+        }
         __bf16* out = reinterpret_cast<__bf16*>(a.o);
 #pragma unroll
         for (int k = 0; k < 2 * VT; k++) {
@@ -447,7 +602,7 @@ __global__ __launch_bounds__(256, 2) void window_decode_kernel(const WindowArgs 
         }
         return;
     }
-    const size_t at = ((size_t)ri * a.heads + head) * a.splits + split;
+    const size_t at = (((size_t)ri * a.heads + head) * MAPS + map) * a.splits + split;
     if (g == 0) {
         a.part_ml[at * 2] = mx;
         a.part_ml[at * 2 + 1] = sum;
@@ -459,29 +614,55 @@ __global__ __launch_bounds__(256, 2) void window_decode_kernel(const WindowArgs 
 constexpr uint32_t kWindowSplits = 64;          // shares of the keys at most: a lane each
 
 // grid (rows of the launch, heads), one wave: the shares of one row and head together
-template <int VT>
+template <int VT, int MAPS>
 __global__ __launch_bounds__(64) void window_combine_kernel(const WindowArgs a)
 {
+    constexpr int COLS = (VT * 32 + 63) / 64;
     __shared__ float wt[kWindowSplits];
     const uint32_t h = blockIdx.y, r = a.drows[blockIdx.x].row, t = threadIdx.x;
-    const size_t at = ((size_t)blockIdx.x * a.heads + h) * a.splits;
-    const bool has = t < a.splits;
-    const float m = has ? a.part_ml[(at + t) * 2] : kLatentNone, l = has ? a.part_ml[(at + t) * 2 + 1] : 0.f;
-    float mx = m;
+    float o[MAPS][COLS];
 #pragma unroll
-    for (int off = 32; off >= 1; off >>= 1) mx = fmaxf(mx, wave_xor_f32(mx, off));
-    const float w = l != 0.f ? fast_exp2(m - mx) : 0.f;    // zero: a share past the row's keys
-    float sum = w * l;
+    for (int m = 0; m < MAPS; m++) {
+        const size_t at = (((size_t)blockIdx.x * a.heads + h) * MAPS + m) * a.splits;
+        const bool has = t < a.splits;
+        const float mo = has ? a.part_ml[(at + t) * 2] : kLatentNone, l = has ? a.part_ml[(at + t) * 2 + 1] : 0.f;
+        float mx = mo;
 #pragma unroll
-    for (int off = 32; off >= 1; off >>= 1) sum += wave_xor_f32(sum, off);
-    const float inv = a.out_scale / sum;
-    wt[t] = w;
-    __syncthreads();
+        for (int off = 32; off >= 1; off >>= 1) mx = fmaxf(mx, wave_xor_f32(mx, off));
+        const float w = l != 0.f ? fast_exp2(mo - mx) : 0.f;    // zero: a share past the row's keys
+        float sum = w * l;
+#pragma unroll
+        for (int off = 32; off >= 1; off >>= 1) sum += wave_xor_f32(sum, off);
+        const float inv = 1.0f / sum;
+        __syncthreads();
+        wt[t] = w;
+        __syncthreads();
+#pragma unroll
+        for (int i = 0; i < COLS; i++) {
+            const uint32_t col = t + 64 * i;
+            o[m][i] = 0.f;
+            if (col >= VT * 32) continue;
+            for (uint32_t s = 0; s < a.splits; s++) o[m][i] = fmaf(wt[s], a.part_o[(at + s) * VT * 32 + col], o[m][i]);
+            o[m][i] *= inv;
+        }
+    }
+    float factor = window_factor<false>(a, r, h);
+    if constexpr (MAPS == 2) {
+        float ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < COLS; i++) {
+            o[0][i] -= a.diff * o[1][i];
+            ss = fmaf(o[0][i], o[0][i], ss);
+        }
+#pragma unroll
+        for (int off = 32; off >= 1; off >>= 1) ss += wave_xor_f32(ss, off);
+        factor /= sqrtf(ss / (float)a.vdim + a.eps);
+    }
     __bf16* out = reinterpret_cast<__bf16*>(a.o);
-    for (uint32_t col = t; col < VT * 32; col += 64) {
-        float o = 0.f;
-        for (uint32_t s = 0; s < a.splits; s++) o = fmaf(wt[s], a.part_o[(at + s) * VT * 32 + col], o);
-        out[frag_elem(r, h * VT * 32 + col, a.o_kt)] = (__bf16)(o * inv);
+#pragma unroll
+    for (int i = 0; i < COLS; i++) {
+        const uint32_t col = t + 64 * i;
+        if (col < VT * 32) out[frag_elem(r, h * VT * 32 + col, a.o_kt)] = (__bf16)(o[0][i] * factor);
     }
 }
 

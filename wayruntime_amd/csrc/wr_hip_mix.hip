@@ -366,6 +366,7 @@ int wr_hip_mix_residual(wr_hip_mix_step* s, int f32, const wr_hip_mix_resid* q)
     if (!g.inited) return WR_HIP_ERR_STATE;
     if (!s || !s->rows || !q || !q->width || !q->x || (q->post && !q->y) || (q->next && !q->h)) return WR_HIP_ERR_INVAL;
     if (q->top && (!q->y || !q->gate || !q->slot)) return WR_HIP_ERR_INVAL;
+    if (q->side && !q->top) return WR_HIP_ERR_INVAL;
     if (q->wanted && (q->y || q->add || !s->n_want)) return WR_HIP_ERR_INVAL;
     ENTER();
     MixRowArgs a = {};
@@ -382,6 +383,9 @@ int wr_hip_mix_residual(wr_hip_mix_step* s, int f32, const wr_hip_mix_resid* q)
     a.gate = q->gate;
     a.slot = q->slot;
     a.top = q->top;
+    a.side = q->side;
+    a.ident = q->ident;
+    a.shared = q->shared;
     a.gather = q->wanted ? s->d<uint32_t>(s->o_want) : nullptr;
     return launch_residual(f32, false, a);
 }
@@ -441,14 +445,17 @@ int wr_hip_mix_gemm_run(int f32, const wr_hip_mix_gemm* q)
     if (!q || !q->w || !q->x || !q->rows) return WR_HIP_ERR_INVAL;
     const uint32_t ktiles = q->w->n_in / 32, batch = q->group_expert ? 1 : q->w->batch;
     if ((uint64_t)q->x_kt0 + (uint64_t)q->x_kt_z * (batch - 1) + ktiles > q->x_kt) return WR_HIP_ERR_INVAL;
-    const bool frag = q->out == WR_HIP_MIX_OUT_FRAG || q->out == WR_HIP_MIX_OUT_SPLIT || q->out == WR_HIP_MIX_OUT_GATED;
-    if (q->out > WR_HIP_MIX_OUT_GATED || (frag && !q->h)) return WR_HIP_ERR_INVAL;
-    const uint32_t n_frag = q->out == WR_HIP_MIX_OUT_SPLIT ? q->n_split : (q->out == WR_HIP_MIX_OUT_GATED ? q->w->n_out / 2 : q->w->n_out);
+    const bool split_gated = q->out == WR_HIP_MIX_OUT_SPLIT_GATED, gated = q->out == WR_HIP_MIX_OUT_GATED || split_gated;
+    const bool frag = q->out == WR_HIP_MIX_OUT_FRAG || q->out == WR_HIP_MIX_OUT_SPLIT || gated;
+    if (q->out > WR_HIP_MIX_OUT_SPLIT_GATED || (frag && !q->h)) return WR_HIP_ERR_INVAL;
+    if (split_gated && (q->n_split % 32 || q->n_split > q->w->n_out || batch != 1 || q->group_expert)) return WR_HIP_ERR_INVAL;
+    const uint32_t n_frag = q->out == WR_HIP_MIX_OUT_SPLIT ? q->n_split
+                            : gated ? (q->w->n_out - (split_gated ? q->n_split : 0)) / 2 : q->w->n_out;
     if (frag && ((uint64_t)q->col_z * (batch - 1) + n_frag > (uint64_t)q->h_kt * 32)) return WR_HIP_ERR_INVAL;
     if (q->out == WR_HIP_MIX_OUT_SPLIT && (q->n_split % 16 || q->n_split > q->w->n_out)) return WR_HIP_ERR_INVAL;
-    if (q->out == WR_HIP_MIX_OUT_GATED && q->w->n_out % 32) return WR_HIP_ERR_INVAL;
-    const bool rows32 = q->out == WR_HIP_MIX_OUT_ROWS_F32 || (q->out == WR_HIP_MIX_OUT_SPLIT && q->n_split < q->w->n_out);
-    const uint32_t n_rows = q->out == WR_HIP_MIX_OUT_SPLIT ? q->w->n_out - q->n_split : q->w->n_out;
+    if (gated && q->w->n_out % 32) return WR_HIP_ERR_INVAL;
+    const bool rows32 = q->out == WR_HIP_MIX_OUT_ROWS_F32 || (q->out == WR_HIP_MIX_OUT_SPLIT && q->n_split < q->w->n_out) || split_gated;
+    const uint32_t n_rows = q->out == WR_HIP_MIX_OUT_SPLIT ? q->w->n_out - q->n_split : split_gated ? q->n_split : q->w->n_out;
     if (rows32 && (!q->y_f32 || q->ldy % 4 || q->ldy < n_rows)) return WR_HIP_ERR_INVAL;
     if (q->out == WR_HIP_MIX_OUT_ROWS_F32 && batch > 1 && (q->col_z % 4 || (uint64_t)q->col_z * (batch - 1) + n_rows > q->ldy))
         return WR_HIP_ERR_INVAL;
@@ -456,6 +463,8 @@ int wr_hip_mix_gemm_run(int f32, const wr_hip_mix_gemm* q)
     if (((q->out == WR_HIP_MIX_OUT_ROWS_F32 && !q->col_z) || q->out == WR_HIP_MIX_OUT_ROWS) && batch != 1) return WR_HIP_ERR_INVAL;
     if (q->group_expert && (q->rows % 16 || (q->tile_groups != 1 && q->tile_groups != 8))) return WR_HIP_ERR_INVAL;
     if (q->group_expert && q->rows / 16 % q->tile_groups) return WR_HIP_ERR_INVAL;
+    if (q->bias && (batch != 1 || gated || q->group_expert)) return WR_HIP_ERR_INVAL;
+    if (q->x_perm && (!q->group_expert || q->tile_groups != 1)) return WR_HIP_ERR_INVAL;
     ENTER();
     MixGemmArgs a = {};
     a.w = reinterpret_cast<const bf16x8*>(q->w->tiles);
@@ -478,10 +487,14 @@ int wr_hip_mix_gemm_run(int f32, const wr_hip_mix_gemm* q)
     a.relu2 = q->relu2;
     a.gelu = q->gelu;
     a.scale = q->scale;
+    a.limit = q->limit;
+    a.slope = q->slope;
+    a.up_bias = q->up_bias;
+    a.bias = q->bias;
+    a.x_perm = q->x_perm;
     a.y = q->y_f32;
     a.ya = q->y_act;
     a.h = q->h;
-    const bool gated = q->out == WR_HIP_MIX_OUT_GATED;
     if (q->group_expert) {
         if (!f32 && q->tile_groups == 8) return launch_lds<4>(a, 1);
         if (f32) return gated ? launch_stream<true, 2, 1>(a, 1) : launch_stream<true, 1, 1>(a, 1);
@@ -976,9 +989,9 @@ static int check_window(const wr_hip_mix_step* s, const wr_hip_mix_pool* pool, u
 {
     if (!s || !s->rows || !pool || run >= pool->latent.size() || pool->f32 != (f32 != 0) || !q || !q->heads || !q->kv_heads ||
         q->heads % q->kv_heads || !q->dim || !q->vdim || q->dim_pad % 32 || q->vdim_pad % 32 || q->dim > q->dim_pad ||
-        q->vdim > q->vdim_pad || q->rot_half * 2 > q->dim || !q->window)
+        q->vdim > q->vdim_pad || q->rot_half * 2 > q->dim || !q->window || q->maps < 1 || q->maps > 2)
         return WR_HIP_ERR_INVAL;
-    if ((uint64_t)q->kv_heads * (q->dim_pad + q->vdim_pad) != pool->latent_dim[run]) return WR_HIP_ERR_INVAL;
+    if ((uint64_t)q->kv_heads * ((uint64_t)q->maps * q->dim_pad + q->vdim_pad) != pool->latent_dim[run]) return WR_HIP_ERR_INVAL;
     return WR_HIP_OK;
 }
 
@@ -1000,6 +1013,13 @@ static WindowArgs window_args(const wr_hip_mix_step* s, const wr_hip_mix_pool* p
     a.half = q->rot_half;
     a.window = q->window;
     a.norm_values = q->norm_values;
+    a.maps = q->maps;
+    a.dimk = q->maps * q->dim_pad;
+    a.neighbours = q->neighbours;
+    a.softcap = q->softcap;
+    a.diff = q->diff;
+    a.q_norm = q->q_norm;
+    a.k_norm = q->k_norm;
     a.scale = q->scale;
     a.out_scale = q->out_scale;
     a.eps = q->eps;
@@ -1014,8 +1034,10 @@ int wr_hip_mix_window_append(wr_hip_mix_step* s, wr_hip_mix_pool* pool, uint32_t
     if (!g.inited) return WR_HIP_ERR_STATE;
     int rc = check_window(s, pool, run, f32, q);
     if (rc) return rc;
-    if (!in_dev || !q_dev || (q->rot_half && !table_dev) || (uint64_t)col_q + (uint64_t)q->heads * q->dim > ld ||
-        (uint64_t)col_k + (uint64_t)q->kv_heads * q->dim > ld || (uint64_t)col_v + (uint64_t)q->kv_heads * q->vdim > ld)
+    const bool keys = col_k != WR_HIP_MIX_NO_KEYS;
+    if (!in_dev || !q_dev || (q->rot_half && !table_dev) || (uint64_t)col_q + (uint64_t)q->heads * q->maps * q->dim > ld ||
+        (keys && ((uint64_t)col_k + (uint64_t)q->kv_heads * q->maps * q->dim > ld ||
+                  (uint64_t)col_v + (uint64_t)q->kv_heads * q->vdim > ld)))
         return WR_HIP_ERR_INVAL;
     ENTER();
     WindowArgs a = window_args(s, pool, run, q);
@@ -1026,24 +1048,26 @@ int wr_hip_mix_window_append(wr_hip_mix_step* s, wr_hip_mix_pool* pool, uint32_t
     a.col_v = col_v;
     a.table = table_dev;
     a.q = q_dev;
-    const dim3 grid((s->rows + 3) / 4, a.kvh + (4 * a.heads * (a.dimp / 8) + kWindowQUnits - 1) / kWindowQUnits);
+    a.key_heads = keys ? a.kvh : 0;
+    const dim3 grid((s->rows + 3) / 4, a.key_heads + (4 * a.heads * (a.dimk / 8) + kWindowQUnits - 1) / kWindowQUnits);
     if (f32) MIX_LAUNCH(window_append_kernel<true>, grid, dim3(256), 0, a);
     else MIX_LAUNCH(window_append_kernel<false>, grid, dim3(256), 0, a);
     return WR_HIP_OK;
 }
 
-template <int KQ, int VT>
+template <int KQ, int VT, int MAPS>
 static int window_mfma(wr_hip_mix_step* s, WindowArgs& a)
 {
     if (s->n_long) {
+        constexpr uint32_t tile = 128 / MAPS;
         uint64_t tiles = 0;
-        for (uint32_t i = 0; i < s->n_long; i++) tiles += ((uint64_t)s->long_rows[i] * a.group + 127) / 128;
+        for (uint32_t i = 0; i < s->n_long; i++) tiles += ((uint64_t)s->long_rows[i] * a.group + tile - 1) / tile;
         a.list = s->d<uint32_t>(s->o_long);
         a.n_list = s->n_long;
-        constexpr size_t lds = window_prefill_lds(KQ, VT);
-        int rc = allow_lds<window_prefill_kernel<KQ, VT>>(lds);
+        constexpr size_t lds = window_prefill_lds(MAPS * KQ, VT);
+        int rc = allow_lds<window_prefill_kernel<KQ, VT, MAPS>>(lds);
         if (rc) return rc;
-        launch_main(window_prefill_kernel<KQ, VT>, dim3((uint32_t)(tiles * a.kvh)), dim3(256), a, lds);
+        launch_main(window_prefill_kernel<KQ, VT, MAPS>, dim3((uint32_t)(tiles * a.kvh)), dim3(256), a, lds);
         HIP_TRY(hipGetLastError(), "windowed prefill launch", 0);
     }
     const uint32_t n = s->n_short_rows;
@@ -1054,7 +1078,7 @@ static int window_mfma(wr_hip_mix_step* s, WindowArgs& a)
         const uint32_t lo = rows[i].pos + 1 > a.window ? rows[i].pos + 1 - a.window : 0;
         keys = std::max(keys, rows[i].pos + 1 - lo / 32 * 32);
     }
-    const uint32_t groups = a.kvh * ((a.group + 15) / 16);
+    const uint32_t groups = a.kvh * ((a.group * MAPS + 15) / 16);
     // Shares: two workgroups per compute unit at a time; a round costs about three iterations before its first and one
     // for each it makes, and the shares' sums about two more to put together.
     uint64_t best = ~(uint64_t)0;
@@ -1072,47 +1096,56 @@ static int window_mfma(wr_hip_mix_step* s, WindowArgs& a)
     }
     a.drows = s->d<LatentRow>(s->o_short_rows);
     if (a.splits > 1) {
-        const size_t part = (size_t)n * a.heads * a.splits;
+        const size_t part = (size_t)n * a.heads * MAPS * a.splits;
         int rc = ensure_device(s->partial, part * (VT * 32 + 2) * 4);
         if (rc) return rc;
         a.part_o = reinterpret_cast<float*>(s->partial.p);
         a.part_ml = a.part_o + part * VT * 32;
     }
-    launch_main(window_decode_kernel<KQ, VT>, dim3(n * groups, a.splits), dim3(256), a);
+    launch_main(window_decode_kernel<MAPS * KQ, VT, MAPS>, dim3(n * groups, a.splits), dim3(256), a);
     HIP_TRY(hipGetLastError(), "windowed decode launch", 0);
-    if (a.splits > 1) MIX_LAUNCH(window_combine_kernel<VT>, dim3(n, a.heads), dim3(64), 0, a);
+    if (a.splits > 1) MIX_LAUNCH((window_combine_kernel<VT, MAPS>), dim3(n, a.heads), dim3(64), 0, a);
     return WR_HIP_OK;
 }
 
-template <int KQ>
+template <int KQ, int MAPS>
 static int window_mfma_v(wr_hip_mix_step* s, WindowArgs& a)
 {
-    if (a.vdimp == 32) return window_mfma<KQ, 1>(s, a);
-    if (a.vdimp == 64) return window_mfma<KQ, 2>(s, a);
-    return window_mfma<KQ, 4>(s, a);
+    if (a.vdimp == 32) return window_mfma<KQ, 1, MAPS>(s, a);
+    if (a.vdimp == 64) return window_mfma<KQ, 2, MAPS>(s, a);
+    return window_mfma<KQ, 4, MAPS>(s, a);
+}
+
+template <int MAPS>
+static int window_mfma_k(wr_hip_mix_step* s, WindowArgs& a)
+{
+    if (a.dimp == 32) return window_mfma_v<1, MAPS>(s, a);
+    if (a.dimp == 64) return window_mfma_v<2, MAPS>(s, a);
+    return window_mfma_v<4, MAPS>(s, a);
 }
 
 int wr_hip_mix_window_attend(wr_hip_mix_step* s, wr_hip_mix_pool* pool, uint32_t run, int f32, const wr_hip_mix_window* q,
-                             const void* q_dev, const float* sink_dev, void* o_dev, uint32_t o_kt)
+                             const void* q_dev, const float* sink_dev, const float* gate_dev, uint32_t ldg, void* o_dev,
+                             uint32_t o_kt)
 {
     if (!g.inited) return WR_HIP_ERR_STATE;
     int rc = check_window(s, pool, run, f32, q);
     if (rc) return rc;
-    if (!q_dev || !o_dev || (uint64_t)q->heads * q->vdim_pad > (uint64_t)o_kt * 32) return WR_HIP_ERR_INVAL;
+    if (!q_dev || !o_dev || (uint64_t)q->heads * q->vdim_pad > (uint64_t)o_kt * 32 || (gate_dev && ldg < q->heads)) return WR_HIP_ERR_INVAL;
     ENTER();
     g.calls.fetch_add(s->n_seq, std::memory_order_relaxed);
     WindowArgs a = window_args(s, pool, run, q);
     a.q = const_cast<void*>(q_dev);
     a.sink = sink_dev;
+    a.gate = gate_dev;
+    a.ldg = ldg;
     a.o = o_dev;
     a.o_kt = o_kt;
     auto fits = [](uint32_t p) { return p == 32 || p == 64 || p == 128; };
     if (!f32 && !g.force_generic && fits(a.dimp) && fits(a.vdimp)) {
-        if (a.dimp == 32) return window_mfma_v<1>(s, a);
-        if (a.dimp == 64) return window_mfma_v<2>(s, a);
-        return window_mfma_v<4>(s, a);
+        return a.maps == 2 ? window_mfma_k<2>(s, a) : window_mfma_k<1>(s, a);
     }
-    const size_t lds = ((size_t)a.dimp + a.vdimp + 64) * 4;
+    const size_t lds = ((size_t)a.dimp + (size_t)a.maps * a.vdimp + 64) * 4;
     rc = f32 ? allow_lds<window_attend_any_kernel<true>>(lds) : allow_lds<window_attend_any_kernel<false>>(lds);
     if (rc) return rc;
     if (f32) MIX_LAUNCH(window_attend_any_kernel<true>, dim3(s->rows, a.heads), dim3(64), lds, a);
@@ -1130,18 +1163,40 @@ uint32_t wr_hip_mix_route_groups(uint32_t rows, uint32_t experts, uint32_t top, 
     return (uint32_t)(runs * tile_groups);
 }
 
-int wr_hip_mix_route(wr_hip_mix_step* s, const float* z_dev, uint32_t ldz, uint32_t experts, uint32_t top,
-                     uint32_t tile_groups, float* gate_dev, uint32_t* slot_dev, uint32_t* perm_dev,
-                     int32_t* group_expert_dev)
+int wr_hip_mix_route(wr_hip_mix_step* s, const float* z_dev, uint32_t ldz, const wr_hip_mix_router* q, uint32_t tile_groups,
+                     float* gate_dev, float* side_dev, uint32_t* slot_dev, uint32_t* perm_dev, int32_t* group_expert_dev)
 {
     if (!g.inited) return WR_HIP_ERR_STATE;
-    if (!s || !s->rows || !z_dev || !experts || !top || top > experts || ldz < experts || !tile_groups || !gate_dev ||
-        !slot_dev || !perm_dev || !group_expert_dev)
+    if (!s || !s->rows || !z_dev || !q || !q->experts || !q->top || !tile_groups || !gate_dev || !slot_dev || !perm_dev ||
+        !group_expert_dev)
         return WR_HIP_ERR_INVAL;
-    if (experts > WR_HIP_MIX_MAX_EXPERTS || top > WR_HIP_MIX_MAX_TOP) return WR_HIP_ERR_LIMIT;
+    const uint64_t outputs = (uint64_t)q->experts + q->identity;
+    if (outputs > WR_HIP_MIX_MAX_EXPERTS || q->top > WR_HIP_MIX_MAX_TOP || q->groups > WR_HIP_MIX_MAX_GROUPS) return WR_HIP_ERR_LIMIT;
+    if (ldz < outputs + (q->shared_gate != 0) || ((q->identity || q->shared_gate) && !side_dev) || (q->correction && !q->softmax_all))
+        return WR_HIP_ERR_INVAL;
+    if (q->groups && (outputs % q->groups || !q->keep || q->keep > q->groups)) return WR_HIP_ERR_INVAL;
+    if (q->top > (q->groups ? outputs / q->groups * q->keep : outputs)) return WR_HIP_ERR_INVAL;
     ENTER();
-    MixRouteArgs a = {z_dev, ldz, s->rows, experts, top, tile_groups, wr_hip_mix_route_groups(s->rows, experts, top, tile_groups),
-                      gate_dev, slot_dev, perm_dev, group_expert_dev};
+    MixRouteArgs a = {};
+    a.z = z_dev;
+    a.ldz = ldz;
+    a.rows = s->rows;
+    a.outputs = (uint32_t)outputs;
+    a.experts = q->experts;
+    a.top = q->top;
+    a.tile_groups = tile_groups;
+    a.n_groups = wr_hip_mix_route_groups(s->rows, q->experts, q->top, tile_groups);
+    a.kinds = q->groups;
+    a.keep = q->keep;
+    a.softmax_all = q->softmax_all;
+    a.shared_gate = q->shared_gate;
+    a.scale = q->scale;
+    a.correction = q->correction;
+    a.gate = gate_dev;
+    a.side = side_dev;
+    a.slot = slot_dev;
+    a.perm = perm_dev;
+    a.group_expert = group_expert_dev;
     if (s->rows <= 64) {
         MIX_LAUNCH(mix_order_kernel<true>, dim3(1), dim3(1024), 0, a);
     } else {

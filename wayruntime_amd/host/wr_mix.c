@@ -158,11 +158,16 @@ typedef struct parallel_rows {
     float *in, *z;
 } parallel_rows;
 
+typedef struct window_rows {
+    float *in;
+    void  *q, *oh;
+} window_rows;
+
 typedef struct moe_rows {
-    float    *z, *gate, *ys;
+    float    *z, *gate, *side, *ys, *shared;
     uint32_t *slot, *perm;
     int32_t  *group_expert;
-    void     *xs, *act;
+    void     *xs, *act, *shared_act;
     uint32_t  groups, tile_groups;
 } moe_rows;
 
@@ -232,10 +237,19 @@ static parallel_rows take_parallel(bump *b, const wrh_mix_layer *L, size_t R, si
     return r;
 }
 
+static window_rows take_window(bump *b, const wrh_mix_layer *L, size_t R, size_t e)
+{
+    window_rows r;
+    r.in = take(b, R * L->ld_in * 4);
+    r.q = take(b, r16(R) * L->heads * L->win.maps * L->win.dim_pad * e);
+    r.oh = take(b, r16(R) * L->heads * L->win.vdim_pad * e);
+    return r;
+}
+
 /* Experts whose rows fill whole tiles take the prompt-sized product. */
 static uint32_t moe_tile(const struct wrh_mix_model *mm, const wrh_mix_layer *L, size_t R)
 {
-    return (!mm->f32 && R * L->top >= (size_t)L->experts * 32) ? 8 : 1;
+    return (!mm->f32 && R * L->router.top >= (size_t)L->router.experts * 32) ? 8 : 1;
 }
 
 static moe_rows take_moe(bump *b, const struct wrh_mix_model *mm, const wrh_mix_layer *L, size_t R, uint32_t tile)
@@ -243,16 +257,19 @@ static moe_rows take_moe(bump *b, const struct wrh_mix_model *mm, const wrh_mix_
     moe_rows r;
     const size_t e = mm->f32 ? 4 : 2;
     r.tile_groups = tile;
-    r.groups = wr_hip_mix_route_groups((uint32_t)R, L->experts, L->top, tile);
+    r.groups = wr_hip_mix_route_groups((uint32_t)R, L->router.experts, L->router.top, tile);
     const size_t slots = (size_t)r.groups * 16;
-    r.z = take(b, R * L->experts_p * 4);
-    r.gate = take(b, R * L->top * 4);
-    r.slot = take(b, R * L->top * 4);
+    r.z = take(b, R * L->router_p * 4);
+    r.gate = take(b, R * L->router.top * 4);
+    r.side = take(b, R * 2 * 4);
+    r.slot = take(b, R * L->router.top * 4);
     r.perm = take(b, slots * 4);
     r.group_expert = take(b, (size_t)r.groups * 4);
     r.xs = take(b, slots * mm->width_p * e);
     r.act = take(b, slots * L->ff_p * e);
     r.ys = take(b, slots * mm->width_p * 4);
+    r.shared_act = L->shared_p ? take(b, r16(R) * L->shared_p * e) : NULL;
+    r.shared = L->shared_p ? take(b, R * mm->width_p * 4) : NULL;
     return r;
 }
 
@@ -272,6 +289,7 @@ static size_t scratch_bytes(const struct wrh_mix_model *mm, size_t R)
         case WRH_MIXER_LATENT: (void)take_latent(&b, L, R, e); break;
         case WRH_MIXER_WKV: (void)take_wkv(&b, mm, L, R); break;
         case WRH_MIXER_PARALLEL: (void)take_parallel(&b, L, R, e); break;
+        case WRH_MIXER_WINDOW: (void)take_window(&b, L, R, e); break;
         }
         if (b.at > most) most = b.at;
         bump f = {NULL, 0};
@@ -441,13 +459,32 @@ static wr_status walk_parallel(wr_model *m, const wrh_mix_layer *L, uint32_t r, 
     TRY(wr_hip_mix_gemm_run(mm->f32, &in), "both halves' projections");
     TRY(wr_hip_mix_window_append(mm->step, mm->pool, store, mm->f32, &L->win, t.in, L->ld_in, L->col_q, L->col_k, L->col_v,
                                  w->rope[L->rope], t.q), "rotation + cache append");
-    TRY(wr_hip_mix_window_attend(mm->step, mm->pool, store, mm->f32, &L->win, t.q, L->sink, t.oh, kt_o), "windowed attention");
+    TRY(wr_hip_mix_window_attend(mm->step, mm->pool, store, mm->f32, &L->win, t.q, L->sink, NULL, 0, t.oh, kt_o),
+        "windowed attention");
     wr_hip_mix_recurrence rec = {.rule = WR_HIP_MIX_RULE_DELTA, .gain = WRH_DELTA_GAIN, .unit_eps = WRH_DELTA_UNIT_EPS,
                                  .out_scale = L->right_scale, .a_bias = q->a_bias, .in = t.in, .ld = L->ld_in,
                                  .col_r = L->col_rr, .col_k = L->col_rk, .col_v = L->col_rv, .col_a = L->col_ra,
                                  .col_g = L->col_rg, .h = t.oh, .h_kt = kt_o, .col_h = L->heads * L->win.vdim_pad};
     const wr_status st = walk_recur(m, q, r, mm->runs[r].store2, t.low, t.z, &rec);
     if (st != WR_OK) return st;
+    const wr_hip_mix_gemm out = {.w = L->w_o, .x = t.oh, .x_kt = kt_o, .rows = R, .out = WR_HIP_MIX_OUT_ROWS_F32,
+                                 .y_f32 = w->y, .ldy = mm->width_p};
+    TRY(wr_hip_mix_gemm_run(mm->f32, &out), "output projection");
+    return WR_OK;
+}
+
+static wr_status walk_window(wr_model *m, const wrh_mix_layer *L, uint32_t r, const walk *w, bump b, uint32_t R)
+{
+    struct wrh_mix_model *mm = m->mix;
+    const window_rows t = take_window(&b, L, R, mm->f32 ? 4 : 2);
+    const uint32_t kt_o = L->heads * L->win.vdim_pad / 32, store = mm->runs[r].store;
+    const wr_hip_mix_gemm in = {.w = L->w_in, .x = w->h, .x_kt = mm->width_p / 32, .rows = R, .out = WR_HIP_MIX_OUT_ROWS_F32,
+                                .y_f32 = t.in, .ldy = L->ld_in, .bias = L->b_in};
+    TRY(wr_hip_mix_gemm_run(mm->f32, &in), "q/k/v projection");
+    TRY(wr_hip_mix_window_append(mm->step, mm->pool, store, mm->f32, &L->win, t.in, L->ld_in, L->col_q, L->col_k, L->col_v,
+                                 w->rope[L->rope], t.q), "rotation + cache append");
+    TRY(wr_hip_mix_window_attend(mm->step, mm->pool, store, mm->f32, &L->win, t.q, L->sink, L->has_gate ? t.in + L->col_rg : NULL,
+                                 L->ld_in, t.oh, kt_o), "windowed attention");
     const wr_hip_mix_gemm out = {.w = L->w_o, .x = t.oh, .x_kt = kt_o, .rows = R, .out = WR_HIP_MIX_OUT_ROWS_F32,
                                  .y_f32 = w->y, .ldy = mm->width_p};
     TRY(wr_hip_mix_gemm_run(mm->f32, &out), "output projection");
@@ -472,24 +509,54 @@ static wr_status walk_mlp(wr_model *m, const wrh_mix_layer *L, uint32_t r, const
         return WR_OK;
     }
     const moe_rows t = take_moe(&b, mm, L, R, moe_tile(mm, L, R));
-    const wr_hip_mix_gemm router = {.w = L->w_router, .x = w->h, .x_kt = wkt, .rows = R, .out = WR_HIP_MIX_OUT_ROWS_F32,
-                                    .y_f32 = t.z, .ldy = L->experts_p};
+    wr_hip_mix_gemm router = {.w = L->w_router, .x = w->h, .x_kt = wkt, .rows = R, .out = WR_HIP_MIX_OUT_ROWS_F32,
+                              .y_f32 = t.z, .ldy = L->router_p};
+    if (L->shared_p) {                                     /* the shared expert's gate and up ride along */
+        router.out = WR_HIP_MIX_OUT_SPLIT_GATED;
+        router.n_split = L->router_p;
+        router.h = t.shared_act;
+        router.h_kt = L->shared_p / 32;
+        router.limit = L->shared_limit;
+        router.slope = WRH_CLAMPED_SLOPE;
+        router.up_bias = WRH_CLAMPED_UP_BIAS;
+    }
     TRY(wr_hip_mix_gemm_run(mm->f32, &router), "router");
-    TRY(wr_hip_mix_route(mm->step, t.z, L->experts_p, L->experts, L->top, t.tile_groups, t.gate, t.slot, t.perm,
-                         t.group_expert), "routing");
-    TRY(wr_hip_mix_route_gather(mm->step, mm->f32, w->h, wkt, t.groups, t.perm, t.group_expert, t.xs), "expert rows");
-    const wr_hip_mix_gemm up = {.w = L->w_eup, .x = t.xs, .x_kt = wkt, .rows = t.groups * 16, .group_expert = t.group_expert,
-                                .tile_groups = t.tile_groups, .out = WR_HIP_MIX_OUT_FRAG, .h = t.act,
-                                .h_kt = L->ff_p / 32, .relu2 = 1};
+    TRY(wr_hip_mix_route(mm->step, t.z, L->router_p, &L->router, t.tile_groups, t.gate, t.side, t.slot, t.perm, t.group_expert),
+        "routing");
+    wr_hip_mix_gemm up = {.w = L->w_eup, .x = t.xs, .x_kt = wkt, .rows = t.groups * 16, .group_expert = t.group_expert,
+                          .tile_groups = t.tile_groups, .out = WR_HIP_MIX_OUT_FRAG, .h = t.act, .h_kt = L->ff_p / 32, .relu2 = 1};
+    if (t.tile_groups == 1) {                              /* few rows: the product fetches them where they are */
+        up.x = w->h;
+        up.x_perm = t.perm;
+    } else {
+        TRY(wr_hip_mix_route_gather(mm->step, mm->f32, w->h, wkt, t.groups, t.perm, t.group_expert, t.xs), "expert rows");
+    }
+    if (L->limit > 0) {
+        up.out = WR_HIP_MIX_OUT_GATED;
+        up.relu2 = 0;
+        up.limit = L->limit;
+        up.slope = WRH_CLAMPED_SLOPE;
+        up.up_bias = WRH_CLAMPED_UP_BIAS;
+    }
     TRY(wr_hip_mix_gemm_run(mm->f32, &up), "experts' up projection");
     const wr_hip_mix_gemm down = {.w = L->w_edown, .x = t.act, .x_kt = L->ff_p / 32, .rows = t.groups * 16,
                                   .group_expert = t.group_expert, .tile_groups = t.tile_groups,
                                   .out = WR_HIP_MIX_OUT_ROWS_F32, .y_f32 = t.ys, .ldy = mm->width_p};
     TRY(wr_hip_mix_gemm_run(mm->f32, &down), "experts' down projection");
+    if (L->shared_p) {
+        const wr_hip_mix_gemm sh = {.w = L->w_down, .x = t.shared_act, .x_kt = L->shared_p / 32, .rows = R,
+                                    .out = WR_HIP_MIX_OUT_ROWS_F32, .y_f32 = t.shared, .ldy = mm->width_p};
+        TRY(wr_hip_mix_gemm_run(mm->f32, &sh), "shared expert's down projection");
+    }
     res->y = t.ys;
     res->gate = t.gate;
     res->slot = t.slot;
-    res->top = L->top;
+    res->top = L->router.top;
+    if (L->router.identity || L->shared_p) {
+        res->side = t.side;
+        res->ident = L->router.identity ? w->h : NULL;
+        res->shared = t.shared;
+    }
     return WR_OK;
 }
 
@@ -528,6 +595,7 @@ static wr_status walk_layers(wr_model *m, walk *w, bump b, uint32_t R, int fail_
         case WRH_MIXER_LATENT: st = walk_latent(m, L, r, w, b, R); break;
         case WRH_MIXER_WKV: st = walk_wkv(m, L, r, w, b, R, y); break;
         case WRH_MIXER_PARALLEL: st = walk_parallel(m, L, r, w, b, R); break;
+        case WRH_MIXER_WINDOW: st = walk_window(m, L, r, w, b, R); break;
         }
         if (st != WR_OK) return st;
         y = NULL;

@@ -1,8 +1,8 @@
 /*
  * wr_mix.h — mixer-stack models: a list of layers, each a mixer (decayed linear
  * attention, windowed attention through a latent, a matrix-state recurrence behind
- * a token shift, or windowed grouped-query attention and such a recurrence side by
- * side) and an optional feed-forward (dense or a mixture of experts), with norms
+ * a token shift, windowed grouped-query attention, or that and such a recurrence side
+ * by side) and an optional feed-forward (dense or a mixture of experts), with norms
  * before and, in some designs, after each, part of the list possibly run several
  * times.  A design (wrh_mix_design) says which of these its models use.  Read from a folder with config.json and
  * model.safetensors.  wr_mix_model.c reads and uploads, wr_mix.c keeps the cache
@@ -15,7 +15,7 @@
 #include "wr_json.h"
 #include "../../include/wr_hip_mix.h"
 
-typedef enum { WRH_MIXER_LIGHTNING, WRH_MIXER_LATENT, WRH_MIXER_WKV, WRH_MIXER_PARALLEL } wrh_mixer_kind;
+typedef enum { WRH_MIXER_LIGHTNING, WRH_MIXER_LATENT, WRH_MIXER_WKV, WRH_MIXER_PARALLEL, WRH_MIXER_WINDOW } wrh_mixer_kind;
 typedef enum { WRH_MLP_NONE, WRH_MLP_DENSE, WRH_MLP_MOE } wrh_mlp_kind;
 
 /* A matrix-state recurrence: its own part of a layer's products and vectors. */
@@ -49,11 +49,22 @@ typedef struct wrh_mix_layer {
     wr_hip_mat *w_in;
     uint32_t col_q, col_k, col_v, col_rr, col_rk, col_rv, col_rg, col_ra, ld_in;
     const float *sink;
+    /* window: one stacked product [q | k | v | gate] (values that are the keys take no part of it), w_o */
+    uint8_t has_gate;                     /* a logistic gate per head, its logits at col_rg */
+    int32_t kv_from;                      /* layer whose keys and values it reads, or -1 */
+    const float *b_in;                    /* ld_in biases, or NULL */
     /* feed-forward */
     wrh_mlp_kind mlp;
     uint8_t gelu;
-    uint32_t ff, ff_p, experts, experts_p, top;
+    uint32_t ff, ff_p;
     wr_hip_mat *w_gu, *w_down, *w_router, *w_eup, *w_edown;
+    /* experts: the router's outputs, padded (logit rows); with limit > 0 gated experts, clamped (w_eup: gate and up) */
+    wr_hip_mix_router router;
+    uint32_t router_p;
+    float limit;
+    /* shared expert: w_router carries its gate's logit and, behind router_p rows, its gate and up; w_down takes it out */
+    uint32_t shared_p;                    /* its width, or 0 */
+    float shared_limit;
     const float *norm1, *norm1b, *norm2, *norm2b;
 } wrh_mix_layer;
 
@@ -106,6 +117,10 @@ struct wrh_mix_model {
 /* The delta rule's own constants: log w = -exp(-1/2) * logistic, unit keys over sqrt(k . k + 1e-6). */
 #define WRH_DELTA_GAIN     0.60653065971263342360f
 #define WRH_DELTA_UNIT_EPS 1e-6f
+
+/* Clamped gated units: g * logistic(1.702 g) * (u + 1). */
+#define WRH_CLAMPED_SLOPE   1.702f
+#define WRH_CLAMPED_UP_BIAS 1.0f
 
 typedef struct wrh_mix_session {
     uint32_t slot, buf;                   /* state slot; which of its buffers is current */

@@ -21,7 +21,7 @@ static uint32_t p32(uint32_t n) { return (n + 31) / 32 * 32; }
 static uint32_t p16(uint32_t n) { return (n + 15) / 16 * 16; }
 
 /* What tells the designs of this family apart. */
-typedef enum { DESIGN_BIPOTAR = 1, DESIGN_TAREDRA = 2 } design_bit;
+typedef enum { DESIGN_BIPOTAR = 1, DESIGN_TAREDRA = 2, DESIGN_FEDIRAX = 4 } design_bit;
 typedef struct wrh_mix_design {
     const char *arch;
     design_bit  bit;
@@ -35,6 +35,7 @@ typedef struct wrh_mix_design {
 static const wrh_mix_design designs[] = {
     {.arch = "Bipotar", .bit = DESIGN_BIPOTAR, .post_norms = 1, .embed_norm = 1},
     {.arch = "Taredra", .bit = DESIGN_TAREDRA, .norms_around_zero = 1, .tied_head = 1, .gelu = 1},
+    {.arch = "Fedirax", .bit = DESIGN_FEDIRAX, .norms_around_zero = 1},
 };
 
 /* Everything the reading functions share; `st` keeps the first failure. */
@@ -85,6 +86,13 @@ static const wrh_json *need_obj(loader *l, const wrh_json *o, const char *key)
         return NULL;
     }
     return v;
+}
+
+/* A key that may be absent or null. */
+static const wrh_json *given(const wrh_json *o, const char *key)
+{
+    const wrh_json *v = wrh_json_get(o, key);
+    return v && v->type != WRH_JSON_NULL ? v : NULL;
 }
 
 static const char *need_str(loader *l, const wrh_json *o, const char *key)
@@ -474,6 +482,7 @@ static void read_parallel(loader *l, uint32_t i, const wrh_json *c, wrh_mix_laye
     g->out_scale = (float)ls;
     g->norm_values = 1;
     g->eps = mm->eps;
+    g->maps = 1;
     L->right_scale = (float)rs;
     if ((uint64_t)H * g->dim_pad > DIM_MAX || (uint64_t)H * g->vdim_pad > DIM_MAX) {
         fail(l, WR_ERR_LIMIT, "config: layer %u is too wide", i);
@@ -514,6 +523,140 @@ static void read_parallel(loader *l, uint32_t i, const wrh_json *c, wrh_mix_laye
     L->w_o = operand_up(l, &o);
 }
 
+/* What windowed attention mixers of their own share: sizes, rotation of neighbours, window, scale. */
+static int read_window_sizes(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *L, uint32_t maps)
+{
+    wr_hip_mix_window *g = &L->win;
+    L->kind = WRH_MIXER_WINDOW;
+    L->kv_from = -1;
+    const uint32_t H = g->heads = L->heads = need_u32(l, c, "heads", 1, HEADS_MAX);
+    const uint32_t G = g->kv_heads = need_u32(l, c, "kv_heads", 1, HEADS_MAX);
+    g->dim = L->dim = need_u32(l, c, "dim", 1, 4096);
+    g->vdim = L->vdim = need_u32(l, c, "vdim", 1, 4096);
+    const wrh_json *rot = need_obj(l, c, "rot"), *mask = need_obj(l, c, "mask");
+    g->scale = (float)need_num(l, c, "scale");
+    if (l->st != WR_OK) return 0;
+    const double base = need_num(l, rot, "base");
+    const uint32_t dims = need_u32(l, rot, "dims", 0, g->dim);
+    g->window = need_u32(l, mask, "size", 1, 0xFFFFFFFFu);
+    if (l->st == WR_OK && (dims % 2 || base <= 0)) fail(l, WR_ERR_FORMAT, "config: layer %u: rotation of %u dimensions, base %g", i, dims, base);
+    if (l->st == WR_OK && H % G) fail(l, WR_ERR_FORMAT, "config: layer %u: %u heads over %u key/value heads", i, H, G);
+    if (l->st != WR_OK) return 0;
+    g->dim_pad = wr_hip_mix_window_pad(g->dim);
+    g->vdim_pad = wr_hip_mix_window_pad(g->vdim);
+    g->rot_half = dims / 2;
+    g->neighbours = 1;
+    g->maps = maps;
+    g->out_scale = 1.0f;
+    g->eps = l->mm->eps;
+    if ((uint64_t)H * maps * g->dim_pad > DIM_MAX || (uint64_t)H * g->vdim_pad > DIM_MAX) {
+        fail(l, WR_ERR_LIMIT, "config: layer %u is too wide", i);
+        return 0;
+    }
+    L->rope = rope_index(l, base, dims);
+    return l->st == WR_OK;
+}
+
+/* One product of a layer's input out of several matrices: where each one's outputs lie, then the operand. */
+typedef struct in_part {
+    const char *name;
+    uint32_t    rows, *col;
+} in_part;
+
+static operand stack_inputs(loader *l, uint32_t i, const in_part *parts, size_t n, uint32_t *ld)
+{
+    *ld = 0;
+    for (size_t k = 0; k < n; k++) {
+        *parts[k].col = *ld;
+        *ld += p32(parts[k].rows);
+    }
+    operand o = operand_new(l, 1, *ld, l->mm->width_p);
+    for (size_t k = 0; k < n; k++)
+        operand_put(l, &o, 0, *parts[k].col, ltensor(l, i, parts[k].name, parts[k].rows, l->mm->width), parts[k].rows, l->mm->width);
+    return o;
+}
+
+static void read_window_out(loader *l, uint32_t i, wrh_mix_layer *L)
+{
+    const wr_hip_mix_window *g = &L->win;
+    operand o = operand_new(l, 1, l->mm->width_p, g->heads * g->vdim_pad);
+    put_heads_out(l, &o, ltensor(l, i, "mix.o", l->mm->width, g->heads * g->vdim), 0, g->heads, g->vdim, g->vdim_pad);
+    L->w_o = operand_up(l, &o);
+}
+
+/* Values that are the keys ahead of their rotation, biases, capped scores, sinks, a gate per head. */
+static void read_window_keys(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *L)
+{
+    if (!read_window_sizes(l, i, c, L, 1)) return;
+    wr_hip_mix_window *g = &L->win;
+    const uint32_t hq = g->heads * g->dim, hk = g->kv_heads * g->dim;
+    if (given(c, "softcap")) g->softcap = (float)need_num(l, c, "softcap");
+    if (l->st == WR_OK && (g->vdim != g->dim || g->softcap < 0))
+        fail(l, WR_ERR_FORMAT, "config: layer %u: values of %u from keys of %u, scores capped at %g", i, g->vdim, g->dim, g->softcap);
+    const in_part parts[] = {{"mix.q", hq, &L->col_q}, {"mix.k", hk, &L->col_k}, {"mix.g", g->heads, &L->col_rg}};
+    operand o = stack_inputs(l, i, parts, sizeof parts / sizeof *parts, &L->ld_in);
+    L->w_in = operand_up(l, &o);
+    L->col_v = L->col_k;
+    L->has_gate = 1;
+    const uint16_t *bq = ltensor(l, i, "mix.q.b", hq, 0), *bk = ltensor(l, i, "mix.k.b", hk, 0);
+    size_t at = 0;
+    float *b = l->st == WR_OK ? vec_take(l, L->ld_in, &at) : NULL;
+    if (b) {
+        for (uint32_t k = 0; k < hq; k++) b[L->col_q + k] = widen(bq[k]);
+        for (uint32_t k = 0; k < hk; k++) b[L->col_k + k] = widen(bk[k]);
+        L->b_in = (const float *)(uintptr_t)(at + 1);
+    }
+    L->sink = vec_put(l, ltensor(l, i, "mix.sink", g->heads, 0), g->heads);
+    read_window_out(l, i, L);
+}
+
+static double dot_of(loader *l, uint32_t i, const char *a, const char *b, uint32_t n)
+{
+    const uint16_t *x = ltensor(l, i, a, n, 0), *y = ltensor(l, i, b, n, 0);
+    double s = 0;
+    for (uint32_t k = 0; x && y && k < n; k++) s += (double)widen(x[k]) * widen(y[k]);
+    return s;
+}
+
+/* Two maps per head over the same values, normed queries and keys; possibly over another layer's keys and values. */
+static void read_window_difference(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *L)
+{
+    if (!read_window_sizes(l, i, c, L, 2)) return;
+    wr_hip_mix_window *g = &L->win;
+    const double diff = need_num(l, c, "diff");
+    if (given(c, "kv_from")) L->kv_from = (int32_t)need_u32(l, c, "kv_from", 0, 0x7FFFFFFFu);
+    if (l->st != WR_OK) return;
+    if (L->kv_from >= 0) {
+        const wrh_mix_layer *S = (uint32_t)L->kv_from < i ? &l->mm->layers[L->kv_from] : NULL;
+        if (!S || S->kind != WRH_MIXER_WINDOW || S->win.maps != 2 || S->kv_from >= 0 || S->win.kv_heads != g->kv_heads ||
+            S->win.dim != g->dim || S->win.vdim != g->vdim) {
+            fail(l, WR_ERR_FORMAT, "config: layer %u cannot use the keys and values of layer %d", i, L->kv_from);
+            return;
+        }
+    }
+    const double lambda = exp(dot_of(l, i, "mix.lq1", "mix.lk1", g->dim)) - exp(dot_of(l, i, "mix.lq2", "mix.lk2", g->dim)) + diff;
+    g->diff = (float)lambda;
+    g->out_scale = (float)(1.0 - diff);
+    const in_part parts[] = {{"mix.q", g->heads * 2 * g->dim, &L->col_q}, {"mix.k", g->kv_heads * 2 * g->dim, &L->col_k},
+                             {"mix.v", g->kv_heads * g->vdim, &L->col_v}};
+    operand o = stack_inputs(l, i, parts, L->kv_from >= 0 ? 1 : sizeof parts / sizeof *parts, &L->ld_in);
+    L->w_in = operand_up(l, &o);
+    g->q_norm = vec_put(l, ltensor(l, i, "mix.q.norm", g->dim, 0), g->dim);
+    if (L->kv_from < 0) g->k_norm = vec_put(l, ltensor(l, i, "mix.k.norm", g->dim, 0), g->dim);
+    else L->col_k = L->col_v = WR_HIP_MIX_NO_KEYS;
+    read_window_out(l, i, L);
+}
+
+/* gate and up [rows][cols] to rows at, at + 1, ... of matrix z, interleaved by tiles of 16 */
+static void put_gated(loader *l, operand *o, uint32_t z, uint32_t at, const uint16_t *gate, const uint16_t *up, uint32_t rows,
+                      uint32_t cols)
+{
+    for (uint32_t r = 0; r < rows && l->st == WR_OK; r++) {
+        operand_put(l, o, z, at + r / 16 * 32 + r % 16, gate + (size_t)r * cols, 1, cols);
+        operand_put(l, o, z, at + r / 16 * 32 + 16 + r % 16, up + (size_t)r * cols, 1, cols);
+    }
+}
+
 static void read_dense(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *L)
 {
     const uint32_t W = l->mm->width, Wp = l->mm->width_p;
@@ -524,10 +667,7 @@ static void read_dense(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *
     L->ff_p = p32(L->ff);
     const uint16_t *gate = ltensor(l, i, "mlp.gate", L->ff, W), *up = ltensor(l, i, "mlp.up", L->ff, W);
     operand o = operand_new(l, 1, 2 * L->ff_p, Wp);
-    for (uint32_t r = 0; r < L->ff && l->st == WR_OK; r++) {
-        operand_put(l, &o, 0, r / 16 * 32 + r % 16, gate + (size_t)r * W, 1, W);
-        operand_put(l, &o, 0, r / 16 * 32 + 16 + r % 16, up + (size_t)r * W, 1, W);
-    }
+    put_gated(l, &o, 0, 0, gate, up, L->ff, W);
     L->w_gu = operand_up(l, &o);
     L->w_down = plain(l, ltensor(l, i, "mlp.down", W, L->ff), W, L->ff, Wp);
 }
@@ -539,20 +679,83 @@ static void read_moe(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *L)
     const wrh_json *ex = need_obj(l, c, "expert"), *ro = need_obj(l, c, "router");
     if (l->st != WR_OK) return;
     L->ff = need_u32(l, ex, "ff", 1, DIM_MAX);
-    L->experts = need_u32(l, ro, "experts", 1, WR_HIP_MIX_MAX_EXPERTS);
-    L->top = need_u32(l, ro, "top", 1, WR_HIP_MIX_MAX_TOP);
-    if (l->st == WR_OK && L->top > L->experts) fail(l, WR_ERR_FORMAT, "config: layer %u: more experts per token than experts", i);
+    wr_hip_mix_router *q = &L->router;
+    q->experts = need_u32(l, ro, "experts", 1, WR_HIP_MIX_MAX_EXPERTS);
+    q->top = need_u32(l, ro, "top", 1, WR_HIP_MIX_MAX_TOP);
+    if (l->st == WR_OK && q->top > q->experts) fail(l, WR_ERR_FORMAT, "config: layer %u: more experts per token than experts", i);
     if (l->st != WR_OK) return;
     L->ff_p = p32(L->ff);
-    L->experts_p = p16(L->experts);
-    L->w_router = plain(l, ltensor(l, i, "mlp.router", L->experts, W), L->experts, W, L->experts_p);
-    operand up = operand_new(l, L->experts, L->ff_p, Wp), down = operand_new(l, L->experts, Wp, L->ff_p);
-    for (uint32_t x = 0; x < L->experts && l->st == WR_OK; x++) {
+    L->router_p = p16(q->experts);
+    L->w_router = plain(l, ltensor(l, i, "mlp.router", q->experts, W), q->experts, W, L->router_p);
+    operand up = operand_new(l, q->experts, L->ff_p, Wp), down = operand_new(l, q->experts, Wp, L->ff_p);
+    for (uint32_t x = 0; x < q->experts && l->st == WR_OK; x++) {
         char nb[64];
         snprintf(nb, sizeof nb, "mlp.e%u.up", x);
         operand_put(l, &up, x, 0, ltensor(l, i, nb, L->ff, W), L->ff, W);
         snprintf(nb, sizeof nb, "mlp.e%u.down", x);
         operand_put(l, &down, x, 0, ltensor(l, i, nb, W, L->ff), W, L->ff);
+    }
+    L->w_eup = operand_up(l, &up);
+    L->w_edown = operand_up(l, &down);
+}
+
+/* Clamped gated experts behind a corrected softmax router with groups and outputs that pass the input on; a shared
+ * expert with a gate of its own. */
+static void read_grouped_moe(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *L)
+{
+    const uint32_t W = l->mm->width, Wp = l->mm->width_p;
+    L->mlp = WRH_MLP_MOE;
+    const wrh_json *ex = need_obj(l, c, "expert"), *ro = need_obj(l, c, "router"), *sh = given(c, "shared");
+    if (l->st != WR_OK) return;
+    wr_hip_mix_router *q = &L->router;
+    L->ff = need_u32(l, ex, "ff", 1, DIM_MAX);
+    L->limit = (float)need_num(l, ex, "limit");
+    q->experts = need_u32(l, ro, "experts", 1, WR_HIP_MIX_MAX_EXPERTS);
+    q->top = need_u32(l, ro, "top", 1, WR_HIP_MIX_MAX_TOP);
+    q->identity = given(ro, "identity") ? need_u32(l, ro, "identity", 0, WR_HIP_MIX_MAX_EXPERTS) : 0;
+    q->scale = (float)need_num(l, ro, "scale");
+    q->softmax_all = 1;
+    const uint32_t outputs = q->experts + q->identity;
+    if (l->st == WR_OK && outputs > WR_HIP_MIX_MAX_EXPERTS) fail(l, WR_ERR_LIMIT, "config: layer %u: %u router outputs", i, outputs);
+    const wrh_json *groups = given(ro, "groups");
+    if (groups) {
+        q->groups = need_u32(l, groups, "count", 1, WR_HIP_MIX_MAX_GROUPS);
+        q->keep = need_u32(l, groups, "keep", 1, q->groups);
+        if (l->st == WR_OK && outputs % q->groups)
+            fail(l, WR_ERR_FORMAT, "config: layer %u: %u router outputs in %u groups", i, outputs, q->groups);
+    }
+    uint32_t shared = 0;
+    if (sh) {
+        shared = need_u32(l, sh, "ff", 1, DIM_MAX);
+        L->shared_limit = (float)need_num(l, sh, "limit");
+        q->shared_gate = 1;
+    }
+    if (l->st != WR_OK) return;
+    if (q->top > (q->groups ? outputs / q->groups * q->keep : outputs) || L->limit <= 0 || (sh && L->shared_limit <= 0)) {
+        fail(l, WR_ERR_FORMAT, "config: layer %u: %u of %u router outputs, limits %g and %g", i, q->top, outputs, L->limit, L->shared_limit);
+        return;
+    }
+    L->ff_p = p32(L->ff);
+    L->shared_p = p32(shared);
+    L->router_p = p32(outputs + q->shared_gate);
+    operand o = operand_new(l, 1, L->router_p + 2 * L->shared_p, Wp);
+    operand_put(l, &o, 0, 0, ltensor(l, i, "mlp.router", outputs, W), outputs, W);
+    if (sh) {
+        operand_put(l, &o, 0, outputs, ltensor(l, i, "mlp.shared.sg", 1, W), 1, W);
+        const uint16_t *gate = ltensor(l, i, "mlp.shared.gate", shared, W), *up = ltensor(l, i, "mlp.shared.up", shared, W);
+        put_gated(l, &o, 0, L->router_p, gate, up, shared, W);
+        L->w_down = plain(l, ltensor(l, i, "mlp.shared.down", W, shared), W, shared, Wp);
+    }
+    L->w_router = operand_up(l, &o);
+    q->correction = vec_put(l, ltensor(l, i, "mlp.correction", outputs, 0), outputs);
+    operand up = operand_new(l, q->experts, 2 * L->ff_p, Wp), down = operand_new(l, q->experts, Wp, L->ff_p);
+    for (uint32_t x = 0; x < q->experts && l->st == WR_OK; x++) {
+        char nb[3][64];
+        static const char *const ends[] = {"gate", "up", "down"};
+        for (uint32_t k = 0; k < 3; k++) snprintf(nb[k], sizeof nb[k], "mlp.e%u.%s", x, ends[k]);
+        const uint16_t *g = ltensor(l, i, nb[0], L->ff, W), *u = ltensor(l, i, nb[1], L->ff, W);
+        put_gated(l, &up, x, 0, g, u, L->ff, W);
+        operand_put(l, &down, x, 0, ltensor(l, i, nb[2], W, L->ff), W, L->ff);
     }
     L->w_eup = operand_up(l, &up);
     L->w_edown = operand_up(l, &down);
@@ -571,8 +774,12 @@ static void read_layer(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *
     } mixers[] = {{"lightning", read_lightning, DESIGN_BIPOTAR},
                   {"latent_attention", read_latent, DESIGN_BIPOTAR},
                   {"wkv", read_wkv, DESIGN_TAREDRA},
-                  {"parallel", read_parallel, DESIGN_TAREDRA}},
-      mlps[] = {{"dense", read_dense, DESIGN_BIPOTAR | DESIGN_TAREDRA}, {"moe", read_moe, DESIGN_BIPOTAR}};
+                  {"parallel", read_parallel, DESIGN_TAREDRA},
+                  {"attention", read_window_keys, DESIGN_FEDIRAX},
+                  {"attention_2", read_window_difference, DESIGN_FEDIRAX}},
+      mlps[] = {{"dense", read_dense, DESIGN_BIPOTAR | DESIGN_TAREDRA},
+                {"moe", read_moe, DESIGN_BIPOTAR},
+                {"moe", read_grouped_moe, DESIGN_FEDIRAX}};
     const size_t n_mixers = sizeof mixers / sizeof *mixers, n_mlps = sizeof mlps / sizeof *mlps;
     const wrh_mix_design *d = l->design;
     size_t k = 0;
@@ -653,6 +860,15 @@ static void plan_runs(loader *l, const wrh_json *cfg)
             mm->runs[r].store2 = mm->n_state;
             mm->state_elems[mm->n_state++] = matrix;
             break;
+        case WRH_MIXER_WINDOW:
+            if (L->kv_from >= 0) {                         /* the pages of that layer's last run before this one */
+                for (uint32_t k = 0; k < r; k++)
+                    if (mm->runs[k].layer == (uint32_t)L->kv_from) mm->runs[r].store = mm->runs[k].store;
+                break;
+            }
+            mm->runs[r].store = mm->n_latent;
+            mm->latent_dim[mm->n_latent++] = L->win.kv_heads * (L->win.maps * L->win.dim_pad + L->win.vdim_pad);
+            break;
         }
     }
 }
@@ -671,7 +887,8 @@ static void upload_small(loader *l)
     for (uint32_t i = 0; i < mm->n_layers; i++) {
         wrh_mix_layer *L = &mm->layers[i];
         const float **p[] = {&L->decay, &L->mix_norm, &L->dq_norm, &L->dkv_norm, &L->norm1, &L->norm1b, &L->norm2, &L->norm2b,
-                             &L->mu, &L->sink, &L->rec.w0, &L->rec.u, &L->rec.a_bias, &L->rec.norm};
+                             &L->mu, &L->sink, &L->rec.w0, &L->rec.u, &L->rec.a_bias, &L->rec.norm, &L->b_in, &L->win.q_norm,
+                             &L->win.k_norm, &L->router.correction};
         for (size_t k = 0; k < sizeof p / sizeof *p; k++) vec_fix(mm, p[k]);
     }
     for (uint32_t r = 0; r < mm->n_ropes && l->st == WR_OK; r++) {
@@ -804,7 +1021,7 @@ wr_status wrh_mix_load(wr_engine *e, const char *dir, const char *arch, const wr
             if (L->geo.window > m->sliding_window) m->sliding_window = L->geo.window;
             m->rope_base = (float)mm->ropes[L->rope].base;
         }
-        if (L->kind == WRH_MIXER_PARALLEL) {
+        if (L->kind == WRH_MIXER_PARALLEL || L->kind == WRH_MIXER_WINDOW) {
             m->has_swa = 1;
             if (L->win.kv_heads > m->n_kv) m->n_kv = L->win.kv_heads;
             if (L->win.window > m->sliding_window) m->sliding_window = L->win.window;

@@ -1,4 +1,4 @@
-"""Writes mixer-stack models (architectures "Bipotar" and "Taredra") as a folder with
+"""Writes mixer-stack models (architectures "Bipotar", "Taredra" and "Fedirax") as a folder with
 config.json and model.safetensors: random-init models for the tests and the benchmark, and any
 set of bfloat16 tensors a caller has."""
 from __future__ import annotations
@@ -38,12 +38,37 @@ def window_and_delta(heads: int, kv_heads: int, dim: int, vdim: int, window: int
                                           "left_scale": left_scale, "right_scale": right_scale}}
 
 
+def keys_as_values(heads: int, kv_heads: int, dim: int, window: int, rot_dims: int | None = None, base: float = 10000.0,
+                   scale: float | None = None, softcap: float | None = 30.0) -> dict:
+    """Grouped-query attention whose values are the keys ahead of their rotation."""
+    m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "mask": {"size": window},
+         "rot": {"base": base, "dims": dim if rot_dims is None else rot_dims}, "scale": dim ** -0.5 if scale is None else scale}
+    return {"type": "attention", "mixer": m if softcap is None else dict(m, softcap=softcap)}
+
+
+def difference(heads: int, kv_heads: int, dim: int, vdim: int, window: int, rot_dims: int | None = None, base: float = 10000.0,
+               scale: float | None = None, diff: float = 0.5, kv_from: int | None = None) -> dict:
+    """Attention of two maps per head, the second taken off the first."""
+    m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "mask": {"size": window}, "diff": diff,
+         "rot": {"base": base, "dims": dim if rot_dims is None else rot_dims}, "scale": dim ** -0.5 if scale is None else scale}
+    return {"type": "attention_2", "mixer": m if kv_from is None else dict(m, kv_from=kv_from)}
+
+
 def dense(ff: int) -> dict:
     return {"kind": "dense", "ff": ff}
 
 
 def moe(experts: int, top: int, ff: int) -> dict:
     return {"kind": "moe", "router": {"experts": experts, "top": top}, "expert": {"ff": ff}}
+
+
+def grouped_moe(experts: int, top: int, ff: int, identity: int = 0, groups=None, scale: float = 1.0, limit: float = 7.0,
+                shared=None) -> dict:
+    """groups: (count, keep) or None; shared: (ff, limit) of a shared expert, or None."""
+    return {"kind": "moe", "expert": {"ff": ff, "limit": limit},
+            "router": {"experts": experts, "identity": identity, "top": top, "scale": scale,
+                       "groups": None if groups is None else dict(zip(("count", "keep"), groups))},
+            "shared": None if shared is None else dict(zip(("ff", "limit"), shared))}
 
 
 def config(width: int, vocab: int, layers, loop=None, eps: float = 1e-6, logit_scale: float = 1.0) -> dict:
@@ -58,6 +83,42 @@ def prenorm_config(width: int, vocab: int, layers, eps: float = 1e-6, embed_scal
     return {"architecture": "Taredra", "width": width, "vocab": vocab, "norm": {"eps": eps},
             "embedding": {"scale": width ** 0.5 if embed_scale is None else embed_scale},
             "layers": [dict(m, mlp=f) for m, f in layers]}
+
+
+def shared_kv_config(width: int, vocab: int, layers, eps: float = 1e-6, embed_scale: float = 1.0) -> dict:
+    """layers: [(mixer, feed-forward or None)] of keys_as_values and difference mixers."""
+    return dict(prenorm_config(width, vocab, layers, eps, embed_scale), architecture="Fedirax")
+
+
+def _shared_kv_shapes(cfg: dict) -> dict:
+    W, out = cfg["width"], {"embed": (cfg["vocab"], cfg["width"])}
+    for i, layer in enumerate(cfg["layers"]):
+        p, m, f = f"l{i}.", layer["mixer"], layer["mlp"]
+        H, G, D, V = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        for n in ("norm1",) + (("norm2",) if f else ()):
+            out[p + n] = (W,)
+        q = p + "mix."
+        if layer["type"] == "attention":
+            out.update({q + "q": (H * D, W), q + "q.b": (H * D,), q + "k": (G * D, W), q + "k.b": (G * D,), q + "sink": (H,),
+                        q + "g": (H, W), q + "o": (W, H * D)})
+        else:
+            out.update({q + "q": (H * 2 * D, W), q + "q.norm": (D,)})
+            if m.get("kv_from") is None:
+                out.update({q + "k": (G * 2 * D, W), q + "v": (G * V, W), q + "k.norm": (D,)})
+            out.update({q + n: (D,) for n in ("lq1", "lk1", "lq2", "lk2")})
+            out[q + "o"] = (W, H * V)
+        if f:
+            r, q = f["router"], p + "mlp."
+            parts = [(f"e{e}.", f["expert"]["ff"]) for e in range(r["experts"])]
+            if f["shared"]:
+                parts.append(("shared.", f["shared"]["ff"]))
+                out[q + "shared.sg"] = (1, W)
+            out.update({q + "router": (r["experts"] + r["identity"], W), q + "correction": (r["experts"] + r["identity"],)})
+            for n, ff in parts:
+                out.update({q + n + "gate": (ff, W), q + n + "up": (ff, W), q + n + "down": (W, ff)})
+    out["final.norm"] = (W,)
+    out["head"] = (cfg["vocab"], W)
+    return out
 
 
 def _recur_shapes(p: str, hd: int, W: int, rank: int) -> dict:
@@ -95,6 +156,8 @@ def tensor_shapes(cfg: dict, rank: int = 24) -> dict:
     """`rank`: of the decays' low-rank products, which no configuration names."""
     if cfg["architecture"] == "Taredra":
         return _prenorm_shapes(cfg, rank)
+    if cfg["architecture"] == "Fedirax":
+        return _shared_kv_shapes(cfg)
     W, out = cfg["width"], {"embed": (cfg["vocab"], cfg["width"]), "embed.norm": (cfg["width"],)}
     for i, layer in enumerate(cfg["layers"]):
         p, m, f = f"l{i}.", layer["mixer"], layer["mlp"]
@@ -128,14 +191,16 @@ def to_bf16(x: np.ndarray) -> np.ndarray:
 
 
 # what the vectors of a pre-norm model are drawn around, and how widely
-_VECTORS = {"norm1": (0, 0.1), "norm2": (0, 0.1), "final.norm": (0, 0.1), "sink": (0, 1), "w0": (-3, 2), "a.b": (0, 1)}
+_VECTORS = {"norm1": (0, 0.1), "norm2": (0, 0.1), "final.norm": (0, 0.1), "sink": (0, 1), "w0": (-3, 2), "a.b": (0, 1),
+            "q.b": (0, 0.5), "k.b": (0, 0.5), "correction": (0, 0.05), "lq1": (0, 0.1), "lk1": (0, 0.1), "lq2": (0, 0.1),
+            "lk2": (0, 0.1)}
 
 
 def random_tensors(cfg: dict, seed: int = 0, gain: float = 1.0, rank: int = 24):
     """Yields (name, bfloat16 bits): norms 1 + 0.1 N(0, 1), matrices gain * N(0, 1 / inputs), the embedding N(0, 1);
     of a pre-norm model the vectors as _VECTORS says, mixing factors in [0, 1], bonuses N(0, 1/4), the embedding N(0, 1 / width).
     Large matrices repeat a pool of samples at different offsets."""
-    prenorm = cfg["architecture"] == "Taredra"
+    prenorm = cfg["architecture"] != "Bipotar"
     rng = np.random.default_rng(seed)
     pool = rng.standard_normal(1 << 22, dtype=np.float32)
     for i, (name, shape) in enumerate(tensor_shapes(cfg, rank).items()):
@@ -148,7 +213,7 @@ def random_tensors(cfg: dict, seed: int = 0, gain: float = 1.0, rank: int = 24):
             x = 1.0 / (1.0 + np.exp(-x))
         elif prenorm and end == "u":
             x = 0.5 * x
-        elif prenorm and name == "embed":
+        elif prenorm and name == "embed" and cfg["architecture"] == "Taredra":
             x = x * np.float32(shape[1] ** -0.5)
         elif prenorm and end in _VECTORS:
             at, spread = _VECTORS[end]
