@@ -202,12 +202,14 @@ def mixer_workload(args) -> None:
     from wayruntime_amd import mix_timing
 
     steps = min(args.steps, 200)
-    kind = "taredra" if args.workload == "taredra" else "mixer"
-    beside = ("mixer", "gqa") if kind == "taredra" else ("gqa",)
+    kind = args.workload
+    beside = {"mixer": ("gqa",), "taredra": ("mixer", "gqa"), "fedirax": ("mixer", "taredra", "gqa")}[kind]
     model = {"mixer": "Bipotar, 4 layers (linear attention x 2, latent attention x 2; dense and expert feed-forwards), "
                       "width 4096, random init",
              "taredra": "Taredra, 4 layers (windowed attention beside a delta-rule recurrence x 2, wkv recurrence x 2; dense "
-                        "feed-forwards), width 4096, random init"}[kind]
+                        "feed-forwards), width 4096, random init",
+             "fedirax": "Fedirax, 4 layers (differential attention x 2, one more over the first's keys and values, "
+                        "keys-as-values attention; expert feed-forwards), width 4096, random init"}[kind]
     figures = mix_timing.run(list(mix_timing.SIZES), reps=3, steps=steps, only=(kind,) + beside,
                              log=lambda *a: print(*a, file=sys.stderr, flush=True))
     top = figures["w4096"][kind]
@@ -238,7 +240,7 @@ def main() -> None:
     ap.add_argument("--no-decode-configs", action="store_true")
     ap.add_argument("--keys-per-wg", type=int, default=0)
     ap.add_argument("--workload", default="headline",
-                    choices=["headline", "ragged16", "long16", "long16-hd256", "batch1", "mixer", "taredra"],
+                    choices=["headline", "ragged16", "long16", "long16-hd256", "batch1", "mixer", "taredra", "fedirax"],
                     help="headline: 16 sessions x --ctx, 32/8/128 (the metric's configuration), with "
                          "the other decode workloads as secondary keys; "
                          "ragged16: 16 sessions with contexts drawn from [256, 4096]; "
@@ -247,7 +249,8 @@ def main() -> None:
                          "run that one workload as the timed steps and report the decode figures only; "
                          "mixer: prefill and decode throughput of mixer-stack models (Bipotar) with layers "
                          "of real sizes, random weights, beside a grouped-query model of the same width; "
-                         "taredra: the same of Taredra models, beside both")
+                         "taredra: the same of Taredra models, beside both; "
+                         "fedirax: the same of Fedirax models, beside all three")
     args = ap.parse_args()
 
     if args.gpus != 1:
@@ -255,7 +258,7 @@ def main() -> None:
               "(nothing here uses a second device)" % args.gpus, file=sys.stderr)
         sys.exit(2)
 
-    if args.workload in ("mixer", "taredra"):
+    if args.workload in ("mixer", "taredra", "fedirax"):
         mixer_workload(args)
         return
 

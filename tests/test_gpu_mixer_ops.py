@@ -11,7 +11,7 @@ from wayruntime_amd import hipattn
 
 pytestmark = pytest.mark.gpu
 
-ROWS_F32, ROWS, FRAG, SPLIT, GATED = range(5)
+ROWS_F32, ROWS, FRAG, SPLIT, GATED, SPLIT_GATED = range(6)
 u32, vp = C.c_uint32, C.c_void_p
 
 
@@ -19,7 +19,8 @@ class Gemm(C.Structure):
     _fields_ = [("w", vp), ("x", vp), ("x_kt", u32), ("x_kt_z", u32), ("rows", u32), ("group_expert", vp),
                 ("tile_groups", u32), ("out", u32), ("y_f32", vp), ("y_act", vp), ("ldy", u32), ("h", vp), ("h_kt", u32),
                 ("col_z", u32), ("n_split", u32), ("silu_end", u32), ("sigmoid_end", u32), ("relu2", u32), ("scale", C.c_float),
-                ("tanh_end", u32), ("gelu", u32), ("x_kt0", u32)]
+                ("tanh_end", u32), ("gelu", u32), ("x_kt0", u32), ("bias", vp), ("limit", C.c_float), ("slope", C.c_float),
+                ("up_bias", C.c_float), ("x_perm", vp)]
 
 
 @pytest.fixture(scope="module")
@@ -112,8 +113,12 @@ def test_rows_out(lib, f32, N, K, rows):
     act[:, :N // 4] = O.silu(want[:, :N // 4])
     act[:, N // 4:N - 7] = np.tanh(want[:, N // 4:N - 7])
     r.close(y.to_host((rows, N)), act)
+    bias = r.rng.standard_normal(N).astype(np.float32)
+    bd = hipattn.DeviceBuffer.from_host(bias)
+    r.go(xd, out=ROWS_F32, y_f32=y.p, ldy=N, bias=bd.p)
+    r.close(y.to_host((rows, N)), want + bias)
     r.end()
-    for b in (y, xd):
+    for b in (y, xd, bd):
         b.free()
 
 
@@ -138,6 +143,20 @@ def test_frag_split_and_gated_out(lib, f32, N, K, rows):
     r.close(r.frag_down(h, rows, N // 2), (O.silu(t[:, :, 0]) * t[:, :, 1]).reshape(rows, -1), eight_bits=True)
     r.go(xd, out=GATED, h=h.p, h_kt=N // 64, gelu=1)
     r.close(r.frag_down(h, rows, N // 2), (O.gelu_tanh(t[:, :, 0]) * t[:, :, 1]).reshape(rows, -1), eight_bits=True)
+
+    def clamped(g, u, limit, slope, more):
+        g = np.minimum(g, limit)
+        return g * O.sigmoid(slope * g) * (np.clip(u, -limit, limit) + more)
+    for limit in (0.3, 5.0):
+        r.go(xd, out=GATED, h=h.p, h_kt=N // 64, limit=limit, slope=1.5, up_bias=0.75)
+        r.close(r.frag_down(h, rows, N // 2), clamped(t[:, :, 0], t[:, :, 1], limit, 1.5, 0.75).reshape(rows, -1), eight_bits=True)
+    # rows ahead of the gated outputs
+    for split in (32, N // 2 // 32 * 32):
+        r.go(xd, out=SPLIT_GATED, h=h.p, h_kt=(N - split) // 64 + 1, n_split=split, y_f32=y.p, ldy=split, limit=0.6, slope=2.0, up_bias=1.0)
+        r.close(y.to_host((rows, split)), want[:, :split])
+        u = want[:, split:].reshape(rows, -1, 2, 16)
+        got = r.frag_down(h, rows, ((N - split) // 64 + 1) * 32)[:, :(N - split) // 2]
+        r.close(got, clamped(u[:, :, 0], u[:, :, 1], 0.6, 2.0, 1.0).reshape(rows, -1), eight_bits=True)
     r.end()
     for b in (y, xd, h):
         b.free()
@@ -181,6 +200,20 @@ def test_matrix_per_row_group(lib, f32, N, K, tile):
         if e >= 0:
             want[16 * g:16 * g + 16] = x[16 * g:16 * g + 16].astype(np.float64) @ r.w[e].T.astype(np.float64)
     r.close(y.to_host((rows, N)), want)
+    if tile == 1:                                          # rows picked one by one out of fewer
+        pick = r.rng.integers(0, 21, rows).astype(np.uint32)
+        used = r.rng.random(rows) < 0.8
+        few = r.act(21, K)
+        fd = r.up(few)
+        pd = hipattn.DeviceBuffer.from_host(np.where(used, pick, np.uint32(0xFFFFFFFF)).astype(np.uint32).view(np.float32))
+        r.go(fd, rows=rows, group_expert=gd.p, tile_groups=1, out=ROWS_F32, y_f32=y.p, ldy=N, x_perm=pd.p)
+        got = y.to_host((rows, N))
+        for g, e in enumerate(which):
+            for i in range(16 * g, 16 * g + 16):
+                if e >= 0 and used[i]:
+                    r.close(got[i], few[pick[i]].astype(np.float64) @ r.w[e].T.astype(np.float64))
+        for b in (fd, pd):
+            b.free()
     r.end()
     for b in (xd, gd, y):
         b.free()
@@ -191,7 +224,8 @@ def test_refusals(lib):
     y = hipattn.DeviceBuffer(16 * 32 * 4)
     ok = dict(w=r.h, x=y.p, x_kt=1, rows=16, out=ROWS_F32, y_f32=y.p, ldy=32)
     for change in (dict(x_kt=0), dict(ldy=28), dict(ldy=33), dict(y_f32=None), dict(out=9), dict(rows=0), dict(w=None),
-                   dict(out=FRAG, h=y.p, h_kt=0), dict(out=SPLIT, h=y.p, h_kt=1, n_split=8), dict(out=GATED), dict(x_kt0=1)):
+                   dict(out=FRAG, h=y.p, h_kt=0), dict(out=SPLIT, h=y.p, h_kt=1, n_split=8), dict(out=GATED), dict(x_kt0=1),
+                   dict(out=GATED, h=y.p, h_kt=1, bias=y.p), dict(x_perm=y.p), dict(out=SPLIT_GATED, h=y.p, h_kt=1, n_split=16)):
         assert lib.wr_hip_mix_gemm_run(0, C.byref(Gemm(**dict(ok, **change)))) == hipattn.ERR_INVAL, change
     h = vp()
     for shape in ((1, 8, 32), (1, 16, 16), (0, 16, 32)):

@@ -2,12 +2,14 @@
 real sizes) beside a grouped-query model of the same width, through the host
 engine.
 
-    python -m wayruntime_amd.mix_timing [--size w2048 w4096] [--only mixer taredra gqa] [--json]
+    python -m wayruntime_amd.mix_timing [--size w2048 w4096] [--only mixer taredra fedirax gqa] [--json]
 
 Each size has four layers.  mixer: linear attention with a dense feed-forward and
 with experts, latent attention with experts and with a dense feed-forward.
 taredra: windowed grouped-query attention beside a delta-rule recurrence, and a
-wkv recurrence, each twice, all with dense feed-forwards.  gqa: the engine's
+wkv recurrence, each twice, all with dense feed-forwards.  fedirax: differential
+attention, keys-as-values attention, differential attention and such over the first
+layer's keys and values, all with experts and a shared one.  gqa: the engine's
 Llama-style model with four layers of the same width, head dimension and
 feed-forward width (F16 weights)."""
 from __future__ import annotations
@@ -40,12 +42,23 @@ def taredra_config(width: int, heads: int, ff: int) -> dict:
     return mw.prenorm_config(width, VOCAB, [(m, mw.dense(ff)) for m in (par, mw.wkv(width // 64, 64)) * 2])
 
 
-KINDS = ("mixer", "taredra", "gqa")
+def fedirax_config(width: int, heads: int, experts: int, top: int, expert_ff: int, shared_ff: int) -> dict:
+    """Two maps of 64 per head over values of 128, eight key/value heads; an eighth of the outputs pass the input on."""
+    diff = dict(heads=heads, kv_heads=8, dim=64, vdim=128, window=4096)
+    keys = mw.keys_as_values(heads, 8, 128, window=4096)
+    moe = mw.grouped_moe(experts, top, expert_ff, identity=experts // 8, groups=(8, 4), scale=2.0, shared=(shared_ff, 7.0))
+    return mw.shared_kv_config(width, VOCAB, [(m, moe) for m in (mw.difference(**diff), keys, mw.difference(**diff),
+                                                                 mw.difference(**diff, kv_from=0))])
+
+
+KINDS = ("mixer", "taredra", "fedirax", "gqa")
 RANK = 64                                   # of the decays' low-rank products
 SIZES = {
     "w2048": (mixer_config(2048, 16, 768, 8192, 64, 6, 1024), taredra_config(2048, 16, 8192),
+              fedirax_config(2048, 16, 64, 6, 1024, 2048),
               gw.ModelShape(arch="llama", n_layers=4, hidden=2048, ffn=8192, n_q=16, n_kv=8, vocab=VOCAB, context=8192)),
     "w4096": (mixer_config(4096, 32, 1536, 12288, 32, 4, 2048), taredra_config(4096, 32, 12288),
+              fedirax_config(4096, 32, 32, 4, 2048, 4096),
               gw.ModelShape(arch="llama", n_layers=4, hidden=4096, ffn=12288, n_q=32, n_kv=8, vocab=VOCAB, context=8192)),
 }
 
@@ -106,16 +119,16 @@ def run(sizes, reps: int = 3, steps: int = 40, only=KINDS, log=print) -> dict:
     with tempfile.TemporaryDirectory() as tmp:
         eng = E.Engine(E.HOST_SO)
         for name in sizes:
-            mixer, taredra, shape = SIZES[name]
+            models = dict(zip(KINDS, SIZES[name]))
             fig = figures[name] = {}
             for kind in only:
                 t = time.perf_counter()
                 path = os.path.join(tmp, name + "_" + kind)
                 if kind == "gqa":
                     path += ".gguf"
-                    gw.write_model(path, shape)
+                    gw.write_model(path, models[kind])
                 else:
-                    mw.write_model(path, mixer if kind == "mixer" else taredra, rank=RANK)
+                    mw.write_model(path, models[kind], rank=RANK)
                 log(f"{name}: {kind} model written in {time.perf_counter() - t:.1f} s")
                 fig[kind] = measure(eng, path, reps, steps)
                 log(f"{name}: {kind} {fig[kind]}")
