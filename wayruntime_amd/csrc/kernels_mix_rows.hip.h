@@ -105,14 +105,24 @@ __device__ __forceinline__ void mix_sub_chunk(const MixRowArgs& a, uint32_t r, u
     }
 #pragma unroll
     for (int j = 0; j < 8; j++) v[j] = 0.f;
-    for (uint32_t t = 0; t < a.top; t++) {
-        const float gt = a.gate[(size_t)r * a.top + t];
-        const uint32_t slot = a.slot[(size_t)r * a.top + t];
-        if (slot == 0xFFFFFFFFu) continue;
-        float e[8];
-        mix_load8(a.y + (size_t)slot * a.wpad + q * 8, e);
+    for (uint32_t t0 = 0; t0 < a.top; t0 += 4) {           // four experts' rows in flight
+        float gt[4], e[4][8];
+        uint32_t slot[4];
 #pragma unroll
-        for (int j = 0; j < 8; j++) v[j] = fmaf(gt, e[j], v[j]);
+        for (uint32_t i = 0; i < 4; i++) {
+            const size_t at = (size_t)r * a.top + min(t0 + i, a.top - 1);
+            gt[i] = a.gate[at];
+            slot[i] = t0 + i < a.top ? a.slot[at] : 0xFFFFFFFFu;
+        }
+#pragma unroll
+        for (uint32_t i = 0; i < 4; i++)
+            if (slot[i] != 0xFFFFFFFFu) mix_load8(a.y + (size_t)slot[i] * a.wpad + q * 8, e[i]);
+#pragma unroll
+        for (uint32_t i = 0; i < 4; i++)
+            if (slot[i] != 0xFFFFFFFFu) {
+#pragma unroll
+                for (int j = 0; j < 8; j++) v[j] = fmaf(gt[i], e[i][j], v[j]);
+            }
     }
     if (!a.side) return;
     float e[8];
@@ -487,28 +497,28 @@ __device__ __forceinline__ float mix_wave_max(float v)
 }
 
 // One wave: the `top` outputs of a row with the largest choice value (lowest index among equals) and their weights.
-// Lane l holds outputs l, l + 64, ...
-__device__ __forceinline__ void mix_top(const MixRouteArgs& a, uint32_t row, int lane)
+// Lane l holds outputs l, l + 64, ...; put(t, output) is called by lane t.
+template <int PER, typename Put>
+__device__ __forceinline__ void mix_top(const MixRouteArgs& a, uint32_t row, int lane, Put put)
 {
-    constexpr int PER = (int)(1024 / 64);
-    float v[PER];
+    float v[PER], s[PER];                                  // choice values (NaN: none, or taken) and softmax terms
     const float* z = a.z + (size_t)row * a.ldz;
+    const float shared = a.shared_gate ? z[a.outputs] : 0.f;
 #pragma unroll
     for (int i = 0; i < PER; i++) {
         const uint32_t e = lane + 64 * i;
-        v[i] = e < a.outputs ? z[e] : -INFINITY;
+        v[i] = e < a.outputs ? z[e] : __builtin_nanf("");
     }
-    float zmax = 0.f, zinv = 1.f;
+    float zinv = 1.f;
     if (a.softmax_all) {                                   // choice: the softmax over all outputs, corrected
-        zmax = v[0];
+        float zmax = v[0], zs = 0.f;
 #pragma unroll
         for (int i = 1; i < PER; i++) zmax = fmaxf(zmax, v[i]);
         zmax = mix_wave_max(zmax);
-        float zs = 0.f;
 #pragma unroll
         for (int i = 0; i < PER; i++) {
-            v[i] = expf(v[i] - zmax);                      // (zero past the outputs)
-            zs += v[i];
+            s[i] = lane + 64u * i < a.outputs ? expf(v[i] - zmax) : 0.f;
+            zs += s[i];
         }
 #pragma unroll
         for (int off = 32; off >= 1; off >>= 1) zs += wave_xor_f32(zs, off);
@@ -516,7 +526,7 @@ __device__ __forceinline__ void mix_top(const MixRouteArgs& a, uint32_t row, int
 #pragma unroll
         for (int i = 0; i < PER; i++) {
             const uint32_t e = lane + 64 * i;
-            if (e < a.outputs) v[i] = v[i] * zinv + (a.correction ? a.correction[e] : 0.f);
+            if (e < a.outputs) v[i] = s[i] * zinv + (a.correction ? a.correction[e] : 0.f);
         }
     }
     if (a.kinds) {                                         // lane g holds the largest choice value of group g
@@ -534,7 +544,7 @@ __device__ __forceinline__ void mix_top(const MixRouteArgs& a, uint32_t row, int
         }
         uint32_t ahead = 0;                                // groups that are better than this lane's
         for (uint32_t k = 0; k < a.kinds; k++) {
-            const float other = __shfl(mine, (int)k, 64);
+            const float other = __int_as_float(__builtin_amdgcn_readlane(__float_as_int(mine), k));
             ahead += other > mine || (other == mine && k < (uint32_t)lane);
         }
         const uint64_t kept = __ballot((uint32_t)lane < a.kinds && ahead < a.keep);
@@ -544,92 +554,101 @@ __device__ __forceinline__ void mix_top(const MixRouteArgs& a, uint32_t row, int
             if (e < a.outputs && !((kept >> (e / size)) & 1u)) v[i] = -INFINITY;
         }
     }
-    uint32_t taken = 0;                                    // bit i: this lane's output i is chosen
     float best0 = 0.f, sum = 0.f, mine = 0.f, own = 0.f;
     for (uint32_t t = 0; t < a.top; t++) {
-        float bv = -INFINITY;
-        uint32_t be = 0xFFFFFFFFu;
+        float bv = v[0];
 #pragma unroll
-        for (int i = 0; i < PER; i++) {
-            const uint32_t e = lane + 64 * i;
-            if (e < a.outputs && !((taken >> i) & 1u) && (be == 0xFFFFFFFFu || v[i] > bv)) {
-                bv = v[i];
-                be = e;
-            }
-        }
+        for (int i = 1; i < PER; i++) bv = fmaxf(bv, v[i]);
+        bv = mix_wave_max(bv);
+        uint32_t be = a.outputs - 1;                       // (NaN logits: still an output)
 #pragma unroll
-        for (int off = 32; off >= 1; off >>= 1) {
-            const float ov = __shfl_xor(bv, off, 64);
-            const uint32_t oe = (uint32_t)__shfl_xor((int)be, off, 64);
-            if (oe != 0xFFFFFFFFu && (be == 0xFFFFFFFFu || ov > bv || (ov == bv && oe < be))) {
-                bv = ov;
-                be = oe;
-            }
+        for (int i = PER - 1; i >= 0; i--) {
+            const uint64_t at = __ballot(v[i] == bv);
+            if (at) be = 64 * i + __ffsll((unsigned long long)at) - 1;
         }
-        be = min(be, a.outputs - 1);                       // NaN logits: still an output
-        if ((be & 63u) == (uint32_t)lane) taken |= 1u << (be >> 6);
+        float term = 0.f;
+#pragma unroll
+        for (int i = 0; i < PER; i++)
+            if (lane + 64u * i == be) {
+                v[i] = __builtin_nanf("");
+                if (a.softmax_all) term = s[i];
+            }
         if (t == 0) best0 = bv;
-        const float g = a.softmax_all ? expf(z[be] - zmax) * zinv : expf(bv - best0);
+        const float g = a.softmax_all ? __int_as_float(__builtin_amdgcn_readlane(__float_as_int(term), be & 63u)) * zinv : expf(bv - best0);
         sum += g;
         if (be >= a.experts) own += g;
         if ((uint32_t)lane == t) {
             mine = g;
-            a.slot[(size_t)row * a.top + t] = be;
+            put(t, be);
         }
     }
     const float over = a.softmax_all ? a.scale / (sum + 1e-20f) : 1.0f;
     if ((uint32_t)lane < a.top) a.gate[(size_t)row * a.top + lane] = a.softmax_all ? mine * over : mine / sum;
     if (a.side && lane == 0) {
         a.side[(size_t)row * 2] = a.softmax_all ? own * over : own / sum;
-        a.side[(size_t)row * 2 + 1] = a.shared_gate ? 1.0f / (1.0f + expf(-z[a.outputs])) : 0.f;
+        a.side[(size_t)row * 2 + 1] = a.shared_gate ? 1.0f / (1.0f + expf(-shared)) : 0.f;
     }
 }
 
+template <int PER>
 __global__ __launch_bounds__(256) void mix_top_kernel(const MixRouteArgs a)
 {
     const uint32_t row = blockIdx.x * 4 + (threadIdx.x >> 6);
-    if (row < a.rows) mix_top(a, row, threadIdx.x & 63);
+    if (row < a.rows) mix_top<PER>(a, row, threadIdx.x & 63, [&](uint32_t t, uint32_t e) { a.slot[(size_t)row * a.top + t] = e; });
 }
+
+constexpr uint32_t kOrderRows = 64, kOrderPairs = kOrderRows * 64;      // of a step whose choice is made with the order
 
 // One workgroup: orders the chosen (row, expert) pairs by expert.  Each expert's
 // pairs take whole runs of tile_groups groups of 16 slots.  Which slot of its
 // expert a pair gets may differ from run to run; nothing computed for it does
 // (a slot's column of a matrix product depends on that column alone).
-template <bool TOP>
+// PER: outputs a lane holds where the choice is made here too (few rows), else 0.
+template <int PER>
 __global__ __launch_bounds__(1024) void mix_order_kernel(const MixRouteArgs a)
 {
-    __shared__ uint32_t count[1024], base[1024], scan[1024];
-    const uint32_t t = threadIdx.x;
-    if constexpr (TOP)                                     // few rows: the choice is made here too
-        for (uint32_t r = t >> 6; r < a.rows; r += 16) mix_top(a, r, t & 63);
-    count[t] = 0;
+    constexpr bool TOP = PER > 0;
+    __shared__ uint32_t count[1024], wave_sum[16];
+    __shared__ uint16_t pick[TOP ? kOrderPairs : 1];
+    const uint32_t t = threadIdx.x, lane = t & 63, wave = t >> 6;
     const uint32_t n_slots = a.n_groups * 16, pairs = a.rows * a.top, run = a.tile_groups * 16;
+    count[t] = 0;
     for (uint32_t i = t; i < n_slots; i += 1024) a.perm[i] = 0xFFFFFFFFu;
     for (uint32_t i = t; i < a.n_groups; i += 1024) a.group_expert[i] = -1;
     __syncthreads();
-    for (uint32_t i = t; i < pairs; i += 1024)
-        if (a.slot[i] < a.experts) atomicAdd(&count[a.slot[i]], 1u);
+    if constexpr (TOP) {
+        for (uint32_t r = wave; r < a.rows; r += 16)
+            mix_top<PER>(a, r, lane, [&](uint32_t k, uint32_t e) {
+                pick[r * a.top + k] = (uint16_t)e;
+                if (e < a.experts) atomicAdd(&count[e], 1u);
+            });
+    } else {
+        for (uint32_t i = t; i < pairs; i += 1024)
+            if (a.slot[i] < a.experts) atomicAdd(&count[a.slot[i]], 1u);
+    }
     __syncthreads();
     const uint32_t mine = (count[t] + run - 1) / run * run;
-    scan[t] = mine;
-    __syncthreads();
-    for (uint32_t off = 1; off < 1024; off <<= 1) {
-        const uint32_t v = t >= off ? scan[t - off] : 0;
-        __syncthreads();
-        scan[t] += v;
-        __syncthreads();
+    uint32_t upto = mine;                                  // slots of the experts up to this one
+#pragma unroll
+    for (int off = 1; off < 64; off <<= 1) {
+        const uint32_t v = __shfl_up(upto, off, 64);
+        if (lane >= (uint32_t)off) upto += v;
     }
-    base[t] = scan[t] - mine;
-    for (uint32_t g = 0; g < mine / 16; g++) a.group_expert[base[t] / 16 + g] = (int32_t)t;
-    count[t] = 0;
+    if (lane == 63) wave_sum[wave] = upto;
+    __syncthreads();
+    for (uint32_t w = 0; w < wave; w++) upto += wave_sum[w];
+    for (uint32_t g = 0; g < mine / 16; g++) a.group_expert[(upto - mine) / 16 + g] = (int32_t)t;
+    count[t] = upto - mine;                                // from here on: the expert's next slot
     __syncthreads();
     for (uint32_t i = t; i < pairs; i += 1024) {
-        const uint32_t e = a.slot[i];
+        uint32_t e;
+        if constexpr (TOP) e = pick[i];
+        else e = a.slot[i];
         if (e >= a.experts) {                              // the input itself: nothing to compute
             a.slot[i] = 0xFFFFFFFFu;
             continue;
         }
-        const uint32_t s = base[e] + atomicAdd(&count[e], 1u);
+        const uint32_t s = atomicAdd(&count[e], 1u);
         a.slot[i] = s;
         a.perm[s] = i / a.top;
     }

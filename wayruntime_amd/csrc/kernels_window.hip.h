@@ -613,46 +613,46 @@ __global__ __launch_bounds__(256, KQ + VT > 8 ? 1 : 2) void window_decode_kernel
 
 constexpr uint32_t kWindowSplits = 64;          // shares of the keys at most: a lane each
 
-// grid (rows of the launch, heads), one wave: the shares of one row and head together
+// grid (rows of the launch, heads), a wave per map: the shares of one row and head together
 template <int VT, int MAPS>
-__global__ __launch_bounds__(64) void window_combine_kernel(const WindowArgs a)
+__global__ __launch_bounds__(64 * MAPS) void window_combine_kernel(const WindowArgs a)
 {
     constexpr int COLS = (VT * 32 + 63) / 64;
-    __shared__ float wt[kWindowSplits];
-    const uint32_t h = blockIdx.y, r = a.drows[blockIdx.x].row, t = threadIdx.x;
-    float o[MAPS][COLS];
-#pragma unroll
-    for (int m = 0; m < MAPS; m++) {
-        const size_t at = (((size_t)blockIdx.x * a.heads + h) * MAPS + m) * a.splits;
-        const bool has = t < a.splits;
-        const float mo = has ? a.part_ml[(at + t) * 2] : kLatentNone, l = has ? a.part_ml[(at + t) * 2 + 1] : 0.f;
-        float mx = mo;
-#pragma unroll
-        for (int off = 32; off >= 1; off >>= 1) mx = fmaxf(mx, wave_xor_f32(mx, off));
-        const float w = l != 0.f ? fast_exp2(mo - mx) : 0.f;    // zero: a share past the row's keys
-        float sum = w * l;
-#pragma unroll
-        for (int off = 32; off >= 1; off >>= 1) sum += wave_xor_f32(sum, off);
-        const float inv = 1.0f / sum;
-        __syncthreads();
-        wt[t] = w;
-        __syncthreads();
-#pragma unroll
-        for (int i = 0; i < COLS; i++) {
-            const uint32_t col = t + 64 * i;
-            o[m][i] = 0.f;
-            if (col >= VT * 32) continue;
-            for (uint32_t s = 0; s < a.splits; s++) o[m][i] = fmaf(wt[s], a.part_o[(at + s) * VT * 32 + col], o[m][i]);
-            o[m][i] *= inv;
-        }
-    }
+    __shared__ float wt[MAPS][kWindowSplits], second[MAPS == 2 ? COLS * 64 : 1];
+    const uint32_t h = blockIdx.y, r = a.drows[blockIdx.x].row, t = threadIdx.x & 63, map = threadIdx.x >> 6;
+    const size_t at = (((size_t)blockIdx.x * a.heads + h) * MAPS + map) * a.splits;
+    const bool has = t < a.splits;
+    const float m = has ? a.part_ml[(at + t) * 2] : kLatentNone, l = has ? a.part_ml[(at + t) * 2 + 1] : 0.f;
     float factor = window_factor<false>(a, r, h);
+    const float mx = mix_wave_max(m);
+    const float w = l != 0.f ? fast_exp2(m - mx) : 0.f;    // zero: a share past the row's keys
+    float sum = w * l;
+#pragma unroll
+    for (int off = 32; off >= 1; off >>= 1) sum += wave_xor_f32(sum, off);
+    const float inv = 1.0f / sum;
+    wt[map][t] = w * inv;
+    __syncthreads();
+    float o[COLS];
+#pragma unroll
+    for (int i = 0; i < COLS; i++) {
+        const uint32_t col = t + 64 * i;
+        o[i] = 0.f;
+        if (col >= VT * 32) continue;
+#pragma unroll 4
+        for (uint32_t s = 0; s < a.splits; s++) o[i] = fmaf(wt[map][s], a.part_o[(at + s) * VT * 32 + col], o[i]);
+    }
     if constexpr (MAPS == 2) {
+        if (map) {
+#pragma unroll
+            for (int i = 0; i < COLS; i++) second[t + 64 * i] = o[i];
+        }
+        __syncthreads();
+        if (map) return;
         float ss = 0.f;
 #pragma unroll
         for (int i = 0; i < COLS; i++) {
-            o[0][i] -= a.diff * o[1][i];
-            ss = fmaf(o[0][i], o[0][i], ss);
+            o[i] -= a.diff * second[t + 64 * i];
+            ss = fmaf(o[i], o[i], ss);
         }
 #pragma unroll
         for (int off = 32; off >= 1; off >>= 1) ss += wave_xor_f32(ss, off);
@@ -662,7 +662,7 @@ __global__ __launch_bounds__(64) void window_combine_kernel(const WindowArgs a)
 #pragma unroll
     for (int i = 0; i < COLS; i++) {
         const uint32_t col = t + 64 * i;
-        if (col < VT * 32) out[frag_elem(r, h * VT * 32 + col, a.o_kt)] = (__bf16)(o[0][i] * factor);
+        if (col < VT * 32) out[frag_elem(r, h * VT * 32 + col, a.o_kt)] = (__bf16)(o[i] * factor);
     }
 }
 

@@ -1104,7 +1104,7 @@ static int window_mfma(wr_hip_mix_step* s, WindowArgs& a)
     }
     launch_main(window_decode_kernel<MAPS * KQ, VT, MAPS>, dim3(n * groups, a.splits), dim3(256), a);
     HIP_TRY(hipGetLastError(), "windowed decode launch", 0);
-    if (a.splits > 1) MIX_LAUNCH((window_combine_kernel<VT, MAPS>), dim3(n, a.heads), dim3(64), 0, a);
+    if (a.splits > 1) MIX_LAUNCH((window_combine_kernel<VT, MAPS>), dim3(n, a.heads), dim3(64 * MAPS), 0, a);
     return WR_HIP_OK;
 }
 
@@ -1197,12 +1197,18 @@ int wr_hip_mix_route(wr_hip_mix_step* s, const float* z_dev, uint32_t ldz, const
     a.slot = slot_dev;
     a.perm = perm_dev;
     a.group_expert = group_expert_dev;
-    if (s->rows <= 64) {
-        MIX_LAUNCH(mix_order_kernel<true>, dim3(1), dim3(1024), 0, a);
-    } else {
-        MIX_LAUNCH(mix_top_kernel, dim3((s->rows + 3) / 4), dim3(256), 0, a);
-        MIX_LAUNCH(mix_order_kernel<false>, dim3(1), dim3(1024), 0, a);
+    static_assert(WR_HIP_MIX_MAX_TOP * kOrderRows <= kOrderPairs, "choices of a short step");
+    if (s->rows <= kOrderRows) {
+        if (outputs <= 64) MIX_LAUNCH(mix_order_kernel<1>, dim3(1), dim3(1024), 0, a);
+        else if (outputs <= 256) MIX_LAUNCH(mix_order_kernel<4>, dim3(1), dim3(1024), 0, a);
+        else MIX_LAUNCH(mix_order_kernel<16>, dim3(1), dim3(1024), 0, a);
+        return WR_HIP_OK;
     }
+    const dim3 grid((s->rows + 3) / 4), block(256);
+    if (outputs <= 64) MIX_LAUNCH(mix_top_kernel<1>, grid, block, 0, a);
+    else if (outputs <= 256) MIX_LAUNCH(mix_top_kernel<4>, grid, block, 0, a);
+    else MIX_LAUNCH(mix_top_kernel<16>, grid, block, 0, a);
+    MIX_LAUNCH(mix_order_kernel<0>, dim3(1), dim3(1024), 0, a);
     return WR_HIP_OK;
 }
 

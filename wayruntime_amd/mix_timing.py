@@ -43,10 +43,10 @@ def taredra_config(width: int, heads: int, ff: int) -> dict:
 
 
 def fedirax_config(width: int, heads: int, experts: int, top: int, expert_ff: int, shared_ff: int) -> dict:
-    """Two maps of 64 per head over values of 128, eight key/value heads; an eighth of the outputs pass the input on."""
+    """Two maps of 64 per head over values of 128, eight key/value heads; eight of the router's outputs pass the input on."""
     diff = dict(heads=heads, kv_heads=8, dim=64, vdim=128, window=4096)
     keys = mw.keys_as_values(heads, 8, 128, window=4096)
-    moe = mw.grouped_moe(experts, top, expert_ff, identity=experts // 8, groups=(8, 4), scale=2.0, shared=(shared_ff, 7.0))
+    moe = mw.grouped_moe(experts, top, expert_ff, identity=8, groups=(8, 4), scale=2.0, shared=(shared_ff, 7.0))
     return mw.shared_kv_config(width, VOCAB, [(m, moe) for m in (mw.difference(**diff), keys, mw.difference(**diff),
                                                                  mw.difference(**diff, kv_from=0))])
 
