@@ -429,6 +429,25 @@ def test_positions_far_out(eng, tmp_path, prec, kind):
     case.close()
 
 
+@pytest.mark.parametrize("dim", [8, 40, 100])
+def test_prompts_that_fill_the_device(eng, tmp_path, dim):
+    # so many heads and rows that a wave of the prompt's attention takes twice the rows; an unequal request beside it
+    cfg = mw.shared_kv_config(64, 90, [(mw.keys_as_values(96, 48, dim, 130, scale=0.5), None)])
+    case = Case(eng, tmp_path, cfg, "bf16", pool=2048)
+    t, u = case.tokens(1090), case.tokens(77, seed=8)
+    want, other = case.oracle(t), case.oracle(u)
+    a, b = case.m.session(), case.m.session()
+    rc, lg = E.mixed_step([(a, t[:1050], range(1050)), (b, u, range(77))])
+    assert rc == 1127
+    case.check(lg[0], want[:1050], f"dim {dim} prompt")
+    case.check(lg[1], other, f"dim {dim} beside it")
+    rc, lg = E.mixed_step([(a, t[1050:], range(40))])
+    case.check(lg[0], want[1050:], f"dim {dim} going on")
+    a.close()
+    b.close()
+    case.close()
+
+
 def test_long_decoding(eng, tmp_path, prec):
     case = Case(eng, tmp_path, stack(prec), prec)
     t = case.tokens(420)

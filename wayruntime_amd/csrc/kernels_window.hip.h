@@ -20,8 +20,8 @@
 // O^T = V^T P^T in the order V is stored.
 //
 //   window_append_kernel    queries normed and rotated into an operand, keys the same way and values into the cache
-//   window_prefill_kernel   128 (token, head, map) rows of one key/value head a workgroup, a page at a time
-//                           through LDS
+//   window_prefill_kernel   128 or 64 (token, head, map) rows of one key/value head a workgroup, a page at a
+//                           time through LDS
 //   window_decode_kernel    a workgroup per (token, key/value head, share of the keys)
 //   window_attend_any_kernel  any geometry, both activation types
 #pragma once
@@ -355,13 +355,14 @@ __device__ __forceinline__ float window_difference(const WindowArgs& a, f32x4 (&
     return 1.0f / sqrtf(ss / (float)a.vdim + a.eps);
 }
 
-// KQ, VT: head sizes in tiles of 32.  Grid: tiles of 128 (token, head of the group, map) rows times key/value heads, the
+// KQ, VT: head sizes in tiles of 32.  Grid: tiles of 64 NR (token, head of the group, map) rows times key/value heads, the
 // key/value head innermost: with eight of them each XCD keeps to one.  A wave's two row tiles are 32 rows, or the two
 // maps of 16.
-template <int KQ, int VT, int MAPS>
+template <int KQ, int VT, int MAPS, int NR>
 __global__ __launch_bounds__(256, 2) void window_prefill_kernel(const WindowArgs a)
 {
-    constexpr int NR = 2, CPW = MAPS * KQ + VT, STAGE = 4 * CPW * 1024, WROWS = 32 / MAPS, ROWS = 4 * WROWS;
+    static_assert(NR % MAPS == 0, "a wave has all maps of its rows");
+    constexpr int CPW = MAPS * KQ + VT, STAGE = 4 * CPW * 1024, WROWS = 16 * NR / MAPS, ROWS = 4 * WROWS;
     extern __shared__ __attribute__((aligned(16))) unsigned char window_lds[];
     const int lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4;
     const uint32_t wave = (uint32_t)__builtin_amdgcn_readfirstlane(threadIdx.x >> 6);

@@ -1055,20 +1055,39 @@ int wr_hip_mix_window_append(wr_hip_mix_step* s, wr_hip_mix_pool* pool, uint32_t
     return WR_HIP_OK;
 }
 
+// Workgroups of a prefill launch of `rows` (token, head of the group) rows each.
+static uint64_t window_tiles(const wr_hip_mix_step* s, const WindowArgs& a, uint32_t rows)
+{
+    uint64_t tiles = 0;
+    for (uint32_t i = 0; i < s->n_long; i++) tiles += ((uint64_t)s->long_rows[i] * a.group + rows - 1) / rows;
+    return tiles * a.kvh;
+}
+
+template <int KQ, int VT, int MAPS, int NR>
+static int window_prefill(wr_hip_mix_step* s, WindowArgs& a)
+{
+    const uint64_t tiles = window_tiles(s, a, 64 * NR / MAPS);
+    a.list = s->d<uint32_t>(s->o_long);
+    a.n_list = s->n_long;
+    constexpr size_t lds = window_prefill_lds(MAPS * KQ, VT);
+    int rc = allow_lds<window_prefill_kernel<KQ, VT, MAPS, NR>>(lds);
+    if (rc) return rc;
+    launch_main(window_prefill_kernel<KQ, VT, MAPS, NR>, dim3((uint32_t)tiles), dim3(256), a, lds);
+    HIP_TRY(hipGetLastError(), "windowed prefill launch", 0);
+    return WR_HIP_OK;
+}
+
 template <int KQ, int VT, int MAPS>
 static int window_mfma(wr_hip_mix_step* s, WindowArgs& a)
 {
     if (s->n_long) {
-        constexpr uint32_t tile = 128 / MAPS;
-        uint64_t tiles = 0;
-        for (uint32_t i = 0; i < s->n_long; i++) tiles += ((uint64_t)s->long_rows[i] * a.group + tile - 1) / tile;
-        a.list = s->d<uint32_t>(s->o_long);
-        a.n_list = s->n_long;
-        constexpr size_t lds = window_prefill_lds(MAPS * KQ, VT);
-        int rc = allow_lds<window_prefill_kernel<KQ, VT, MAPS>>(lds);
+        // 32 rows a wave, or 16 where the launch would be little more than what the device holds at once (two workgroups
+        // a compute unit): its time is then that of the workgroup with the most keys
+        int rc;
+        if constexpr (MAPS == 2) rc = window_prefill<KQ, VT, 2, 2>(s, a);
+        else if (window_tiles(s, a, 128) > 3 * (uint64_t)g.n_cus) rc = window_prefill<KQ, VT, 1, 2>(s, a);
+        else rc = window_prefill<KQ, VT, 1, 1>(s, a);
         if (rc) return rc;
-        launch_main(window_prefill_kernel<KQ, VT, MAPS>, dim3((uint32_t)(tiles * a.kvh)), dim3(256), a, lds);
-        HIP_TRY(hipGetLastError(), "windowed prefill launch", 0);
     }
     const uint32_t n = s->n_short_rows;
     if (n == 0) return WR_HIP_OK;
