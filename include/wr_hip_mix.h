@@ -2,7 +2,7 @@
  * wr_hip_mix.h — C ABI of the device steps of mixer-stack models: models whose
  * layers pair a mixer (decayed linear attention, sliding-window attention through
  * a low-rank latent or over grouped keys and values, a matrix-state recurrence
- * with input-made decays) with a feed-forward (dense or a mixture of experts),
+ * with input-made decays, a gated recurrence element by element) with a feed-forward (dense or a mixture of experts),
  * with norms before and, in some designs, after each, and bfloat16 weights.
  *
  * Conventions are those of wr_hip_attn.h: plain C, status returns, every call
@@ -99,10 +99,11 @@ int wr_hip_mix_embed(wr_hip_mix_step *s, int f32, const uint16_t *table_dev, uin
  *                                     row r of y is sum_t gate[r][t] * y[slot[r][t]], the
  *                                     experts' rows, slots of ~0 left out; with `side` as well
  *                                     + side[r][0] * ident[r] + side[r][1] * shared[r])
+ *   x += rmsnorm(pair_y[i]) * pair_post[i], i = 0, 1   (when given, both or neither)
  *   x += add                         (when given)
  *   h = rmsnorm(x) * next            (when given; only the step's wanted rows, packed,
  *                                     with `wanted` set)
- * ident: frag rows of the width, may be h itself; shared: 32-bit rows like y; either may
+ * gate may be NULL: ones.  ident: frag rows of the width, may be h itself; shared: 32-bit rows like y; either may
  * be NULL. */
 typedef struct wr_hip_mix_resid {
     uint32_t width;
@@ -117,6 +118,7 @@ typedef struct wr_hip_mix_resid {
     const float *side;
     const void *ident;
     const float *shared;
+    const float *pair_y[2], *pair_post[2];
 } wr_hip_mix_resid;
 int wr_hip_mix_residual(wr_hip_mix_step *s, int f32, const wr_hip_mix_resid *a);
 /* Token shift.  x += y first (y may be NULL).  With h[r] = rmsnorm(x[r]) * norm and p[r]
@@ -137,16 +139,16 @@ int wr_hip_mix_shift(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, in
  * out says where output n of row r goes:
  *   ROWS_F32   y_f32[r][z * col_z + n]     32-bit rows, row stride ldy
  *   ROWS       y_act[r][n]                 activation type, row stride ldy
- *   FRAG       h (frag, h_kt tiles): row r, input z * col_z + n
+ *   FRAG       h (frag, h_kt tiles): row r, input h_kt0 * 32 + z * col_z + n
  *   SPLIT      n < n_split: FRAG; else y_f32[r][n - n_split]
  *   GATED      tiles 2j / 2j+1 of W are gate / up: silu(gate) * up to FRAG
  *              (with gelu: 0.5 g (1 + tanh(sqrt(2/pi) (g + 0.044715 g^3))) * up;
  *              with limit > 0: g = min(gate, limit), u = up within [-limit, limit],
  *              g * logistic(slope * g) * (u + up_bias))
  *   SPLIT_GATED n < n_split (a multiple of 32): y_f32[r][n]; the tiles behind as GATED
- * after `bias` (n_out floats, batch 1) and an activation: SiLU for n < silu_end, else the logistic for n <
+ * after a factor per row (x_scale, with group_expert), `bias` (a float for each of the n_out outputs, batch 1) and an activation: SiLU for n < silu_end, else the logistic for n <
  * sigmoid_end, else the hyperbolic tangent for n < tanh_end; square of ReLU
- * everywhere with relu2; times `scale` when not 0.  (GATED outputs take neither.) */
+ * everywhere with relu2; times `scale` when not 0.  (GATED outputs take the factor alone; `scale` is not for SPLIT_GATED.) */
 enum { WR_HIP_MIX_OUT_ROWS_F32 = 0, WR_HIP_MIX_OUT_ROWS = 1, WR_HIP_MIX_OUT_FRAG = 2,
        WR_HIP_MIX_OUT_SPLIT = 3, WR_HIP_MIX_OUT_GATED = 4, WR_HIP_MIX_OUT_SPLIT_GATED = 5 };
 typedef struct wr_hip_mix_gemm {
@@ -169,6 +171,8 @@ typedef struct wr_hip_mix_gemm {
     const float *bias;
     float limit, slope, up_bias;
     const uint32_t *x_perm;        /* with group_expert and tile_groups 1: row i is row x_perm[i] of x (any row for ~0) */
+    uint32_t h_kt0;                /* input tile of h where its outputs begin */
+    const float *x_scale;          /* with group_expert: row i's outputs are those of x_scale[i] times its input */
 } wr_hip_mix_gemm;
 int wr_hip_mix_gemm_run(int f32, const wr_hip_mix_gemm *a);
 
@@ -186,12 +190,16 @@ int wr_hip_mix_gate_norm(wr_hip_mix_step *s, int f32, const float *o_dev, uint32
                          const void *g_dev, uint32_t ldg, const float *norm_dev, float eps, void *h_dev);
 
 /* ---- matrix-state recurrence with input-made decays -----------------------------
- * Per head a state S [dim][dim], key channel by value column, 32-bit.  Every token
+ * Per head a state S [dim][vdim], key channel by value column, 32-bit.  Every token
  * brings r, k, v and a decay per key channel, w = exp(-exp(z + w0)), or
- * exp(-gain * sigmoid(z + w0)) with `gain` > 0, z = w_decay . low.  Two rules:
+ * exp(-gain * sigmoid(z + w0)) with `gain` > 0, z = w_decay . low.  Three rules:
  *   BONUS  o = (S + diag(u) k v^T)^T r;  then S <- diag(w) S + k v^T
  *   DELTA  with n = k / sqrt(k . k + unit_eps) and a = sigmoid(za + a_bias):
  *          S <- diag(w) S - (a n) (n^T S) + k v^T (old S on the right);  o = S^T r
+ *   FORGET w = lower + (1 - lower) logistic(z + w0) with z the rows at col_k, k = 1 - w:
+ *          S <- diag(w) S + k v^T;  o = S^T r    (no low-rank product, no gate; norm is
+ *          one of vdim weights that the heads share)
+ * vdim is dim but in FORGET.
  * Then each head's o is divided by its root mean square (eps), times norm, times the
  * gate (SiLU or logistic of the rows at col_g), times out_scale, and goes to h (frag,
  * h_kt tiles) at input col_h + head * dim + column; inputs up to the next multiple of
@@ -199,7 +207,7 @@ int wr_hip_mix_gate_norm(wr_hip_mix_step *s, int f32, const float *o_dev, uint32
  * in: 32-bit rows, stride ld; r, k, v, za, g at their columns, head by head.
  * low: frag rows of w_decay's inputs; z: room for the products, 32-bit rows of w_decay's
  * outputs (used where they are not made in passing).  State `run` of the pool; position 0 starts from zero. */
-enum { WR_HIP_MIX_RULE_BONUS = 0, WR_HIP_MIX_RULE_DELTA = 1 };
+enum { WR_HIP_MIX_RULE_BONUS = 0, WR_HIP_MIX_RULE_DELTA = 1, WR_HIP_MIX_RULE_FORGET = 2 };
 typedef struct wr_hip_mix_recurrence {
     uint32_t heads, dim, rule;
     float gain, unit_eps, eps, out_scale;
@@ -212,9 +220,25 @@ typedef struct wr_hip_mix_recurrence {
     float *z;
     void *h;
     uint32_t h_kt, col_h;
+    uint32_t vdim;                            /* FORGET */
+    const float *lower;                       /* FORGET: device, heads * dim */
 } wr_hip_mix_recurrence;
 int wr_hip_mix_recur(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, int f32,
                      const wr_hip_mix_recurrence *a);
+
+/* ---- gated recurrence element by element ------------------------------------------
+ * z = logistic of the rows at col_z, u the rows at col_x, c = u + 1/2 where u >= 0, else
+ * logistic(u):  S <- (1 - z) S + z c, 32-bit;  S times SiLU of the rows at col_g goes to h
+ * (frag, h_kt tiles) at input col_h.  `width` elements, padded to 32 (rows, state and
+ * operand alike; the rows' pads are zeros).  State `run` of the pool; position 0 starts from zero. */
+typedef struct wr_hip_mix_gru {
+    uint32_t width;
+    const float *in;                          /* 32-bit rows, stride ld */
+    uint32_t ld, col_z, col_x, col_g;
+    void *h;
+    uint32_t h_kt, col_h;
+} wr_hip_mix_gru;
+int wr_hip_mix_min_gru(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, int f32, const wr_hip_mix_gru *a);
 
 /* ---- windowed attention over grouped keys and values ----------------------------
  * `heads` query heads, `kv_heads` key/value heads (query head h reads h / (heads /
@@ -224,6 +248,9 @@ int wr_hip_mix_recur(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, in
  * Queries and keys may be normed (each map's vector over its root mean square, times a
  * weight of dim), then the first 2 * rot_half dimensions are rotated, i with
  * i + rot_half, or with `neighbours` 2i with 2i + 1.
+ * With `chunk` a row sees what came before it in its own chunk of that many positions, counted
+ * from the request's first.  With turn_values, element 2m of a value is turned with element
+ * 2m + 1 by the angles in that table ahead of the cache, and a head's output back by its row's.
  * Cached per position: kv_heads * (maps * dim_pad + vdim_pad) elements. */
 typedef struct wr_hip_mix_window {
     uint32_t heads, kv_heads, dim, dim_pad, vdim, vdim_pad, rot_half;
@@ -236,6 +263,9 @@ typedef struct wr_hip_mix_window {
     float softcap;                 /* > 0: scores are softcap * tanh(score / softcap) */
     float diff;                    /* maps = 2: how much of the second map's output is taken off */
     const float *q_norm, *k_norm;  /* device, dim floats each, or NULL */
+    uint32_t chunk;                /* > 0: in place of the window */
+    uint32_t gate_wide;            /* the gate has a logit for every output element */
+    const float *turn_values;      /* device, [rows][vdim / 2][2], or NULL */
 } wr_hip_mix_window;
 /* The padded head size to use: what the matrix kernels take, else a multiple of 32. */
 uint32_t wr_hip_mix_window_pad(uint32_t dim);
@@ -250,16 +280,17 @@ int wr_hip_mix_window_append(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t
 /* Softmax attention over the cached rows inside the window; with `sink`, a head's weights
  * are exp(score) / (exp(sink[head]) + sum of exp(score)).  With two maps a head's output is
  * first - diff * second, over its root mean square (eps).  Head h's output times out_scale,
- * and times logistic(gate[row * ldg + h]) where `gate` is given, goes to o (frag, o_kt
+ * and times logistic(gate[row * ldg + h]) where `gate` is given (with gate_wide element by
+ * element, gate[row * ldg + h * vdim + column]), goes to o (frag, o_kt
  * tiles) at input h * vdim_pad. */
 int wr_hip_mix_window_attend(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, int f32,
                              const wr_hip_mix_window *g, const void *q_dev, const float *sink_dev,
                              const float *gate_dev, uint32_t ldg, void *o_dev, uint32_t o_kt);
 
 /* ---- attention through a latent -----------------------------------------------
- * Table of (cos, sin) of position * freq[i] for the step's rows, [rows][half][2];
+ * Table of (cos, sin) of position * freq[i], both times gain, for the step's rows, [rows][half][2];
  * freq: device doubles. */
-int wr_hip_mix_rope_table(wr_hip_mix_step *s, const double *freq_dev, uint32_t half, float *table_dev);
+int wr_hip_mix_rope_table(wr_hip_mix_step *s, const double *freq_dev, uint32_t half, float gain, float *table_dev);
 /* The geometry of one attention layer.  A cached row is [rank_pad | rot_pad]. */
 typedef struct wr_hip_mix_latent {
     uint32_t heads, rank, rank_pad, rot, rot_pad, rot_half;
@@ -291,7 +322,8 @@ int wr_hip_mix_latent_attend(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t
  * outputs that pass the layer's input on: the `top` outputs with the largest choice value
  * (lowest index first among equals), their weights, and an order of the (row, choice)
  * pairs by expert: each expert's pairs take runs of tile_groups groups of 16 slots.
- * The choice value is the logit and the weights are the softmax over the chosen; with
+ * The choice value is the logit and the weights are the softmax over the chosen, or with
+ * logistic their logits' logistic as it is; with
  * softmax_all it is the softmax over all outputs plus `correction`, and the weights are
  * the chosen outputs' softmax over (their sum + 1e-20), times scale.  With groups > 0 the
  * outputs form that many equal groups of neighbours, and only those of the `keep` groups
@@ -300,6 +332,7 @@ int wr_hip_mix_latent_attend(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t
  * group_expert: expert of each group of 16 slots, or -1; side[r] (may be NULL): the sum of
  * the identity outputs' weights, and, with shared_gate, the logistic of the logit behind
  * the outputs' (else 0).
+ * slot_weight (may be NULL): the weight of each slot's pair, 0 for an empty slot.
  * wr_hip_mix_route_groups: how many groups that can take at most. */
 typedef struct wr_hip_mix_router {
     uint32_t experts, identity, top;
@@ -307,12 +340,13 @@ typedef struct wr_hip_mix_router {
     uint32_t softmax_all, shared_gate;
     float scale;
     const float *correction;       /* device, or NULL */
+    uint32_t logistic;
 } wr_hip_mix_router;
 #define WR_HIP_MIX_MAX_GROUPS 64u
 uint32_t wr_hip_mix_route_groups(uint32_t rows, uint32_t experts, uint32_t top, uint32_t tile_groups);
 int wr_hip_mix_route(wr_hip_mix_step *s, const float *z_dev, uint32_t ldz, const wr_hip_mix_router *g,
-                     uint32_t tile_groups, float *gate_dev, float *side_dev, uint32_t *slot_dev, uint32_t *perm_dev,
-                     int32_t *group_expert_dev);
+                     uint32_t tile_groups, float *gate_dev, float *side_dev, float *slot_weight_dev, uint32_t *slot_dev,
+                     uint32_t *perm_dev, int32_t *group_expert_dev);
 /* The rows of h in slot order: xs (frag). */
 int wr_hip_mix_route_gather(wr_hip_mix_step *s, int f32, const void *h_dev, uint32_t kt, uint32_t n_groups,
                             const uint32_t *perm_dev, const int32_t *group_expert_dev, void *xs_dev);

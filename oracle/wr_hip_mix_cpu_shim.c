@@ -175,13 +175,17 @@ int wr_hip_mix_residual(wr_hip_mix_step *s, int f32, const wr_hip_mix_resid *a)
                 y[k] = a->top ? 0.0f : a->y[(size_t)r * wp + k];
                 for (uint32_t t = 0; t < a->top; t++) {
                     const uint32_t slot = a->slot[(size_t)r * a->top + t];
-                    if (slot != ~0u) y[k] += a->gate[(size_t)r * a->top + t] * a->y[(size_t)slot * wp + k];
+                    if (slot != ~0u) y[k] += (a->gate ? a->gate[(size_t)r * a->top + t] : 1.0f) * a->y[(size_t)slot * wp + k];
                 }
                 if (a->side && a->ident) y[k] += a->side[2 * r] * ((const float *)a->ident)[(size_t)r * wp + k];
                 if (a->side && a->shared) y[k] += a->side[2 * r + 1] * a->shared[(size_t)r * wp + k];
             }
             const float inv = a->post ? inv_rms(y, a->width, a->eps) : 1.0f;
             for (uint32_t k = 0; k < wp; k++) x[k] += a->post ? y[k] * inv * a->post[k] : y[k];
+        }
+        for (int i2 = 0; i2 < 2 && a->pair_y[i2]; i2++) {
+            const float *p = a->pair_y[i2] + (size_t)r * wp, inv = inv_rms(p, a->width, a->eps);
+            for (uint32_t k = 0; k < wp; k++) x[k] += p[k] * inv * a->pair_post[i2][k];
         }
         if (a->add)
             for (uint32_t k = 0; k < wp; k++) x[k] += a->add[(size_t)r * wp + k];
@@ -232,12 +236,21 @@ static float gated_unit(const wr_hip_mix_gemm *a, float g, float u)
     return a->gelu ? 0.5f * g * (1.0f + tanhf(0.79788456080286536f * (g + 0.044715f * g * g * g))) * u : g * sig(g) * u;
 }
 
+static float row_value(const wr_hip_mix_gemm *a, uint32_t n, float o)
+{
+    const uint32_t sig_end = a->sigmoid_end > a->silu_end ? a->sigmoid_end : a->silu_end;
+    if (a->bias) o += a->bias[n];
+    if (n < a->silu_end) return o * sig(o);
+    if (n < sig_end) return sig(o);
+    if (n < a->tanh_end) return tanhf(o);
+    return a->relu2 ? (o > 0 ? o * o : 0) : o;
+}
+
 int wr_hip_mix_gemm_run(int f32, const wr_hip_mix_gemm *a)
 {
     if (!f32) return WR_HIP_ERR_UNSUPPORTED;
     if (g_late > 0 && --g_late == 0) return WR_HIP_ERR_INTERNAL;
     const uint32_t N = a->w->n_out, K = a->w->n_in, batch = a->group_expert ? 1 : a->w->batch, ldx = a->x_kt * 32;
-    const uint32_t sig_end = a->sigmoid_end > a->silu_end ? a->sigmoid_end : a->silu_end;
     float *v = malloc(N * 4);
     for (uint32_t z = 0; z < batch; z++)
         for (uint32_t r = 0; r < a->rows; r++) {
@@ -252,22 +265,18 @@ int wr_hip_mix_gemm_run(int f32, const wr_hip_mix_gemm *a)
             for (uint32_t n = 0; n < N; n++) {
                 float acc = 0;
                 for (uint32_t k = 0; k < K; k++) acc += w[(size_t)n * K + k] * x[k];
-                v[n] = acc;
+                v[n] = a->x_scale ? acc * a->x_scale[r] : acc;
             }
-            float *h = a->h ? (float *)a->h + (size_t)r * a->h_kt * 32 + (size_t)z * a->col_z : NULL;
+            float *h = a->h ? (float *)a->h + (size_t)r * a->h_kt * 32 + (size_t)a->h_kt0 * 32 + (size_t)z * a->col_z : NULL;
             if (a->out >= WR_HIP_MIX_OUT_GATED) {
                 const uint32_t rows = a->out == WR_HIP_MIX_OUT_SPLIT_GATED ? a->n_split : 0;
-                for (uint32_t n = 0; n < rows; n++) a->y_f32[(size_t)r * a->ldy + n] = v[n];
+                for (uint32_t n = 0; n < rows; n++) a->y_f32[(size_t)r * a->ldy + n] = row_value(a, n, v[n]);
                 for (uint32_t n = 0; n < (N - rows) / 2; n++)
                     h[n] = gated_unit(a, v[rows + n / 16 * 32 + n % 16], v[rows + n / 16 * 32 + 16 + n % 16]);
                 continue;
             }
             for (uint32_t n = 0; n < N; n++) {
-                float o = v[n] + (a->bias ? a->bias[n] : 0.0f);
-                if (n < a->silu_end) o *= sig(o);
-                else if (n < sig_end) o = sig(o);
-                else if (n < a->tanh_end) o = tanhf(o);
-                else if (a->relu2) o = o > 0 ? o * o : 0;
+                float o = row_value(a, n, v[n]);
                 if (a->scale != 0) o *= a->scale;
                 if (a->out == WR_HIP_MIX_OUT_ROWS_F32) a->y_f32[(size_t)r * a->ldy + (size_t)z * a->col_z + n] = o;
                 else if (a->out == WR_HIP_MIX_OUT_ROWS) ((float *)a->y_act)[(size_t)r * a->ldy + n] = o;
@@ -322,19 +331,79 @@ int wr_hip_mix_gate_norm(wr_hip_mix_step *s, int f32, const float *o, uint32_t l
     return WR_HIP_OK;
 }
 
-int wr_hip_mix_rope_table(wr_hip_mix_step *s, const double *freq, uint32_t half, float *table)
+int wr_hip_mix_rope_table(wr_hip_mix_step *s, const double *freq, uint32_t half, float gain, float *table)
 {
     for (uint32_t r = 0; r < s->rows; r++)
         for (uint32_t i = 0; i < half; i++) {
-            table[2 * ((size_t)r * half + i)] = (float)cos(s->pos[r] * freq[i]);
-            table[2 * ((size_t)r * half + i) + 1] = (float)sin(s->pos[r] * freq[i]);
+            table[2 * ((size_t)r * half + i)] = (float)cos(s->pos[r] * freq[i]) * gain;
+            table[2 * ((size_t)r * half + i) + 1] = (float)sin(s->pos[r] * freq[i]) * gain;
         }
+    return WR_HIP_OK;
+}
+
+/* S <- diag(w) S + (1 - w) v^T, o = S^T r, normed head by head. */
+static int recur_forget(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, const wr_hip_mix_recurrence *a)
+{
+    const uint32_t D = a->dim, V = a->vdim, hv = a->heads * V;
+    const size_t all = (size_t)a->heads * D * V;
+    if (pool->state_elems[run] != all) return WR_HIP_ERR_INVAL;
+    for (uint32_t i = 0; i < s->n_seq; i++) {
+        const wr_hip_mix_seq *q = &s->seqs[i];
+        float *S = calloc(all, 4), *o = malloc(V * 4);
+        if (q->pos0) memcpy(S, pool->state[run] + (size_t)(q->slot * 2 + q->buf_in) * all, all * 4);
+        for (uint32_t t = s->row0[i]; t < s->row0[i] + q->rows; t++) {
+            const float *row = a->in + (size_t)t * a->ld;
+            float *to = (float *)a->h + (size_t)t * a->h_kt * 32 + a->col_h;
+            for (uint32_t h = 0; h < a->heads; h++) {
+                memset(o, 0, V * 4);
+                for (uint32_t d = 0; d < D; d++) {
+                    const uint32_t n = h * D + d;
+                    const float z = row[a->col_k + n] + a->w0[n], w = a->lower[n] + (1 - a->lower[n]) * sig(z);
+                    const float k = (1 - a->lower[n]) * sig(-z);
+                    for (uint32_t c = 0; c < V; c++) {
+                        float *e = &S[((size_t)h * D + d) * V + c];
+                        *e = w * *e + k * row[a->col_v + h * V + c];
+                        o[c] += *e * row[a->col_r + n];
+                    }
+                }
+                const float inv = a->out_scale * inv_rms(o, V, a->eps);
+                for (uint32_t c = 0; c < V; c++) to[h * V + c] = o[c] * inv * a->norm[c];
+            }
+            for (uint32_t c = hv; c < p32(hv); c++) to[c] = 0.0f;
+        }
+        memcpy(pool->state[run] + (size_t)(q->slot * 2 + q->buf_out) * all, S, all * 4);
+        free(S);
+        free(o);
+    }
+    return WR_HIP_OK;
+}
+
+int wr_hip_mix_min_gru(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, int f32, const wr_hip_mix_gru *a)
+{
+    if (!f32) return WR_HIP_ERR_UNSUPPORTED;
+    const uint32_t wp = p32(a->width);
+    if (pool->state_elems[run] != wp) return WR_HIP_ERR_INVAL;
+    for (uint32_t i = 0; i < s->n_seq; i++) {
+        const wr_hip_mix_seq *q = &s->seqs[i];
+        const float *in = pool->state[run] + (size_t)(q->slot * 2 + q->buf_in) * wp;
+        float *out = pool->state[run] + (size_t)(q->slot * 2 + q->buf_out) * wp;
+        for (uint32_t k = 0; k < wp; k++) {
+            float S = q->pos0 ? in[k] : 0.0f;
+            for (uint32_t t = s->row0[i]; t < s->row0[i] + q->rows; t++) {
+                const float *row = a->in + (size_t)t * a->ld, z = row[a->col_z + k], u = row[a->col_x + k], g = row[a->col_g + k];
+                S = sig(-z) * S + sig(z) * (u >= 0 ? u + 0.5f : sig(u));
+                ((float *)a->h)[(size_t)t * a->h_kt * 32 + a->col_h + k] = S * g * sig(g);
+            }
+            out[k] = S;
+        }
+    }
     return WR_HIP_OK;
 }
 
 int wr_hip_mix_recur(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, int f32, const wr_hip_mix_recurrence *a)
 {
     if (!f32) return WR_HIP_ERR_UNSUPPORTED;
+    if (a->rule == WR_HIP_MIX_RULE_FORGET) return recur_forget(s, pool, run, a);
     const uint32_t D = a->dim, hd = a->heads * D, delta = a->rule == WR_HIP_MIX_RULE_DELTA;
     const size_t all = (size_t)hd * D;
     if (pool->state_elems[run] != all) return WR_HIP_ERR_INVAL;
@@ -509,6 +578,11 @@ int wr_hip_mix_window_append(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t
             memset(cv, 0, g->vdim_pad * 4);
             const float *v = row + col_v + h * g->vdim, inv = g->norm_values ? inv_rms(v, g->vdim, g->eps) : 1.0f;
             for (uint32_t k = 0; k < g->vdim; k++) cv[k] = v[k] * inv;
+            for (uint32_t k = 0; g->turn_values && k < g->vdim; k += 2) {
+                const float *cs = g->turn_values + (size_t)r * g->vdim + k, x = cv[k], y = cv[k + 1];
+                cv[k] = x * cs[0] - y * cs[1];
+                cv[k + 1] = y * cs[0] + x * cs[1];
+            }
         }
     }
     return WR_HIP_OK;
@@ -521,7 +595,8 @@ int wr_hip_mix_window_attend(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t
     const uint32_t V = g->vdim_pad;
     for (uint32_t r = 0; r < s->rows; r++) {
         const wr_hip_mix_seq *sq = &s->seqs[s->seq[r]];
-        const uint32_t pos = s->pos[r], lo = pos + 1 > g->window ? pos + 1 - g->window : 0;
+        const uint32_t pos = s->pos[r];
+        const uint32_t lo = g->chunk ? pos / g->chunk * g->chunk : pos + 1 > g->window ? pos + 1 - g->window : 0;
         double *w = malloc(sizeof(double) * (pos - lo + 1)), *a2 = malloc(sizeof(double) * 2 * V);
         for (uint32_t h = 0; h < g->heads; h++) {
             const uint32_t kvh = h / (g->heads / g->kv_heads);
@@ -546,13 +621,19 @@ int wr_hip_mix_window_attend(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t
                     a2[m * V + k] = a / sum;
                 }
             }
-            double f = gate ? g->out_scale * sig(gate[(size_t)r * ldg + h]) : g->out_scale, ss = 0;
+            double f = gate && !g->gate_wide ? g->out_scale * sig(gate[(size_t)r * ldg + h]) : g->out_scale, ss = 0;
             for (uint32_t k = 0; g->maps == 2 && k < V; k++) {
                 a2[k] -= g->diff * a2[V + k];
                 ss += a2[k] * a2[k];
             }
             if (g->maps == 2) f /= sqrt(ss / g->vdim + g->eps);
-            for (uint32_t k = 0; k < V; k++) o[k] = (float)(a2[k] * f);
+            for (uint32_t k = 0; g->turn_values && k < g->vdim; k += 2) {
+                const float *cs = g->turn_values + (size_t)r * g->vdim + k;
+                const double x = a2[k], y = a2[k + 1];
+                a2[k] = x * cs[0] + y * cs[1];
+                a2[k + 1] = y * cs[0] - x * cs[1];
+            }
+            for (uint32_t k = 0; k < V; k++) o[k] = (float)(a2[k] * f * (g->gate_wide && k < g->vdim ? sig(gate[(size_t)r * ldg + h * g->vdim + k]) : 1.0f));
         }
         free(w);
         free(a2);
@@ -567,7 +648,7 @@ uint32_t wr_hip_mix_route_groups(uint32_t rows, uint32_t experts, uint32_t top, 
 }
 
 int wr_hip_mix_route(wr_hip_mix_step *s, const float *z, uint32_t ldz, const wr_hip_mix_router *g, uint32_t tile_groups,
-                     float *gate, float *side, uint32_t *slot, uint32_t *perm, int32_t *group_expert)
+                     float *gate, float *side, float *slot_weight, uint32_t *slot, uint32_t *perm, int32_t *group_expert)
 {
     const uint32_t experts = g->experts, top = g->top, N = experts + g->identity;
     const uint32_t groups = wr_hip_mix_route_groups(s->rows, experts, top, tile_groups), run = tile_groups * 16;
@@ -595,11 +676,11 @@ int wr_hip_mix_route(wr_hip_mix_step *s, const float *z, uint32_t ldz, const wr_
                 if (c[e] > c[best]) best = e;
             c[best] = -INFINITY;
             slot[r * top + t] = best;
-            sum += gate[r * top + t] = g->softmax_all ? p[best] / all : p[best];
+            sum += gate[r * top + t] = g->logistic ? sig(zr[best]) : g->softmax_all ? p[best] / all : p[best];
         }
         for (uint32_t t = 0; t < top; t++) {
             float *w = &gate[r * top + t];
-            *w = g->softmax_all ? *w / (sum + 1e-20f) * g->scale : *w / sum;
+            if (!g->logistic) *w = g->softmax_all ? *w / (sum + 1e-20f) * g->scale : *w / sum;
             if (slot[r * top + t] >= experts) own += *w;
         }
         if (side) {
@@ -611,6 +692,7 @@ int wr_hip_mix_route(wr_hip_mix_step *s, const float *z, uint32_t ldz, const wr_
     free(p);
     free(lead);
     for (uint32_t i = 0; i < groups * 16; i++) perm[i] = ~0u;
+    for (uint32_t i = 0; slot_weight && i < groups * 16; i++) slot_weight[i] = 0;
     for (uint32_t i = 0; i < groups; i++) group_expert[i] = -1;
     uint32_t at = 0;
     uint32_t *out = malloc((size_t)s->rows * top * 4);
@@ -620,6 +702,7 @@ int wr_hip_mix_route(wr_hip_mix_step *s, const float *z, uint32_t ldz, const wr_
         for (uint32_t i = 0; i < s->rows * top; i++)
             if (slot[i] == e) {
                 perm[at] = i / top;
+                if (slot_weight) slot_weight[at] = gate[i];
                 out[i] = at++;
             }
         at = (at + run - 1) / run * run;

@@ -1,5 +1,5 @@
 """Plain, slow restatement of the mixer-stack models (architectures "Bipotar",
-"Taredra" and "Fedirax"): one function per mechanism, numpy, one sequence at a time, every
+"Taredra", "Fedirax" and "Marosun"): one function per mechanism, numpy, one sequence at a time, every
 position from the definition (no cache, no chunks, no absorbed products).  Shares
 no code with the product path; the tests compare the engine with it.
 
@@ -354,6 +354,162 @@ def shared_kv_layer(x, w, cfg, eps, kvs, margins=None):
     return x
 
 
+def rotation(rot):
+    """(frequencies, factor of cosine and sine) of a rotation, the far pairs slowed down where it is scaled: a pair that
+    turns more than `fast` times over the original length keeps its frequency, one that turns less than `slow` times has
+    it divided by the factor, with a ramp over the pairs between."""
+    dims, base, sc = rot["dims"], float(rot["base"]), rot.get("scaling")
+    f = base ** (-2.0 * np.arange(dims // 2) / dims)
+    if not sc:
+        return f, 1.0
+    pair = lambda turns: dims * np.log(sc["original"] / (2 * np.pi * turns)) / (2 * np.log(base))
+    lo, hi = max(np.floor(pair(sc["fast"])), 0), min(np.ceil(pair(sc["slow"])), dims - 1)
+    ramp = np.clip((np.arange(dims // 2) - lo) / max(hi - lo, 0.001), 0, 1)
+    return f / sc["factor"] * ramp + f * (1 - ramp), 0.1 * np.log(sc["factor"]) + 1
+
+
+def turn_neighbours(x, positions, freq, gain=1.0):
+    """x [T, heads, >= 2 len(freq)]: dimension 2i turns with dimension 2i + 1 by position * freq[i]."""
+    out, n = x.copy(), len(freq)
+    ang = np.asarray(positions, dtype=np.float64)[:, None, None] * freq
+    c, s = (np.cos(ang) * gain).astype(x.dtype), (np.sin(ang) * gain).astype(x.dtype)
+    u, v = x[..., 0:2 * n:2], x[..., 1:2 * n:2]
+    out[..., 0:2 * n:2], out[..., 1:2 * n:2] = u * c - v * s, v * c + u * s
+    return out
+
+
+def in_chunk(pos, size):
+    """[T, T]: row i sees what came before it in its own chunk of positions, itself included."""
+    return (pos[:, None] >= pos[None, :]) & (pos[:, None] // size == pos[None, :] // size)
+
+
+def sunk_weights(score, sink):
+    """Softmax of the rows of `score` (-inf: unseen) with exp(sink) added to the denominator."""
+    top = np.maximum(score.max(axis=1, keepdims=True), sink)
+    e = np.exp(score - top)
+    return e / (e.sum(axis=1, keepdims=True) + np.exp(sink - top))
+
+
+def sink_heads(q, k, v, scale, seen, sink):
+    """Every head's weighted values [T, H, vdim]; heads share the key/value heads in equal runs."""
+    H, G = q.shape[1], k.shape[1]
+    out = np.empty((q.shape[0], H, v.shape[-1]), dtype=q.dtype)
+    for hh in range(H):
+        g = hh // (H // G)
+        score = np.where(seen, (q[:, hh] @ k[:, g].T) * q.dtype.type(scale), -np.inf)
+        out[:, hh] = sunk_weights(score, sink[hh]) @ v[:, g]
+    return out
+
+
+def biased(h, w, name):
+    return h @ w[name].T + w[name + ".b"]
+
+
+def normed_turned(h, w, cfg, eps, pos):
+    """Queries and keys with biases, normed head by head and rotated; values with biases."""
+    H, G, D, V, T = cfg["heads"], cfg["kv_heads"], cfg["dim"], cfg["vdim"], h.shape[0]
+    turn = rotation(cfg["rot"])
+    q = turn_neighbours(rms_norm(biased(h, w, "q").reshape(T, H, D), w["q.norm"], eps), pos, *turn)
+    k = turn_neighbours(rms_norm(biased(h, w, "k").reshape(T, G, D), w["k.norm"], eps), pos, *turn)
+    return q, k, biased(h, w, "v").reshape(T, G, V)
+
+
+def turned_values_attention(h, w, cfg, eps, positions=None):
+    """Causal attention whose values are rotated by their position and whose outputs are turned back by the row's."""
+    pos = np.arange(h.shape[0]) if positions is None else np.asarray(positions)
+    q, k, v = normed_turned(h, w, cfg, eps, pos)
+    freq, _ = rotation({"base": cfg["rot"]["base"], "dims": cfg["vdim"]})
+    o = sink_heads(q, k, turn_neighbours(v, pos, freq), cfg["scale"], pos[:, None] >= pos[None, :], w["sink"])
+    return biased(turn_neighbours(o, -pos, freq).reshape(len(h), -1), w, "o")
+
+
+def one_more_attention(h, w, cfg, eps, positions=None):
+    """Causal attention with one added to the softmax's denominator."""
+    pos = np.arange(h.shape[0]) if positions is None else np.asarray(positions)
+    q, k, v = normed_turned(h, w, cfg, eps, pos)
+    o = sink_heads(q, k, v, cfg["scale"], pos[:, None] >= pos[None, :], np.zeros(cfg["heads"], dtype=h.dtype))
+    return biased(o.reshape(len(h), -1), w, "o")
+
+
+def chunked_attention(h, w, cfg, eps, positions=None):
+    """Attention inside chunks of positions, without rotation, every output element with a logistic gate."""
+    pos, T = np.arange(h.shape[0]) if positions is None else np.asarray(positions), len(h)
+    q, k, v = ((h @ w[n].T).reshape(T, c, d) for n, c, d in (("q", cfg["heads"], cfg["dim"]), ("k", cfg["kv_heads"], cfg["dim"]),
+                                                            ("v", cfg["kv_heads"], cfg["vdim"])))
+    o = sink_heads(q, k, v, cfg["scale"], in_chunk(pos, cfg["mask"]["size"]), w["sink"])
+    return (o.reshape(T, -1) * sigmoid(h @ w["g"].T)) @ w["o"].T
+
+
+def forget_gate_recurrence(h, w, cfg, eps):
+    """Linear attention whose keys are what the forget gate lets go; returns (out [T, width], final state [heads, dim, vdim])."""
+    H, D, V, T = cfg["heads"], cfg["dim"], cfg["vdim"], h.shape[0]
+    q, v = silu(h @ w["q"].T).reshape(T, H, D), (h @ w["v"].T).reshape(T, H, V)
+    low = w["lower"]
+    f = (low + (1 - low) * sigmoid(h @ w["f"].T + w["f.b"])).reshape(T, H, D)
+    S = np.zeros((H, D, V), dtype=h.dtype)
+    o = np.empty((T, H, V), dtype=h.dtype)
+    for t in range(T):
+        S = f[t][:, :, None] * S + (1 - f[t])[:, :, None] * v[t][:, None, :]
+        o[t] = np.einsum("hdv,hd->hv", S, q[t])
+    return rms_norm(o, w["norm"], eps).reshape(T, H * V) @ w["o"].T, S
+
+
+def min_gru(h, w, cfg, eps):
+    """A gated recurrence element by element; returns (out [T, width], final state [size])."""
+    z, u = sigmoid(biased(h, w, "z")), biased(h, w, "x")
+    candidate = np.where(u >= 0, u + h.dtype.type(0.5), sigmoid(u))
+    S = np.zeros(cfg["width"], dtype=h.dtype)
+    states = np.empty_like(z)
+    for t in range(len(h)):
+        S = (1 - z[t]) * S + z[t] * candidate[t]
+        states[t] = S
+    return (states * silu(h @ w["g"].T)) @ w["o"].T, S
+
+
+def chunked_beside_forget_gate(h, w, cfg, eps):
+    left = chunked_attention(h, _sub(w, "left."), cfg["left"], eps)
+    right, _ = forget_gate_recurrence(h, _sub(w, "right."), cfg["right"], eps)
+    return h.dtype.type(cfg["left_scale"]) * left + h.dtype.type(cfg["right_scale"]) * right
+
+
+def one_more_beside_gru(h, w, cfg, eps):
+    left = one_more_attention(h, _sub(w, "left."), cfg["left"], eps)
+    right, _ = min_gru(h, _sub(w, "right."), cfg["right"], eps)
+    return (rms_norm(left, w["left.out"], eps) + rms_norm(right, w["right.out"], eps)) / 2
+
+
+def logistic_choice(z, top):
+    """One token's logits: the chosen experts and their scores."""
+    s = sigmoid(z)
+    chosen = np.argsort(-s, kind="stable")[:top]
+    return chosen, s[chosen]
+
+
+def weighted_input_moe(h, w, cfg):
+    """Gated experts whose input, not output, is multiplied by the weight."""
+    out = np.zeros_like(h)
+    for t in range(h.shape[0]):
+        for e, s in zip(*logistic_choice(w["router"] @ h[t], cfg["router"]["top"])):
+            out[t] += dense_mlp(s * h[t], _sub(w, f"e{e}."))
+    return out
+
+
+SIDE_MIXERS = {"attention": turned_values_attention, "parallel": chunked_beside_forget_gate, "parallel_2": one_more_beside_gru}
+
+
+def side_by_side_layer(x, w, cfg, eps, margins=None):
+    """A layer whose mixer and feed-forward read the same norm and join the residual together."""
+    h, f = rms_norm(x, 1 + w["norm1"], eps), cfg.get("mlp")
+    y = SIDE_MIXERS[cfg["type"]](h, _sub(w, "mix."), cfg["mixer"], eps)
+    if f and f["kind"] == "dense":
+        y = y + clamped_expert(h, _sub(w, "mlp."), f["limit"])
+    elif f:
+        y = y + weighted_input_moe(h, _sub(w, "mlp."), f)
+        if margins is not None:
+            margins.append(router_margin(h, _sub(w, "mlp."), f))
+    return x + y
+
+
 MIXERS = {"lightning": lambda *a: lightning(*a)[0], "latent_attention": latent_attention,
           "wkv": lambda *a: wkv(*a)[0], "parallel": parallel}
 
@@ -402,6 +558,13 @@ def forward(cfg, tensors, tokens, prec=np.float32, capture=None, margins=None):
             if capture is not None:
                 capture.append(x.copy())
         return rms_norm(x, 1 + w["final.norm"], eps) @ w["embed"].T
+    if cfg["architecture"] == "Marosun":
+        x = w["embed"][np.asarray(tokens)]
+        for i, c in enumerate(cfg["layers"]):
+            x = side_by_side_layer(x, _sub(w, f"l{i}."), c, eps, margins)
+            if capture is not None:
+                capture.append(x.copy())
+        return rms_norm(x, 1 + w["final.norm"], eps) @ w["head"].T
     if cfg["architecture"] == "Fedirax":
         x, kvs = w["embed"][np.asarray(tokens)] * prec(cfg["embedding"]["scale"]), []
         for i, c in enumerate(cfg["layers"]):

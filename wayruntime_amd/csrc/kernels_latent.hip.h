@@ -38,9 +38,9 @@ struct LatentArgs {
     void* q_out;
 };
 
-// (cos, sin) of position * freq, angles reduced in double
+// (cos, sin) of position * freq, times gain; angles reduced in double
 __global__ __launch_bounds__(256) void mix_rope_table_kernel(const uint32_t* row_pos, uint32_t rows, const double* freq,
-                                                             uint32_t half, float* table)
+                                                             uint32_t half, float gain, float* table)
 {
     const uint32_t i = blockIdx.x * 256 + threadIdx.x;
     if (i >= rows * half) return;
@@ -49,8 +49,8 @@ __global__ __launch_bounds__(256) void mix_rope_table_kernel(const uint32_t* row
     const float x = (float)((turns - rint(turns)) * 6.283185307179586477);
     float s, c;
     sincosf(x, &s, &c);
-    table[2 * (size_t)i] = c;
-    table[2 * (size_t)i + 1] = s;
+    table[2 * (size_t)i] = c * gain;
+    table[2 * (size_t)i + 1] = s * gain;
 }
 
 // Eight rotated elements i0 .. i0 + 7 of x (zero past rot).

@@ -29,6 +29,7 @@ struct MixGemmArgs {
     float scale, limit, slope, up_bias;
     const float* bias;
     const uint32_t* x_perm;
+    const float* x_scale;            // a factor per row of the input (applied to its products), or nullptr
     float* y;
     void* ya;
     void* h;
@@ -69,26 +70,10 @@ __device__ __forceinline__ float mix_gated(const MixGemmArgs& a, float gate, flo
     return gate * mix_sigmoid<F32>(y) * up;
 }
 
-// Accumulator tile nt of row group `group`: lane 16g + c holds outputs
-// 16 nt + 4g .. +3 of row 16 group + c.  `up`: the tile's partner (GATED, SPLIT_GATED).
+// Bias and activation of outputs n .. n + 3.
 template <bool F32>
-__device__ __forceinline__ void mix_store_tile(const MixGemmArgs& a, f32x4 v, f32x4 up, uint32_t nt, uint32_t group,
-                                               uint32_t z, int lane)
+__device__ __forceinline__ f32x4 mix_activate(const MixGemmArgs& a, f32x4 v, uint32_t n)
 {
-    const uint32_t c = lane & 15, g = lane >> 4, row = group * 16 + c, n = nt * 16 + 4 * g;
-    if (row >= a.rows || nt >= a.ntiles) return;
-    if (a.out >= kMixOutGated) {
-        if (a.out == kMixOutSplitGated && nt * 16 < a.n_split) {
-            *reinterpret_cast<f32x4*>(a.y + (size_t)row * a.ldy + n) = v;
-            *reinterpret_cast<f32x4*>(a.y + (size_t)row * a.ldy + n + 16) = up;
-            return;
-        }
-#pragma unroll
-        for (int i = 0; i < 4; i++) v[i] = mix_gated<F32>(a, v[i], up[i]);
-        const uint32_t to = nt - (a.out == kMixOutSplitGated ? a.n_split / 16 : 0u);
-        mix_put4<F32>(a.h, frag_elem(row, to / 2 * 16 + 4 * g, a.h_kt), v);
-        return;
-    }
     if (a.bias) {
         const f32x4 b = *reinterpret_cast<const f32x4*>(a.bias + n);
 #pragma unroll
@@ -110,6 +95,38 @@ __device__ __forceinline__ void mix_store_tile(const MixGemmArgs& a, f32x4 v, f3
             v[i] = p * p;
         }
     }
+    return v;
+}
+
+// Accumulator tile nt of row group `group`: lane 16g + c holds outputs
+// 16 nt + 4g .. +3 of row 16 group + c.  `up`: the tile's partner (GATED, SPLIT_GATED).
+template <bool F32>
+__device__ __forceinline__ void mix_store_tile(const MixGemmArgs& a, f32x4 v, f32x4 up, uint32_t nt, uint32_t group,
+                                               uint32_t z, int lane)
+{
+    const uint32_t c = lane & 15, g = lane >> 4, row = group * 16 + c, n = nt * 16 + 4 * g;
+    if (row >= a.rows || nt >= a.ntiles) return;
+    if (a.x_scale) {
+        const float s = a.x_scale[row];
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            v[i] *= s;
+            up[i] *= s;
+        }
+    }
+    if (a.out >= kMixOutGated) {
+        if (a.out == kMixOutSplitGated && nt * 16 < a.n_split) {
+            *reinterpret_cast<f32x4*>(a.y + (size_t)row * a.ldy + n) = mix_activate<F32>(a, v, n);
+            *reinterpret_cast<f32x4*>(a.y + (size_t)row * a.ldy + n + 16) = mix_activate<F32>(a, up, n + 16);
+            return;
+        }
+#pragma unroll
+        for (int i = 0; i < 4; i++) v[i] = mix_gated<F32>(a, v[i], up[i]);
+        const uint32_t to = nt - (a.out == kMixOutSplitGated ? a.n_split / 16 : 0u);
+        mix_put4<F32>(a.h, frag_elem(row, to / 2 * 16 + 4 * g, a.h_kt), v);
+        return;
+    }
+    v = mix_activate<F32>(a, v, n);
     if (a.scale != 0.f) {
 #pragma unroll
         for (int i = 0; i < 4; i++) v[i] *= a.scale;

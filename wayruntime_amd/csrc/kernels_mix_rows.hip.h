@@ -80,7 +80,8 @@ struct MixRowArgs {
     float eps;
     float* x;
     const float *y, *post, *add, *next;
-    const float* gate;
+    const float *pair_y[2], *pair_post[2];      // two more outputs, each normed
+    const float* gate;                // nullptr: ones
     const uint32_t* slot;
     uint32_t top;
     const float *side, *shared;      // weights of the input's own row and of the shared expert's, [rows][2]
@@ -111,7 +112,7 @@ __device__ __forceinline__ void mix_sub_chunk(const MixRowArgs& a, uint32_t r, u
 #pragma unroll
         for (uint32_t i = 0; i < 4; i++) {
             const size_t at = (size_t)r * a.top + min(t0 + i, a.top - 1);
-            gt[i] = a.gate[at];
+            gt[i] = a.gate ? a.gate[at] : 1.0f;
             slot[i] = t0 + i < a.top ? a.slot[at] : 0xFFFFFFFFu;
         }
 #pragma unroll
@@ -141,8 +142,9 @@ __device__ __forceinline__ void mix_sub_chunk(const MixRowArgs& a, uint32_t r, u
 }
 
 // x <- x + rmsnorm(y) * post (or + y) + add; h <- rmsnorm(x) * next
-// (EMBED: x <- rmsnorm(table[token]) * norm, or table[token] * scale, first).
-template <bool F32, int RPW, bool EMBED, bool HELD>
+// (EMBED: x <- rmsnorm(table[token]) * norm, or table[token] * scale, first;
+// PAIR: + rmsnorm(pair_y[i]) * pair_post[i] for both).
+template <bool F32, int RPW, bool EMBED, bool HELD, bool PAIR>
 __global__ __launch_bounds__(MixRowShape<RPW>::kThreads) void mix_residual_kernel(const MixRowArgs a)
 {
     using Sh = MixRowShape<RPW>;
@@ -205,9 +207,34 @@ __global__ __launch_bounds__(MixRowShape<RPW>::kThreads) void mix_residual_kerne
         }
         if (normed) inv = 1.0f / sqrtf(mix_row_sum<RPW>(ss, red) * invw + a.eps);
     }
+    float pair[PAIR ? 2 : 1][HELD && PAIR ? CH : 1][8], pinv[2];
+    if constexpr (PAIR) {
+#pragma unroll
+        for (int k = 0; k < 2; k++) {
+            const float* p = a.pair_y[k] + (size_t)r * a.wpad;
+            float ps = 0.f;
+            if constexpr (HELD) {
+#pragma unroll
+                for (int i = 0; i < CH; i++) {
+                    const uint32_t q = lr + i * Sh::kPerRow;
+                    if (q >= nq) continue;
+                    mix_load8(p + q * 8, pair[k][i]);
+#pragma unroll
+                    for (int j = 0; j < 8; j++) ps = fmaf(pair[k][i][j], pair[k][i][j], ps);
+                }
+            } else {
+                for (uint32_t q = lr; q < nq; q += Sh::kPerRow) {
+                    mix_load8(p + q * 8, pair[k][0]);
+#pragma unroll
+                    for (int j = 0; j < 8; j++) ps = fmaf(pair[k][0][j], pair[k][0][j], ps);
+                }
+            }
+            pinv[k] = 1.0f / sqrtf(mix_row_sum<RPW>(ps, red) * invw + a.eps);
+        }
+    }
 
     // x of one chunk, from the value above
-    auto second = [&](uint32_t q, float (&v)[8]) {
+    auto second = [&](uint32_t q, float (&v)[8], [[maybe_unused]] int at) {
         if constexpr (EMBED) {
             if (normed) {
                 float w[8];
@@ -230,6 +257,16 @@ __global__ __launch_bounds__(MixRowShape<RPW>::kThreads) void mix_residual_kerne
 #pragma unroll
                 for (int j = 0; j < 8; j++) x[j] += v[j] * inv * w[j];
             }
+            if constexpr (PAIR) {
+#pragma unroll
+                for (int k = 0; k < 2; k++) {
+                    float w[8];
+                    if constexpr (!HELD) mix_load8(a.pair_y[k] + (size_t)r * a.wpad + q * 8, pair[k][0]);
+                    mix_load8(a.pair_post[k] + q * 8, w);
+#pragma unroll
+                    for (int j = 0; j < 8; j++) x[j] = fmaf(pair[k][HELD ? at : 0][j] * pinv[k], w[j], x[j]);
+                }
+            }
             if (a.add) {
                 float w[8];
                 mix_load8(a.add + (size_t)r * a.wpad + q * 8, w);
@@ -239,7 +276,7 @@ __global__ __launch_bounds__(MixRowShape<RPW>::kThreads) void mix_residual_kerne
 #pragma unroll
             for (int j = 0; j < 8; j++) v[j] = x[j];
         }
-        if (live && (EMBED || a.y || a.add)) {
+        if (live && (EMBED || PAIR || a.y || a.add)) {
             mix_store8(xr + q * 8, v);
             if (EMBED && a.x0) mix_store8(a.x0 + (size_t)r * a.wpad + q * 8, v);
         }
@@ -250,7 +287,7 @@ __global__ __launch_bounds__(MixRowShape<RPW>::kThreads) void mix_residual_kerne
         for (int i = 0; i < CH; i++) {
             const uint32_t q = lr + i * Sh::kPerRow;
             if (q < nq) {
-                second(q, held[i]);
+                second(q, held[i], i);
 #pragma unroll
                 for (int j = 0; j < 8; j++) ss = fmaf(held[i][j], held[i][j], ss);
             }
@@ -259,7 +296,7 @@ __global__ __launch_bounds__(MixRowShape<RPW>::kThreads) void mix_residual_kerne
         for (uint32_t q = lr; q < nq; q += Sh::kPerRow) {
             float v[8];
             if (some) first(q, v);
-            second(q, v);
+            second(q, v, 0);
 #pragma unroll
             for (int j = 0; j < 8; j++) ss = fmaf(v[j], v[j], ss);
         }
@@ -282,7 +319,7 @@ __global__ __launch_bounds__(MixRowShape<RPW>::kThreads) void mix_residual_kerne
     } else {
         for (uint32_t q = lr; q < nq; q += Sh::kPerRow) {
             float v[8];
-            if (a.add || a.y || EMBED) {
+            if (a.add || a.y || EMBED || PAIR) {
                 if (live) {
                     mix_load8(xr + q * 8, v);              // this thread's own writes
                 } else {
@@ -480,10 +517,10 @@ __global__ __launch_bounds__(MixRowShape<RPW>::kThreads) void mix_gate_norm_kern
 struct MixRouteArgs {
     const float* z;
     uint32_t ldz, rows, outputs, experts, top, tile_groups, n_groups;     // outputs: experts, then those that pass the input on
-    uint32_t kinds, keep, softmax_all, shared_gate;                       // kinds: groups of neighbouring outputs, or 0
+    uint32_t kinds, keep, softmax_all, shared_gate, logistic;             // kinds: groups of neighbouring outputs, or 0
     float scale;
     const float* correction;
-    float *gate, *side;
+    float *gate, *side, *slot_weight;
     uint32_t* slot;                  // first the chosen output, then the slot
     uint32_t* perm;
     int32_t* group_expert;
@@ -574,7 +611,8 @@ __device__ __forceinline__ void mix_top(const MixRouteArgs& a, uint32_t row, int
                 if (a.softmax_all) term = s[i];
             }
         if (t == 0) best0 = bv;
-        const float g = a.softmax_all ? __int_as_float(__builtin_amdgcn_readlane(__float_as_int(term), be & 63u)) * zinv : expf(bv - best0);
+        const float g = a.softmax_all ? __int_as_float(__builtin_amdgcn_readlane(__float_as_int(term), be & 63u)) * zinv
+                        : a.logistic  ? 1.0f / (1.0f + expf(-bv)) : expf(bv - best0);
         sum += g;
         if (be >= a.experts) own += g;
         if ((uint32_t)lane == t) {
@@ -582,10 +620,11 @@ __device__ __forceinline__ void mix_top(const MixRouteArgs& a, uint32_t row, int
             put(t, be);
         }
     }
+    const bool as_is = a.softmax_all || a.logistic;
     const float over = a.softmax_all ? a.scale / (sum + 1e-20f) : 1.0f;
-    if ((uint32_t)lane < a.top) a.gate[(size_t)row * a.top + lane] = a.softmax_all ? mine * over : mine / sum;
+    if ((uint32_t)lane < a.top) a.gate[(size_t)row * a.top + lane] = as_is ? mine * over : mine / sum;
     if (a.side && lane == 0) {
-        a.side[(size_t)row * 2] = a.softmax_all ? own * over : own / sum;
+        a.side[(size_t)row * 2] = as_is ? own * over : own / sum;
         a.side[(size_t)row * 2 + 1] = a.shared_gate ? 1.0f / (1.0f + expf(-shared)) : 0.f;
     }
 }
@@ -613,7 +652,10 @@ __global__ __launch_bounds__(1024) void mix_order_kernel(const MixRouteArgs a)
     const uint32_t t = threadIdx.x, lane = t & 63, wave = t >> 6;
     const uint32_t n_slots = a.n_groups * 16, pairs = a.rows * a.top, run = a.tile_groups * 16;
     count[t] = 0;
-    for (uint32_t i = t; i < n_slots; i += 1024) a.perm[i] = 0xFFFFFFFFu;
+    for (uint32_t i = t; i < n_slots; i += 1024) {
+        a.perm[i] = 0xFFFFFFFFu;
+        if (a.slot_weight) a.slot_weight[i] = 0.f;
+    }
     for (uint32_t i = t; i < a.n_groups; i += 1024) a.group_expert[i] = -1;
     __syncthreads();
     if constexpr (TOP) {
@@ -651,6 +693,7 @@ __global__ __launch_bounds__(1024) void mix_order_kernel(const MixRouteArgs a)
         const uint32_t s = atomicAdd(&count[e], 1u);
         a.slot[i] = s;
         a.perm[s] = i / a.top;
+        if (a.slot_weight) a.slot_weight[s] = a.gate[i];   // (made here: ahead of two barriers)
     }
 }
 

@@ -1,10 +1,11 @@
 // Matrix-state recurrence with a decay per head and key channel made from the input:
-// per head a state S [dim][dim] (key channel by value column) in 32-bit floats,
+// per head a state S [dim][vdim] (key channel by value column) in 32-bit floats,
 //
-//   BONUS  o_t = (S_(t-1) + diag(u) k_t v_t^T)^T r_t    S_t = diag(w_t) S_(t-1) + k_t v_t^T
-//   DELTA  S_t = diag(w_t) S_(t-1) - b_t (n_t^T S_(t-1)) + k_t v_t^T     o_t = S_t^T r_t
+//   BONUS   o_t = (S_(t-1) + diag(u) k_t v_t^T)^T r_t    S_t = diag(w_t) S_(t-1) + k_t v_t^T
+//   DELTA   S_t = diag(w_t) S_(t-1) - b_t (n_t^T S_(t-1)) + k_t v_t^T     o_t = S_t^T r_t
+//   FORGET  S_t = diag(w_t) S_(t-1) + (1 - w_t) v_t^T     o_t = S_t^T r_t
 //
-// n_t the unit key, b_t = a_t n_t.  Everything between the projections' 32-bit rows
+// n_t the unit key, b_t = a_t n_t (BONUS, DELTA: vdim = dim).  Everything between the projections' 32-bit rows
 // and the next product's operand happens here: decays, rates, unit keys, the
 // recurrence, each head's norm and the gate.
 //
@@ -23,11 +24,12 @@
 //   S_16 = rho(chunk) S_0 + K^T V - B^T P
 //   A_xy[t][s] = sum over channels of x_t y_s rho(s, t or t-1),  K, B: k_s, b_s times rho(s, end)
 //
-// (BONUS: P, N, B fall away.)  Two launches:
+// (BONUS, FORGET: P, N, B fall away; DELTA, FORGET: r_t comes times w_t.)  Two launches:
 //   recur_chunk_kernel   parallel over (chunk, head), a wave each: the operands
 //                        T N~, R~, [K | -B], [A_rk | -A_rb], T A_nk and V
 //   recur_chain_kernel   a workgroup per (request, head), a wave per 16 value columns:
 //                        walks the chunks with S in registers, operands through LDS
+//                        (FORGET: per slice of the value columns, whose number is free)
 // and recur_gate_kernel norms and gates their rows.  Where requests times heads leave
 // most of the device idle, a request's chunks are walked in segments side by side: a
 // first walk takes every segment but the last from S = 0 (and, DELTA, from S = I
@@ -56,9 +58,11 @@ struct RecurArgs {
     const MixSeq* seqs;
     const MixChunk* chunks;
     const uint32_t* list;           // requests of this launch
-    uint32_t heads, dim, vtiles, silu;      // vtiles: value tiles of sixteen, chunked form
+    uint32_t heads, dim, vdim, vtiles;      // vtiles: value tiles of sixteen, chunked form
+    uint32_t gate;                  // kRecurGate*
+    uint32_t norm_step;             // from one head's norm weights to the next's: vdim, or 0 where the heads share them
     float gain, unit_eps, eps, out_scale;
-    const float *w0, *u, *ab, *norm;
+    const float *w0, *u, *ab, *norm;        // FORGET: w0 the gate's bias, u its lower bound
     const float* in;
     uint32_t ld, col_r, col_k, col_v, col_a, col_g;
     const float* z;
@@ -76,6 +80,9 @@ struct RecurArgs {
     float *seg_c, *seg_x;           // [request of the list][segment][heads]: C [32 KT][16 VT], X [32 KT][32 KT] or its diagonal
 };
 
+enum { kRecurBonus = 0, kRecurDelta = 1, kRecurForget = 2 };
+enum { kRecurGateLogistic = 0, kRecurGateSilu = 1, kRecurGateNone = 2 };
+
 __device__ __forceinline__ float recur_decay(const RecurArgs& a, float z)
 {
     return expf(a.gain > 0.f ? -a.gain / (1.0f + expf(-z)) : -expf(z));
@@ -83,7 +90,14 @@ __device__ __forceinline__ float recur_decay(const RecurArgs& a, float z)
 __device__ __forceinline__ float recur_gate(const RecurArgs& a, float g)
 {
     const float s = 1.0f / (1.0f + expf(-g));
-    return a.silu ? g * s : s;
+    return a.gate == kRecurGateSilu ? g * s : s;
+}
+// FORGET: the decay low + (1 - low) logistic(z) and what it leaves of one.
+__device__ __forceinline__ void recur_forget(float z, float low, float& w, float& k)
+{
+    const float e = expf(-fabsf(z)), over = 1.0f / (1.0f + e), s = z < 0.f ? e * over : over, t = z < 0.f ? over : e * over;
+    w = fmaf(1.0f - low, s, low);
+    k = (1.0f - low) * t;
 }
 
 // ---- token by token ---------------------------------------------------------
@@ -232,6 +246,66 @@ __global__ __launch_bounds__(4 * DP) void recur_step_kernel(const RecurArgs a)
 #pragma unroll
     for (int j = 0; j < DPT; j++)
         if (has && d0 + j < D) out[(size_t)(d0 + j) * D + c] = S[j];
+}
+
+// FORGET.  grid (requests, heads), 4 CP threads: thread t has value column t % CP, channels DPT (t / CP) .. +DPT
+template <bool F32, int DPT, int CP>
+__global__ __launch_bounds__(4 * CP) void recur_forget_step_kernel(const RecurArgs a)
+{
+    using E = typename MixAct<F32>::E;
+    constexpr int DP = 4 * DPT, WV = CP >= 64 ? CP / 64 : 1;       // waves that put the columns together
+    __shared__ float sr[DP], sk[DP], sw[DP], red[4 * CP], sq[WV];
+    const uint32_t t = threadIdx.x, head = blockIdx.y, part = t / CP, c = t % CP, d0 = part * DPT, D = a.dim, V = a.vdim;
+    const uint32_t lane = t & 63, wave = t >> 6;
+    const bool has = c < V, own = t < CP && has;
+    const MixSeq s = a.seqs[a.list[blockIdx.x]];
+    const size_t head_elems = (size_t)D * V;
+    const float* in = a.state + ((size_t)s.state_in * a.heads + head) * head_elems;
+    float* out = a.state + ((size_t)s.state_out * a.heads + head) * head_elems;
+    float S[DPT];
+#pragma unroll
+    for (int j = 0; j < DPT; j++) S[j] = (s.pos0 > 0 && has && d0 + j < D) ? in[(size_t)(d0 + j) * V + c] : 0.f;
+    const float nrm = own ? a.norm[head * a.norm_step + c] * a.out_scale : 0.f;
+    const uint32_t npad = (a.heads * V + 31) / 32 * 32;
+    for (uint32_t i = 0; i < s.rows; i++) {
+        const uint32_t r = s.row0 + i;
+        const float* row = a.in + (size_t)r * a.ld;
+        const float vv = has ? row[a.col_v + head * V + c] : 0.f;
+        for (uint32_t d = t; d < DP; d += 4 * CP) {
+            float w = 1.0f, k = 0.f;
+            if (d < D) recur_forget(row[a.col_k + head * D + d] + a.w0[head * D + d], a.u[head * D + d], w, k);
+            sw[d] = w;
+            sk[d] = k;
+            sr[d] = d < D ? row[a.col_r + head * D + d] : 0.f;
+        }
+        __syncthreads();
+        float o = 0.f;
+#pragma unroll
+        for (int j = 0; j < DPT; j++) {
+            S[j] = fmaf(sk[d0 + j], vv, sw[d0 + j] * S[j]);
+            o = fmaf(sr[d0 + j], S[j], o);
+        }
+        red[t] = o;
+        __syncthreads();
+        o = own ? (red[c] + red[CP + c]) + (red[2 * CP + c] + red[3 * CP + c]) : 0.f;
+        if (wave < WV) {
+            const float ss = recur_wave_sum(o * o);
+            if (lane == 0) sq[wave] = ss;
+        }
+        __syncthreads();
+        if (own) {
+            float ss = 0.f;
+#pragma unroll
+            for (int x = 0; x < WV; x++) ss += sq[x];
+            reinterpret_cast<E*>(a.h)[frag_elem(r, a.col_h + head * V + c, a.h_kt)] = (E)(o / sqrtf(ss / (float)V + a.eps) * nrm);
+        }
+        // (sr, sk, sw: read ahead of the last two barriers; red and sq: written again only after the next row's)
+        if (head + 1 == a.heads && t < npad - a.heads * V)        // pads of the operand
+            reinterpret_cast<E*>(a.h)[frag_elem(r, a.col_h + a.heads * V + t, a.h_kt)] = (E)0.f;
+    }
+#pragma unroll
+    for (int j = 0; j < DPT; j++)
+        if (has && d0 + j < D) out[(size_t)(d0 + j) * V + c] = S[j];
 }
 
 // ---- by chunks --------------------------------------------------------------
@@ -419,9 +493,10 @@ __host__ __device__ constexpr int recur_chunk_lds(int kt, bool delta)
 
 // grid (chunks of 64 rows, heads): wave w of four has rows 16w .. 16w + 15.  `whole`: dim and every column are
 // multiples of four.
-template <bool F32, int KT, bool DELTA>
+template <bool F32, int KT, int RULE>
 __global__ __launch_bounds__(256, KT <= 2 ? 2 : 1) void recur_chunk_kernel(const RecurArgs a, const uint32_t whole)
 {
+    constexpr bool DELTA = RULE == kRecurDelta, FORGET = RULE == kRecurForget;
     using U = RecurUnit<KT, DELTA>;
     constexpr int LD = 32 * KT + 4;
     extern __shared__ __attribute__((aligned(16))) float recur_smem[];
@@ -442,7 +517,7 @@ __global__ __launch_bounds__(256, KT <= 2 ? 2 : 1) void recur_chunk_kernel(const
     unsigned char* unit = a.ops + ((size_t)(blockIdx.x * kRecurSubs + wave) * a.heads + head) *
                                       (size_t)recur_unit_kib(KT, DELTA, vtiles) * 1024;
 
-    float q[KT][8], k[KT][8], n[DELTA ? KT : 1][8], b[DELTA ? KT : 1][8];      // q: r, in DELTA times this token's decay
+    float q[KT][8], k[KT][8], n[DELTA ? KT : 1][8], b[DELTA ? KT : 1][8];      // q: r, times this token's decay but in BONUS
     float E[KT][8], F[KT][8], B[KT][8];                           // rho: after the token in its block, ahead of it, the block
     float k2 = 0.f, drk = 0.f, drb = 0.f;
 #pragma unroll
@@ -450,7 +525,9 @@ __global__ __launch_bounds__(256, KT <= 2 ? 2 : 1) void recur_chunk_kernel(const
 #pragma unroll
         for (int h = 0; h < 2; h++) {
             const uint32_t d = 32 * t + 16 * h + 4 * g;
-            const f32x4 r4 = recur_load4(row + a.col_r, d, D, whole), k4 = recur_load4(row + a.col_k, d, D, whole);
+            const f32x4 r4 = recur_load4(row + a.col_r, d, D, whole);
+            f32x4 k4 = r4;
+            if constexpr (!FORGET) k4 = recur_load4(row + a.col_k, d, D, whole);
             const f32x4 z4 = recur_load4(zrow, d, D, whole), w4 = recur_load4(a.w0 + hd, d, D, whole);
             const f32x4 x4 = recur_load4((DELTA ? a.ab : a.u) + hd, d, D, whole);
             f32x4 a4 = x4;
@@ -458,9 +535,18 @@ __global__ __launch_bounds__(256, KT <= 2 ? 2 : 1) void recur_chunk_kernel(const
 #pragma unroll
             for (int j = 0; j < 4; j++) {
                 const bool on = live && d + j < D;
-                const float rr = on ? r4[j] : 0.f, kk = on ? k4[j] : 0.f, w = on ? recur_decay(a, z4[j] + w4[j]) : 1.0f;
+                const float rr = on ? r4[j] : 0.f;
+                float kk, w;
+                if constexpr (FORGET) {
+                    recur_forget(z4[j] + w4[j], x4[j], w, kk);
+                    w = on ? w : 1.0f;
+                    kk = on ? kk : 0.f;
+                } else {
+                    kk = on ? k4[j] : 0.f;
+                    w = on ? recur_decay(a, z4[j] + w4[j]) : 1.0f;
+                }
                 const int e = 4 * h + j;
-                q[t][e] = DELTA ? rr * w : rr;
+                q[t][e] = DELTA || FORGET ? rr * w : rr;
                 k[t][e] = kk;
                 B[t][e] = w;
                 E[t][e] = F[t][e] = 1.0f;
@@ -472,7 +558,7 @@ __global__ __launch_bounds__(256, KT <= 2 ? 2 : 1) void recur_chunk_kernel(const
                     drk = fmaf(rr, kk, drk);
                     drb = fmaf(rr, rate * kk, drb);
                 } else {
-                    drk = fmaf(rr * x4[j], kk, drk);
+                    drk = fmaf(FORGET ? rr : rr * x4[j], kk, drk);
                 }
             }
         }
@@ -643,7 +729,7 @@ __global__ __launch_bounds__(256, KT <= 2 ? 2 : 1) void recur_chunk_kernel(const
 #pragma unroll
         for (int j = 0; j < 4; j++) {
             const uint32_t tok = wave * kRecurSub + 4 * g + j, col = 16 * t + c;
-            v[j] = tok < ch.rows && col < D ? a.in[(size_t)(ch.row0 + tok) * a.ld + a.col_v + hd + col] : 0.f;
+            v[j] = tok < ch.rows && col < a.vdim ? a.in[(size_t)(ch.row0 + tok) * a.ld + a.col_v + head * a.vdim + col] : 0.f;
         }
         recur_put<F32>(unit, U::kV + t, lane, recur_op4<F32>(v));
     }
@@ -712,17 +798,19 @@ __device__ __forceinline__ f32x4 recur_mm_many(const RecurOp8<false> (&a)[N], co
 
 // Grid (requests * segments, heads), a wave per 16 value columns (1, 2, 4 or 8 of them, VT).  A stage of the ring is
 // read into registers a step before it is used, and copied over from then on.  CARRY: the walk without outputs, of
-// every segment but the last; DELTA has z = 1 for the walk from S = I.
+// every segment but the last; DELTA has z = 1 for the walk from S = I.  Without DELTA z is the slice of VT value tiles.
 template <bool F32, int KT, bool DELTA, int VT, bool CARRY>
 __global__ __launch_bounds__(64 * VT, 2) void recur_chain_kernel(const RecurArgs a)
 {
     using U = RecurUnit<KT, DELTA>;
-    constexpr int ALL = recur_unit_kib(KT, DELTA, VT), K0 = CARRY ? U::kG : 0, UNIT = ALL - K0;
+    constexpr int K0 = CARRY ? U::kG : 0, UNIT = recur_unit_kib(KT, DELTA, VT) - K0;
     constexpr int RING = recur_ring(KT, DELTA), CPW = (UNIT + VT - 1) / VT, STORES = CARRY ? 0 : 4;
     // what is on its way behind the stage waited for: RING - 2 stages, and the stores of each step made since
     constexpr int EARLY = (RING - 2) * CPW, FULL = (RING - 2) * (CPW + STORES) + STORES, FIRST = (RING - 1) * CPW;
     static_assert(FULL < 64 && FIRST < 64, "vmcnt");
-    constexpr uint32_t KP = 32 * KT, CP = 16 * VT;
+    constexpr uint32_t KP = 32 * KT;
+    // a sub-chunk's operands and value columns in all, and those ahead of this slice
+    const uint32_t all = (uint32_t)U::kV + a.vtiles, CP = 16 * a.vtiles, first_tile = DELTA ? 0 : blockIdx.z * VT;
     extern __shared__ __attribute__((aligned(16))) unsigned char recur_lds[];
     const uint32_t segs = CARRY ? a.n_seg - 1 : a.n_seg, item = blockIdx.x / segs, seg = blockIdx.x % segs;
     const MixSeq s = a.seqs[a.list[item]];
@@ -731,19 +819,21 @@ __global__ __launch_bounds__(64 * VT, 2) void recur_chain_kernel(const RecurArgs
     const bool values = !(CARRY && DELTA) || blockIdx.z == 0;     // (else: from S = I, without values)
     const uint32_t head = blockIdx.y, D = a.dim, sub0 = s.chunk0 * kRecurSubs;
     const int lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4;
-    const uint32_t wave = (uint32_t)__builtin_amdgcn_readfirstlane(threadIdx.x >> 6), col = wave * 16 + c;
+    const uint32_t wave = (uint32_t)__builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const uint32_t col = (first_tile + wave) * 16 + c, V = a.vdim;
     const uint32_t lds0 = (uint32_t)__builtin_amdgcn_readfirstlane((uint32_t)(uintptr_t)recur_lds);
     auto issue = [&](uint32_t sub) {                              // (past the end: the last one again)
         const unsigned char* base =
-            uniform_ptr(a.ops + (((size_t)(sub0 + min(begin + sub, end - 1)) * a.heads + head) * ALL + K0) * 1024);
+            uniform_ptr(a.ops + (((size_t)(sub0 + min(begin + sub, end - 1)) * a.heads + head) * all + K0) * 1024);
         const uint32_t to = lds0 + sub % RING * UNIT * 1024;
 #pragma unroll
         for (int i = 0; i < CPW; i++) {
             const uint32_t k = min(wave * CPW + i, (uint32_t)(UNIT - 1));        // (a repeat copies the same bytes)
-            lds_direct_load(to + k * 1024, base + (size_t)k * 1024, lane * 16);
+            const uint32_t from = k + (k >= (uint32_t)(U::kV - K0) ? first_tile : 0u);
+            lds_direct_load(to + k * 1024, base + (size_t)from * 1024, lane * 16);
         }
     };
-    const size_t head_elems = (size_t)D * D;
+    const size_t head_elems = (size_t)D * V;
     const float* in = a.state + ((size_t)s.state_in * a.heads + head) * head_elems;
     float* out = a.state + ((size_t)s.state_out * a.heads + head) * head_elems;
     auto seg_at = [&](uint32_t q) { return ((size_t)item * a.n_seg + q) * a.heads + head; };
@@ -754,7 +844,7 @@ __global__ __launch_bounds__(64 * VT, 2) void recur_chain_kernel(const RecurArgs
         for (int i = 0; i < 4; i++) {
             const uint32_t d = 16 * t + 4 * g + i;
             if constexpr (CARRY) S[t][i] = values || d != col ? 0.f : 1.0f;
-            else S[t][i] = (s.pos0 > 0 && d < D && col < D) ? in[(size_t)d * D + col] : 0.f;
+            else S[t][i] = (s.pos0 > 0 && d < D && col < V) ? in[(size_t)d * V + col] : 0.f;
             gp[t][i] = 1.0f;
         }
     if constexpr (!CARRY) {
@@ -776,7 +866,7 @@ __global__ __launch_bounds__(64 * VT, 2) void recur_chain_kernel(const RecurArgs
                     for (int k = 0; k < KT; k++) {
                         const f32x4 lo = *reinterpret_cast<const f32x4*>(X + (size_t)16 * t * KP + 32 * k);
                         f32x4 hi = f32x4{0.f, 0.f, 0.f, 0.f};
-                        if (32 * k + 16 < (int)CP) hi = *reinterpret_cast<const f32x4*>(X + (size_t)16 * t * KP + 32 * k + 16);
+                        if (32 * k + 16 < 16 * VT) hi = *reinterpret_cast<const f32x4*>(X + (size_t)16 * t * KP + 32 * k + 16);
                         next[t] = recur_mm(recur_op8<F32>(lo, hi), So[k], next[t]);
                     }
                     if constexpr (KT >= 4) __builtin_amdgcn_sched_barrier(0);    // (not every row's operands at once)
@@ -863,7 +953,7 @@ __global__ __launch_bounds__(64 * VT, 2) void recur_chain_kernel(const RecurArgs
         for (int t = 0; t < 2 * KT; t++)
 #pragma unroll
             for (int i = 0; i < 4; i++) to[(size_t)(16 * t + 4 * g + i) * ld] = S[t][i];
-        if (!DELTA && wave == 0 && c == 0) {
+        if (!DELTA && first_tile + wave == 0 && c == 0) {
 #pragma unroll
             for (int t = 0; t < 2 * KT; t++) *reinterpret_cast<f32x4*>(a.seg_x + seg_at(seg) * KP + 16 * t + 4 * g) = gp[t];
         }
@@ -875,7 +965,7 @@ __global__ __launch_bounds__(64 * VT, 2) void recur_chain_kernel(const RecurArgs
 #pragma unroll
         for (int i = 0; i < 4; i++) {
             const uint32_t d = 16 * t + 4 * g + i;
-            if (d < D && col < D) out[(size_t)d * D + col] = S[t][i];
+            if (d < D && col < V) out[(size_t)d * V + col] = S[t][i];
         }
 }
 
@@ -885,7 +975,8 @@ __global__ __launch_bounds__(256) void recur_gate_kernel(const RecurArgs a)
 {
     using E = typename MixAct<F32>::E;
     const MixChunk ch = a.chunks[blockIdx.x];
-    const uint32_t head = blockIdx.y, D = a.dim, hd = head * D, vp = a.vtiles * 16;
+    const uint32_t head = blockIdx.y, D = a.vdim, hd = head * D, vp = a.vtiles * 16;
+    const float* norm = a.norm + head * a.norm_step;
     const uint32_t i = threadIdx.x / 4, q = threadIdx.x % 4;
     if (i >= ch.rows) return;                                     // (no barrier below)
     const uint32_t r = ch.row0 + i, npad = (a.heads * D + 31) / 32 * 32;
@@ -911,15 +1002,19 @@ __global__ __launch_bounds__(256) void recur_gate_kernel(const RecurArgs a)
         for (uint32_t d = q * 8; d < D; d += 32) {
             float v[8], w[8], x[8];
             mix_load8(o + d, v);
-            mix_load8(g + d, x);
-            mix_load8(a.norm + hd + d, w);
+            mix_load8(norm + d, w);
+            if (a.gate != kRecurGateNone) {                       // (uniform)
+                mix_load8(g + d, x);
 #pragma unroll
-            for (int j = 0; j < 8; j++) v[j] *= inv * w[j] * recur_gate(a, x[j]);
+                for (int j = 0; j < 8; j++) w[j] *= recur_gate(a, x[j]);
+            }
+#pragma unroll
+            for (int j = 0; j < 8; j++) v[j] *= inv * w[j];
             mix_store_unit<F32>(h, frag_unit(r, (a.col_h + hd + d) / 8, a.h_kt), v);
         }
     } else {
         for (uint32_t d = q; d < D; d += 4)
-            h[frag_elem(r, a.col_h + hd + d, a.h_kt)] = (E)(o[d] * inv * a.norm[hd + d] * recur_gate(a, g[d]));
+            h[frag_elem(r, a.col_h + hd + d, a.h_kt)] = (E)(o[d] * inv * norm[d] * (a.gate != kRecurGateNone ? recur_gate(a, g[d]) : 1.0f));
     }
     if (head + 1 == a.heads)
         for (uint32_t d = a.heads * D + q; d < npad; d += 4) h[frag_elem(r, a.col_h + d, a.h_kt)] = (E)0.f;

@@ -1,6 +1,9 @@
-// Sliding-window attention over grouped keys and values.  Optionally each head has a sink
-// s: its weights are exp(score) / (exp(s) + sum of exp(score)), so a row may attend to
-// nothing at all.  Scores may be capped (cap * tanh(score / cap)) and a head's output gated.
+// Attention over grouped keys and values inside a sliding window, or inside chunks of
+// positions (a row sees its own chunk from the chunk's first position on).  Optionally each
+// head has a sink s: its weights are exp(score) / (exp(s) + sum of exp(score)), so a row may
+// attend to nothing at all.  Scores may be capped (cap * tanh(score / cap)), and a head's
+// output gated, whole or element by element.  Values may be turned by their position like
+// the keys; a row's output is then turned back by the row's.
 //
 // With two maps every head weighs the same values twice, by two queries over two keys, and
 // its output is the first sum less `diff` times the second, over its root mean square.
@@ -34,11 +37,12 @@ struct WindowArgs {
     const MixSeq* seqs;
     const uint32_t *row_seq, *row_pos, *pages;
     uint32_t rows, heads, kvh, group;            // group = heads / kvh
-    uint32_t dim, dimp, vdim, vdimp, half, window, norm_values;
+    uint32_t dim, dimp, vdim, vdimp, half, window, chunk, norm_values;
     uint32_t maps, dimk, neighbours, key_heads;  // dimk = maps * dimp; key_heads: key/value heads to append (0 or kvh)
     float scale, out_scale, eps, softcap, diff;
     const float *q_norm, *k_norm, *gate;
-    uint32_t ldg;
+    uint32_t ldg, gate_wide;                     // gate_wide: an element's own, head by head
+    const float* vtable;                         // angles of the step's rows over the values, [rows][vdim / 2][2]
     void* cache;
     const float* in;
     uint32_t ld, col_q, col_k, col_v;
@@ -52,6 +56,13 @@ struct WindowArgs {
     uint32_t splits, split_keys;
     float *part_o, *part_ml;
 };
+
+// First position the row at `pos` sees.
+__host__ __device__ __forceinline__ uint32_t window_lo(uint32_t pos, uint32_t window, uint32_t chunk)
+{
+    if (chunk) return pos - pos % chunk;
+    return pos + 1 > window ? pos + 1 - window : 0;
+}
 
 // element of (position in page, column) inside a head's V block
 __device__ __forceinline__ uint32_t window_v_elem(uint32_t at, uint32_t d, uint32_t vdimp)
@@ -113,6 +124,15 @@ __device__ __forceinline__ float window_inv_rms(const WindowArgs& a, const float
     return 1.0f / sqrtf(ss / (float)a.dim + a.eps);
 }
 
+// Element d of row r's value, turned where values are.
+__device__ __forceinline__ float window_value(const WindowArgs& a, uint32_t r, uint32_t kvh, uint32_t d)
+{
+    const float* v = a.in + (size_t)r * a.ld + a.col_v + kvh * a.vdim;
+    if (!a.vtable) return v[d];                            // uniform
+    const float* cs = a.vtable + (size_t)r * a.vdim + (d & ~1u);
+    return v[d] * cs[0] + (d & 1 ? v[d - 1] : -v[d + 1]) * cs[1];
+}
+
 // grid (rows / 4, key_heads + slices of 4 rows' query units)
 template <bool F32>
 __global__ __launch_bounds__(256) void window_append_kernel(const WindowArgs a)
@@ -166,7 +186,7 @@ __global__ __launch_bounds__(256) void window_append_kernel(const WindowArgs a)
         V4 x;
 #pragma unroll
         for (uint32_t i = 0; i < 4; i++)
-            x[i] = (E)(i < n && d < a.vdim ? a.in[(size_t)(r0 + min(i, n - 1)) * a.ld + a.col_v + kvh * a.vdim + d] * s_inv[i] : 0.f);
+            x[i] = (E)(i < n && d < a.vdim ? window_value(a, r0 + min(i, n - 1), kvh, d) * s_inv[i] : 0.f);
         if (run) {                                         // four positions of one column side by side
             *reinterpret_cast<V4*>(head_block(r0) + kMixPage * a.dimk + window_v_elem(p0 % kMixPage, d, a.vdimp)) = x;
         } else {
@@ -180,7 +200,41 @@ __global__ __launch_bounds__(256) void window_append_kernel(const WindowArgs a)
 template <bool F32>
 __device__ __forceinline__ float window_factor(const WindowArgs& a, uint32_t r, uint32_t h)
 {
-    return a.gate ? a.out_scale * mix_sigmoid<F32>(a.gate[(size_t)r * a.ldg + h]) : a.out_scale;
+    return a.gate && !a.gate_wide ? a.out_scale * mix_sigmoid<F32>(a.gate[(size_t)r * a.ldg + h]) : a.out_scale;
+}
+
+// Column col of head h's output of row r, turned back and times the element's gate; pair: the column it is paired with.
+template <bool F32>
+__device__ __forceinline__ float window_finish(const WindowArgs& a, uint32_t r, uint32_t h, uint32_t col, float v, float pair)
+{
+    if (col >= a.vdim) return v;                           // (zeros)
+    if (a.vtable) {                                        // uniform, like the gate
+        const float* cs = a.vtable + (size_t)r * a.vdim + (col & ~1u);
+        v = v * cs[0] + (col & 1 ? -pair : pair) * cs[1];
+    }
+    return a.gate_wide ? v * mix_sigmoid<F32>(a.gate[(size_t)r * a.ldg + h * a.vdim + col]) : v;
+}
+
+// Columns col .. col + 3 of it (col a multiple of four).
+__device__ __forceinline__ f32x4 window_finish4(const WindowArgs& a, uint32_t r, uint32_t h, uint32_t col, f32x4 v)
+{
+    if (a.vdim % 4 == 0) {
+        if (col >= a.vdim) return v;
+        if (a.vtable) {
+            const f32x4 cs = *reinterpret_cast<const f32x4*>(a.vtable + (size_t)r * a.vdim + col);
+            v = f32x4{v[0] * cs[0] + v[1] * cs[1], v[1] * cs[0] - v[0] * cs[1], v[2] * cs[2] + v[3] * cs[3], v[3] * cs[2] - v[2] * cs[3]};
+        }
+        if (a.gate_wide) {
+            const f32x4 gt = *reinterpret_cast<const f32x4*>(a.gate + (size_t)r * a.ldg + h * a.vdim + col);
+#pragma unroll
+            for (int i = 0; i < 4; i++) v[i] *= mix_sigmoid<false>(gt[i]);
+        }
+        return v;
+    }
+    f32x4 o;
+#pragma unroll
+    for (int i = 0; i < 4; i++) o[i] = window_finish<false>(a, r, h, col + i, v[i], v[i ^ 1]);
+    return o;
 }
 
 // One wave per (row, head), a lane per key of a page.  LDS: a query row and every map's output row as floats, 64 weights.
@@ -194,7 +248,7 @@ __global__ __launch_bounds__(64) void window_attend_any_kernel(const WindowArgs 
     float *q = window_smem, *w = q + a.dimp, *outs = w + 64;
     const V8* qf = reinterpret_cast<const V8*>(a.q);
     const MixSeq s = a.seqs[a.row_seq[r]];
-    const uint32_t pos = a.row_pos[r], lo = pos + 1 > a.window ? pos + 1 - a.window : 0;
+    const uint32_t pos = a.row_pos[r], lo = window_lo(pos, a.window, a.chunk);
     for (uint32_t m = 0; m < a.maps; m++) {
         float* o = outs + m * a.vdimp;
         for (uint32_t u = lane; u < per_map; u += 64) {
@@ -260,7 +314,9 @@ __global__ __launch_bounds__(64) void window_attend_any_kernel(const WindowArgs 
         factor /= sqrtf(ss / (float)a.vdim + a.eps);
     }
     E* out = reinterpret_cast<E*>(a.o);
-    for (uint32_t k = lane; k < a.vdimp; k += 64) out[frag_elem(r, h * a.vdimp + k, a.o_kt)] = (E)(outs[k] * factor);
+    __syncthreads();                                       // (a pair's other column is another lane's)
+    for (uint32_t k = lane; k < a.vdimp; k += 64)
+        out[frag_elem(r, h * a.vdimp + k, a.o_kt)] = (E)(window_finish<F32>(a, r, h, k, outs[k], outs[k ^ 1u]) * factor);
 }
 
 // ---- matrix forms (bfloat16; head sizes padded to 32, 64 or 128) -------------
@@ -378,7 +434,7 @@ __global__ __launch_bounds__(256, 2) void window_prefill_kernel(const WindowArgs
     const MixSeq s = a.seqs[pick_seq];
     const uint32_t m_end = s.rows * H, m0 = tile * ROWS;
     const uint32_t pos_first = s.pos0 + m0 / H, pos_last = s.pos0 + (min(m0 + ROWS, m_end) - 1) / H;
-    const uint32_t j_begin = (pos_first + 1 > a.window ? pos_first + 1 - a.window : 0) / kMixPage * kMixPage, j_end = pos_last + 1;
+    const uint32_t j_begin = window_lo(pos_first, a.window, a.chunk) / kMixPage * kMixPage, j_end = pos_last + 1;
     const WindowScore score(a);
 
     uint32_t m[NR], pos[NR], lo[NR];
@@ -389,7 +445,7 @@ __global__ __launch_bounds__(256, 2) void window_prefill_kernel(const WindowArgs
         m[t] = m0 + wave * WROWS + (MAPS == 1 ? t * 16 : 0) + c;
         const uint32_t mm = min(m[t], m_end - 1), head = kvh * H + mm % H;
         pos[t] = s.pos0 + mm / H;
-        lo[t] = pos[t] + 1 > a.window ? pos[t] + 1 - a.window : 0;
+        lo[t] = window_lo(pos[t], a.window, a.chunk);
 #pragma unroll
         for (int k = 0; k < KQ; k++)
             qv[t][k] = reinterpret_cast<const bf16x8*>(a.q)[frag_unit(
@@ -399,8 +455,8 @@ __global__ __launch_bounds__(256, 2) void window_prefill_kernel(const WindowArgs
     }
     // positions this wave's rows span: a page between them needs no mask
     const uint32_t w0 = min(m0 + wave * WROWS, m_end - 1), w1 = min(m0 + wave * WROWS + WROWS - 1, m_end - 1);
-    const uint32_t w_pos0 = s.pos0 + w0 / H, w_pos1 = s.pos0 + w1 / H, w_lo1 = w_pos1 + 1 > a.window ? w_pos1 + 1 - a.window : 0;
-    const uint32_t w_lo0 = w_pos0 + 1 > a.window ? w_pos0 + 1 - a.window : 0;
+    const uint32_t w_pos0 = s.pos0 + w0 / H, w_pos1 = s.pos0 + w1 / H;
+    const uint32_t w_lo0 = window_lo(w_pos0, a.window, a.chunk), w_lo1 = window_lo(w_pos1, a.window, a.chunk);
     f32x4 acc[NR][2 * VT];
 #pragma unroll
     for (int t = 0; t < NR; t++)
@@ -479,8 +535,9 @@ __global__ __launch_bounds__(256, 2) void window_prefill_kernel(const WindowArgs
 #pragma unroll
         for (int k = 0; k < 2 * VT; k++) {
             bf16x4 o;
+            const f32x4 v = window_finish4(a, r, h, k * 16 + 4 * g, acc[t][k]);
 #pragma unroll
-            for (int i = 0; i < 4; i++) o[i] = (__bf16)(acc[t][k][i] * inv);
+            for (int i = 0; i < 4; i++) o[i] = (__bf16)(v[i] * inv);
             *reinterpret_cast<bf16x4*>(out + frag_elem(r, h * VT * 32 + k * 16 + 4 * g, a.o_kt)) = o;
         }
     }
@@ -497,7 +554,7 @@ __global__ __launch_bounds__(256, KQ + VT > 8 ? 1 : 2) void window_decode_kernel
     const uint32_t columns = a.group * MAPS, tiles = (columns + 15) / 16, split = blockIdx.y;
     const uint32_t kvh = blockIdx.x % a.kvh, tile = blockIdx.x / a.kvh % tiles, ri = blockIdx.x / a.kvh / tiles;
     const LatentRow lr = a.drows[ri];
-    const uint32_t r = lr.row, pos = lr.pos, lo = pos + 1 > a.window ? pos + 1 - a.window : 0;
+    const uint32_t r = lr.row, pos = lr.pos, lo = window_lo(pos, a.window, a.chunk);
     const uint32_t first = lo / 32 * 32 + split * a.split_keys, end = min(pos + 1, first + a.split_keys);
     const WindowScore score(a);
     const uint32_t member = tile * 16 + c, column = min(member, columns - 1), head = kvh * a.group + column / MAPS, map = column % MAPS;
@@ -597,8 +654,9 @@ __global__ __launch_bounds__(256, KQ + VT > 8 ? 1 : 2) void window_decode_kernel
 #pragma unroll
         for (int k = 0; k < 2 * VT; k++) {
             bf16x4 o;
+            const f32x4 v = window_finish4(a, r, head, k * 16 + 4 * g, acc[k]);
 #pragma unroll
-            for (int i = 0; i < 4; i++) o[i] = (__bf16)(acc[k][i] * inv);
+            for (int i = 0; i < 4; i++) o[i] = (__bf16)(v[i] * inv);
             *reinterpret_cast<bf16x4*>(out + frag_elem(r, head * VT * 32 + k * 16 + 4 * g, a.o_kt)) = o;
         }
         return;
@@ -663,7 +721,8 @@ __global__ __launch_bounds__(64 * MAPS) void window_combine_kernel(const WindowA
 #pragma unroll
     for (int i = 0; i < COLS; i++) {
         const uint32_t col = t + 64 * i;
-        if (col < VT * 32) out[frag_elem(r, h * VT * 32 + col, a.o_kt)] = (__bf16)(o[i] * factor);
+        const float pair = wave_xor_f32(o[i], 1);
+        if (col < VT * 32) out[frag_elem(r, h * VT * 32 + col, a.o_kt)] = (__bf16)(window_finish<false>(a, r, h, col, o[i], pair) * factor);
     }
 }
 

@@ -21,6 +21,7 @@
 #include "kernels_latent_mfma.hip.h"
 #include "kernels_recur.hip.h"
 #include "kernels_window.hip.h"
+#include "kernels_gru.hip.h"
 
 using namespace wr;
 
@@ -318,23 +319,25 @@ int wr_hip_mix_step_set(wr_hip_mix_step* s, const wr_hip_mix_pool* pool, uint32_
 
 static int launch_residual(int f32, bool embed, const MixRowArgs& a)
 {
-    const bool many = a.rows >= 64, held = a.wpad <= 4096;
+    const bool many = a.rows >= 64, held = a.wpad <= 4096, pair = a.pair_y[0] != nullptr;
     const dim3 g1(a.rows), b1(MixRowShape<1>::kThreads), g4((a.rows + 3) / 4), b4(MixRowShape<4>::kThreads);
-#define WR_RESID(F, EMB)                                                                         \
+#define WR_RESID(F, EMB, PAIR)                                                                   \
     do {                                                                                         \
         if (many && held)                                                                        \
-            MIX_LAUNCH((mix_residual_kernel<F, 4, EMB, true>), g4, b4, 0, a);  \
+            MIX_LAUNCH((mix_residual_kernel<F, 4, EMB, true, PAIR>), g4, b4, 0, a);              \
         else if (many)                                                                           \
-            MIX_LAUNCH((mix_residual_kernel<F, 4, EMB, false>), g4, b4, 0, a); \
+            MIX_LAUNCH((mix_residual_kernel<F, 4, EMB, false, PAIR>), g4, b4, 0, a);             \
         else if (held)                                                                           \
-            MIX_LAUNCH((mix_residual_kernel<F, 1, EMB, true>), g1, b1, 0, a);     \
+            MIX_LAUNCH((mix_residual_kernel<F, 1, EMB, true, PAIR>), g1, b1, 0, a);              \
         else                                                                                     \
-            MIX_LAUNCH((mix_residual_kernel<F, 1, EMB, false>), g1, b1, 0, a);    \
+            MIX_LAUNCH((mix_residual_kernel<F, 1, EMB, false, PAIR>), g1, b1, 0, a);             \
     } while (0)
-    if (f32 && embed) WR_RESID(true, true);
-    else if (f32) WR_RESID(true, false);
-    else if (embed) WR_RESID(false, true);
-    else WR_RESID(false, false);
+    if (f32 && embed) WR_RESID(true, true, false);
+    else if (f32 && pair) WR_RESID(true, false, true);
+    else if (f32) WR_RESID(true, false, false);
+    else if (embed) WR_RESID(false, true, false);
+    else if (pair) WR_RESID(false, false, true);
+    else WR_RESID(false, false, false);
 #undef WR_RESID
     return WR_HIP_OK;
 }
@@ -365,9 +368,11 @@ int wr_hip_mix_residual(wr_hip_mix_step* s, int f32, const wr_hip_mix_resid* q)
 {
     if (!g.inited) return WR_HIP_ERR_STATE;
     if (!s || !s->rows || !q || !q->width || !q->x || (q->post && !q->y) || (q->next && !q->h)) return WR_HIP_ERR_INVAL;
-    if (q->top && (!q->y || !q->gate || !q->slot)) return WR_HIP_ERR_INVAL;
+    if (q->top && (!q->y || !q->slot)) return WR_HIP_ERR_INVAL;
+    const bool pair = q->pair_y[0] != nullptr;
+    if (pair != (q->pair_y[1] != nullptr) || (pair && (!q->pair_post[0] || !q->pair_post[1]))) return WR_HIP_ERR_INVAL;
     if (q->side && !q->top) return WR_HIP_ERR_INVAL;
-    if (q->wanted && (q->y || q->add || !s->n_want)) return WR_HIP_ERR_INVAL;
+    if (q->wanted && (q->y || q->add || pair || !s->n_want)) return WR_HIP_ERR_INVAL;
     ENTER();
     MixRowArgs a = {};
     a.rows = q->wanted ? s->n_want : s->rows;
@@ -380,6 +385,10 @@ int wr_hip_mix_residual(wr_hip_mix_step* s, int f32, const wr_hip_mix_resid* q)
     a.add = q->add;
     a.next = q->next;
     a.h = q->h;
+    for (int i = 0; i < 2; i++) {
+        a.pair_y[i] = q->pair_y[i];
+        a.pair_post[i] = q->pair_post[i];
+    }
     a.gate = q->gate;
     a.slot = q->slot;
     a.top = q->top;
@@ -451,7 +460,7 @@ int wr_hip_mix_gemm_run(int f32, const wr_hip_mix_gemm* q)
     if (split_gated && (q->n_split % 32 || q->n_split > q->w->n_out || batch != 1 || q->group_expert)) return WR_HIP_ERR_INVAL;
     const uint32_t n_frag = q->out == WR_HIP_MIX_OUT_SPLIT ? q->n_split
                             : gated ? (q->w->n_out - (split_gated ? q->n_split : 0)) / 2 : q->w->n_out;
-    if (frag && ((uint64_t)q->col_z * (batch - 1) + n_frag > (uint64_t)q->h_kt * 32)) return WR_HIP_ERR_INVAL;
+    if (frag && ((uint64_t)q->h_kt0 * 32 + (uint64_t)q->col_z * (batch - 1) + n_frag > (uint64_t)q->h_kt * 32)) return WR_HIP_ERR_INVAL;
     if (q->out == WR_HIP_MIX_OUT_SPLIT && (q->n_split % 16 || q->n_split > q->w->n_out)) return WR_HIP_ERR_INVAL;
     if (gated && q->w->n_out % 32) return WR_HIP_ERR_INVAL;
     const bool rows32 = q->out == WR_HIP_MIX_OUT_ROWS_F32 || (q->out == WR_HIP_MIX_OUT_SPLIT && q->n_split < q->w->n_out) || split_gated;
@@ -463,7 +472,8 @@ int wr_hip_mix_gemm_run(int f32, const wr_hip_mix_gemm* q)
     if (((q->out == WR_HIP_MIX_OUT_ROWS_F32 && !q->col_z) || q->out == WR_HIP_MIX_OUT_ROWS) && batch != 1) return WR_HIP_ERR_INVAL;
     if (q->group_expert && (q->rows % 16 || (q->tile_groups != 1 && q->tile_groups != 8))) return WR_HIP_ERR_INVAL;
     if (q->group_expert && q->rows / 16 % q->tile_groups) return WR_HIP_ERR_INVAL;
-    if (q->bias && (batch != 1 || gated || q->group_expert)) return WR_HIP_ERR_INVAL;
+    if (q->bias && (batch != 1 || q->out == WR_HIP_MIX_OUT_GATED || q->group_expert)) return WR_HIP_ERR_INVAL;
+    if (q->x_scale && !q->group_expert) return WR_HIP_ERR_INVAL;
     if (q->x_perm && (!q->group_expert || q->tile_groups != 1)) return WR_HIP_ERR_INVAL;
     ENTER();
     MixGemmArgs a = {};
@@ -492,9 +502,10 @@ int wr_hip_mix_gemm_run(int f32, const wr_hip_mix_gemm* q)
     a.up_bias = q->up_bias;
     a.bias = q->bias;
     a.x_perm = q->x_perm;
+    a.x_scale = q->x_scale;
     a.y = q->y_f32;
     a.ya = q->y_act;
-    a.h = q->h;
+    a.h = frag ? static_cast<uint8_t*>(q->h) + (size_t)q->h_kt0 * 512 * (f32 ? 4 : 2) : q->h;
     if (q->group_expert) {
         if (!f32 && q->tile_groups == 8) return launch_lds<4>(a, 1);
         if (f32) return gated ? launch_stream<true, 2, 1>(a, 1) : launch_stream<true, 1, 1>(a, 1);
@@ -653,16 +664,19 @@ static int recur_steps(const RecurArgs& a, uint32_t n)
 
 constexpr uint32_t kSegMax = 8, kSegSubs = 6;
 
-template <bool F32, int KT, bool DELTA, int VT>
+template <bool F32, int KT, int RULE, int VT>
 static int recur_chunks(wr_hip_mix_step* s, RecurArgs& a)
 {
-    a.vtiles = VT;
+    constexpr bool DELTA = RULE == kRecurDelta;
+    // FORGET: the value columns in slices of VT tiles, a workgroup each
+    const uint32_t slices = RULE == kRecurForget ? (a.vdim + 16 * VT - 1) / (16 * VT) : 1;
+    a.vtiles = VT * slices;
     constexpr size_t unit = (size_t)recur_unit_kib(KT, DELTA, VT) * 1024;
-    int rc = ensure_device(s->recur_ops, (size_t)s->n_chunks * kRecurSubs * a.heads * unit);
-    if (rc == WR_HIP_OK) rc = ensure_device(s->recur_out, (size_t)s->n_chunks * kMixChunk * a.heads * VT * 16 * 4);
+    int rc = ensure_device(s->recur_ops, (size_t)s->n_chunks * kRecurSubs * a.heads * recur_unit_kib(KT, DELTA, a.vtiles) * 1024);
+    if (rc == WR_HIP_OK) rc = ensure_device(s->recur_out, (size_t)s->n_chunks * kMixChunk * a.heads * a.vtiles * 16 * 4);
     constexpr size_t l1 = (size_t)4 * recur_chunk_lds(KT, DELTA) * 4, l2 = recur_ring(KT, DELTA) * unit;
     constexpr size_t l3 = l2 - (size_t)recur_ring(KT, DELTA) * RecurUnit<KT, DELTA>::kG * 1024;      // without the outputs' part
-    if (rc == WR_HIP_OK) rc = allow_lds<recur_chunk_kernel<F32, KT, DELTA>>(l1);
+    if (rc == WR_HIP_OK) rc = allow_lds<recur_chunk_kernel<F32, KT, RULE>>(l1);
     if (rc == WR_HIP_OK) rc = allow_lds<recur_chain_kernel<F32, KT, DELTA, VT, false>>(l2);
     if (rc == WR_HIP_OK) rc = allow_lds<recur_chain_kernel<F32, KT, DELTA, VT, true>>(l2);
     if (rc) return rc;
@@ -670,11 +684,11 @@ static int recur_chunks(wr_hip_mix_step* s, RecurArgs& a)
     for (uint32_t i = 0; i < s->n_long; i++) longest = std::max(longest, (s->long_rows[i] + kRecurSub - 1) / kRecurSub);
     // Segments: as many as give every compute unit a walk (below three the two walks cost more than one), none shorter
     // than kSegSubs.
-    a.n_seg = std::min({(uint32_t)g.n_cus / (s->n_long * a.heads), longest / kSegSubs, kSegMax});
+    a.n_seg = std::min({(uint32_t)g.n_cus / (s->n_long * a.heads * slices), longest / kSegSubs, kSegMax});
     if (a.n_seg < 3) a.n_seg = 1;
     a.seg_len = (longest + a.n_seg - 1) / a.n_seg;
     if (a.n_seg > 1) {
-        constexpr size_t c = (size_t)32 * KT * 16 * VT, x = DELTA ? (size_t)32 * KT * 32 * KT : 32 * KT;
+        const size_t c = (size_t)32 * KT * 16 * a.vtiles, x = DELTA ? (size_t)32 * KT * 32 * KT : 32 * KT;
         const size_t items = (size_t)s->n_long * a.n_seg * a.heads;
         rc = ensure_device(s->recur_segs, items * (c + x) * 4);
         if (rc) return rc;
@@ -684,11 +698,11 @@ static int recur_chunks(wr_hip_mix_step* s, RecurArgs& a)
     a.ops = reinterpret_cast<unsigned char*>(s->recur_ops.p);
     a.o = reinterpret_cast<float*>(s->recur_out.p);
     const uint32_t whole = !((a.dim | a.ld | a.ldz | a.col_r | a.col_k | a.col_a) % 4);
-    MIX_LAUNCH((recur_chunk_kernel<F32, KT, DELTA>), dim3(s->n_chunks, a.heads), dim3(256), l1, a, whole);
+    MIX_LAUNCH((recur_chunk_kernel<F32, KT, RULE>), dim3(s->n_chunks, a.heads), dim3(256), l1, a, whole);
     if (a.n_seg > 1)
-        MIX_LAUNCH((recur_chain_kernel<F32, KT, DELTA, VT, true>), dim3(s->n_long * (a.n_seg - 1), a.heads, DELTA ? 2 : 1),
+        MIX_LAUNCH((recur_chain_kernel<F32, KT, DELTA, VT, true>), dim3(s->n_long * (a.n_seg - 1), a.heads, DELTA ? 2 : slices),
                    dim3(64 * VT), l3, a);
-    MIX_LAUNCH((recur_chain_kernel<F32, KT, DELTA, VT, false>), dim3(s->n_long * a.n_seg, a.heads), dim3(64 * VT), l2, a);
+    MIX_LAUNCH((recur_chain_kernel<F32, KT, DELTA, VT, false>), dim3(s->n_long * a.n_seg, a.heads, slices), dim3(64 * VT), l2, a);
     MIX_LAUNCH(recur_gate_kernel<F32>, dim3(s->n_chunks, a.heads), dim3(256), 0, a);
     return WR_HIP_OK;
 }
@@ -718,43 +732,84 @@ static int recur_run(wr_hip_mix_step* s, RecurArgs& a, const wr_hip_mix_recurren
     if (chunked) {
         a.list = s->d<uint32_t>(s->o_long);
         int rc;
-        if (a.dim <= 16) rc = recur_chunks<F32, 1, DELTA, 1>(s, a);
-        else if (a.dim <= 32) rc = recur_chunks<F32, 1, DELTA, 2>(s, a);
-        else if (a.dim <= 64) rc = recur_chunks<F32, 2, DELTA, 4>(s, a);
-        else rc = recur_chunks<F32, 4, DELTA, 8>(s, a);
+        constexpr int RULE = DELTA ? kRecurDelta : kRecurBonus;
+        if (a.dim <= 16) rc = recur_chunks<F32, 1, RULE, 1>(s, a);
+        else if (a.dim <= 32) rc = recur_chunks<F32, 1, RULE, 2>(s, a);
+        else if (a.dim <= 64) rc = recur_chunks<F32, 2, RULE, 4>(s, a);
+        else rc = recur_chunks<F32, 4, RULE, 8>(s, a);
         if (rc) return rc;
     }
     a.list = s->d<uint32_t>(chunked ? s->o_short : s->o_all);
     return recur_steps<F32, DELTA>(a, chunked ? s->n_short : s->n_seq);
 }
 
+template <bool F32, int DPT>
+static int forget_steps_v(const RecurArgs& a, uint32_t n)
+{
+    const dim3 grid(n, a.heads);
+    if (a.vdim <= 32) MIX_LAUNCH((recur_forget_step_kernel<F32, DPT, 32>), grid, dim3(128), 0, a);
+    else if (a.vdim <= 64) MIX_LAUNCH((recur_forget_step_kernel<F32, DPT, 64>), grid, dim3(256), 0, a);
+    else if (a.vdim <= 128) MIX_LAUNCH((recur_forget_step_kernel<F32, DPT, 128>), grid, dim3(512), 0, a);
+    else MIX_LAUNCH((recur_forget_step_kernel<F32, DPT, 256>), grid, dim3(1024), 0, a);
+    return WR_HIP_OK;
+}
+
+template <bool F32, int KT>
+static int forget_chunks(wr_hip_mix_step* s, RecurArgs& a)
+{
+    return a.vdim <= 32 ? recur_chunks<F32, KT, kRecurForget, 2>(s, a) : recur_chunks<F32, KT, kRecurForget, 4>(s, a);
+}
+
+template <bool F32>
+static int forget_run(wr_hip_mix_step* s, RecurArgs& a)
+{
+    const bool chunked = s->n_long && a.dim <= (uint32_t)kRecurMaxDim;
+    if (chunked) {
+        a.list = s->d<uint32_t>(s->o_long);
+        const int rc = a.dim <= 32 ? forget_chunks<F32, 1>(s, a) : a.dim <= 64 ? forget_chunks<F32, 2>(s, a) : forget_chunks<F32, 4>(s, a);
+        if (rc) return rc;
+    }
+    a.list = s->d<uint32_t>(chunked ? s->o_short : s->o_all);
+    const uint32_t n = chunked ? s->n_short : s->n_seq;
+    if (n == 0) return WR_HIP_OK;
+    if (a.dim <= 32) return forget_steps_v<F32, 8>(a, n);
+    if (a.dim <= 64) return forget_steps_v<F32, 16>(a, n);
+    if (a.dim <= 128) return forget_steps_v<F32, 32>(a, n);
+    return forget_steps_v<F32, 64>(a, n);
+}
+
 int wr_hip_mix_recur(wr_hip_mix_step* s, wr_hip_mix_pool* pool, uint32_t run, int f32, const wr_hip_mix_recurrence* q)
 {
     if (!g.inited) return WR_HIP_ERR_STATE;
     if (!s || !s->rows || !pool || run >= pool->state.size() || !q || !q->heads || !q->dim || !q->w0 || !q->norm || !q->in ||
-        !q->w_decay || !q->low || !q->z || !q->h || q->rule > WR_HIP_MIX_RULE_DELTA)
+        !q->h || q->rule > WR_HIP_MIX_RULE_FORGET)
         return WR_HIP_ERR_INVAL;
-    const bool delta = q->rule == WR_HIP_MIX_RULE_DELTA;
-    if (delta ? !q->a_bias : !q->u) return WR_HIP_ERR_INVAL;
-    if (q->dim > WR_HIP_MIX_MAX_RECUR_DIM) return WR_HIP_ERR_LIMIT;
-    const uint64_t hd = (uint64_t)q->heads * q->dim;
-    if (hd * q->dim != pool->state_elems[run]) return WR_HIP_ERR_INVAL;
-    if (q->w_decay->batch != 1 || q->w_decay->n_out < hd || q->col_r + hd > q->ld || q->col_k + hd > q->ld || q->col_v + hd > q->ld || q->col_g + hd > q->ld ||
-        (delta && q->col_a + hd > q->ld) || q->col_h + (hd + 31) / 32 * 32 > (uint64_t)q->h_kt * 32)
+    const bool delta = q->rule == WR_HIP_MIX_RULE_DELTA, forget = q->rule == WR_HIP_MIX_RULE_FORGET;
+    if (delta ? !q->a_bias : forget ? !q->lower || !q->vdim : !q->u) return WR_HIP_ERR_INVAL;
+    if (!forget && (!q->w_decay || !q->low || !q->z)) return WR_HIP_ERR_INVAL;
+    const uint32_t vdim = forget ? q->vdim : q->dim;
+    if (q->dim > WR_HIP_MIX_MAX_RECUR_DIM || vdim > WR_HIP_MIX_MAX_RECUR_DIM) return WR_HIP_ERR_LIMIT;
+    const uint64_t hd = (uint64_t)q->heads * q->dim, hv = (uint64_t)q->heads * vdim;
+    if (hd * vdim != pool->state_elems[run]) return WR_HIP_ERR_INVAL;
+    if (q->col_r + hd > q->ld || q->col_k + hd > q->ld || q->col_v + hv > q->ld || (!forget && q->col_g + hd > q->ld) ||
+        (delta && q->col_a + hd > q->ld) || q->col_h + (hv + 31) / 32 * 32 > (uint64_t)q->h_kt * 32)
         return WR_HIP_ERR_INVAL;
+    if (!forget && (q->w_decay->batch != 1 || q->w_decay->n_out < hd)) return WR_HIP_ERR_INVAL;
     ENTER();
     RecurArgs a = {};
     a.seqs = s->d<MixSeq>(s->o_seqs);
     a.chunks = s->d<MixChunk>(s->o_chunks);
     a.heads = q->heads;
     a.dim = q->dim;
-    a.silu = q->gate_silu;
+    a.vdim = vdim;
+    a.gate = forget ? kRecurGateNone : q->gate_silu ? kRecurGateSilu : kRecurGateLogistic;
+    a.norm_step = forget ? 0 : vdim;
     a.gain = q->gain;
     a.unit_eps = q->unit_eps;
     a.eps = q->eps;
     a.out_scale = q->out_scale;
     a.w0 = q->w0;
-    a.u = q->u;
+    a.u = forget ? q->lower : q->u;
     a.ab = q->a_bias;
     a.norm = q->norm;
     a.in = q->in;
@@ -763,16 +818,45 @@ int wr_hip_mix_recur(wr_hip_mix_step* s, wr_hip_mix_pool* pool, uint32_t run, in
     a.col_k = q->col_k;
     a.col_v = q->col_v;
     a.col_a = delta ? q->col_a : 0;
-    a.col_g = q->col_g;
-    a.z = q->z;
-    a.ldz = q->w_decay->n_out;
-    a.low_kt = q->w_decay->n_in / 32;
+    a.col_g = forget ? 0 : q->col_g;
+    a.z = forget ? q->in + q->col_k : q->z;
+    a.ldz = forget ? q->ld : q->w_decay->n_out;
+    a.low_kt = forget ? 0 : q->w_decay->n_in / 32;
     a.state = pool->state[run];
     a.h = q->h;
     a.h_kt = q->h_kt;
     a.col_h = q->col_h;
+    if (forget) return f32 ? forget_run<true>(s, a) : forget_run<false>(s, a);
     if (f32) return delta ? recur_run<true, true>(s, a, q) : recur_run<true, false>(s, a, q);
     return delta ? recur_run<false, true>(s, a, q) : recur_run<false, false>(s, a, q);
+}
+
+int wr_hip_mix_min_gru(wr_hip_mix_step* s, wr_hip_mix_pool* pool, uint32_t run, int f32, const wr_hip_mix_gru* q)
+{
+    if (!g.inited) return WR_HIP_ERR_STATE;
+    if (!s || !s->rows || !pool || run >= pool->state.size() || !q || !q->width || !q->in || !q->h) return WR_HIP_ERR_INVAL;
+    const uint32_t wp = round32(q->width);
+    if (pool->state_elems[run] != wp || (q->ld | q->col_z | q->col_x | q->col_g) % 4 || q->col_h % 8 ||
+        (uint64_t)std::max({q->col_z, q->col_x, q->col_g}) + wp > q->ld || (uint64_t)q->col_h + wp > (uint64_t)q->h_kt * 32)
+        return WR_HIP_ERR_INVAL;
+    ENTER();
+    GruArgs a = {s->d<MixSeq>(s->o_seqs), s->d<uint32_t>(s->o_long), wp, q->in, q->ld, q->col_z, q->col_x, q->col_g,
+                 pool->state[run], q->h, q->h_kt, q->col_h};
+    if (s->n_long) {
+        const dim3 grid(wp / 32, s->n_long);
+        const bool many = *std::max_element(s->long_rows, s->long_rows + s->n_long) > 64;
+        if (many && f32) MIX_LAUNCH((gru_scan_kernel<true, 16>), grid, dim3(1024), 0, a);
+        else if (many) MIX_LAUNCH((gru_scan_kernel<false, 16>), grid, dim3(1024), 0, a);
+        else if (f32) MIX_LAUNCH((gru_scan_kernel<true, 4>), grid, dim3(256), 0, a);
+        else MIX_LAUNCH((gru_scan_kernel<false, 4>), grid, dim3(256), 0, a);
+    }
+    if (s->n_short) {
+        a.list = s->d<uint32_t>(s->o_short);
+        const dim3 grid(wp / 32, s->n_short);
+        if (f32) MIX_LAUNCH((gru_scan_kernel<true, 1>), grid, dim3(64), 0, a);
+        else MIX_LAUNCH((gru_scan_kernel<false, 1>), grid, dim3(64), 0, a);
+    }
+    return WR_HIP_OK;
 }
 
 // ----------------------------------------------------------------- latent --
@@ -811,13 +895,13 @@ static LatentArgs latent_args(const wr_hip_mix_step* s, const wr_hip_mix_latent*
     return a;
 }
 
-int wr_hip_mix_rope_table(wr_hip_mix_step* s, const double* freq_dev, uint32_t half, float* table_dev)
+int wr_hip_mix_rope_table(wr_hip_mix_step* s, const double* freq_dev, uint32_t half, float gain, float* table_dev)
 {
     if (!g.inited) return WR_HIP_ERR_STATE;
     if (!s || !s->rows || !freq_dev || !half || !table_dev) return WR_HIP_ERR_INVAL;
     ENTER();
     MIX_LAUNCH(mix_rope_table_kernel, dim3((s->rows * half + 255) / 256), dim3(256), 0, s->d<uint32_t>(s->o_pos), s->rows,
-               freq_dev, half, table_dev);
+               freq_dev, half, gain, table_dev);
     return WR_HIP_OK;
 }
 
@@ -989,8 +1073,9 @@ static int check_window(const wr_hip_mix_step* s, const wr_hip_mix_pool* pool, u
 {
     if (!s || !s->rows || !pool || run >= pool->latent.size() || pool->f32 != (f32 != 0) || !q || !q->heads || !q->kv_heads ||
         q->heads % q->kv_heads || !q->dim || !q->vdim || q->dim_pad % 32 || q->vdim_pad % 32 || q->dim > q->dim_pad ||
-        q->vdim > q->vdim_pad || q->rot_half * 2 > q->dim || !q->window || q->maps < 1 || q->maps > 2)
+        q->vdim > q->vdim_pad || q->rot_half * 2 > q->dim || (!q->window && !q->chunk) || q->maps < 1 || q->maps > 2)
         return WR_HIP_ERR_INVAL;
+    if (q->turn_values && (q->vdim % 2 || q->maps != 1)) return WR_HIP_ERR_INVAL;
     if ((uint64_t)q->kv_heads * ((uint64_t)q->maps * q->dim_pad + q->vdim_pad) != pool->latent_dim[run]) return WR_HIP_ERR_INVAL;
     return WR_HIP_OK;
 }
@@ -1012,6 +1097,9 @@ static WindowArgs window_args(const wr_hip_mix_step* s, const wr_hip_mix_pool* p
     a.vdimp = q->vdim_pad;
     a.half = q->rot_half;
     a.window = q->window;
+    a.chunk = q->chunk;
+    a.gate_wide = q->gate_wide;
+    a.vtable = q->turn_values;
     a.norm_values = q->norm_values;
     a.maps = q->maps;
     a.dimk = q->maps * q->dim_pad;
@@ -1094,7 +1182,7 @@ static int window_mfma(wr_hip_mix_step* s, WindowArgs& a)
     const LatentRow* rows = s->h<LatentRow>(s->o_short_rows);
     uint32_t keys = 1;                                     // of the row that sees the most, from its first block on
     for (uint32_t i = 0; i < n; i++) {
-        const uint32_t lo = rows[i].pos + 1 > a.window ? rows[i].pos + 1 - a.window : 0;
+        const uint32_t lo = window_lo(rows[i].pos, a.window, a.chunk);
         keys = std::max(keys, rows[i].pos + 1 - lo / 32 * 32);
     }
     const uint32_t groups = a.kvh * ((a.group * MAPS + 15) / 16);
@@ -1150,7 +1238,9 @@ int wr_hip_mix_window_attend(wr_hip_mix_step* s, wr_hip_mix_pool* pool, uint32_t
     if (!g.inited) return WR_HIP_ERR_STATE;
     int rc = check_window(s, pool, run, f32, q);
     if (rc) return rc;
-    if (!q_dev || !o_dev || (uint64_t)q->heads * q->vdim_pad > (uint64_t)o_kt * 32 || (gate_dev && ldg < q->heads)) return WR_HIP_ERR_INVAL;
+    if (!q_dev || !o_dev || (uint64_t)q->heads * q->vdim_pad > (uint64_t)o_kt * 32 || (gate_dev && ldg < (q->gate_wide ? q->heads * q->vdim : q->heads)))
+        return WR_HIP_ERR_INVAL;
+    if (q->gate_wide && (!gate_dev || ldg % 4)) return WR_HIP_ERR_INVAL;
     ENTER();
     g.calls.fetch_add(s->n_seq, std::memory_order_relaxed);
     WindowArgs a = window_args(s, pool, run, q);
@@ -1183,7 +1273,8 @@ uint32_t wr_hip_mix_route_groups(uint32_t rows, uint32_t experts, uint32_t top, 
 }
 
 int wr_hip_mix_route(wr_hip_mix_step* s, const float* z_dev, uint32_t ldz, const wr_hip_mix_router* q, uint32_t tile_groups,
-                     float* gate_dev, float* side_dev, uint32_t* slot_dev, uint32_t* perm_dev, int32_t* group_expert_dev)
+                     float* gate_dev, float* side_dev, float* slot_weight_dev, uint32_t* slot_dev, uint32_t* perm_dev,
+                     int32_t* group_expert_dev)
 {
     if (!g.inited) return WR_HIP_ERR_STATE;
     if (!s || !s->rows || !z_dev || !q || !q->experts || !q->top || !tile_groups || !gate_dev || !slot_dev || !perm_dev ||
@@ -1193,6 +1284,7 @@ int wr_hip_mix_route(wr_hip_mix_step* s, const float* z_dev, uint32_t ldz, const
     if (outputs > WR_HIP_MIX_MAX_EXPERTS || q->top > WR_HIP_MIX_MAX_TOP || q->groups > WR_HIP_MIX_MAX_GROUPS) return WR_HIP_ERR_LIMIT;
     if (ldz < outputs + (q->shared_gate != 0) || ((q->identity || q->shared_gate) && !side_dev) || (q->correction && !q->softmax_all))
         return WR_HIP_ERR_INVAL;
+    if (q->logistic && q->softmax_all) return WR_HIP_ERR_INVAL;
     if (q->groups && (outputs % q->groups || !q->keep || q->keep > q->groups)) return WR_HIP_ERR_INVAL;
     if (q->top > (q->groups ? outputs / q->groups * q->keep : outputs)) return WR_HIP_ERR_INVAL;
     ENTER();
@@ -1209,6 +1301,8 @@ int wr_hip_mix_route(wr_hip_mix_step* s, const float* z_dev, uint32_t ldz, const
     a.keep = q->keep;
     a.softmax_all = q->softmax_all;
     a.shared_gate = q->shared_gate;
+    a.logistic = q->logistic;
+    a.slot_weight = slot_weight_dev;
     a.scale = q->scale;
     a.correction = q->correction;
     a.gate = gate_dev;

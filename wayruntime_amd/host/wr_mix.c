@@ -163,8 +163,16 @@ typedef struct window_rows {
     void  *q, *oh;
 } window_rows;
 
+/* Where a joint layer's parts of the output product's input lie: buffers of their own with out_norm, else one. */
+typedef struct joint_rows {
+    float *in;
+    void  *q, *attn, *beside, *act;
+    uint32_t attn_kt, beside_kt, beside_col, act_kt, act_kt0;
+    float *y_attn, *y_beside;
+} joint_rows;
+
 typedef struct moe_rows {
-    float    *z, *gate, *side, *ys, *shared;
+    float    *z, *gate, *side, *slot_weight, *ys, *shared;
     uint32_t *slot, *perm;
     int32_t  *group_expert;
     void     *xs, *act, *shared_act;
@@ -246,6 +254,37 @@ static window_rows take_window(bump *b, const wrh_mix_layer *L, size_t R, size_t
     return r;
 }
 
+static uint32_t beside_out(const wrh_mix_layer *L)
+{
+    return L->beside == WRH_BESIDE_FORGET ? L->rec.hv_p : L->beside == WRH_BESIDE_GRU ? L->gru_p : 0;
+}
+
+static joint_rows take_joint(bump *b, const struct wrh_mix_model *mm, const wrh_mix_layer *L, size_t R)
+{
+    joint_rows r;
+    memset(&r, 0, sizeof r);
+    const size_t e = mm->f32 ? 4 : 2;
+    const uint32_t heads = L->heads * L->win.vdim_pad, beside = beside_out(L), ff = L->mlp == WRH_MLP_DENSE ? L->ff_p : 0;
+    r.in = take(b, R * L->ld_in * 4);
+    r.q = take(b, r16(R) * L->heads * L->win.dim_pad * e);
+    if (L->out_norm[0]) {
+        r.attn = take(b, r16(R) * heads * e);
+        r.beside = take(b, r16(R) * beside * e);
+        r.act = take(b, r16(R) * ff * e);
+        r.attn_kt = heads / 32;
+        r.beside_kt = beside / 32;
+        r.act_kt = ff / 32;
+        r.y_attn = take(b, R * mm->width_p * 4);
+        r.y_beside = take(b, R * mm->width_p * 4);
+        return r;
+    }
+    r.attn = r.beside = r.act = take(b, r16(R) * (heads + beside + ff) * e);
+    r.attn_kt = r.beside_kt = r.act_kt = (heads + beside + ff) / 32;
+    r.beside_col = heads;
+    r.act_kt0 = (heads + beside) / 32;
+    return r;
+}
+
 /* Experts whose rows fill whole tiles take the prompt-sized product. */
 static uint32_t moe_tile(const struct wrh_mix_model *mm, const wrh_mix_layer *L, size_t R)
 {
@@ -265,6 +304,7 @@ static moe_rows take_moe(bump *b, const struct wrh_mix_model *mm, const wrh_mix_
     r.slot = take(b, R * L->router.top * 4);
     r.perm = take(b, slots * 4);
     r.group_expert = take(b, (size_t)r.groups * 4);
+    r.slot_weight = L->weigh_input ? take(b, slots * 4) : NULL;
     r.xs = take(b, slots * mm->width_p * e);
     r.act = take(b, slots * L->ff_p * e);
     r.ys = take(b, slots * mm->width_p * 4);
@@ -290,8 +330,13 @@ static size_t scratch_bytes(const struct wrh_mix_model *mm, size_t R)
         case WRH_MIXER_WKV: (void)take_wkv(&b, mm, L, R); break;
         case WRH_MIXER_PARALLEL: (void)take_parallel(&b, L, R, e); break;
         case WRH_MIXER_WINDOW: (void)take_window(&b, L, R, e); break;
+        case WRH_MIXER_JOINT:
+            (void)take_joint(&b, mm, L, R);
+            if (L->mlp == WRH_MLP_MOE) (void)take_moe(&b, mm, L, R, 8);
+            break;
         }
         if (b.at > most) most = b.at;
+        if (L->kind == WRH_MIXER_JOINT) continue;
         bump f = {NULL, 0};
         if (L->mlp == WRH_MLP_DENSE) (void)take(&f, r16(R) * L->ff_p * e);
         if (L->mlp == WRH_MLP_MOE) (void)take_moe(&f, mm, L, R, 8);      /* the larger of the two forms */
@@ -491,6 +536,105 @@ static wr_status walk_window(wr_model *m, const wrh_mix_layer *L, uint32_t r, co
     return WR_OK;
 }
 
+/* The experts: the router's logits `z` (row stride ldz) to expert rows that `res` is told to combine. */
+static wr_status walk_experts(wr_model *m, const wrh_mix_layer *L, uint32_t r, const walk *w, const moe_rows *t, const float *z,
+                              uint32_t ldz, wr_hip_mix_resid *res)
+{
+    struct wrh_mix_model *mm = m->mix;
+    const uint32_t wkt = mm->width_p / 32;
+    TRY(wr_hip_mix_route(mm->step, z, ldz, &L->router, t->tile_groups, t->gate, t->side, t->slot_weight, t->slot, t->perm,
+                         t->group_expert), "routing");
+    wr_hip_mix_gemm up = {.w = L->w_eup, .x = t->xs, .x_kt = wkt, .rows = t->groups * 16, .group_expert = t->group_expert,
+                          .tile_groups = t->tile_groups, .out = WR_HIP_MIX_OUT_FRAG, .h = t->act, .h_kt = L->ff_p / 32,
+                          .x_scale = t->slot_weight};
+    if (t->tile_groups == 1) {                             /* few rows: the product fetches them where they are */
+        up.x = w->h;
+        up.x_perm = t->perm;
+    } else {
+        TRY(wr_hip_mix_route_gather(mm->step, mm->f32, w->h, wkt, t->groups, t->perm, t->group_expert, t->xs), "expert rows");
+    }
+    if (L->gated || L->limit > 0) up.out = WR_HIP_MIX_OUT_GATED;
+    else up.relu2 = 1;
+    if (L->limit > 0) {
+        up.limit = L->limit;
+        up.slope = WRH_CLAMPED_SLOPE;
+        up.up_bias = WRH_CLAMPED_UP_BIAS;
+    }
+    TRY(wr_hip_mix_gemm_run(mm->f32, &up), "experts' up projection");
+    const wr_hip_mix_gemm down = {.w = L->w_edown, .x = t->act, .x_kt = L->ff_p / 32, .rows = t->groups * 16,
+                                  .group_expert = t->group_expert, .tile_groups = t->tile_groups,
+                                  .out = WR_HIP_MIX_OUT_ROWS_F32, .y_f32 = t->ys, .ldy = mm->width_p};
+    TRY(wr_hip_mix_gemm_run(mm->f32, &down), "experts' down projection");
+    res->y = t->ys;
+    res->gate = L->weigh_input ? NULL : t->gate;
+    res->slot = t->slot;
+    res->top = L->router.top;
+    return WR_OK;
+}
+
+/* A whole joint layer: mixers and feed-forward from the rows in w->h; `res` is told what joins the residual. */
+static wr_status walk_joint(wr_model *m, const wrh_mix_layer *L, uint32_t r, const walk *w, bump b, uint32_t R, wr_hip_mix_resid *res)
+{
+    struct wrh_mix_model *mm = m->mix;
+    const joint_rows t = take_joint(&b, mm, L, R);
+    const uint32_t store = mm->runs[r].store, store2 = mm->runs[r].store2;
+    const int dense = L->mlp == WRH_MLP_DENSE, apart = L->out_norm[0] != NULL;
+    wr_hip_mix_gemm in = {.w = L->w_in, .x = w->h, .x_kt = mm->width_p / 32, .rows = R, .out = WR_HIP_MIX_OUT_ROWS_F32,
+                          .y_f32 = t.in, .ldy = L->ld_in, .bias = L->b_in, .silu_end = L->silu_end};
+    if (dense) {
+        in.out = WR_HIP_MIX_OUT_SPLIT_GATED;
+        in.n_split = L->ld_in;
+        in.h = t.act;
+        in.h_kt = t.act_kt;
+        in.h_kt0 = t.act_kt0;
+        in.limit = L->limit;
+        in.slope = WRH_CLAMPED_SLOPE;
+        in.up_bias = WRH_CLAMPED_UP_BIAS;
+    }
+    TRY(wr_hip_mix_gemm_run(mm->f32, &in), "layer's input projections");
+    wr_hip_mix_window g = L->win;
+    g.turn_values = L->turn >= 0 ? w->rope[L->turn] : NULL;
+    TRY(wr_hip_mix_window_append(mm->step, mm->pool, store, mm->f32, &g, t.in, L->ld_in, L->col_q, L->col_k, L->col_v,
+                                 w->rope[L->rope], t.q), "rotation + cache append");
+    TRY(wr_hip_mix_window_attend(mm->step, mm->pool, store, mm->f32, &g, t.q, L->sink, L->has_gate ? t.in + L->col_rg : NULL,
+                                 L->ld_in, t.attn, t.attn_kt), "attention");
+    if (L->beside == WRH_BESIDE_FORGET) {
+        const wr_hip_mix_recurrence rec = {.heads = L->rec.heads, .dim = L->rec.dim, .vdim = L->rec.vdim,
+                                           .rule = WR_HIP_MIX_RULE_FORGET, .eps = mm->eps, .out_scale = L->right_scale,
+                                           .w0 = L->rec.w0, .lower = L->rec.lower, .norm = L->rec.norm, .in = t.in,
+                                           .ld = L->ld_in, .col_r = L->col_rr, .col_k = L->col_rk, .col_v = L->col_rv,
+                                           .h = t.beside, .h_kt = t.beside_kt, .col_h = t.beside_col};
+        TRY(wr_hip_mix_recur(mm->step, mm->pool, store2, mm->f32, &rec), "matrix-state recurrence");
+    } else if (L->beside == WRH_BESIDE_GRU) {
+        const wr_hip_mix_gru gru = {.width = L->gru, .in = t.in, .ld = L->ld_in, .col_z = L->col_rr, .col_x = L->col_rk,
+                                    .col_g = L->col_rv, .h = t.beside, .h_kt = t.beside_kt, .col_h = t.beside_col};
+        TRY(wr_hip_mix_min_gru(mm->step, mm->pool, store2, mm->f32, &gru), "gated recurrence");
+    }
+    wr_hip_mix_gemm out = {.w = L->w_o, .x = t.attn, .x_kt = t.attn_kt, .rows = R, .out = WR_HIP_MIX_OUT_ROWS_F32,
+                           .y_f32 = apart ? t.y_attn : w->y, .ldy = mm->width_p, .bias = L->b_o};
+    TRY(wr_hip_mix_gemm_run(mm->f32, &out), "output projection");
+    if (apart) {
+        out = (wr_hip_mix_gemm){.w = L->w_o2, .x = t.beside, .x_kt = t.beside_kt, .rows = R, .out = WR_HIP_MIX_OUT_ROWS_F32,
+                                .y_f32 = t.y_beside, .ldy = mm->width_p};
+        TRY(wr_hip_mix_gemm_run(mm->f32, &out), "second output projection");
+        res->pair_y[0] = t.y_attn;
+        res->pair_y[1] = t.y_beside;
+        for (int k = 0; k < 2; k++) res->pair_post[k] = L->out_norm[k];
+        if (dense) {
+            out = (wr_hip_mix_gemm){.w = L->w_down, .x = t.act, .x_kt = t.act_kt, .rows = R, .out = WR_HIP_MIX_OUT_ROWS_F32,
+                                    .y_f32 = w->y, .ldy = mm->width_p};
+            TRY(wr_hip_mix_gemm_run(mm->f32, &out), "down projection");
+        }
+    }
+    if (dense || !apart) res->y = w->y;
+    if (L->mlp == WRH_MLP_MOE) {
+        const moe_rows x = take_moe(&b, mm, L, R, moe_tile(mm, L, R));
+        res->add = res->y;
+        return walk_experts(m, L, r, w, &x, t.in + L->col_router, L->ld_in, res);
+    }
+    return WR_OK;
+}
+
 /* The feed-forward's output: plain rows in w->y, or expert rows that `res` is told to combine. */
 static wr_status walk_mlp(wr_model *m, const wrh_mix_layer *L, uint32_t r, const walk *w, bump b, uint32_t R,
                           wr_hip_mix_resid *res)
@@ -521,37 +665,13 @@ static wr_status walk_mlp(wr_model *m, const wrh_mix_layer *L, uint32_t r, const
         router.up_bias = WRH_CLAMPED_UP_BIAS;
     }
     TRY(wr_hip_mix_gemm_run(mm->f32, &router), "router");
-    TRY(wr_hip_mix_route(mm->step, t.z, L->router_p, &L->router, t.tile_groups, t.gate, t.side, t.slot, t.perm, t.group_expert),
-        "routing");
-    wr_hip_mix_gemm up = {.w = L->w_eup, .x = t.xs, .x_kt = wkt, .rows = t.groups * 16, .group_expert = t.group_expert,
-                          .tile_groups = t.tile_groups, .out = WR_HIP_MIX_OUT_FRAG, .h = t.act, .h_kt = L->ff_p / 32, .relu2 = 1};
-    if (t.tile_groups == 1) {                              /* few rows: the product fetches them where they are */
-        up.x = w->h;
-        up.x_perm = t.perm;
-    } else {
-        TRY(wr_hip_mix_route_gather(mm->step, mm->f32, w->h, wkt, t.groups, t.perm, t.group_expert, t.xs), "expert rows");
-    }
-    if (L->limit > 0) {
-        up.out = WR_HIP_MIX_OUT_GATED;
-        up.relu2 = 0;
-        up.limit = L->limit;
-        up.slope = WRH_CLAMPED_SLOPE;
-        up.up_bias = WRH_CLAMPED_UP_BIAS;
-    }
-    TRY(wr_hip_mix_gemm_run(mm->f32, &up), "experts' up projection");
-    const wr_hip_mix_gemm down = {.w = L->w_edown, .x = t.act, .x_kt = L->ff_p / 32, .rows = t.groups * 16,
-                                  .group_expert = t.group_expert, .tile_groups = t.tile_groups,
-                                  .out = WR_HIP_MIX_OUT_ROWS_F32, .y_f32 = t.ys, .ldy = mm->width_p};
-    TRY(wr_hip_mix_gemm_run(mm->f32, &down), "experts' down projection");
+    const wr_status st = walk_experts(m, L, r, w, &t, t.z, L->router_p, res);
+    if (st != WR_OK) return st;
     if (L->shared_p) {
         const wr_hip_mix_gemm sh = {.w = L->w_down, .x = t.shared_act, .x_kt = L->shared_p / 32, .rows = R,
                                     .out = WR_HIP_MIX_OUT_ROWS_F32, .y_f32 = t.shared, .ldy = mm->width_p};
         TRY(wr_hip_mix_gemm_run(mm->f32, &sh), "shared expert's down projection");
     }
-    res->y = t.ys;
-    res->gate = t.gate;
-    res->slot = t.slot;
-    res->top = L->router.top;
     if (L->router.identity || L->shared_p) {
         res->side = t.side;
         res->ident = L->router.identity ? w->h : NULL;
@@ -559,7 +679,6 @@ static wr_status walk_mlp(wr_model *m, const wrh_mix_layer *L, uint32_t r, const
     }
     return WR_OK;
 }
-
 static wr_status capture(struct wrh_mix_model *mm, const walk *w, uint32_t R)
 {
     const size_t n = (size_t)R * mm->width;
@@ -579,7 +698,8 @@ static wr_status walk_layers(wr_model *m, walk *w, bump b, uint32_t R, int fail_
     uint32_t r = 0;
     for (uint32_t i = 0; i < mm->n_ropes; i++)
         if (mm->ropes[i].dims)
-            TRY(wr_hip_mix_rope_table(mm->step, mm->ropes[i].freq_dev, mm->ropes[i].dims / 2, w->rope[i]), "angles");
+            TRY(wr_hip_mix_rope_table(mm->step, mm->ropes[i].freq_dev, mm->ropes[i].dims / 2, mm->ropes[i].gain, w->rope[i]),
+                "angles");
     const wrh_mix_layer *next = &mm->layers[mm->runs[0].layer];
     /* a layer behind a token shift makes its input from the residual itself */
     TRY(wr_hip_mix_embed(mm->step, mm->f32, mm->embed_dev, mm->width, mm->embed_norm, mm->embed_scale, mm->eps, w->x, w->x0,
@@ -590,17 +710,23 @@ static wr_status walk_layers(wr_model *m, walk *w, bump b, uint32_t R, int fail_
         next = r + 1 < mm->n_runs ? &mm->layers[mm->runs[r + 1].layer] : NULL;
         if (fail_run == (int)r) return op_fail(m, "mixer (injected)", r, WR_ERR_INTERNAL);
         wr_status st = WR_ERR_INTERNAL;
+        wr_hip_mix_resid res = {.width = mm->width, .eps = mm->eps};
         switch (L->kind) {
         case WRH_MIXER_LIGHTNING: st = walk_lightning(m, L, r, w, b, R); break;
         case WRH_MIXER_LATENT: st = walk_latent(m, L, r, w, b, R); break;
         case WRH_MIXER_WKV: st = walk_wkv(m, L, r, w, b, R, y); break;
         case WRH_MIXER_PARALLEL: st = walk_parallel(m, L, r, w, b, R); break;
         case WRH_MIXER_WINDOW: st = walk_window(m, L, r, w, b, R); break;
+        case WRH_MIXER_JOINT: st = walk_joint(m, L, r, w, b, R, &res); break;
         }
         if (st != WR_OK) return st;
         y = NULL;
-        wr_hip_mix_resid res = {.width = mm->width, .eps = mm->eps, .x = w->x, .y = w->y, .post = L->norm1b};
-        if (L->mlp != WRH_MLP_NONE) {
+        res.x = w->x;
+        if (L->kind != WRH_MIXER_JOINT) {
+            res.y = w->y;
+            res.post = L->norm1b;
+        }
+        if (L->kind != WRH_MIXER_JOINT && L->mlp != WRH_MLP_NONE) {
             /* the mixer's output joins the residual and the feed-forward's input is made */
             res.next = L->norm2;
             res.h = w->h;
@@ -617,16 +743,22 @@ static wr_status walk_layers(wr_model *m, walk *w, bump b, uint32_t R, int fail_
             res = (wr_hip_mix_resid){.width = mm->width, .eps = mm->eps, .x = w->x};
         }
         if (next) {
-            if (mm->runs[r + 1].add_embedding) res.add = w->x0;
+            if (mm->runs[r + 1].add_embedding) {
+                if (res.add) {                             /* the layer's outputs first */
+                    TRY(wr_hip_mix_residual(mm->step, mm->f32, &res), "post-norm + residual");
+                    res = (wr_hip_mix_resid){.width = mm->width, .eps = mm->eps, .x = w->x};
+                }
+                res.add = w->x0;
+            }
             if (next->kind != WRH_MIXER_WKV) {
                 res.next = next->norm1;
                 res.h = w->h;
-            } else if (res.y && !res.post && !res.top && !res.add) {
+            } else if (res.y && !res.post && !res.top && !res.add && !res.pair_y[0]) {
                 y = res.y;                                 /* the token shift adds it */
                 res.y = NULL;
             }
         }
-        if (res.y || res.add || res.next) TRY(wr_hip_mix_residual(mm->step, mm->f32, &res), "post-norm + residual");
+        if (res.y || res.add || res.pair_y[0] || res.next) TRY(wr_hip_mix_residual(mm->step, mm->f32, &res), "post-norm + residual");
     }
     return WR_OK;
 }

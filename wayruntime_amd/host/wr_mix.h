@@ -3,8 +3,8 @@
  * attention, windowed attention through a latent, a matrix-state recurrence behind
  * a token shift, windowed grouped-query attention, or that and such a recurrence side
  * by side) and an optional feed-forward (dense or a mixture of experts), with norms
- * before and, in some designs, after each, part of the list possibly run several
- * times.  A design (wrh_mix_design) says which of these its models use.  Read from a folder with config.json and
+ * before and, in some designs, after each, or one norm whose rows both read, part of
+ * the list possibly run several times.  A design (wrh_mix_design) says which of these its models use.  Read from a folder with config.json and
  * model.safetensors.  wr_mix_model.c reads and uploads, wr_mix.c keeps the cache
  * pool and walks the layers.
  */
@@ -15,7 +15,10 @@
 #include "wr_json.h"
 #include "../../include/wr_hip_mix.h"
 
-typedef enum { WRH_MIXER_LIGHTNING, WRH_MIXER_LATENT, WRH_MIXER_WKV, WRH_MIXER_PARALLEL, WRH_MIXER_WINDOW } wrh_mixer_kind;
+typedef enum { WRH_MIXER_LIGHTNING, WRH_MIXER_LATENT, WRH_MIXER_WKV, WRH_MIXER_PARALLEL, WRH_MIXER_WINDOW,
+               WRH_MIXER_JOINT } wrh_mixer_kind;
+/* What stands beside a joint layer's attention. */
+typedef enum { WRH_BESIDE_NOTHING, WRH_BESIDE_FORGET, WRH_BESIDE_GRU } wrh_beside_kind;
 typedef enum { WRH_MLP_NONE, WRH_MLP_DENSE, WRH_MLP_MOE } wrh_mlp_kind;
 
 /* A matrix-state recurrence: its own part of a layer's products and vectors. */
@@ -23,6 +26,8 @@ typedef struct wrh_mix_recur {
     uint32_t heads, dim, hd_p, rank_p;    /* hd = heads * dim; rank of the decay's low-rank product */
     wr_hip_mat *w_decay;                  /* [hd_p][rank_p] */
     const float *w0, *u, *a_bias, *norm;
+    uint32_t vdim, hv_p;                  /* a forget gate's: values of their own size */
+    const float *lower;
 } wrh_mix_recur;
 
 /* Feature counts ending in _p are padded to a multiple of 32. */
@@ -53,6 +58,15 @@ typedef struct wrh_mix_layer {
     uint8_t has_gate;                     /* a logistic gate per head, its logits at col_rg */
     int32_t kv_from;                      /* layer whose keys and values it reads, or -1 */
     const float *b_in;                    /* ld_in biases, or NULL */
+    /* joint: mixers and feed-forward read one norm.  One stacked product of the mixers' inputs and, behind ld_in rows, a
+     * dense feed-forward's gate and up, or the router's logits among the rows; w_o takes out everything, or with
+     * out_norm the attention alone (w_o2 what stands beside it, w_down the feed-forward), each mixer's output normed */
+    wrh_beside_kind beside;
+    int32_t turn;                         /* rotary table of the values, or -1 */
+    uint32_t gru, gru_p;                  /* elements of the gated recurrence */
+    uint32_t col_router, silu_end;        /* rows below silu_end leave the product through SiLU */
+    wr_hip_mat *w_o2;
+    const float *b_o, *out_norm[2];       /* (halved: the outputs are averaged) */
     /* feed-forward */
     wrh_mlp_kind mlp;
     uint8_t gelu;
@@ -61,6 +75,7 @@ typedef struct wrh_mix_layer {
     /* experts: the router's outputs, padded (logit rows); with limit > 0 gated experts, clamped (w_eup: gate and up) */
     wr_hip_mix_router router;
     uint32_t router_p;
+    uint8_t gated, weigh_input;           /* gated experts without a clamp; the weights multiply the experts' input */
     float limit;
     /* shared expert: w_router carries its gate's logit and, behind router_p rows, its gate and up; w_down takes it out */
     uint32_t shared_p;                    /* its width, or 0 */
@@ -79,6 +94,8 @@ typedef struct wrh_mix_run {
 typedef struct wrh_mix_rope {
     double   base;
     uint32_t dims;
+    double   factor, original, fast, slow;    /* far pairs slowed down by factor (0: none) */
+    float    gain;                            /* of cosine and sine */
     double  *freq_dev;
 } wrh_mix_rope;
 

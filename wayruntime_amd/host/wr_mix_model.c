@@ -21,13 +21,15 @@ static uint32_t p32(uint32_t n) { return (n + 31) / 32 * 32; }
 static uint32_t p16(uint32_t n) { return (n + 15) / 16 * 16; }
 
 /* What tells the designs of this family apart. */
-typedef enum { DESIGN_BIPOTAR = 1, DESIGN_TAREDRA = 2, DESIGN_FEDIRAX = 4 } design_bit;
+typedef enum { DESIGN_BIPOTAR = 1, DESIGN_TAREDRA = 2, DESIGN_FEDIRAX = 4, DESIGN_MAROSUN = 8 } design_bit;
 typedef struct wrh_mix_design {
     const char *arch;
     design_bit  bit;
     uint8_t post_norms;                   /* a sublayer's output is normed before it joins the residual */
     uint8_t norms_around_zero;            /* stored w means 1 + w */
-    uint8_t embed_norm;                   /* the embedding is normed; else multiplied by embedding.scale */
+    uint8_t embed_norm;                   /* the embedding is normed; else multiplied by embedding.scale, */
+    uint8_t embed_plain;                  /* or taken as it is */
+    uint8_t joint;                        /* one norm per layer: mixers and feed-forward read the same rows */
     uint8_t tied_head;                    /* the head is the embedding table */
     uint8_t gelu;                         /* dense feed-forwards gate with the tanh form of GELU, else SiLU */
 } wrh_mix_design;
@@ -36,7 +38,17 @@ static const wrh_mix_design designs[] = {
     {.arch = "Bipotar", .bit = DESIGN_BIPOTAR, .post_norms = 1, .embed_norm = 1},
     {.arch = "Taredra", .bit = DESIGN_TAREDRA, .norms_around_zero = 1, .tied_head = 1, .gelu = 1},
     {.arch = "Fedirax", .bit = DESIGN_FEDIRAX, .norms_around_zero = 1},
+    {.arch = "Marosun", .bit = DESIGN_MAROSUN, .norms_around_zero = 1, .embed_plain = 1, .joint = 1},
 };
+
+/* One of the matrices that a product of a layer's input is stacked from: where its outputs lie, and its bias if any. */
+typedef struct in_part {
+    const char *name;
+    uint32_t    rows, *col;
+    const char *bias;
+} in_part;
+
+#define PARTS_MAX 12
 
 /* Everything the reading functions share; `st` keeps the first failure. */
 typedef struct loader {
@@ -46,6 +58,8 @@ typedef struct loader {
     wrh_safetensors       f;
     float                *vec;            /* host copy of the vector block being gathered */
     size_t                vec_n, vec_cap;
+    in_part               parts[PARTS_MAX];   /* of the joint layer being read */
+    size_t                n_parts;
     wr_status             st;
 } loader;
 
@@ -304,21 +318,48 @@ static void read_lightning(loader *l, uint32_t i, const wrh_json *c, wrh_mix_lay
     L->mix_norm = vec_put(l, ltensor(l, i, "mix.norm", hv, 0), hv);
 }
 
-/* The model's table of this rotation. */
-static uint32_t rope_index(loader *l, double base, uint32_t dims)
+/* The model's table of this rotation.  `scaling`: what slows its far pairs down (factor, original, fast, slow), or NULL. */
+static uint32_t rope_index(loader *l, double base, uint32_t dims, const wrh_json *scaling)
 {
     struct wrh_mix_model *mm = l->mm;
     uint32_t k = 0;
-    while (k < mm->n_ropes && !(mm->ropes[k].base == base && mm->ropes[k].dims == dims)) k++;
+    wrh_mix_rope q = {.base = base, .dims = dims, .gain = 1.0f};
+    if (scaling) {
+        q.factor = need_num(l, scaling, "factor");
+        q.original = need_num(l, scaling, "original");
+        q.fast = need_num(l, scaling, "fast");
+        q.slow = need_num(l, scaling, "slow");
+        if (l->st == WR_OK && (q.factor <= 0 || q.original <= 0 || q.fast <= 0 || q.slow <= 0 || base == 1.0))
+            fail(l, WR_ERR_FORMAT, "config: rotation of base %g scaled by %g over %g, between %g and %g turns", base, q.factor,
+                 q.original, q.fast, q.slow);
+        if (l->st != WR_OK) return 0;
+        q.gain = (float)(0.1 * log(q.factor) + 1.0);
+    }
+    for (; k < mm->n_ropes; k++) {
+        const wrh_mix_rope *o = &mm->ropes[k];
+        if (o->base == base && o->dims == dims && o->factor == q.factor && o->original == q.original && o->fast == q.fast &&
+            o->slow == q.slow)
+            break;
+    }
     if (k == WRH_MAX_LAYERS) {
         fail(l, WR_ERR_LIMIT, "config: more than %u different rotations", WRH_MAX_LAYERS);
         return 0;
     }
-    if (k == mm->n_ropes) {
-        mm->ropes[mm->n_ropes].base = base;
-        mm->ropes[mm->n_ropes++].dims = dims;
-    }
+    if (k == mm->n_ropes) mm->ropes[mm->n_ropes++] = q;
     return k;
+}
+
+/* Frequency of pair i of a rotation: a pair that turns more than `fast` times over the original length keeps its own, one
+ * that turns less than `slow` times has it divided by the factor, with a ramp over the pairs between. */
+static double rope_freq(const wrh_mix_rope *q, uint32_t i)
+{
+    const double f = pow(q->base, -2.0 * i / q->dims), two_pi = 6.283185307179586477;
+    if (q->factor == 0) return f;
+    const double fast = q->dims * log(q->original / (two_pi * q->fast)) / (2.0 * log(q->base));
+    const double slow = q->dims * log(q->original / (two_pi * q->slow)) / (2.0 * log(q->base));
+    const double lo = fmax(floor(fast), 0.0), hi = fmin(ceil(slow), q->dims - 1.0);
+    const double ramp = fmin(fmax((i - lo) / fmax(hi - lo, 0.001), 0.0), 1.0);
+    return f / q->factor * ramp + f * (1.0 - ramp);
 }
 
 /* The output matrix over heads whose inputs are padded one by one: [Wp][H * vp], zeros between.  `at`: its first
@@ -366,7 +407,7 @@ static void read_latent(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer 
     g->rot_half = dims / 2;
     g->window = window;
     g->scale = (float)scale;
-    L->rope = rope_index(l, base, dims);
+    L->rope = rope_index(l, base, dims, NULL);
     if (l->st != WR_OK) return;
 
     const uint32_t kp = p32(L->kv_rank), rp = p32(L->rot_dim);
@@ -488,7 +529,7 @@ static void read_parallel(loader *l, uint32_t i, const wrh_json *c, wrh_mix_laye
         fail(l, WR_ERR_LIMIT, "config: layer %u is too wide", i);
         return;
     }
-    L->rope = rope_index(l, base, dims);
+    L->rope = rope_index(l, base, dims, NULL);
     wrh_mix_recur *q = &L->rec;
     read_recur(l, i, "mix.right.", right, q);
     if (l->st != WR_OK) return;
@@ -523,28 +564,19 @@ static void read_parallel(loader *l, uint32_t i, const wrh_json *c, wrh_mix_laye
     L->w_o = operand_up(l, &o);
 }
 
-/* What windowed attention mixers of their own share: sizes, rotation of neighbours, window, scale. */
-static int read_window_sizes(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *L, uint32_t maps)
+/* What attention mixers over grouped keys and values share: sizes and scale. */
+static int read_heads(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *L, uint32_t maps)
 {
     wr_hip_mix_window *g = &L->win;
-    L->kind = WRH_MIXER_WINDOW;
-    L->kv_from = -1;
     const uint32_t H = g->heads = L->heads = need_u32(l, c, "heads", 1, HEADS_MAX);
     const uint32_t G = g->kv_heads = need_u32(l, c, "kv_heads", 1, HEADS_MAX);
     g->dim = L->dim = need_u32(l, c, "dim", 1, 4096);
     g->vdim = L->vdim = need_u32(l, c, "vdim", 1, 4096);
-    const wrh_json *rot = need_obj(l, c, "rot"), *mask = need_obj(l, c, "mask");
     g->scale = (float)need_num(l, c, "scale");
-    if (l->st != WR_OK) return 0;
-    const double base = need_num(l, rot, "base");
-    const uint32_t dims = need_u32(l, rot, "dims", 0, g->dim);
-    g->window = need_u32(l, mask, "size", 1, 0xFFFFFFFFu);
-    if (l->st == WR_OK && (dims % 2 || base <= 0)) fail(l, WR_ERR_FORMAT, "config: layer %u: rotation of %u dimensions, base %g", i, dims, base);
     if (l->st == WR_OK && H % G) fail(l, WR_ERR_FORMAT, "config: layer %u: %u heads over %u key/value heads", i, H, G);
     if (l->st != WR_OK) return 0;
     g->dim_pad = wr_hip_mix_window_pad(g->dim);
     g->vdim_pad = wr_hip_mix_window_pad(g->vdim);
-    g->rot_half = dims / 2;
     g->neighbours = 1;
     g->maps = maps;
     g->out_scale = 1.0f;
@@ -553,27 +585,60 @@ static int read_window_sizes(loader *l, uint32_t i, const wrh_json *c, wrh_mix_l
         fail(l, WR_ERR_LIMIT, "config: layer %u is too wide", i);
         return 0;
     }
-    L->rope = rope_index(l, base, dims);
+    return 1;
+}
+
+/* The rotation of queries and keys; returns its base. */
+static double read_rotation(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *L)
+{
+    const wrh_json *rot = need_obj(l, c, "rot");
+    if (l->st != WR_OK) return 0;
+    const double base = need_num(l, rot, "base");
+    const uint32_t dims = need_u32(l, rot, "dims", 0, L->win.dim);
+    if (l->st == WR_OK && (dims % 2 || base <= 0)) fail(l, WR_ERR_FORMAT, "config: layer %u: rotation of %u dimensions, base %g", i, dims, base);
+    if (l->st != WR_OK) return 0;
+    L->win.rot_half = dims / 2;
+    L->rope = rope_index(l, base, dims, given(rot, "scaling"));
+    return base;
+}
+
+/* What windowed attention mixers of their own share: sizes, rotation of neighbours, window, scale. */
+static int read_window_sizes(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *L, uint32_t maps)
+{
+    L->kind = WRH_MIXER_WINDOW;
+    L->kv_from = -1;
+    if (!read_heads(l, i, c, L, maps)) return 0;
+    (void)read_rotation(l, i, c, L);
+    const wrh_json *mask = need_obj(l, c, "mask");
+    if (l->st == WR_OK) L->win.window = need_u32(l, mask, "size", 1, 0xFFFFFFFFu);
     return l->st == WR_OK;
 }
 
-/* One product of a layer's input out of several matrices: where each one's outputs lie, then the operand. */
-typedef struct in_part {
-    const char *name;
-    uint32_t    rows, *col;
-} in_part;
-
-static operand stack_inputs(loader *l, uint32_t i, const in_part *parts, size_t n, uint32_t *ld)
+/* One product of a layer's input out of several matrices: where each one's outputs lie, then the operand, with `more`
+ * rows behind theirs. */
+static operand stack_inputs(loader *l, uint32_t i, const in_part *parts, size_t n, uint32_t *ld, uint32_t more)
 {
     *ld = 0;
     for (size_t k = 0; k < n; k++) {
         *parts[k].col = *ld;
         *ld += p32(parts[k].rows);
     }
-    operand o = operand_new(l, 1, *ld, l->mm->width_p);
+    operand o = operand_new(l, 1, *ld + more, l->mm->width_p);
     for (size_t k = 0; k < n; k++)
         operand_put(l, &o, 0, *parts[k].col, ltensor(l, i, parts[k].name, parts[k].rows, l->mm->width), parts[k].rows, l->mm->width);
     return o;
+}
+
+/* Their biases, and zeros for those that have none and for `more` outputs behind. */
+static const float *stack_biases(loader *l, uint32_t i, const in_part *parts, size_t n, uint32_t ld, uint32_t more)
+{
+    size_t at = 0;
+    float *b = l->st == WR_OK ? vec_take(l, ld + more, &at) : NULL;
+    for (size_t k = 0; k < n && b; k++) {
+        const uint16_t *src = parts[k].bias ? ltensor(l, i, parts[k].bias, parts[k].rows, 0) : NULL;
+        for (uint32_t j = 0; src && j < parts[k].rows; j++) b[*parts[k].col + j] = widen(src[j]);
+    }
+    return b ? (const float *)(uintptr_t)(at + 1) : NULL;
 }
 
 static void read_window_out(loader *l, uint32_t i, wrh_mix_layer *L)
@@ -593,19 +658,13 @@ static void read_window_keys(loader *l, uint32_t i, const wrh_json *c, wrh_mix_l
     if (given(c, "softcap")) g->softcap = (float)need_num(l, c, "softcap");
     if (l->st == WR_OK && (g->vdim != g->dim || g->softcap < 0))
         fail(l, WR_ERR_FORMAT, "config: layer %u: values of %u from keys of %u, scores capped at %g", i, g->vdim, g->dim, g->softcap);
-    const in_part parts[] = {{"mix.q", hq, &L->col_q}, {"mix.k", hk, &L->col_k}, {"mix.g", g->heads, &L->col_rg}};
-    operand o = stack_inputs(l, i, parts, sizeof parts / sizeof *parts, &L->ld_in);
+    const in_part parts[] = {{"mix.q", hq, &L->col_q, "mix.q.b"}, {"mix.k", hk, &L->col_k, "mix.k.b"}, {"mix.g", g->heads, &L->col_rg, NULL}};
+    const size_t n = sizeof parts / sizeof *parts;
+    operand o = stack_inputs(l, i, parts, n, &L->ld_in, 0);
     L->w_in = operand_up(l, &o);
+    L->b_in = stack_biases(l, i, parts, n, L->ld_in, 0);
     L->col_v = L->col_k;
     L->has_gate = 1;
-    const uint16_t *bq = ltensor(l, i, "mix.q.b", hq, 0), *bk = ltensor(l, i, "mix.k.b", hk, 0);
-    size_t at = 0;
-    float *b = l->st == WR_OK ? vec_take(l, L->ld_in, &at) : NULL;
-    if (b) {
-        for (uint32_t k = 0; k < hq; k++) b[L->col_q + k] = widen(bq[k]);
-        for (uint32_t k = 0; k < hk; k++) b[L->col_k + k] = widen(bk[k]);
-        L->b_in = (const float *)(uintptr_t)(at + 1);
-    }
     L->sink = vec_put(l, ltensor(l, i, "mix.sink", g->heads, 0), g->heads);
     read_window_out(l, i, L);
 }
@@ -637,9 +696,9 @@ static void read_window_difference(loader *l, uint32_t i, const wrh_json *c, wrh
     const double lambda = exp(dot_of(l, i, "mix.lq1", "mix.lk1", g->dim)) - exp(dot_of(l, i, "mix.lq2", "mix.lk2", g->dim)) + diff;
     g->diff = (float)lambda;
     g->out_scale = (float)(1.0 - diff);
-    const in_part parts[] = {{"mix.q", g->heads * 2 * g->dim, &L->col_q}, {"mix.k", g->kv_heads * 2 * g->dim, &L->col_k},
-                             {"mix.v", g->kv_heads * g->vdim, &L->col_v}};
-    operand o = stack_inputs(l, i, parts, L->kv_from >= 0 ? 1 : sizeof parts / sizeof *parts, &L->ld_in);
+    const in_part parts[] = {{"mix.q", g->heads * 2 * g->dim, &L->col_q, NULL}, {"mix.k", g->kv_heads * 2 * g->dim, &L->col_k, NULL},
+                             {"mix.v", g->kv_heads * g->vdim, &L->col_v, NULL}};
+    operand o = stack_inputs(l, i, parts, L->kv_from >= 0 ? 1 : sizeof parts / sizeof *parts, &L->ld_in, 0);
     L->w_in = operand_up(l, &o);
     g->q_norm = vec_put(l, ltensor(l, i, "mix.q.norm", g->dim, 0), g->dim);
     if (L->kv_from < 0) g->k_norm = vec_put(l, ltensor(l, i, "mix.k.norm", g->dim, 0), g->dim);
@@ -699,6 +758,24 @@ static void read_moe(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *L)
     L->w_edown = operand_up(l, &down);
 }
 
+/* Experts of gated units: gate and up interleaved, down. */
+static void read_gated_experts(loader *l, uint32_t i, wrh_mix_layer *L)
+{
+    const uint32_t W = l->mm->width, Wp = l->mm->width_p;
+    const wr_hip_mix_router *q = &L->router;
+    operand up = operand_new(l, q->experts, 2 * L->ff_p, Wp), down = operand_new(l, q->experts, Wp, L->ff_p);
+    for (uint32_t x = 0; x < q->experts && l->st == WR_OK; x++) {
+        char nb[3][64];
+        static const char *const ends[] = {"gate", "up", "down"};
+        for (uint32_t k = 0; k < 3; k++) snprintf(nb[k], sizeof nb[k], "mlp.e%u.%s", x, ends[k]);
+        const uint16_t *g = ltensor(l, i, nb[0], L->ff, W), *u = ltensor(l, i, nb[1], L->ff, W);
+        put_gated(l, &up, x, 0, g, u, L->ff, W);
+        operand_put(l, &down, x, 0, ltensor(l, i, nb[2], W, L->ff), W, L->ff);
+    }
+    L->w_eup = operand_up(l, &up);
+    L->w_edown = operand_up(l, &down);
+}
+
 /* Clamped gated experts behind a corrected softmax router with groups and outputs that pass the input on; a shared
  * expert with a gate of its own. */
 static void read_grouped_moe(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *L)
@@ -748,17 +825,172 @@ static void read_grouped_moe(loader *l, uint32_t i, const wrh_json *c, wrh_mix_l
     }
     L->w_router = operand_up(l, &o);
     q->correction = vec_put(l, ltensor(l, i, "mlp.correction", outputs, 0), outputs);
-    operand up = operand_new(l, q->experts, 2 * L->ff_p, Wp), down = operand_new(l, q->experts, Wp, L->ff_p);
-    for (uint32_t x = 0; x < q->experts && l->st == WR_OK; x++) {
-        char nb[3][64];
-        static const char *const ends[] = {"gate", "up", "down"};
-        for (uint32_t k = 0; k < 3; k++) snprintf(nb[k], sizeof nb[k], "mlp.e%u.%s", x, ends[k]);
-        const uint16_t *g = ltensor(l, i, nb[0], L->ff, W), *u = ltensor(l, i, nb[1], L->ff, W);
-        put_gated(l, &up, x, 0, g, u, L->ff, W);
-        operand_put(l, &down, x, 0, ltensor(l, i, nb[2], W, L->ff), W, L->ff);
+    read_gated_experts(l, i, L);
+}
+
+/* ---- joint layers: the mixer's and the feed-forward's readers gather, finish_joint makes the products ---- */
+
+static void joint_part(loader *l, const char *name, uint32_t rows, uint32_t *col, const char *bias)
+{
+    if (l->n_parts < PARTS_MAX) l->parts[l->n_parts++] = (in_part){name, rows, col, bias};
+    else fail(l, WR_ERR_INTERNAL, "too many input products in a layer");
+}
+
+static int read_joint_attention(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *L)
+{
+    L->kind = WRH_MIXER_JOINT;
+    L->kv_from = L->turn = -1;
+    L->win.window = 0xFFFFFFFFu;
+    return c && read_heads(l, i, c, L, 1);
+}
+
+/* Biases, normed and rotated queries and keys, a sink per head, values turned with their position. */
+static void read_joint_turned(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *L)
+{
+    if (!read_joint_attention(l, i, c, L)) return;
+    wr_hip_mix_window *g = &L->win;
+    const double base = read_rotation(l, i, c, L);
+    if (l->st == WR_OK && g->vdim % 2) fail(l, WR_ERR_FORMAT, "config: layer %u: values of %u elements turn in pairs", i, g->vdim);
+    if (l->st != WR_OK) return;
+    L->turn = (int32_t)rope_index(l, base, g->vdim, NULL);
+    joint_part(l, "mix.q", g->heads * g->dim, &L->col_q, "mix.q.b");
+    joint_part(l, "mix.k", g->kv_heads * g->dim, &L->col_k, "mix.k.b");
+    joint_part(l, "mix.v", g->kv_heads * g->vdim, &L->col_v, "mix.v.b");
+    g->q_norm = vec_put(l, ltensor(l, i, "mix.q.norm", g->dim, 0), g->dim);
+    g->k_norm = vec_put(l, ltensor(l, i, "mix.k.norm", g->dim, 0), g->dim);
+    L->sink = vec_put(l, ltensor(l, i, "mix.sink", g->heads, 0), g->heads);
+    L->b_o = vec_put(l, ltensor(l, i, "mix.o.b", l->mm->width, 0), l->mm->width);
+}
+
+/* Attention in chunks with sinks and a gate per output element, beside the recurrence whose forget gate makes the keys. */
+static void read_joint_chunks(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *L)
+{
+    const wrh_json *left = need_obj(l, c, "left"), *right = need_obj(l, c, "right");
+    if (!read_joint_attention(l, i, left, L)) return;
+    wr_hip_mix_window *g = &L->win;
+    wrh_mix_recur *q = &L->rec;
+    const wrh_json *mask = need_obj(l, left, "mask");
+    if (l->st != WR_OK) return;
+    g->chunk = need_u32(l, mask, "size", 1, 0xFFFFFFFFu);
+    g->out_scale = (float)need_num(l, c, "left_scale");
+    L->right_scale = (float)need_num(l, c, "right_scale");
+    q->heads = need_u32(l, right, "heads", 1, HEADS_MAX);
+    q->dim = need_u32(l, right, "dim", 1, WR_HIP_MIX_MAX_RECUR_DIM);
+    q->vdim = need_u32(l, right, "vdim", 1, WR_HIP_MIX_MAX_RECUR_DIM);
+    if (l->st != WR_OK) return;
+    const uint32_t hd = q->heads * q->dim;
+    L->beside = WRH_BESIDE_FORGET;
+    q->hd_p = p32(hd);
+    q->hv_p = p32(q->heads * q->vdim);
+    L->has_gate = 1;
+    g->gate_wide = 1;
+    joint_part(l, "mix.right.q", hd, &L->col_rr, NULL);    /* first: it leaves the product through SiLU */
+    L->silu_end = q->hd_p;
+    joint_part(l, "mix.right.f", hd, &L->col_rk, NULL);    /* (its bias is the recurrence's) */
+    joint_part(l, "mix.right.v", q->heads * q->vdim, &L->col_rv, NULL);
+    joint_part(l, "mix.left.q", g->heads * g->dim, &L->col_q, NULL);
+    joint_part(l, "mix.left.k", g->kv_heads * g->dim, &L->col_k, NULL);
+    joint_part(l, "mix.left.v", g->kv_heads * g->vdim, &L->col_v, NULL);
+    joint_part(l, "mix.left.g", g->heads * g->vdim, &L->col_rg, NULL);
+    q->w0 = vec_put(l, ltensor(l, i, "mix.right.f.b", hd, 0), hd);
+    q->lower = vec_put(l, ltensor(l, i, "mix.right.lower", hd, 0), hd);
+    q->norm = vec_put(l, ltensor(l, i, "mix.right.norm", q->vdim, 0), q->vdim);
+    L->sink = vec_put(l, ltensor(l, i, "mix.left.sink", g->heads, 0), g->heads);
+}
+
+/* Attention with one added to the softmax's denominator beside a gated recurrence, each output normed, and their mean. */
+static void read_joint_averaged(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *L)
+{
+    const wrh_json *left = need_obj(l, c, "left"), *right = need_obj(l, c, "right");
+    if (!read_joint_attention(l, i, left, L)) return;
+    wr_hip_mix_window *g = &L->win;
+    const uint32_t W = l->mm->width;
+    (void)read_rotation(l, i, left, L);
+    L->gru = need_u32(l, right, "width", 1, DIM_MAX);
+    if (l->st != WR_OK) return;
+    L->beside = WRH_BESIDE_GRU;
+    L->gru_p = p32(L->gru);
+    joint_part(l, "mix.left.q", g->heads * g->dim, &L->col_q, "mix.left.q.b");
+    joint_part(l, "mix.left.k", g->kv_heads * g->dim, &L->col_k, "mix.left.k.b");
+    joint_part(l, "mix.left.v", g->kv_heads * g->vdim, &L->col_v, "mix.left.v.b");
+    joint_part(l, "mix.right.z", L->gru, &L->col_rr, "mix.right.z.b");
+    joint_part(l, "mix.right.x", L->gru, &L->col_rk, "mix.right.x.b");
+    joint_part(l, "mix.right.g", L->gru, &L->col_rv, NULL);
+    g->q_norm = vec_put(l, ltensor(l, i, "mix.left.q.norm", g->dim, 0), g->dim);
+    g->k_norm = vec_put(l, ltensor(l, i, "mix.left.k.norm", g->dim, 0), g->dim);
+    size_t at = 0;
+    if (vec_take(l, g->heads, &at)) L->sink = (const float *)(uintptr_t)(at + 1);      /* scores of zero */
+    L->b_o = vec_put(l, ltensor(l, i, "mix.left.o.b", W, 0), W);
+    static const char *const outs[] = {"mix.left.out", "mix.right.out"};
+    for (uint32_t k = 0; k < 2; k++) {
+        L->out_norm[k] = vec_put(l, ltensor(l, i, outs[k], W, 0), W);
+        for (uint32_t j = 0; j < W && L->out_norm[k]; j++) l->vec[(uintptr_t)L->out_norm[k] - 1 + j] *= 0.5f;
     }
-    L->w_eup = operand_up(l, &up);
-    L->w_edown = operand_up(l, &down);
+}
+
+/* Clamped gated units. */
+static void read_joint_dense(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *L)
+{
+    L->mlp = WRH_MLP_DENSE;
+    L->ff = need_u32(l, c, "ff", 1, DIM_MAX);
+    L->limit = (float)need_num(l, c, "limit");
+    if (l->st == WR_OK && !(L->limit > 0)) fail(l, WR_ERR_FORMAT, "config: layer %u: units clamped at %g", i, L->limit);
+    L->ff_p = p32(L->ff);
+}
+
+/* Gated experts behind a logistic router, whose weights multiply the experts' input. */
+static void read_joint_moe(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *L)
+{
+    L->mlp = WRH_MLP_MOE;
+    const wrh_json *ex = need_obj(l, c, "expert"), *ro = need_obj(l, c, "router");
+    if (l->st != WR_OK) return;
+    wr_hip_mix_router *q = &L->router;
+    L->ff = need_u32(l, ex, "ff", 1, DIM_MAX);
+    q->experts = need_u32(l, ro, "experts", 1, WR_HIP_MIX_MAX_EXPERTS);
+    q->top = need_u32(l, ro, "top", 1, WR_HIP_MIX_MAX_TOP);
+    if (l->st == WR_OK && q->top > q->experts) fail(l, WR_ERR_FORMAT, "config: layer %u: more experts per token than experts", i);
+    if (l->st != WR_OK) return;
+    q->logistic = 1;
+    L->gated = L->weigh_input = 1;
+    L->ff_p = p32(L->ff);
+    L->router_p = p32(q->experts);
+    joint_part(l, "mlp.router", q->experts, &L->col_router, NULL);
+    read_gated_experts(l, i, L);
+}
+
+static void finish_joint(loader *l, uint32_t i, wrh_mix_layer *L)
+{
+    const uint32_t W = l->mm->width, Wp = l->mm->width_p, ff = L->mlp == WRH_MLP_DENSE ? L->ff_p : 0;
+    const wr_hip_mix_window *g = &L->win;
+    const uint32_t heads = g->heads * g->vdim_pad, beside = L->beside == WRH_BESIDE_FORGET ? L->rec.hv_p : L->gru_p;
+    if (l->st != WR_OK) return;
+    int biased = 0;
+    for (size_t k = 0; k < l->n_parts; k++) biased |= l->parts[k].bias != NULL;
+    operand o = stack_inputs(l, i, l->parts, l->n_parts, &L->ld_in, 2 * ff);
+    const uint16_t *wd = NULL;
+    if (ff) {
+        const uint16_t *gate = ltensor(l, i, "mlp.gate", L->ff, W), *up = ltensor(l, i, "mlp.up", L->ff, W);
+        put_gated(l, &o, 0, L->ld_in, gate, up, L->ff, W);
+        wd = ltensor(l, i, "mlp.down", W, L->ff);
+    }
+    L->w_in = operand_up(l, &o);
+    if (biased) L->b_in = stack_biases(l, i, l->parts, l->n_parts, L->ld_in, 2 * ff);
+    const char *first = L->beside ? "mix.left.o" : "mix.o";
+    const uint16_t *wo = ltensor(l, i, first, W, g->heads * g->vdim), *wo2 = NULL;
+    const uint32_t n2 = L->beside == WRH_BESIDE_FORGET ? L->rec.heads * L->rec.vdim : L->gru;
+    if (L->beside) wo2 = ltensor(l, i, "mix.right.o", W, n2);
+    const int apart = L->out_norm[0] != NULL;
+    o = operand_new(l, 1, Wp, apart ? heads : heads + beside + ff);
+    put_heads_out(l, &o, wo, 0, g->heads, g->vdim, g->vdim_pad);
+    if (apart) {
+        L->w_o = operand_up(l, &o);
+        L->w_o2 = plain(l, wo2, W, n2, Wp);
+        if (ff) L->w_down = plain(l, wd, W, L->ff, Wp);
+        return;
+    }
+    put_heads_out(l, &o, wo2, heads, 1, n2, beside);
+    put_heads_out(l, &o, wd, heads + beside, 1, L->ff, ff);
+    L->w_o = operand_up(l, &o);
 }
 
 static void read_layer(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *L)
@@ -776,10 +1008,15 @@ static void read_layer(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *
                   {"wkv", read_wkv, DESIGN_TAREDRA},
                   {"parallel", read_parallel, DESIGN_TAREDRA},
                   {"attention", read_window_keys, DESIGN_FEDIRAX},
-                  {"attention_2", read_window_difference, DESIGN_FEDIRAX}},
+                  {"attention_2", read_window_difference, DESIGN_FEDIRAX},
+                  {"attention", read_joint_turned, DESIGN_MAROSUN},
+                  {"parallel", read_joint_chunks, DESIGN_MAROSUN},
+                  {"parallel_2", read_joint_averaged, DESIGN_MAROSUN}},
       mlps[] = {{"dense", read_dense, DESIGN_BIPOTAR | DESIGN_TAREDRA},
                 {"moe", read_moe, DESIGN_BIPOTAR},
-                {"moe", read_grouped_moe, DESIGN_FEDIRAX}};
+                {"moe", read_grouped_moe, DESIGN_FEDIRAX},
+                {"dense", read_joint_dense, DESIGN_MAROSUN},
+                {"moe", read_joint_moe, DESIGN_MAROSUN}};
     const size_t n_mixers = sizeof mixers / sizeof *mixers, n_mlps = sizeof mlps / sizeof *mlps;
     const wrh_mix_design *d = l->design;
     size_t k = 0;
@@ -788,11 +1025,15 @@ static void read_layer(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *
         fail(l, WR_ERR_UNSUPPORTED, "layer %u: mixer '%s' is not served by this engine", i, type);
         return;
     }
+    l->n_parts = 0;
     mixers[k].read(l, i, mixer, L);
     L->norm1 = norm_put(l, ltensor(l, i, "norm1", W, 0), W);
     if (d->post_norms) L->norm1b = norm_put(l, ltensor(l, i, "norm1b", W, 0), W);
     const wrh_json *mlp = wrh_json_get(c, "mlp");
-    if (!mlp || mlp->type == WRH_JSON_NULL) return;
+    if (!mlp || mlp->type == WRH_JSON_NULL) {
+        if (d->joint) finish_joint(l, i, L);
+        return;
+    }
     const char *kind = need_str(l, mlp, "kind");
     if (l->st != WR_OK) return;
     for (k = 0; k < n_mlps && (strcmp(kind, mlps[k].name) || !(mlps[k].designs & d->bit)); k++) {}
@@ -801,6 +1042,10 @@ static void read_layer(loader *l, uint32_t i, const wrh_json *c, wrh_mix_layer *
         return;
     }
     mlps[k].read(l, i, mlp, L);
+    if (d->joint) {
+        finish_joint(l, i, L);
+        return;
+    }
     L->norm2 = norm_put(l, ltensor(l, i, "norm2", W, 0), W);
     if (d->post_norms) L->norm2b = norm_put(l, ltensor(l, i, "norm2b", W, 0), W);
 }
@@ -869,6 +1114,14 @@ static void plan_runs(loader *l, const wrh_json *cfg)
             mm->runs[r].store = mm->n_latent;
             mm->latent_dim[mm->n_latent++] = L->win.kv_heads * (L->win.maps * L->win.dim_pad + L->win.vdim_pad);
             break;
+        case WRH_MIXER_JOINT:
+            mm->runs[r].store = mm->n_latent;
+            mm->latent_dim[mm->n_latent++] = L->win.kv_heads * (L->win.dim_pad + L->win.vdim_pad);
+            if (L->beside == WRH_BESIDE_NOTHING) break;
+            mm->runs[r].store2 = mm->n_state;
+            mm->state_elems[mm->n_state++] = L->beside == WRH_BESIDE_GRU ? L->gru_p
+                                                                         : (uint64_t)L->rec.heads * L->rec.dim * L->rec.vdim;
+            break;
         }
     }
 }
@@ -888,7 +1141,8 @@ static void upload_small(loader *l)
         wrh_mix_layer *L = &mm->layers[i];
         const float **p[] = {&L->decay, &L->mix_norm, &L->dq_norm, &L->dkv_norm, &L->norm1, &L->norm1b, &L->norm2, &L->norm2b,
                              &L->mu, &L->sink, &L->rec.w0, &L->rec.u, &L->rec.a_bias, &L->rec.norm, &L->b_in, &L->win.q_norm,
-                             &L->win.k_norm, &L->router.correction};
+                             &L->win.k_norm, &L->router.correction, &L->rec.lower, &L->b_o, &L->out_norm[0],
+                             &L->out_norm[1]};
         for (size_t k = 0; k < sizeof p / sizeof *p; k++) vec_fix(mm, p[k]);
     }
     for (uint32_t r = 0; r < mm->n_ropes && l->st == WR_OK; r++) {
@@ -898,7 +1152,7 @@ static void upload_small(loader *l)
         double *f = malloc(bytes);
         R->freq_dev = wr_hip_attn_dev_alloc(bytes);
         if (f)
-            for (uint32_t i = 0; i < R->dims / 2; i++) f[i] = pow(R->base, -2.0 * i / R->dims);
+            for (uint32_t i = 0; i < R->dims / 2; i++) f[i] = rope_freq(R, i);
         if (!f || !R->freq_dev || wr_hip_attn_h2d(R->freq_dev, f, bytes) != WR_HIP_OK)
             fail(l, WR_ERR_NOMEM, "upload of the rotary frequencies failed");
         free(f);
@@ -911,7 +1165,7 @@ void wrh_mix_free(struct wrh_mix_model *mm)
     for (uint32_t i = 0; mm->layers && i < mm->n_layers; i++) {
         wrh_mix_layer *L = &mm->layers[i];
         wr_hip_mat *w[] = {L->w_qkvg, L->w_o, L->w_d, L->w_uq, L->w_uk, L->w_uv, L->w_gu, L->w_down, L->w_router, L->w_eup,
-                           L->w_edown, L->w_rkvg, L->w_low, L->w_in, L->rec.w_decay};
+                           L->w_edown, L->w_rkvg, L->w_low, L->w_in, L->rec.w_decay, L->w_o2};
         for (size_t k = 0; k < sizeof w / sizeof *w; k++) wr_hip_mix_mat_destroy(w[k]);
     }
     for (uint32_t r = 0; mm->ropes && r < mm->n_ropes; r++) wr_hip_attn_dev_free(mm->ropes[r].freq_dev);
@@ -947,7 +1201,7 @@ wr_status wrh_mix_load(wr_engine *e, const char *dir, const char *arch, const wr
     pthread_mutex_init(&mm->lock, NULL);
     const wrh_mix_design *design = designs;
     while (strcmp(design->arch, arch)) design++;           /* (the registry holds no other name) */
-    loader l = {e, design, mm, {0}, NULL, 0, 0, WR_OK};
+    loader l = {.e = e, .design = design, .mm = mm, .st = WR_OK};
     const wrh_json *layers = wrh_json_get(cfg, "layers");
     if (!layers || layers->type != WRH_JSON_ARRAY || layers->count == 0)
         fail(&l, WR_ERR_FORMAT, "config: 'layers' missing or empty");
@@ -961,14 +1215,16 @@ wr_status wrh_mix_load(wr_engine *e, const char *dir, const char *arch, const wr
     double scale = 1.0;
     if (wrh_json_get(cfg, "logit_scale")) scale = need_num(&l, cfg, "logit_scale");
     mm->logit_scale = (float)scale;
-    if (!design->embed_norm) {
+    if (design->embed_plain) {
+        mm->embed_scale = 1.0f;
+    } else if (!design->embed_norm) {
         const wrh_json *emb = need_obj(&l, cfg, "embedding");
         if (emb) mm->embed_scale = (float)need_num(&l, emb, "scale");
     }
     if (l.st == WR_OK) {
         mm->n_layers = layers->count;
         mm->layers = calloc(mm->n_layers, sizeof *mm->layers);
-        mm->ropes = calloc(mm->n_layers, sizeof *mm->ropes);
+        mm->ropes = calloc((size_t)2 * mm->n_layers, sizeof *mm->ropes);
         if (!mm->layers || !mm->ropes) fail(&l, WR_ERR_NOMEM, "out of memory");
     }
     if (l.st == WR_OK) {
@@ -1026,6 +1282,12 @@ wr_status wrh_mix_load(wr_engine *e, const char *dir, const char *arch, const wr
             if (L->win.kv_heads > m->n_kv) m->n_kv = L->win.kv_heads;
             if (L->win.window > m->sliding_window) m->sliding_window = L->win.window;
             m->rope_base = (float)mm->ropes[L->rope].base;
+        }
+        if (L->kind == WRH_MIXER_JOINT) {
+            if (L->win.kv_heads > m->n_kv) m->n_kv = L->win.kv_heads;
+            if (L->win.chunk) m->has_swa = 1;
+            if (L->win.chunk > m->sliding_window) m->sliding_window = L->win.chunk;
+            if (L->win.rot_half) m->rope_base = (float)mm->ropes[L->rope].base;
         }
     }
     m->max_context = p->max_context ? p->max_context : WRH_DEFAULT_CTX;

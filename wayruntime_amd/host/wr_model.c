@@ -502,7 +502,8 @@ static int bind_vector(wr_engine *e, const gguf_file *g, const char *name, uint3
 static const struct {
     const char *name;
     wr_status (*load)(wr_engine *, const char *, const char *, const wrh_json *, const wr_model_params *, wr_model *);
-} folder_archs[] = {{"Bipotar", wrh_mix_load}, {"Taredra", wrh_mix_load}, {"Fedirax", wrh_mix_load}};
+} folder_archs[] = {{"Bipotar", wrh_mix_load}, {"Taredra", wrh_mix_load}, {"Fedirax", wrh_mix_load},
+                    {"Marosun", wrh_mix_load}};
 
 static wr_status load_folder(wr_engine *e, const char *dir, const wr_model_params *p, wr_model **out)
 {
