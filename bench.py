@@ -203,13 +203,17 @@ def mixer_workload(args) -> None:
 
     steps = min(args.steps, 200)
     kind = args.workload
-    beside = {"mixer": ("gqa",), "taredra": ("mixer", "gqa"), "fedirax": ("mixer", "taredra", "gqa")}[kind]
+    beside = {"mixer": ("gqa",), "taredra": ("mixer", "gqa"), "fedirax": ("mixer", "taredra", "gqa"),
+              "marosun": ("taredra", "fedirax", "gqa")}[kind]
     model = {"mixer": "Bipotar, 4 layers (linear attention x 2, latent attention x 2; dense and expert feed-forwards), "
                       "width 4096, random init",
              "taredra": "Taredra, 4 layers (windowed attention beside a delta-rule recurrence x 2, wkv recurrence x 2; dense "
                         "feed-forwards), width 4096, random init",
              "fedirax": "Fedirax, 4 layers (differential attention x 2, one more over the first's keys and values, "
-                        "keys-as-values attention; expert feed-forwards), width 4096, random init"}[kind]
+                        "keys-as-values attention; expert feed-forwards), width 4096, random init",
+             "marosun": "Marosun, 4 layers (attention over turned values x 2, attention beside an element-wise gated "
+                        "recurrence, chunked attention beside a forget-gate recurrence; dense and expert feed-forwards), "
+                        "width 4096, random init"}[kind]
     figures = mix_timing.run(list(mix_timing.SIZES), reps=3, steps=steps, only=(kind,) + beside,
                              log=lambda *a: print(*a, file=sys.stderr, flush=True))
     top = figures["w4096"][kind]
@@ -240,7 +244,7 @@ def main() -> None:
     ap.add_argument("--no-decode-configs", action="store_true")
     ap.add_argument("--keys-per-wg", type=int, default=0)
     ap.add_argument("--workload", default="headline",
-                    choices=["headline", "ragged16", "long16", "long16-hd256", "batch1", "mixer", "taredra", "fedirax"],
+                    choices=["headline", "ragged16", "long16", "long16-hd256", "batch1", "mixer", "taredra", "fedirax", "marosun"],
                     help="headline: 16 sessions x --ctx, 32/8/128 (the metric's configuration), with "
                          "the other decode workloads as secondary keys; "
                          "ragged16: 16 sessions with contexts drawn from [256, 4096]; "
@@ -250,7 +254,8 @@ def main() -> None:
                          "mixer: prefill and decode throughput of mixer-stack models (Bipotar) with layers "
                          "of real sizes, random weights, beside a grouped-query model of the same width; "
                          "taredra: the same of Taredra models, beside both; "
-                         "fedirax: the same of Fedirax models, beside all three")
+                         "fedirax: the same of Fedirax models, beside all three; "
+                         "marosun: the same of Marosun models, beside Taredra, Fedirax and the grouped-query model")
     args = ap.parse_args()
 
     if args.gpus != 1:
@@ -258,7 +263,7 @@ def main() -> None:
               "(nothing here uses a second device)" % args.gpus, file=sys.stderr)
         sys.exit(2)
 
-    if args.workload in ("mixer", "taredra", "fedirax"):
+    if args.workload in ("mixer", "taredra", "fedirax", "marosun"):
         mixer_workload(args)
         return
 

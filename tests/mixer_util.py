@@ -46,6 +46,16 @@ class Case:
         self.m.close()
 
 
+def f32_edit(change):
+    """An edit of a model's tensors as floats."""
+    def edit(bits):
+        f = {k: O.bf16_to_f32(v).copy() for k, v in bits.items()}
+        change(f)
+        for k, v in f.items():
+            bits[k] = O.f32_to_bf16(v)
+    return edit
+
+
 def run_cut(case, tokens, cuts):
     """All logits of one request whose tokens come in portions of the given sizes (the last repeats)."""
     s, out, at, i = case.m.session(), [], 0, 0

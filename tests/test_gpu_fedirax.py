@@ -5,7 +5,7 @@ import numpy as np
 import pytest
 
 from tests import mixer_oracle as O
-from tests.mixer_util import Case, run_cut
+from tests.mixer_util import Case, f32_edit, run_cut
 from wayruntime_amd import engine as E, hipattn, mix_writer as mw
 
 pytestmark = pytest.mark.gpu
@@ -24,16 +24,6 @@ def eng():
 @pytest.fixture(params=["f32", "bf16"])
 def prec(request):
     return request.param
-
-
-def f32_edit(change):
-    """An edit of a model's tensors as floats."""
-    def edit(bits):
-        f = {k: O.bf16_to_f32(v).copy() for k, v in bits.items()}
-        change(f)
-        for k, v in f.items():
-            bits[k] = O.f32_to_bf16(v)
-    return edit
 
 
 WIDTH, VOCAB = 104, 211            # neither a multiple of 16

@@ -20,7 +20,7 @@ class Gemm(C.Structure):
                 ("tile_groups", u32), ("out", u32), ("y_f32", vp), ("y_act", vp), ("ldy", u32), ("h", vp), ("h_kt", u32),
                 ("col_z", u32), ("n_split", u32), ("silu_end", u32), ("sigmoid_end", u32), ("relu2", u32), ("scale", C.c_float),
                 ("tanh_end", u32), ("gelu", u32), ("x_kt0", u32), ("bias", vp), ("limit", C.c_float), ("slope", C.c_float),
-                ("up_bias", C.c_float), ("x_perm", vp)]
+                ("up_bias", C.c_float), ("x_perm", vp), ("h_kt0", u32), ("x_scale", vp)]
 
 
 @pytest.fixture(scope="module")
@@ -157,8 +157,19 @@ def test_frag_split_and_gated_out(lib, f32, N, K, rows):
         u = want[:, split:].reshape(rows, -1, 2, 16)
         got = r.frag_down(h, rows, ((N - split) // 64 + 1) * 32)[:, :(N - split) // 2]
         r.close(got, clamped(u[:, :, 0], u[:, :, 1], 0.6, 2.0, 1.0).reshape(rows, -1), eight_bits=True)
+    # those rows with a bias and an activation, the gated outputs behind three input tiles of a wider operand
+    split, silu, tiles = N // 2 // 32 * 32, 27, (N - N // 2 // 32 * 32) // 64 + 4
+    bias = np.pad(r.rng.standard_normal(split).astype(np.float32), (0, N - split), constant_values=np.nan)
+    bd, wide = hipattn.DeviceBuffer.from_host(bias), hipattn.DeviceBuffer.from_host(np.full((-(-rows // 16) * 16, tiles * 32), 3.0, np.float32))
+    r.go(xd, out=SPLIT_GATED, h=wide.p, h_kt=tiles, h_kt0=3, n_split=split, y_f32=y.p, ldy=split, bias=bd.p, silu_end=silu)
+    v = want[:, :split] + bias[:split]
+    r.close(y.to_host((rows, split)), np.concatenate([O.silu(v[:, :silu]), v[:, silu:]], axis=1))
+    got, u = r.frag_down(wide, rows, tiles * 32), want[:, split:].reshape(rows, -1, 2, 16)
+    r.close(got[:, 96:96 + (N - split) // 2], (O.silu(u[:, :, 0]) * u[:, :, 1]).reshape(rows, -1), eight_bits=True)
+    blank = 3.0 if f32 else O.bf16_to_f32(np.full(2, 3.0, np.float32).view(np.uint16)[1::2])[0]
+    assert set(np.unique(got[:, :96])) <= {blank, np.float32(0)}
     r.end()
-    for b in (y, xd, h):
+    for b in (y, xd, h, bd, wide):
         b.free()
 
 
@@ -200,6 +211,16 @@ def test_matrix_per_row_group(lib, f32, N, K, tile):
         if e >= 0:
             want[16 * g:16 * g + 16] = x[16 * g:16 * g + 16].astype(np.float64) @ r.w[e].T.astype(np.float64)
     r.close(y.to_host((rows, N)), want)
+    # a factor per row, ahead of the gated units
+    factor = r.rng.uniform(0, 2, rows).astype(np.float32)
+    fd, h = hipattn.DeviceBuffer.from_host(factor), hipattn.DeviceBuffer(rows * (N // 32 * 16 + 32) * 4)
+    if N % 64 == 0:
+        r.go(xd, rows=rows, group_expert=gd.p, tile_groups=tile, out=GATED, h=h.p, h_kt=N // 64, x_scale=fd.p)
+        t = (np.where(np.repeat(which, 16)[:, None] >= 0, want, 0) * factor[:, None]).reshape(rows, N // 32, 2, 16)
+        live = np.repeat(which, 16) >= 0
+        r.close(r.frag_down(h, rows, N // 2)[live], (O.silu(t[:, :, 0]) * t[:, :, 1]).reshape(rows, -1)[live], eight_bits=True)
+    for b in (fd, h):
+        b.free()
     if tile == 1:                                          # rows picked one by one out of fewer
         pick = r.rng.integers(0, 21, rows).astype(np.uint32)
         used = r.rng.random(rows) < 0.8
@@ -225,7 +246,8 @@ def test_refusals(lib):
     ok = dict(w=r.h, x=y.p, x_kt=1, rows=16, out=ROWS_F32, y_f32=y.p, ldy=32)
     for change in (dict(x_kt=0), dict(ldy=28), dict(ldy=33), dict(y_f32=None), dict(out=9), dict(rows=0), dict(w=None),
                    dict(out=FRAG, h=y.p, h_kt=0), dict(out=SPLIT, h=y.p, h_kt=1, n_split=8), dict(out=GATED), dict(x_kt0=1),
-                   dict(out=GATED, h=y.p, h_kt=1, bias=y.p), dict(x_perm=y.p), dict(out=SPLIT_GATED, h=y.p, h_kt=1, n_split=16)):
+                   dict(out=GATED, h=y.p, h_kt=1, bias=y.p), dict(x_perm=y.p), dict(x_scale=y.p),
+                   dict(out=GATED, h=y.p, h_kt=1, h_kt0=1), dict(out=SPLIT_GATED, h=y.p, h_kt=1, n_split=16)):
         assert lib.wr_hip_mix_gemm_run(0, C.byref(Gemm(**dict(ok, **change)))) == hipattn.ERR_INVAL, change
     h = vp()
     for shape in ((1, 8, 32), (1, 16, 16), (0, 16, 32)):

@@ -1,8 +1,8 @@
 """The C11 host engine under AddressSanitizer and UndefinedBehaviorSanitizer, on
 the CPU test double: every host source is compiled with the sanitizers together
 with tests/host_sanitize.c and the oracle-backed stand-in for the device
-library, and the exerciser runs over six toy models (two Qwen3 shapes, a Gemma
-one and three mixer stacks).  A heap error, an undefined operation or a leaked allocation in the
+library, and the exerciser runs over seven toy models (two Qwen3 shapes, a Gemma
+one and four mixer stacks).  A heap error, an undefined operation or a leaked allocation in the
 host code fails the run."""
 import glob
 import os
@@ -47,9 +47,13 @@ def test_host_engine_is_sanitizer_clean(tmp_path):
     cfg = mw.shared_kv_config(24, 40, [(mw.difference(4, 2, 6, 10, 90), mw.grouped_moe(3, 2, 8, identity=1, groups=(2, 1), shared=(12, 1.0))),
                                        (mw.keys_as_values(2, 1, 8, 90), None), (mw.difference(2, 2, 6, 10, 20, kv_from=0), None)])
     args += [mw.write_model(str(tmp_path / "shared_kv"), cfg), "40"]
+    cfg = mw.joint_config(24, 40, [(mw.turned_values(4, 2, 6, 10, rot_dims=4), mw.clamped_dense(12, 1.0)),
+                                   (mw.chunks_and_forget(2, 1, 8, 6, 50, 2, 5, 7), mw.moe(3, 2, 8)),
+                                   (mw.one_more_and_gru(2, 2, 6, 8, 13), None)])
+    args += [mw.write_model(str(tmp_path / "joint"), cfg), "40"]
     env = dict(os.environ, ASAN_OPTIONS="detect_leaks=1:verify_asan_link_order=0", OMP_NUM_THREADS="4")
     run = subprocess.run([exe] + args, capture_output=True, text=True, env=env, timeout=600)
     out = run.stdout + run.stderr
     assert run.returncode == 0, out[-3000:]
-    assert out.count(" ok acc=") == 6
+    assert out.count(" ok acc=") == 7
     assert "AddressSanitizer" not in out and ": runtime error:" not in out, out[-3000:]

@@ -2,14 +2,17 @@
 real sizes) beside a grouped-query model of the same width, through the host
 engine.
 
-    python -m wayruntime_amd.mix_timing [--size w2048 w4096] [--only mixer taredra fedirax gqa] [--json]
+    python -m wayruntime_amd.mix_timing [--size w2048 w4096] [--only mixer taredra fedirax marosun gqa] [--json]
 
 Each size has four layers.  mixer: linear attention with a dense feed-forward and
 with experts, latent attention with experts and with a dense feed-forward.
 taredra: windowed grouped-query attention beside a delta-rule recurrence, and a
 wkv recurrence, each twice, all with dense feed-forwards.  fedirax: differential
 attention, keys-as-values attention, differential attention and such over the first
-layer's keys and values, all with experts and a shared one.  gqa: the engine's
+layer's keys and values, all with experts and a shared one.  marosun: attention over
+turned values, attention beside an element-wise gated recurrence (both with dense
+feed-forwards), chunked attention beside a forget-gate recurrence, attention over turned
+values (both with experts).  gqa: the engine's
 Llama-style model with four layers of the same width, head dimension and
 feed-forward width (F16 weights)."""
 from __future__ import annotations
@@ -51,14 +54,23 @@ def fedirax_config(width: int, heads: int, experts: int, top: int, expert_ff: in
                                                                  mw.difference(**diff, kv_from=0))])
 
 
-KINDS = ("mixer", "taredra", "fedirax", "gqa")
+def marosun_config(width: int, heads: int, ff: int, experts: int, top: int, expert_ff: int) -> dict:
+    """Heads of 128 over eight key/value heads; recurrences with heads of 128 x 128, and of the model's width."""
+    a = dict(heads=heads, kv_heads=8, dim=128, vdim=128)
+    turned, d, m = mw.turned_values(**a, rot_dims=64), mw.clamped_dense(ff), mw.moe(experts, top, expert_ff)
+    return mw.joint_config(width, VOCAB, [
+        (turned, d), (mw.one_more_and_gru(**a, size=width), d),
+        (mw.chunks_and_forget(**a, chunk=4096, right_heads=width // 128, right_dim=128, right_vdim=128), m), (turned, m)])
+
+
+KINDS = ("mixer", "taredra", "fedirax", "marosun", "gqa")
 RANK = 64                                   # of the decays' low-rank products
 SIZES = {
     "w2048": (mixer_config(2048, 16, 768, 8192, 64, 6, 1024), taredra_config(2048, 16, 8192),
-              fedirax_config(2048, 16, 64, 6, 1024, 2048),
+              fedirax_config(2048, 16, 64, 6, 1024, 2048), marosun_config(2048, 16, 8192, 64, 6, 1024),
               gw.ModelShape(arch="llama", n_layers=4, hidden=2048, ffn=8192, n_q=16, n_kv=8, vocab=VOCAB, context=8192)),
     "w4096": (mixer_config(4096, 32, 1536, 12288, 32, 4, 2048), taredra_config(4096, 32, 12288),
-              fedirax_config(4096, 32, 32, 4, 2048, 4096),
+              fedirax_config(4096, 32, 32, 4, 2048, 4096), marosun_config(4096, 32, 12288, 32, 4, 2048),
               gw.ModelShape(arch="llama", n_layers=4, hidden=4096, ffn=12288, n_q=32, n_kv=8, vocab=VOCAB, context=8192)),
 }
 

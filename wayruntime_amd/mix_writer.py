@@ -1,6 +1,6 @@
-"""Writes mixer-stack models (architectures "Bipotar", "Taredra" and "Fedirax") as a folder with
-config.json and model.safetensors: random-init models for the tests and the benchmark, and any
-set of bfloat16 tensors a caller has."""
+"""Writes mixer-stack models (architectures "Bipotar", "Taredra", "Fedirax" and "Marosun") as a
+folder with config.json and model.safetensors: random-init models for the tests and the benchmark,
+and any set of bfloat16 tensors a caller has."""
 from __future__ import annotations
 
 import json
@@ -54,6 +54,40 @@ def difference(heads: int, kv_heads: int, dim: int, vdim: int, window: int, rot_
     return {"type": "attention_2", "mixer": m if kv_from is None else dict(m, kv_from=kv_from)}
 
 
+def _heads(heads: int, kv_heads: int, dim: int, vdim: int, scale: float | None) -> dict:
+    return {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": dim ** -0.5 if scale is None else scale}
+
+
+def turned_values(heads: int, kv_heads: int, dim: int, vdim: int, rot_dims: int | None = None, base: float = 10000.0,
+                  scale: float | None = None, scaling=(4.0, 4096, 32.0, 1.0)) -> dict:
+    """Causal attention with normed queries and keys whose values turn with their positions; scaling: (factor, original
+    length, fast, slow) of the rotation's far pairs, or None."""
+    rot = {"base": base, "dims": dim if rot_dims is None else rot_dims}
+    if scaling is not None:
+        rot["scaling"] = dict(zip(("factor", "original", "fast", "slow"), scaling))
+    return {"type": "attention", "mixer": dict(_heads(heads, kv_heads, dim, vdim, scale), rot=rot)}
+
+
+def chunks_and_forget(heads: int, kv_heads: int, dim: int, vdim: int, chunk: int, right_heads: int, right_dim: int,
+                      right_vdim: int, scale: float | None = None, left_scale: float = 1.0, right_scale: float = 1.0) -> dict:
+    """Attention inside chunks of positions and a recurrence whose forget gate makes the keys, side by side."""
+    return {"type": "parallel", "mixer": {"left": dict(_heads(heads, kv_heads, dim, vdim, scale), mask={"size": chunk}),
+                                          "right": {"heads": right_heads, "dim": right_dim, "vdim": right_vdim},
+                                          "left_scale": left_scale, "right_scale": right_scale}}
+
+
+def one_more_and_gru(heads: int, kv_heads: int, dim: int, vdim: int, size: int, rot_dims: int | None = None,
+                     base: float = 10000.0, scale: float | None = None) -> dict:
+    """Causal attention with one added to the softmax's denominator and a gated recurrence of `size` elements, averaged."""
+    rot = {"base": base, "dims": dim if rot_dims is None else rot_dims}
+    return {"type": "parallel_2", "mixer": {"left": dict(_heads(heads, kv_heads, dim, vdim, scale), rot=rot),
+                                            "right": {"width": size}}}
+
+
+def clamped_dense(ff: int, limit: float = 7.0) -> dict:
+    return {"kind": "dense", "ff": ff, "limit": limit}
+
+
 def dense(ff: int) -> dict:
     return {"kind": "dense", "ff": ff}
 
@@ -88,6 +122,55 @@ def prenorm_config(width: int, vocab: int, layers, eps: float = 1e-6, embed_scal
 def shared_kv_config(width: int, vocab: int, layers, eps: float = 1e-6, embed_scale: float = 1.0) -> dict:
     """layers: [(mixer, feed-forward or None)] of keys_as_values and difference mixers."""
     return dict(prenorm_config(width, vocab, layers, eps, embed_scale), architecture="Fedirax")
+
+
+def joint_config(width: int, vocab: int, layers, eps: float = 1e-6) -> dict:
+    """layers: [(mixer, feed-forward or None)] of turned_values, chunks_and_forget and one_more_and_gru mixers with
+    clamped_dense or moe feed-forwards; both read one norm."""
+    return {"architecture": "Marosun", "width": width, "vocab": vocab, "norm": {"eps": eps},
+            "layers": [dict(m, mlp=f) for m, f in layers]}
+
+
+def _joint_shapes(cfg: dict) -> dict:
+    W, out = cfg["width"], {"embed": (cfg["vocab"], cfg["width"])}
+
+    def heads(p, m, biases):
+        H, G, D, V = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        for n, rows, cols in (("q", H * D, W), ("k", G * D, W), ("v", G * V, W), ("o", W, H * V)):
+            out[p + n] = (rows, cols)
+            if biases:
+                out[p + n + ".b"] = (rows,)
+        if biases:
+            out.update({p + "q.norm": (D,), p + "k.norm": (D,)})
+    for i, layer in enumerate(cfg["layers"]):
+        p, m, f = f"l{i}.", layer["mixer"], layer["mlp"]
+        out[p + "norm1"] = (W,)
+        q = p + "mix."
+        if layer["type"] == "attention":
+            heads(q, m, True)
+            out[q + "sink"] = (m["heads"],)
+        elif layer["type"] == "parallel":
+            a, r = m["left"], m["right"]
+            heads(q + "left.", a, False)
+            out.update({q + "left.sink": (a["heads"],), q + "left.g": (a["heads"] * a["vdim"], W)})
+            hd, hv = r["heads"] * r["dim"], r["heads"] * r["vdim"]
+            out.update({q + "right.q": (hd, W), q + "right.v": (hv, W), q + "right.f": (hd, W), q + "right.f.b": (hd,),
+                        q + "right.lower": (hd,), q + "right.norm": (r["vdim"],), q + "right.o": (W, hv)})
+        else:
+            heads(q + "left.", m["left"], True)
+            n = m["right"]["width"]
+            out.update({q + "right.z": (n, W), q + "right.z.b": (n,), q + "right.x": (n, W), q + "right.x.b": (n,),
+                        q + "right.g": (n, W), q + "right.o": (W, n), q + "left.out": (W,), q + "right.out": (W,)})
+        if f and f["kind"] == "dense":
+            out.update({p + "mlp.gate": (f["ff"], W), p + "mlp.up": (f["ff"], W), p + "mlp.down": (W, f["ff"])})
+        elif f:
+            out[p + "mlp.router"] = (f["router"]["experts"], W)
+            for e in range(f["router"]["experts"]):
+                e, ff = p + f"mlp.e{e}.", f["expert"]["ff"]
+                out.update({e + "gate": (ff, W), e + "up": (ff, W), e + "down": (W, ff)})
+    out["final.norm"] = (W,)
+    out["head"] = (cfg["vocab"], W)
+    return out
 
 
 def _shared_kv_shapes(cfg: dict) -> dict:
@@ -158,6 +241,8 @@ def tensor_shapes(cfg: dict, rank: int = 24) -> dict:
         return _prenorm_shapes(cfg, rank)
     if cfg["architecture"] == "Fedirax":
         return _shared_kv_shapes(cfg)
+    if cfg["architecture"] == "Marosun":
+        return _joint_shapes(cfg)
     W, out = cfg["width"], {"embed": (cfg["vocab"], cfg["width"]), "embed.norm": (cfg["width"],)}
     for i, layer in enumerate(cfg["layers"]):
         p, m, f = f"l{i}.", layer["mixer"], layer["mlp"]
@@ -193,12 +278,12 @@ def to_bf16(x: np.ndarray) -> np.ndarray:
 # what the vectors of a pre-norm model are drawn around, and how widely
 _VECTORS = {"norm1": (0, 0.1), "norm2": (0, 0.1), "final.norm": (0, 0.1), "sink": (0, 1), "w0": (-3, 2), "a.b": (0, 1),
             "q.b": (0, 0.5), "k.b": (0, 0.5), "correction": (0, 0.05), "lq1": (0, 0.1), "lk1": (0, 0.1), "lq2": (0, 0.1),
-            "lk2": (0, 0.1)}
+            "lk2": (0, 0.1), "v.b": (0, 0.5), "o.b": (0, 0.2), "f.b": (1, 1), "z.b": (-1, 1), "x.b": (0, 0.5)}
 
 
 def random_tensors(cfg: dict, seed: int = 0, gain: float = 1.0, rank: int = 24):
     """Yields (name, bfloat16 bits): norms 1 + 0.1 N(0, 1), matrices gain * N(0, 1 / inputs), the embedding N(0, 1);
-    of a pre-norm model the vectors as _VECTORS says, mixing factors in [0, 1], bonuses N(0, 1/4), the embedding N(0, 1 / width).
+    of a pre-norm model the vectors as _VECTORS says, mixing factors and lower bounds in [0, 1], bonuses N(0, 1/4), the embedding N(0, 1 / width).
     Large matrices repeat a pool of samples at different offsets."""
     prenorm = cfg["architecture"] != "Bipotar"
     rng = np.random.default_rng(seed)
@@ -209,7 +294,7 @@ def random_tensors(cfg: dict, seed: int = 0, gain: float = 1.0, rank: int = 24):
         x = pool[(at + np.arange(n)) % pool.size] if n <= pool.size else np.resize(np.roll(pool, at), n)
         end = name.split(".", 2)[-1] if name.startswith("l") else name
         end = end.removeprefix("left.").removeprefix("right.")
-        if prenorm and ".mu." in name:
+        if prenorm and (".mu." in name or end == "lower"):
             x = 1.0 / (1.0 + np.exp(-x))
         elif prenorm and end == "u":
             x = 0.5 * x
