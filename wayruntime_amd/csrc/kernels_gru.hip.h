@@ -4,9 +4,9 @@
 //   out = S_t * SiLU(g_t)
 //
 // zl, u and g are 32-bit rows of the layer's input product.  A token is the map S -> A S + B, so
-// tokens can be put together in any grouping: a workgroup has 32 channels of a request, a wave
-// sixteen rows of them (lane 16g + c: row c, channels 8g .. +7, which is the next product's
-// operand), scans its rows across lanes, and the waves' totals are put together in LDS.  Decoded
+// tokens can be put together in any grouping: a workgroup has sixteen channels of a request, a
+// wave sixteen rows of them (lane 16g + c: row c, channels 4g .. +3), scans its rows across lanes,
+// and the waves' totals are put together in LDS while the next rows are on their way.  Decoded
 // tokens and short portions take one wave.
 #pragma once
 
@@ -34,10 +34,10 @@ __device__ __forceinline__ float gru_up(float v, float none)
 }
 
 template <int BY>
-__device__ __forceinline__ void gru_join(float (&A)[8], float (&B)[8])
+__device__ __forceinline__ void gru_join(f32x4& A, f32x4& B)
 {
 #pragma unroll
-    for (int j = 0; j < 8; j++) {
+    for (int j = 0; j < 4; j++) {
         const float a = gru_up<BY>(A[j], 1.0f), b = gru_up<BY>(B[j], 0.f);
         B[j] = fmaf(A[j], b, B[j]);
         A[j] *= a;
@@ -60,29 +60,34 @@ __device__ __forceinline__ void gru_logistic(float z, float& s, float& t)
     t = z < 0.f ? over : e * over;
 }
 
-// grid (channels / 32, requests), NW waves
+// What this wave did in LDS is done, and everybody's: loads from memory stay on their way.
+__device__ __forceinline__ void gru_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+
+// grid (channels / 16, requests), NW waves
 template <bool F32, int NW>
 __global__ __launch_bounds__(64 * NW) void gru_scan_kernel(const GruArgs a)
 {
-    __shared__ float tot[NW][2][32], start[NW][32];
+    __shared__ __attribute__((aligned(16))) float tot[NW][2][16], start[NW][16];
     const MixSeq s = a.seqs[a.list[blockIdx.y]];
     const uint32_t lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4, wave = threadIdx.x >> 6;
-    const uint32_t ch = blockIdx.x * 32 + 8 * g;
-    float carry = 0.f;                                     // wave 0, lanes below 32: the state of a channel each
-    if (threadIdx.x < 32 && s.pos0 > 0) carry = a.state[(size_t)s.state_in * a.wpad + blockIdx.x * 32 + lane];
-    float z[8], u[8], q[8];
+    // the two halves of a row's 128 bytes go to workgroups of one XCD
+    const uint32_t b = blockIdx.x, slab = gridDim.x % 16 == 0 ? (b / 16 * 8 + b % 8) * 2 + b / 8 % 2 : b;
+    const uint32_t ch = slab * 16 + 4 * g;
+    float carry = 0.f;                                     // wave 0, lanes below 16: the state of a channel each
+    if (threadIdx.x < 16 && s.pos0 > 0) carry = a.state[(size_t)s.state_in * a.wpad + slab * 16 + lane];
+    f32x4 z, u, q;
     auto load = [&](uint32_t row) {                        // (rows past the request's repeat its last one)
         const float* p = a.in + (size_t)(s.row0 + min(row, s.rows - 1)) * a.ld + ch;
-        mix_load8(p + a.col_z, z);
-        mix_load8(p + a.col_x, u);
-        mix_load8(p + a.col_g, q);
+        z = *reinterpret_cast<const f32x4*>(p + a.col_z);
+        u = *reinterpret_cast<const f32x4*>(p + a.col_x);
+        q = *reinterpret_cast<const f32x4*>(p + a.col_g);
     };
     load(wave * 16 + c);
     for (uint32_t row0 = 0; row0 < s.rows; row0 += 16 * NW) {
         const uint32_t row = row0 + wave * 16 + c;
-        float A[8], B[8], o[8];
+        f32x4 A, B, o;
 #pragma unroll
-        for (int j = 0; j < 8; j++) {
+        for (int j = 0; j < 4; j++) {
             float zs, zt, us, ut, qs, qt;
             gru_logistic<F32>(z[j], zs, zt);
             gru_logistic<F32>(u[j], us, ut);
@@ -97,25 +102,28 @@ __global__ __launch_bounds__(64 * NW) void gru_scan_kernel(const GruArgs a)
         gru_join<4>(A, B);
         gru_join<8>(A, B);
         if (c == 15) {
-            mix_store8(&tot[wave][0][8 * g], A);
-            mix_store8(&tot[wave][1][8 * g], B);
+            *reinterpret_cast<f32x4*>(&tot[wave][0][4 * g]) = A;
+            *reinterpret_cast<f32x4*>(&tot[wave][1][4 * g]) = B;
         }
-        __syncthreads();
-        if (threadIdx.x < 32) {
+        gru_barrier();
+        if (threadIdx.x < 16) {
 #pragma unroll
             for (int w = 0; w < NW; w++) {
                 start[w][lane] = carry;
                 carry = fmaf(tot[w][0][lane], carry, tot[w][1][lane]);
             }
         }
-        __syncthreads();                                   // (tot is written again behind it, start behind the next one)
-        float S[8];
-        mix_load8(&start[wave][8 * g], S);
+        gru_barrier();                                     // (tot is written again behind it, start behind the next one)
+        const f32x4 S = *reinterpret_cast<const f32x4*>(&start[wave][4 * g]);
+        if (row < s.rows) {
+            typename MixAct<F32>::V4 out;
 #pragma unroll
-        for (int j = 0; j < 8; j++) o[j] *= fmaf(A[j], S[j], B[j]);
-        if (row < s.rows) mix_store_unit<F32>(a.h, frag_unit(s.row0 + row, (a.col_h + ch) / 8, a.h_kt), o);
+            for (int j = 0; j < 4; j++) out[j] = (typename MixAct<F32>::E)(o[j] * fmaf(A[j], S[j], B[j]));
+            *reinterpret_cast<typename MixAct<F32>::V4*>(reinterpret_cast<typename MixAct<F32>::E*>(a.h) +
+                                                         frag_elem(s.row0 + row, a.col_h + ch, a.h_kt)) = out;
+        }
     }
-    if (threadIdx.x < 32) a.state[(size_t)s.state_out * a.wpad + blockIdx.x * 32 + lane] = carry;
+    if (threadIdx.x < 16) a.state[(size_t)s.state_out * a.wpad + slab * 16 + lane] = carry;
 }
 
 }  // namespace wr

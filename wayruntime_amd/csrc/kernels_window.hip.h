@@ -124,6 +124,50 @@ __device__ __forceinline__ float window_inv_rms(const WindowArgs& a, const float
     return 1.0f / sqrtf(ss / (float)a.dim + a.eps);
 }
 
+// Whether units of eight lie whole inside a vector and inside or outside its rotated part, so that they go in as vectors.
+__device__ __forceinline__ bool window_whole(const WindowArgs& a, uint32_t col)
+{
+    return a.neighbours && a.dim % 8 == 0 && a.half % 4 == 0 && a.ld % 4 == 0 && col % 4 == 0 && (a.dimp == 32 || a.dimp == 64 || a.dimp == 128);
+}
+
+// Unit i0 .. i0 + 7 of the vector x, normed and rotated (neighbours): the other units of x are held by every fourth lane.
+__device__ __forceinline__ void window_unit(const WindowArgs& a, const float* x, const float* norm, const float* tab, uint32_t i0,
+                                            float (&v)[8])
+{
+    const bool some = i0 < a.dim;
+    if (some) {
+        mix_load8(x + i0, v);
+    } else {
+#pragma unroll
+        for (int j = 0; j < 8; j++) v[j] = 0.f;
+    }
+    if (norm) {                                            // uniform
+        float ss = 0.f, w[8];
+#pragma unroll
+        for (int j = 0; j < 8; j++) ss = fmaf(v[j], v[j], ss);
+        ss += wave_xor_f32(ss, 4);
+        ss += wave_xor_f32(ss, 8);
+        if (a.dimp >= 64) ss += wave_xor_f32(ss, 16);
+        if (a.dimp >= 128) ss += wave_xor_f32(ss, 32);
+        const float inv = 1.0f / sqrtf(ss / (float)a.dim + a.eps);
+        if (some) {
+            mix_load8(norm + i0, w);
+#pragma unroll
+            for (int j = 0; j < 8; j++) v[j] *= inv * w[j];
+        }
+    }
+    if (i0 < 2 * a.half) {
+        float cs[8];
+        mix_load8(tab + i0, cs);
+#pragma unroll
+        for (int j = 0; j < 8; j += 2) {
+            const float e = v[j], o = v[j + 1];
+            v[j] = e * cs[j] - o * cs[j + 1];
+            v[j + 1] = o * cs[j] + e * cs[j + 1];
+        }
+    }
+}
+
 // Element d of row r's value, turned where values are.
 __device__ __forceinline__ float window_value(const WindowArgs& a, uint32_t r, uint32_t kvh, uint32_t d)
 {
@@ -141,14 +185,20 @@ __global__ __launch_bounds__(256) void window_append_kernel(const WindowArgs a)
     using V4 = typename MixAct<F32>::V4;
     __shared__ float s_inv[4];
     const uint32_t t = threadIdx.x, r0 = blockIdx.x * 4, n = min(4u, a.rows - r0), per_map = a.dimp / 8;
+    const bool whole = window_whole(a, blockIdx.y >= a.key_heads ? a.col_q : a.col_k);       // uniform
     if (blockIdx.y >= a.key_heads) {
         const uint32_t per = a.heads * a.maps * per_map, u0 = (blockIdx.y - a.key_heads) * kWindowQUnits;
         for (uint32_t u = u0 + t; u < min(u0 + kWindowQUnits, 4 * per); u += 256) {
             const uint32_t i = u % 4, q = u / 4, r = r0 + min(i, n - 1);
             const float* x = a.in + (size_t)r * a.ld + a.col_q + q / per_map * a.dim;
+            float v[8];
+            if (whole) {
+                window_unit(a, x, a.q_norm, a.table + (size_t)r * 2 * a.half, q % per_map * 8, v);
+                if (i < n) mix_store_unit<F32>(a.q, frag_unit(r, q, a.heads * (a.dimk / 32)), v);
+                continue;
+            }
             const float inv = a.q_norm ? window_inv_rms(a, x, q % per_map * 8) : 1.0f;
             if (i >= n) continue;
-            float v[8];
             window_turn8(a, x, a.q_norm, inv, a.table + (size_t)r * 2 * a.half, q % per_map * 8, v);
             mix_store_unit<F32>(a.q, frag_unit(r, q, a.heads * (a.dimk / 32)), v);
         }
@@ -162,9 +212,14 @@ __global__ __launch_bounds__(256) void window_append_kernel(const WindowArgs a)
     for (uint32_t u = t; u < 4 * a.maps * per_map; u += 256) {
         const uint32_t i = u % 4, q = u / 4, r = r0 + min(i, n - 1);
         const float* x = a.in + (size_t)r * a.ld + a.col_k + (kvh * a.maps + q / per_map) * a.dim;
+        float v[8];
+        if (whole) {
+            window_unit(a, x, a.k_norm, a.table + (size_t)r * 2 * a.half, q % per_map * 8, v);
+            if (i < n) mix_store_unit<F32>(head_block(r), frag_unit(a.row_pos[r] % kMixPage, q, a.dimk / 32), v);
+            continue;
+        }
         const float inv = a.k_norm ? window_inv_rms(a, x, q % per_map * 8) : 1.0f;
         if (i >= n) continue;
-        float v[8];
         window_turn8(a, x, a.k_norm, inv, a.table + (size_t)r * 2 * a.half, q % per_map * 8, v);
         mix_store_unit<F32>(head_block(r), frag_unit(a.row_pos[r] % kMixPage, q, a.dimk / 32), v);
     }

@@ -843,7 +843,7 @@ int wr_hip_mix_min_gru(wr_hip_mix_step* s, wr_hip_mix_pool* pool, uint32_t run, 
     GruArgs a = {s->d<MixSeq>(s->o_seqs), s->d<uint32_t>(s->o_long), wp, q->in, q->ld, q->col_z, q->col_x, q->col_g,
                  pool->state[run], q->h, q->h_kt, q->col_h};
     if (s->n_long) {
-        const dim3 grid(wp / 32, s->n_long);
+        const dim3 grid(wp / 16, s->n_long);
         const bool many = *std::max_element(s->long_rows, s->long_rows + s->n_long) > 64;
         if (many && f32) MIX_LAUNCH((gru_scan_kernel<true, 16>), grid, dim3(1024), 0, a);
         else if (many) MIX_LAUNCH((gru_scan_kernel<false, 16>), grid, dim3(1024), 0, a);
@@ -852,7 +852,7 @@ int wr_hip_mix_min_gru(wr_hip_mix_step* s, wr_hip_mix_pool* pool, uint32_t run, 
     }
     if (s->n_short) {
         a.list = s->d<uint32_t>(s->o_short);
-        const dim3 grid(wp / 32, s->n_short);
+        const dim3 grid(wp / 16, s->n_short);
         if (f32) MIX_LAUNCH((gru_scan_kernel<true, 1>), grid, dim3(64), 0, a);
         else MIX_LAUNCH((gru_scan_kernel<false, 1>), grid, dim3(64), 0, a);
     }
