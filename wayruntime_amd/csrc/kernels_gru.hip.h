@@ -75,28 +75,30 @@ __global__ __launch_bounds__(64 * NW) void gru_scan_kernel(const GruArgs a)
     const uint32_t ch = slab * 16 + 4 * g;
     float carry = 0.f;                                     // wave 0, lanes below 16: the state of a channel each
     if (threadIdx.x < 16 && s.pos0 > 0) carry = a.state[(size_t)s.state_in * a.wpad + slab * 16 + lane];
-    f32x4 z, u, q;
-    auto load = [&](uint32_t row) {                        // (rows past the request's repeat its last one)
-        const float* p = a.in + (size_t)(s.row0 + min(row, s.rows - 1)) * a.ld + ch;
-        z = *reinterpret_cast<const f32x4*>(p + a.col_z);
-        u = *reinterpret_cast<const f32x4*>(p + a.col_x);
-        q = *reinterpret_cast<const f32x4*>(p + a.col_g);
+    struct Rows {
+        f32x4 z, u, q;
     };
-    load(wave * 16 + c);
-    for (uint32_t row0 = 0; row0 < s.rows; row0 += 16 * NW) {
+    auto load = [&](Rows& x, uint32_t row) {               // (rows past the request's repeat its last one)
+        const float* p = a.in + (size_t)(s.row0 + min(row, s.rows - 1)) * a.ld + ch;
+        x.z = *reinterpret_cast<const f32x4*>(p + a.col_z);
+        x.u = *reinterpret_cast<const f32x4*>(p + a.col_x);
+        x.q = *reinterpret_cast<const f32x4*>(p + a.col_g);
+    };
+    // sixteen rows a wave from row0 on; x is theirs, and then those of the turn after the next
+    auto turn = [&](Rows& x, uint32_t row0) {
         const uint32_t row = row0 + wave * 16 + c;
         f32x4 A, B, o;
 #pragma unroll
         for (int j = 0; j < 4; j++) {
             float zs, zt, us, ut, qs, qt;
-            gru_logistic<F32>(z[j], zs, zt);
-            gru_logistic<F32>(u[j], us, ut);
-            gru_logistic<F32>(q[j], qs, qt);
+            gru_logistic<F32>(x.z[j], zs, zt);
+            gru_logistic<F32>(x.u[j], us, ut);
+            gru_logistic<F32>(x.q[j], qs, qt);
             A[j] = row < s.rows ? zt : 1.0f;
-            B[j] = row < s.rows ? zs * (u[j] >= 0.f ? u[j] + 0.5f : us) : 0.f;
-            o[j] = q[j] * qs;
+            B[j] = row < s.rows ? zs * (x.u[j] >= 0.f ? x.u[j] + 0.5f : us) : 0.f;
+            o[j] = x.q[j] * qs;
         }
-        if (row0 + 16 * NW < s.rows) load(row + 16 * NW);  // uniform
+        load(x, row + 32 * NW);
         gru_join<1>(A, B);
         gru_join<2>(A, B);
         gru_join<4>(A, B);
@@ -122,6 +124,13 @@ __global__ __launch_bounds__(64 * NW) void gru_scan_kernel(const GruArgs a)
             *reinterpret_cast<typename MixAct<F32>::V4*>(reinterpret_cast<typename MixAct<F32>::E*>(a.h) +
                                                          frag_elem(s.row0 + row, a.col_h + ch, a.h_kt)) = out;
         }
+    };
+    Rows even, odd;
+    load(even, wave * 16 + c);
+    load(odd, 16 * NW + wave * 16 + c);
+    for (uint32_t row0 = 0; row0 < s.rows; row0 += 32 * NW) {      // uniform
+        turn(even, row0);
+        if (row0 + 16 * NW < s.rows) turn(odd, row0 + 16 * NW);
     }
     if (threadIdx.x < 16) a.state[(size_t)s.state_out * a.wpad + slab * 16 + lane] = carry;
 }

@@ -623,6 +623,7 @@ static operand stack_inputs(loader *l, uint32_t i, const in_part *parts, size_t 
         *parts[k].col = *ld;
         *ld += p32(parts[k].rows);
     }
+    if (*ld % 1024 == 0) *ld += 32;                        /* (rows a multiple of 4 KiB apart share too few channels) */
     operand o = operand_new(l, 1, *ld + more, l->mm->width_p);
     for (size_t k = 0; k < n; k++)
         operand_put(l, &o, 0, *parts[k].col, ltensor(l, i, parts[k].name, parts[k].rows, l->mm->width), parts[k].rows, l->mm->width);
