@@ -583,7 +583,7 @@ static wr_status walk_joint(wr_model *m, const wrh_mix_layer *L, uint32_t r, con
                           .y_f32 = t.in, .ldy = L->ld_in, .bias = L->b_in, .silu_end = L->silu_end};
     if (dense) {
         in.out = WR_HIP_MIX_OUT_SPLIT_GATED;
-        in.n_split = L->ld_in;
+        in.n_split = L->n_in;
         in.h = t.act;
         in.h_kt = t.act_kt;
         in.h_kt0 = t.act_kt0;

@@ -57,14 +57,14 @@ typedef struct wrh_mix_layer {
     /* window: one stacked product [q | k | v | gate] (values that are the keys take no part of it), w_o */
     uint8_t has_gate;                     /* a logistic gate per head, its logits at col_rg */
     int32_t kv_from;                      /* layer whose keys and values it reads, or -1 */
-    const float *b_in;                    /* ld_in biases, or NULL */
-    /* joint: mixers and feed-forward read one norm.  One stacked product of the mixers' inputs and, behind ld_in rows, a
+    const float *b_in;                    /* a bias for every output of w_in, or NULL */
+    /* joint: mixers and feed-forward read one norm.  One stacked product of the mixers' inputs and, behind n_in outputs, a
      * dense feed-forward's gate and up, or the router's logits among the rows; w_o takes out everything, or with
      * out_norm the attention alone (w_o2 what stands beside it, w_down the feed-forward), each mixer's output normed */
     wrh_beside_kind beside;
     int32_t turn;                         /* rotary table of the values, or -1 */
     uint32_t gru, gru_p;                  /* elements of the gated recurrence */
-    uint32_t col_router, silu_end;        /* rows below silu_end leave the product through SiLU */
+    uint32_t n_in, col_router, silu_end;        /* rows below silu_end leave the product through SiLU */
     wr_hip_mat *w_o2;
     const float *b_o, *out_norm[2];       /* (halved: the outputs are averaged) */
     /* feed-forward */

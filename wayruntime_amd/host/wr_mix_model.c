@@ -614,6 +614,9 @@ static int read_window_sizes(loader *l, uint32_t i, const wrh_json *c, wrh_mix_l
     return l->st == WR_OK;
 }
 
+/* How far apart the rows of n outputs are kept: rows a multiple of 4 KiB apart share too few memory channels. */
+static uint32_t row_stride(uint32_t n) { return n % 1024 ? n : n + 32; }
+
 /* One product of a layer's input out of several matrices: where each one's outputs lie, then the operand, with `more`
  * rows behind theirs. */
 static operand stack_inputs(loader *l, uint32_t i, const in_part *parts, size_t n, uint32_t *ld, uint32_t more)
@@ -623,7 +626,6 @@ static operand stack_inputs(loader *l, uint32_t i, const in_part *parts, size_t 
         *parts[k].col = *ld;
         *ld += p32(parts[k].rows);
     }
-    if (*ld % 1024 == 0) *ld += 32;                        /* (rows a multiple of 4 KiB apart share too few channels) */
     operand o = operand_new(l, 1, *ld + more, l->mm->width_p);
     for (size_t k = 0; k < n; k++)
         operand_put(l, &o, 0, *parts[k].col, ltensor(l, i, parts[k].name, parts[k].rows, l->mm->width), parts[k].rows, l->mm->width);
@@ -664,6 +666,7 @@ static void read_window_keys(loader *l, uint32_t i, const wrh_json *c, wrh_mix_l
     operand o = stack_inputs(l, i, parts, n, &L->ld_in, 0);
     L->w_in = operand_up(l, &o);
     L->b_in = stack_biases(l, i, parts, n, L->ld_in, 0);
+    L->ld_in = row_stride(L->ld_in);
     L->col_v = L->col_k;
     L->has_gate = 1;
     L->sink = vec_put(l, ltensor(l, i, "mix.sink", g->heads, 0), g->heads);
@@ -701,6 +704,7 @@ static void read_window_difference(loader *l, uint32_t i, const wrh_json *c, wrh
                              {"mix.v", g->kv_heads * g->vdim, &L->col_v, NULL}};
     operand o = stack_inputs(l, i, parts, L->kv_from >= 0 ? 1 : sizeof parts / sizeof *parts, &L->ld_in, 0);
     L->w_in = operand_up(l, &o);
+    L->ld_in = row_stride(L->ld_in);
     g->q_norm = vec_put(l, ltensor(l, i, "mix.q.norm", g->dim, 0), g->dim);
     if (L->kv_from < 0) g->k_norm = vec_put(l, ltensor(l, i, "mix.k.norm", g->dim, 0), g->dim);
     else L->col_k = L->col_v = WR_HIP_MIX_NO_KEYS;
@@ -967,15 +971,16 @@ static void finish_joint(loader *l, uint32_t i, wrh_mix_layer *L)
     if (l->st != WR_OK) return;
     int biased = 0;
     for (size_t k = 0; k < l->n_parts; k++) biased |= l->parts[k].bias != NULL;
-    operand o = stack_inputs(l, i, l->parts, l->n_parts, &L->ld_in, 2 * ff);
+    operand o = stack_inputs(l, i, l->parts, l->n_parts, &L->n_in, 2 * ff);
+    L->ld_in = row_stride(L->n_in);
     const uint16_t *wd = NULL;
     if (ff) {
         const uint16_t *gate = ltensor(l, i, "mlp.gate", L->ff, W), *up = ltensor(l, i, "mlp.up", L->ff, W);
-        put_gated(l, &o, 0, L->ld_in, gate, up, L->ff, W);
+        put_gated(l, &o, 0, L->n_in, gate, up, L->ff, W);
         wd = ltensor(l, i, "mlp.down", W, L->ff);
     }
     L->w_in = operand_up(l, &o);
-    if (biased) L->b_in = stack_biases(l, i, l->parts, l->n_parts, L->ld_in, 2 * ff);
+    if (biased) L->b_in = stack_biases(l, i, l->parts, l->n_parts, L->n_in, 2 * ff);
     const char *first = L->beside ? "mix.left.o" : "mix.o";
     const uint16_t *wo = ltensor(l, i, first, W, g->heads * g->vdim), *wo2 = NULL;
     const uint32_t n2 = L->beside == WRH_BESIDE_FORGET ? L->rec.heads * L->rec.vdim : L->gru;
