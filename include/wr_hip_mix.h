@@ -2,8 +2,9 @@
  * wr_hip_mix.h — C ABI of the device steps of mixer-stack models: models whose
  * layers pair a mixer (decayed linear attention, sliding-window attention through
  * a low-rank latent or over grouped keys and values, a matrix-state recurrence
- * with input-made decays, a gated recurrence element by element) with a feed-forward (dense or a mixture of experts),
- * with norms before and, in some designs, after each, and bfloat16 weights.
+ * with input-made decays, an element-wise gated recurrence) with a feed-forward (dense
+ * or a mixture of experts), with norms before and, in some designs, after each, or one
+ * norm for both, and bfloat16 weights.
  *
  * Conventions are those of wr_hip_attn.h: plain C, status returns, every call
  * enqueues on the calling thread's stream and returns without waiting unless it
@@ -103,8 +104,8 @@ int wr_hip_mix_embed(wr_hip_mix_step *s, int f32, const uint16_t *table_dev, uin
  *   x += add                         (when given)
  *   h = rmsnorm(x) * next            (when given; only the step's wanted rows, packed,
  *                                     with `wanted` set)
- * gate may be NULL: ones.  ident: frag rows of the width, may be h itself; shared: 32-bit rows like y; either may
- * be NULL. */
+ * gate may be NULL: ones.  ident: frag rows of the width, may be h itself; shared: 32-bit rows
+ * like y; either may be NULL. */
 typedef struct wr_hip_mix_resid {
     uint32_t width;
     float eps;
@@ -146,9 +147,11 @@ int wr_hip_mix_shift(wr_hip_mix_step *s, wr_hip_mix_pool *pool, uint32_t run, in
  *              with limit > 0: g = min(gate, limit), u = up within [-limit, limit],
  *              g * logistic(slope * g) * (u + up_bias))
  *   SPLIT_GATED n < n_split (a multiple of 32): y_f32[r][n]; the tiles behind as GATED
- * after a factor per row (x_scale, with group_expert), `bias` (a float for each of the n_out outputs, batch 1) and an activation: SiLU for n < silu_end, else the logistic for n <
- * sigmoid_end, else the hyperbolic tangent for n < tanh_end; square of ReLU
- * everywhere with relu2; times `scale` when not 0.  (GATED outputs take the factor alone; `scale` is not for SPLIT_GATED.) */
+ * after a factor per row (x_scale, with group_expert), `bias` (a float for each of the n_out
+ * outputs, batch 1) and an activation: SiLU for n < silu_end, else the logistic for n <
+ * sigmoid_end, else the hyperbolic tangent for n < tanh_end; square of ReLU everywhere with
+ * relu2; times `scale` when not 0.  (Gated outputs take the factor alone; `scale` is not for
+ * SPLIT_GATED.) */
 enum { WR_HIP_MIX_OUT_ROWS_F32 = 0, WR_HIP_MIX_OUT_ROWS = 1, WR_HIP_MIX_OUT_FRAG = 2,
        WR_HIP_MIX_OUT_SPLIT = 3, WR_HIP_MIX_OUT_GATED = 4, WR_HIP_MIX_OUT_SPLIT_GATED = 5 };
 typedef struct wr_hip_mix_gemm {

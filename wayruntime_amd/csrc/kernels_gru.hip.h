@@ -1,4 +1,4 @@
-// Gated recurrence element by element whose gates read the current token alone (minGRU):
+// Element-wise gated recurrence, gates and candidates made from the input and not from the state (minGRU):
 //
 //   S_t = (1 - z_t) S_(t-1) + z_t c_t      z = logistic(zl), c = u + 1/2 for u >= 0, else logistic(u)
 //   out = S_t * SiLU(g_t)
